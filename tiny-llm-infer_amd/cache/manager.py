@@ -77,12 +77,16 @@ class CacheNeed:
     """What one mixer needs of the paged cache: the records it keeps for every token and
     how far back its rows read (``window`` None: everything, else the last ``window``
     tokens, so that pages before the window can be given back; ``chunk``: only the positions
-    of its own block of that many, so that the pages of blocks that have passed can).  Cache
-    layers whose needs are equal share a group: page ids, block tables and tensors of their own."""
+    of its own block of that many, so that the pages of blocks that have passed can).  With a
+    ``stride`` above 1 a slot of a page stands for that many positions in a row (what is kept is
+    one thing a block of positions, such as the mean of its keys), so a page covers ``stride`` times
+    as many.  Cache layers whose needs are equal share a group: page ids, block tables and tensors
+    of their own.  A mixer may have several needs (``Mixer.cache_need`` gives a tuple of them)."""
     records: Tuple[CacheRecord, ...]
     window: Optional[int] = None
     chunk: Optional[int] = None          # rows read only inside their own block of ``chunk`` positions (counted from 0)
     keep_first: int = 0                  # with a window: the first so many positions of a sequence stay readable for ever
+    stride: int = 1                      # positions that one slot stands for
 
     def __post_init__(self):
         names = [r.name for r in self.records]
@@ -94,6 +98,8 @@ class CacheNeed:
             raise ValueError("a window or a chunk must be positive")
         if self.keep_first < 0 or (self.keep_first and self.window is None):
             raise ValueError("first positions are kept beside a window only, and their number cannot be negative")
+        if self.stride <= 0:
+            raise ValueError("a slot stands for at least one position")
 
     @property
     def keeps_all(self) -> bool:
@@ -104,6 +110,15 @@ class CacheNeed:
     def reach(self) -> Optional[int]:
         """A row reads fewer than this many positions back (None: any number)."""
         return self.window if self.window is not None else self.chunk
+
+    def page_span(self, page_size: int) -> int:
+        """The positions that one page covers."""
+        return page_size * self.stride
+
+    def pages_of_pool(self, num_pages: int, max_requests: int) -> int:
+        """The pages of a group that keeps all its slots when one with a slot a position has
+        ``num_pages``: as many positions, and the page that each request has begun."""
+        return num_pages if self.stride == 1 else _blocks(num_pages, self.stride) + max_requests
 
     def first_read(self, position: int) -> int:
         """The lowest position that a row at ``position``, or any later row, reads."""
@@ -229,8 +244,9 @@ class CacheManager:
             raise ValueError("page_size, num_pages and max_requests must be positive")
         distinct = group_needs(needs)
         if per_group is None:
-            per_group = [num_pages if (n.keeps_all or max_step_tokens is None) else
-                         min(num_pages, window_group_pages(n.reach, page_size, max_requests, max_step_tokens, n.keep_first))
+            per_group = [n.pages_of_pool(num_pages, max_requests) if (n.keeps_all or max_step_tokens is None) else
+                         min(n.pages_of_pool(num_pages, max_requests),
+                             window_group_pages(n.reach, n.page_span(page_size), max_requests, max_step_tokens, n.keep_first))
                          for n in distinct]
         if len(per_group) != len(distinct):
             raise ValueError(f"{len(per_group)} page counts for {len(distinct)} groups of cache layers")
@@ -250,13 +266,15 @@ class CacheManager:
                 self.groups.append(g)
             g.cache_layers.append(layer)
             self.group_of_layer[layer] = g.index
-        self._no_window = all(g.need.keeps_all for g in self.groups)
+        self._alike = all(g.need.keeps_all and g.need.stride == 1 for g in self.groups)    # every group's table grows alike
         self._free_slots = list(range(max_requests - 1, -1, -1))   # pop() gives the lowest
         self._live: Dict[Hashable, RequestCache] = {}
         self.pages_taken_total = 0
         self.pages_returned_total = 0
         if prefix_caching and any(not g.need.keeps_all for g in self.groups):
             raise ValueError("prefix caching needs every layer to keep all keys (no window)")
+        if prefix_caching and any(g.need.stride != 1 for g in self.groups):
+            raise ValueError("prefix caching needs a slot for every position in every group")
         self.prefix_caching = prefix_caching
         # per group: hash -> page, and per page its (hash, token ids) while it is in the cache
         self._page_of_hash: List[Dict[int, int]] = [dict() for _ in self.groups]
@@ -372,19 +390,23 @@ class CacheManager:
     # ---- pages ----------------------------------------------------------
     def _first_needed_block(self, g: GroupLayout, first_query_pos: int) -> int:
         """Lowest block a query at ``first_query_pos`` (and any later one) can read."""
-        return g.need.first_read(first_query_pos) // self.page_size
+        return g.need.first_read(first_query_pos) // self.span(g)
+
+    def span(self, g: GroupLayout) -> int:
+        """The positions that a page of the group covers."""
+        return g.need.page_span(self.page_size)
 
     def _kept_blocks(self, g: GroupLayout) -> int:
         """The leading blocks of a request that a window group never gives back: those of the first
         positions that every later row still reads."""
-        return _blocks(g.need.keep_first, self.page_size)
+        return _blocks(g.need.keep_first, self.span(g))
 
     def pages_needed(self, key: Hashable, new_total: int) -> List[int]:
         """Per group, pages that must be taken so that the request can run the
         tokens at positions [num_tokens, new_total)."""
         rc = self._live[key]
-        nb = _blocks(new_total, self.page_size)
-        if self._no_window:                   # (every step of every request comes through here: the short way)
+        if self._alike:                       # (every step of every request comes through here: the short way)
+            nb = _blocks(new_total, self.page_size)
             return [max(0, nb - len(table)) for table in rc.tables]
         out = []
         for gi, g in enumerate(self.groups):
@@ -392,7 +414,7 @@ class CacheManager:
             # held (``reserve`` filled them, ``advance`` gives back only what lies before): what is
             # missing are the blocks past the table's end
             first = self._first_needed_block(g, rc.num_tokens)
-            out.append(max(0, nb - max(first, len(rc.tables[gi]))))
+            out.append(max(0, _blocks(new_total, self.span(g)) - max(first, len(rc.tables[gi]))))
         return out
 
     def can_reserve(self, key: Hashable, new_total: int) -> bool:
@@ -403,22 +425,21 @@ class CacheManager:
         """Per group, the most pages one request of ``total_tokens`` tokens ever holds when it is
         run in portions of at most ``portion`` tokens: all its blocks where all keys are kept, the
         window's and a portion's where a window passes."""
-        whole = _blocks(total_tokens, self.page_size)
         out = []
         for g in self.groups:
+            whole, span = _blocks(total_tokens, self.span(g)), self.span(g)
             if g.need.keeps_all:
                 out.append(whole)
             else:
-                out.append(min(whole, _blocks(g.need.reach - 1, self.page_size) + 2 + self._kept_blocks(g)
-                               + _blocks(min(portion, total_tokens), self.page_size)))
+                out.append(min(whole, _blocks(g.need.reach - 1, span) + 2 + self._kept_blocks(g)
+                               + _blocks(min(portion, total_tokens), span)))
         return out
 
     def pages_per_group(self) -> List[int]:
         return [g.pool.num_pages for g in self.groups]
 
     def _ahead_needed(self, rc: RequestCache, total: int) -> List[int]:
-        nb = _blocks(total, self.page_size)
-        return [max(0, nb - len(rc.tables[gi])) if g.need.keeps_all else 0
+        return [max(0, _blocks(total, self.span(g)) - len(rc.tables[gi])) if g.need.keeps_all else 0
                 for gi, g in enumerate(self.groups)]
 
     def can_hold_ahead(self, key: Hashable, total: int) -> bool:
@@ -434,10 +455,9 @@ class CacheManager:
         rc = self._live[key]
         if not self.can_hold_ahead(key, total):
             raise CacheFull(f"not enough free pages to hold {total} tokens of {key!r}")
-        nb = _blocks(total, self.page_size)
         for gi, g in enumerate(self.groups):
             if g.need.keeps_all:
-                table = rc.tables[gi]
+                table, nb = rc.tables[gi], _blocks(total, self.span(g))
                 while len(table) < nb:
                     table.append(self._take(gi))
 
@@ -449,16 +469,15 @@ class CacheManager:
         if new_total < rc.num_tokens:
             raise ValueError("a request cannot shrink")
         needs = self.pages_needed(key, new_total)
-        if not any(needs) and self._no_window:            # a token that goes into a page already held
+        if not any(needs) and self._alike:                # a token that goes into a page already held
             if new_total > rc.reserved_tokens:
                 rc.reserved_tokens = new_total
             return
         if any(n > g.pool.free_count for n, g in zip(needs, self.groups)):
             raise CacheFull(f"not enough free pages to hold {new_total} tokens of {key!r}")
-        nb = _blocks(new_total, self.page_size)
         for gi, g in enumerate(self.groups):
             table = rc.tables[gi]
-            held = len(table)
+            held, nb = len(table), _blocks(new_total, self.span(g))
             first = self._first_needed_block(g, rc.num_tokens)
             while len(table) < min(first, nb):
                 table.append(-1)                  # (a window has jumped past these blocks)

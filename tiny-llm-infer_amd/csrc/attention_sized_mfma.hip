@@ -17,10 +17,14 @@
 // meanwhile, and their fragments are read from there; a value cache lies transposed ([dim][slot]), so that a lane's
 // four keys of one dim are 8 bytes (a tile of 16 keys lies inside one page: pages of 16 slots and more).
 //
+// POOLED variants walk, behind the window's tiles of keys, tiles of 16 pooled blocks (pooled.h), which lie in pages of
+// their own with a table of their own.
+//
 // The sizes are arguments, not template parameters, but for the common sizes, which have kernels of their own (EXACT
 // below): the registers for the query's fragments and the output's sums are those of the largest size of a variant
 // (keys up to 128 / 256 / 640 elements, values up to 128 / 256 / 512).
 #include "common.h"
+#include "pooled.h"
 
 typedef __attribute__((ext_vector_type(4))) short bf16x4;
 typedef __attribute__((ext_vector_type(4))) float f32x4;
@@ -62,13 +66,13 @@ __device__ __forceinline__ float asm_sink_factor(float sink, float m, float l) {
     return keys / (l * keys + __expf(sink - top));
 }
 
-template <int NKM, int NVM, bool VKEY, typename TO, bool EXACT>
+template <int NKM, int NVM, bool VKEY, typename TO, bool EXACT, bool POOLED>
 __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
     const bf16_t* __restrict__ q, TO* __restrict__ out, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ row_start, const int* __restrict__ seq_start,
     int num_seqs, const int* __restrict__ tables, int table_width, int page_size, int num_pages, int heads,
     int kv_heads, int maps, int nk_arg, int nv_arg, float scale, int window, int keep_first, int grouped, int col_groups,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, PooledKeys pooled, int out_ld, float out_scale) {
     const int nk = EXACT ? NKM : nk_arg, nv = EXACT ? NVM : nv_arg;
     const int DK = nk * 16, DV = nv * 16, LD = DK + ASM_PAD;
     const int pieces = 2 * nk;                                          // 16-byte pieces of one key
@@ -138,14 +142,27 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
     const int k_low = lo - lo % 16, k_top = hi - hi % 16;
     const int n_main = (k_top - k_low) / 16 + 1;
     const int n_kept = (min(kept_hi, k_low) + 15) / 16;
-    const int n_tiles = n_main + n_kept;
-    auto tile_key = [&](int i) { return i < n_main ? k_top - 16 * i : 16 * (i - n_main); };
+    const int n_tokens = n_main + n_kept;                                // tiles of tokens; those of blocks follow
+    const int blocks_hi = POOLED ? pooled_blocks_seen(hi, window, pooled.pool) : 0;      // of the tile's last row
+    const int blocks_my = POOLED ? pooled_blocks_seen(qpos, window, pooled.pool) : 0;
+    const int* block_table = POOLED ? pooled.tables + (size_t)seq * pooled.width : nullptr;
+    const int n_tiles = n_tokens + (blocks_hi + 15) / 16;
+    auto is_block = [&](int i) { return POOLED && i >= n_tokens; };
+    auto tile_key = [&](int i) {
+        return is_block(i) ? 16 * (i - n_tokens) : i < n_main ? k_top - 16 * i : 16 * (i - n_main);
+    };
 
     uint4 next[PASSES];
     // chunk c = 64 ps + lane is piece c % pieces of key c / pieces: one division a lane, then steps of 64 chunks
     const int key_first = lane / pieces, piece_first = lane - key_first * pieces;
     const int key_step = 64 / pieces, piece_step = 64 - key_step * pieces;
-    auto fetch = [&](int k0) {
+    auto fetch = [&](int i) {
+        const int k0 = tile_key(i);
+        const bool block = is_block(i);
+        const int* tab = block ? block_table : table;
+        const bf16_t* keys = block ? (const bf16_t*)pooled.k : k_cache;
+        const int all = block ? pooled.pages : num_pages;
+        const int t_lo = block ? 0 : lo, t_hi = block ? blocks_hi - 1 : hi, t_kept = block ? 0 : kept_hi;
         int ck = key_first, cp = piece_first;
 #pragma unroll
         for (int ps = 0; ps < PASSES; ++ps) {
@@ -153,10 +170,10 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
             next[ps] = make_uint4(0, 0, 0, 0);
             if (c < chunks) {
                 const int key = k0 + ck;
-                if (key <= hi && (key >= lo || key < kept_hi)) {
-                    const int page = table[key >> page_shift];
-                    if (page >= 0 && page < num_pages)
-                        next[ps] = *reinterpret_cast<const uint4*>(k_cache + (size_t)page * k_page +
+                if (key <= t_hi && (key >= t_lo || key < t_kept)) {
+                    const int page = tab[key >> page_shift];
+                    if (page >= 0 && page < all)
+                        next[ps] = *reinterpret_cast<const uint4*>(keys + (size_t)page * k_page +
                                                                    ((size_t)kh * page_size + (key & page_mask)) * DK + cp * 8);
                 }
             }
@@ -168,7 +185,7 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
             }
         }
     };
-    if (wave < n_tiles) fetch(tile_key(wave));
+    if (wave < n_tiles) fetch(wave);
     for (int it = wave; it < n_tiles; it += ASM_WAVES) {
         const int k0 = tile_key(it);
         {
@@ -185,16 +202,17 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
                 }
             }
         }
-        if (it + ASM_WAVES < n_tiles) fetch(tile_key(it + ASM_WAVES));
+        if (it + ASM_WAVES < n_tiles) fetch(it + ASM_WAVES);
+        const bool block = is_block(it);
         // the values of this tile's keys from their own cache: dim 16 j + col of the keys k0 + 4 grp + i
         SFrag4 vf[VKEY ? 1 : NVM];
         if (!VKEY) {
             const int key = k0 + grp * 4;
             const bf16_t* vp = nullptr;
-            if (key <= hi && (key + 3 >= lo || key < kept_hi)) {
-                const int page = table[key >> page_shift];
-                if (page >= 0 && page < num_pages)
-                    vp = v_cache + (size_t)page * v_page + ((size_t)g * DV + col) * page_size + (key & page_mask);
+            if (block ? key < blocks_hi : key <= hi && (key + 3 >= lo || key < kept_hi)) {
+                const int page = (block ? block_table : table)[key >> page_shift];
+                if (page >= 0 && page < (block ? pooled.pages : num_pages))
+                    vp = (block ? (const bf16_t*)pooled.v : v_cache) + (size_t)page * v_page + ((size_t)g * DV + col) * page_size + (key & page_mask);
             }
 #pragma unroll
             for (int j = 0; j < NVM; ++j) {
@@ -223,10 +241,11 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
         SFrag4 p;
         float w[4];
         float mx = -INFINITY;
+        const int s_hi = block ? blocks_my - 1 : qpos, s_lo = block ? 0 : qlo;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int key = k0 + grp * 4 + i;
-            const bool seen = key <= qpos && (key >= qlo || key < keep_first);
+            const bool seen = key <= s_hi && (key >= s_lo || key < keep_first);
             w[i] = seen ? s[i] * scale : -INFINITY;
             mx = fmaxf(mx, w[i]);
         }
@@ -295,8 +314,8 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
     if (col >= live_cols) return;
     float inv = lt > 0.f ? 1.0f / lt : 0.f;
     if (sinks) inv = asm_sink_factor(sinks[unit], mt, lt);
-    int out_unit = unit, out_row = row0 + my;
-    TO* o_row = out + ((size_t)out_row * units + out_unit) * DV;
+    inv *= out_scale;
+    TO* o_row = out + (size_t)(row0 + my) * out_ld + (size_t)unit * DV;
 #pragma unroll
     for (int j = 0; j < NVM; ++j) {
         if (j < nv) {
@@ -334,13 +353,13 @@ static inline size_t ast_lds_bytes(int DK, int DV) {
     return 2 * ((size_t)16 * (DK + ASM_PAD) + (size_t)DV * AST_VLD) * 2;
 }
 
-template <int NKM, int NVM, bool VKEY, typename TO, bool EXACT, int WAVES>
+template <int NKM, int NVM, bool VKEY, typename TO, bool EXACT, int WAVES, bool POOLED>
 __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
     const bf16_t* __restrict__ q, TO* __restrict__ out, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, const int* __restrict__ row_start, const int* __restrict__ seq_start,
     int num_seqs, const int* __restrict__ tables, int table_width, int page_size, int num_pages, int heads,
     int kv_heads, int maps, int nk_arg, int nv_arg, float scale, int window, int keep_first, int grouped,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, PooledKeys pooled, int out_ld, float out_scale) {
     const int nk = EXACT ? NKM : nk_arg, nv = EXACT ? NVM : nv_arg;
     const int DK = nk * 16, DV = nv * 16, LD = DK + ASM_PAD;
     const int pieces = 2 * nk;                                          // 16-byte pieces of one key
@@ -417,17 +436,27 @@ __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
     const int k_low = lo - lo % 16, k_top = hi - hi % 16;
     const int n_main = (k_top - k_low) / 16 + 1;
     const int n_kept = (min(kept_hi, k_low) + 15) / 16;
-    const int n_tiles = n_main + n_kept;
-    auto tile_key = [&](int i) { return i < n_main ? k_top - 16 * i : 16 * (i - n_main); };
+    const int n_tokens = n_main + n_kept;                               // tiles of tokens; those of blocks follow
+    const int blocks_hi = POOLED ? pooled_blocks_seen(hi, window, pooled.pool) : 0;      // of the workgroup's last row
+    const int blocks_w = POOLED ? pooled_blocks_seen(w_hi, window, pooled.pool) : 0;     // of the wave's
+    const int blocks_my = POOLED ? pooled_blocks_seen(qpos, window, pooled.pool) : 0;
+    const int* block_table = POOLED ? pooled.tables + (size_t)seq * pooled.width : nullptr;
+    const int n_tiles = n_tokens + (blocks_hi + 15) / 16;
+    auto is_block = [&](int i) { return POOLED && i >= n_tokens; };
+    auto tile_key = [&](int i) {
+        return is_block(i) ? 16 * (i - n_tokens) : i < n_main ? k_top - 16 * i : 16 * (i - n_main);
+    };
 
     const int kk = tid % 16, p0 = tid / 16;                             // this thread's key of a tile, its first piece
     uint4 next_k[KPASS];
     uint4 next_v[VPASS];
-    auto fetch = [&](int k0) {
+    auto fetch = [&](int i) {
         // (a tile of 16 keys lies inside one page)
-        const int page = table[k0 >> page_shift];
-        const bool there = page >= 0 && page < num_pages;
-        const bf16_t* src = k_cache + (size_t)(there ? page : 0) * k_page + ((size_t)kh * page_size + ((k0 + kk) & page_mask)) * DK;
+        const int k0 = tile_key(i);
+        const bool block = is_block(i);
+        const int page = (block ? block_table : table)[k0 >> page_shift];
+        const bool there = page >= 0 && page < (block ? pooled.pages : num_pages);
+        const bf16_t* src = (block ? (const bf16_t*)pooled.k : k_cache) + (size_t)(there ? page : 0) * k_page + ((size_t)kh * page_size + ((k0 + kk) & page_mask)) * DK;
 #pragma unroll
         for (int ps = 0; ps < KPASS; ++ps) {
             const int p = ps * (4 * WAVES) + p0;
@@ -435,7 +464,7 @@ __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
             if (there && p < pieces) next_k[ps] = *reinterpret_cast<const uint4*>(src + p * 8);
         }
         if (!VKEY) {
-            const bf16_t* vsrc = v_cache + (size_t)(there ? page : 0) * v_page + (size_t)g * DV * page_size + (k0 & page_mask);
+            const bf16_t* vsrc = (block ? (const bf16_t*)pooled.v : v_cache) + (size_t)(there ? page : 0) * v_page + (size_t)g * DV * page_size + (k0 & page_mask);
 #pragma unroll
             for (int ps = 0; ps < VPASS; ++ps) {
                 const int c = ps * (64 * WAVES) + tid;                           // dim c / 2, keys 8 (c % 2) .. + 7 of the tile
@@ -473,16 +502,18 @@ __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
         }
     };
 
-    fetch(tile_key(0));
+    fetch(0);
     store(lds);
     __syncthreads();
     for (int it = 0; it < n_tiles; ++it) {
         const int k0 = tile_key(it);
         const bool more = it + 1 < n_tiles;
-        if (more) fetch(tile_key(it + 1));
+        if (more) fetch(it + 1);
+        const bool block = is_block(it);
         const bf16_t* kt = lds + (size_t)(it & 1) * buf_elems;
         const bf16_t* vt = kt + (size_t)16 * LD;
-        if (stores && k0 <= w_hi && (k0 + 15 >= w_lo || k0 < keep_first)) {   // (the same for the whole wave)
+        // (the same for the whole wave)
+        if (stores && (block ? k0 < blocks_w : k0 <= w_hi && (k0 + 15 >= w_lo || k0 < keep_first))) {
             // scores, transposed: A = the key k0 + col, this lane group's dims; two sums in turn, so that a matrix
             // instruction does not wait for the one before it
             f32x4 s = (f32x4){0.f, 0.f, 0.f, 0.f}, s_odd = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -501,10 +532,11 @@ __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
             SFrag4 p;
             float w[4];
             float mx = -INFINITY;
+            const int s_hi = block ? blocks_my - 1 : qpos, s_lo = block ? 0 : qlo;
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int key = k0 + grp * 4 + i;
-                const bool seen = key <= qpos && (key >= qlo || key < keep_first);
+                const bool seen = key <= s_hi && (key >= s_lo || key < keep_first);
                 w[i] = seen ? (s[i] + s_odd[i]) * scale : -INFINITY;
                 mx = fmaxf(mx, w[i]);
             }
@@ -541,7 +573,8 @@ __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
     if (!stores || col >= live) return;
     float inv = l > 0.f ? 1.0f / l : 0.f;
     if (sinks) inv = asm_sink_factor(sinks[unit], m, l);
-    TO* o_row = out + ((size_t)row * units + unit) * DV;
+    inv *= out_scale;
+    TO* o_row = out + (size_t)row * out_ld + (size_t)unit * DV;
 #pragma unroll
     for (int j = 0; j < NVM; ++j)
         if (j < nv) asm_store4(o_row + j * 16 + grp * 4, acc[j], inv);
@@ -555,16 +588,11 @@ extern "C" int tli_attention_sized_mfma_takes(int key_dim, int value_dim, int pa
     return 1;
 }
 
-// q [rows, heads * maps, key_dim]; out [rows, heads * maps, value_dim] (float32 with out_f32, else bfloat16);
-// k_cache [pages][kv_heads * maps][slot][key_dim]; v_cache [pages][kv_heads][value_dim][slot] or null;
-// tiles: an upper bound of the sum over the sequences of ceil(rows / 16) (of the rows, with `grouped`);
-// grouped: a tile is one row and its columns are the query heads of one key head, 16 at a time;
-// sinks: float32 [heads * maps] or null
-extern "C" int tli_attention_sized_mfma_bf16(
+static int run_sized_mfma(
     const void* q, void* out, const void* k_cache, const void* v_cache, const int* row_start, const int* seq_start,
     int num_seqs, int tiles, const int* tables, int table_width, int page_size, int num_pages, int heads, int kv_heads,
     int maps, int key_dim, int value_dim, float scale, int window, int keep_first, int grouped, int out_f32,
-    const float* sinks, void* stream) {
+    const float* sinks, const PooledKeys& pooled, int out_ld, float out_scale, void* stream) {
     if (num_seqs <= 0 || tiles <= 0) return 0;
     if (!tli_attention_sized_mfma_takes(key_dim, value_dim, page_size, v_cache != nullptr))
         return tli_fail("attention: the matrix-core kernel does not take keys of %d and values of %d in pages of %d", key_dim,
@@ -572,6 +600,7 @@ extern "C" int tli_attention_sized_mfma_bf16(
     if (heads <= 0 || kv_heads <= 0 || heads % kv_heads || maps <= 0)
         return tli_fail("attention: heads %d must be a multiple of kv heads %d", heads, kv_heads);
     if (table_width <= 0 || num_pages <= 0) return tli_fail("attention: bad cache geometry");
+    if (out_ld < heads * maps * value_dim || out_ld % 4) return tli_fail("attention: output rows of %d elements", out_ld);
     if (window < 0 || keep_first < 0) return tli_fail("attention: bad window %d with %d kept", window, keep_first);
     if ((((uintptr_t)q | (uintptr_t)out | (uintptr_t)k_cache | (uintptr_t)v_cache) & 15))
         return tli_fail("attention: operands must be 16-byte aligned");
@@ -594,9 +623,10 @@ extern "C" int tli_attention_sized_mfma_bf16(
         if (wgs > 0x7fffffffLL || kv_heads * maps > 65535) return tli_fail("attention: too many tiles for one launch");
         const dim3 sgrid((unsigned)wgs, (unsigned)(kv_heads * maps));
         const size_t sbytes = ast_lds_bytes(key_dim, value_dim);
-#define AST_ONE(NKM, NVM, VKEY, TO, EXACT, WAVES)                                                                                        \
+#define AST_ONE(NKM, NVM, VKEY, TO, EXACT, WAVES) AST_RUN(NKM, NVM, VKEY, TO, EXACT, WAVES, false)
+#define AST_RUN(NKM, NVM, VKEY, TO, EXACT, WAVES, POOLED)                                                                  \
     {                                                                                                                      \
-        auto kernel = attention_sized_shared_kernel<NKM, NVM, VKEY, TO, EXACT, WAVES>;                                                   \
+        auto kernel = attention_sized_shared_kernel<NKM, NVM, VKEY, TO, EXACT, WAVES, POOLED>;                                                   \
         static bool allowed = false;                                                                                       \
         if (sbytes > 65536 && !allowed) {                                                                                  \
             if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) !=        \
@@ -606,7 +636,7 @@ extern "C" int tli_attention_sized_mfma_bf16(
         }                                                                                                                  \
         kernel<<<sgrid, 64 * WAVES, sbytes, s>>>((const bf16_t*)q, (TO*)out, (const bf16_t*)k_cache, (const bf16_t*)v_cache,      \
                                           row_start, seq_start, num_seqs, tables, table_width, page_size, num_pages,      \
-                                          heads, kv_heads, maps, nk, nv, scale, window, keep_first, grouped, sinks);      \
+                                          heads, kv_heads, maps, nk, nv, scale, window, keep_first, grouped, sinks, pooled, out_ld, out_scale); \
     }
 #define AST_SIZES(VKEY, TO)                                                   \
     if (nk <= 8 && nv <= 8) AST_ONE(8, 8, VKEY, TO, false, 4)                 \
@@ -614,7 +644,13 @@ extern "C" int tli_attention_sized_mfma_bf16(
     else AST_ONE(40, 32, VKEY, TO, false, 4)
         // (sizes with a kernel of their own: heads of 64 and 128 with values of 64 to 256 in float32, for the
         // attention with two maps; a latent vector of 512 beside a turned part of 64)
-        if (v_cache && out_f32 && nk == 4 && nv == 4) AST_ONE(4, 4, false, float, true, 4)
+        if (pooled.pool > 0) {
+            if (nk == 8 && nv == 8) AST_RUN(8, 8, false, bf16_t, true, 4, true)
+            else if (nk == 4 && nv == 4) AST_RUN(4, 4, false, bf16_t, true, 4, true)
+            else if (nk <= 8 && nv <= 8) AST_RUN(8, 8, false, bf16_t, false, 4, true)
+            else if (nk <= 16 && nv <= 16) AST_RUN(16, 16, false, bf16_t, false, 4, true)
+            else AST_RUN(40, 32, false, bf16_t, false, 4, true)
+        } else if (v_cache && out_f32 && nk == 4 && nv == 4) AST_ONE(4, 4, false, float, true, 4)
         else if (v_cache && out_f32 && nk == 4 && nv == 8) AST_ONE(4, 8, false, float, true, 4)
         else if (v_cache && out_f32 && nk == 8 && nv == 8) AST_ONE(8, 8, false, float, true, 4)
         else if (v_cache && out_f32 && nk == 8 && nv == 16) AST_ONE(8, 16, false, float, true, 4)
@@ -627,15 +663,17 @@ extern "C" int tli_attention_sized_mfma_bf16(
         }
 #undef AST_SIZES
 #undef AST_ONE
+#undef AST_RUN
         return tli_check_launch("attention_sized_shared");
     }
     const dim3 grid(tiles, (unsigned)gy);
     const size_t bytes = asm_lds_bytes(key_dim, value_dim);
 #define ASM_ARGS (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, row_start, seq_start, num_seqs, tables, \
         table_width, page_size, num_pages, heads, kv_heads, maps, nk, nv, scale, window, keep_first, grouped, col_groups
-#define ASM_ONE(NKM, NVM, VKEY, TO, EXACT)                                                                                        \
+#define ASM_ONE(NKM, NVM, VKEY, TO, EXACT) ASM_RUN(NKM, NVM, VKEY, TO, EXACT, false)
+#define ASM_RUN(NKM, NVM, VKEY, TO, EXACT, POOLED)                                                                         \
     {                                                                                                                      \
-        auto kernel = attention_sized_mfma_kernel<NKM, NVM, VKEY, TO, EXACT>;                                                     \
+        auto kernel = attention_sized_mfma_kernel<NKM, NVM, VKEY, TO, EXACT, POOLED>;                                                     \
         static bool allowed = false;                                                                                       \
         if (bytes > 65536 && !allowed) {                                                                                   \
             if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) !=        \
@@ -646,19 +684,57 @@ extern "C" int tli_attention_sized_mfma_bf16(
         kernel<<<grid, 64 * ASM_WAVES, bytes, s>>>((const bf16_t*)q, (TO*)out, (const bf16_t*)k_cache,                      \
                                                    (const bf16_t*)v_cache, row_start, seq_start, num_seqs, tables,         \
                                                    table_width, page_size, num_pages, heads, kv_heads, maps, nk, nv,       \
-                                                   scale, window, keep_first, grouped, col_groups, sinks);                 \
+                                                   scale, window, keep_first, grouped, col_groups, sinks, pooled, out_ld,  \
+                                                   out_scale);                                                             \
     }
 #define ASM_SIZES(VKEY, TO)                                                   \
     if (nk <= 8 && nv <= 8) ASM_ONE(8, 8, VKEY, TO, false)                    \
     else if (nk <= 16 && nv <= 16) ASM_ONE(16, 16, VKEY, TO, false)           \
     else ASM_ONE(40, 32, VKEY, TO, false)
-    if (out_f32 && nk == 4 && nv == 4) ASM_ONE(4, 4, false, float, true)
+    if (pooled.pool > 0) {
+        if (nk == 8 && nv == 8) ASM_RUN(8, 8, false, bf16_t, true, true)
+        else if (nk == 4 && nv == 4) ASM_RUN(4, 4, false, bf16_t, true, true)
+        else if (nk <= 8 && nv <= 8) ASM_RUN(8, 8, false, bf16_t, false, true)
+        else if (nk <= 16 && nv <= 16) ASM_RUN(16, 16, false, bf16_t, false, true)
+        else ASM_RUN(40, 32, false, bf16_t, false, true)
+    } else if (out_f32 && nk == 4 && nv == 4) ASM_ONE(4, 4, false, float, true)
     else if (out_f32 && nk == 4 && nv == 8) ASM_ONE(4, 8, false, float, true)
     else if (out_f32 && nk == 8 && nv == 8) ASM_ONE(8, 8, false, float, true)
     else if (out_f32 && nk == 8 && nv == 16) ASM_ONE(8, 16, false, float, true)
     else if (out_f32) { ASM_SIZES(false, float) } else { ASM_SIZES(false, bf16_t) }
 #undef ASM_SIZES
 #undef ASM_ONE
+#undef ASM_RUN
 #undef ASM_ARGS
     return tli_check_launch("attention_sized_mfma");
+}
+
+// q [rows, heads * maps, key_dim]; out [rows, heads * maps, value_dim] (float32 with out_f32, else bfloat16);
+// k_cache [pages][kv_heads * maps][slot][key_dim]; v_cache [pages][kv_heads][value_dim][slot] or null;
+// tiles: an upper bound of the sum over the sequences of ceil(rows / 16) (of the rows, with `grouped`);
+// grouped: a tile is one row and its columns are the query heads of one key head, 16 at a time;
+// sinks: float32 [heads * maps] or null
+extern "C" int tli_attention_sized_mfma_bf16(
+    const void* q, void* out, const void* k_cache, const void* v_cache, const int* row_start, const int* seq_start,
+    int num_seqs, int tiles, const int* tables, int table_width, int page_size, int num_pages, int heads, int kv_heads,
+    int maps, int key_dim, int value_dim, float scale, int window, int keep_first, int grouped, int out_f32,
+    const float* sinks, void* stream) {
+    return run_sized_mfma(q, out, k_cache, v_cache, row_start, seq_start, num_seqs, tiles, tables, table_width, page_size,
+                          num_pages, heads, kv_heads, maps, key_dim, value_dim, scale, window, keep_first, grouped, out_f32, sinks,
+                          PooledKeys{}, heads * maps * value_dim, 1.0f, stream);
+}
+
+// The same over a window and the pooled blocks before it (pooled.h; their caches hold kv_heads heads): one map, values of
+// their own, bfloat16 output rows out_ld elements apart (a multiple of 4) and times out_scale.
+extern "C" int tli_attention_pooled_mfma_bf16(
+    const void* q, void* out, const void* k_cache, const void* v_cache, const int* row_start, const int* seq_start,
+    int num_seqs, int tiles, const int* tables, int table_width, int page_size, int num_pages, int heads, int kv_heads,
+    int key_dim, int value_dim, float scale, int window, const void* pooled_k, const void* pooled_v, const int* pooled_tables,
+    int pooled_width, int pooled_pages, int pool, int grouped, const float* sinks, int out_ld, float out_scale, void* stream) {
+    if (window <= 0 || pool <= 0 || pooled_width <= 0 || pooled_pages <= 0 || !v_cache)
+        return tli_fail("attention: blocks of %d beside a window of %d", pool, window);
+    if (((uintptr_t)pooled_k | (uintptr_t)pooled_v) & 15) return tli_fail("attention: operands must be 16-byte aligned");
+    return run_sized_mfma(q, out, k_cache, v_cache, row_start, seq_start, num_seqs, tiles, tables, table_width, page_size,
+                          num_pages, heads, kv_heads, 1, key_dim, value_dim, scale, window, 0, grouped, 0, sinks,
+                          PooledKeys{pooled_k, pooled_v, pooled_tables, pooled_width, pooled_pages, pool}, out_ld, out_scale, stream);
 }

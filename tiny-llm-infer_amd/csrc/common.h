@@ -84,6 +84,35 @@ __device__ __forceinline__ float gated_unit(float g, float u, float limit, float
     return g / (1.0f + expf(-slope * g)) * (u + 1.0f);
 }
 
+// The output of a gated product: act(g) * u * scale from the sums g and u of a gate row and an up row, act the silu
+// (`act` 0) or the tanh form of gelu (1), rows `ld` elements apart.  (tanh form: 0.5 z (1 + tanh(t / 2)) with
+// t = 2 sqrt(2 / pi) (z + 0.044715 z^3), which is z / (1 + exp(-t)); silu is the same with t = z.)
+#define TLI_ACT_SILU 0
+#define TLI_ACT_GELU_TANH 1
+struct GateOut {
+    int on;                                  // 0: not a gated product
+    int act;
+    float scale;
+    int ld;
+    __host__ __device__ operator int() const { return on; }
+};
+__device__ __forceinline__ float gate_exponent(float z, int act) {
+    return act == TLI_ACT_GELU_TANH ? z * fmaf(0.07135481282552725f, z * z, 1.5957691216057308f) : z;
+}
+__device__ __forceinline__ float gate_unit(float g, float u, const GateOut& out) {
+    return g / (1.0f + expf(-gate_exponent(g, out.act))) * u * out.scale;
+}
+// (`ld` 0: the rows lie close together, `cols` elements each)
+static inline GateOut gate_out(int gated, int act, float scale, int ld, int cols) {
+    return GateOut{gated, act, scale, ld > 0 ? ld : cols};
+}
+// null if the output can be written
+static inline const char* gate_out_fault(const GateOut& g, int cols) {
+    if (g.on && (g.act < TLI_ACT_SILU || g.act > TLI_ACT_GELU_TANH)) return "unknown activation of a gated product";
+    if (g.on && g.ld < cols) return "the rows of a gated product's output overlap";
+    return nullptr;
+}
+
 // Makes LDS writes of this wavefront's lanes visible to its other lanes.
 __device__ __forceinline__ void wave_lds_sync() {
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");

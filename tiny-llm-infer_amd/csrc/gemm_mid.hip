@@ -46,7 +46,7 @@ union Pack16m {
 template <int RT, int WAVES, int DEPTH, int MT, typename TO, bool GATED>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* __restrict__ y,
-                float* __restrict__ part, int M_all, int N, int K, int splits, int steps_per_split) {
+                float* __restrict__ part, int M_all, int N, int K, int splits, int steps_per_split, GateOut gate) {
     constexpr int ROWS = MT * 16;
     constexpr int STAGES = DEPTH + 1;                        // W: DEPTH slices on their way, one in use
     constexpr int XSLOTS = DEPTH + 2;                        // x: one slice further ahead
@@ -233,7 +233,7 @@ gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* 
     }
     if (GATED) {
         const int n_out = N / 2;
-        y += (size_t)row0 * n_out;
+        y += (size_t)row0 * gate.ld;
 #pragma unroll
         for (int t = 0; t + 1 < RT; t += 2) {
             const int n0 = ((tile0 + t) / 2) * 16 + 4 * c;
@@ -245,9 +245,9 @@ gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* 
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const float g = acc[t][m][i], u = acc[t + 1][m][i];
-                    o[i] = g / (1.0f + expf(-g)) * u;
+                    o[i] = gate_unit(g, u, gate);
                 }
-                store4(y + (size_t)row * n_out + n0, o, n_out - n0, (n_out & 3) == 0);
+                store4(y + (size_t)row * gate.ld + n0, o, n_out - n0, (gate.ld & 3) == 0);
             }
         }
         return;
@@ -268,7 +268,7 @@ gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* 
 
 template <int RT, int WAVES, int DEPTH, int MT>
 static int launch_mid_rows(const bf16_t* x, const bf16_t* w, void* y, float* part, int M, int N, int K,
-                           int y_dtype, int gated, int splits, hipStream_t s) {
+                           int y_dtype, GateOut gated, int splits, hipStream_t s) {
     const int n_tiles = (N + 15) / 16, k_steps = (K + 127) / 128;
     const int steps_per_split = (k_steps + splits - 1) / splits;
     const int groups = (n_tiles + RT * WAVES - 1) / (RT * WAVES), row_blocks = (M + MT * 16 - 1) / (MT * 16);
@@ -285,7 +285,7 @@ static int launch_mid_rows(const bf16_t* x, const bf16_t* w, void* y, float* par
                 return tli_fail("gemm_mid: cannot have %zu bytes of LDS", lds);                            \
             allowed = true;                                                                                \
         }                                                                                                  \
-        kernel<<<grid, WAVES * 64, lds, s>>>(x, w, (TO*)y, part, M, N, K, splits, steps_per_split);        \
+        kernel<<<grid, WAVES * 64, lds, s>>>(x, w, (TO*)y, part, M, N, K, splits, steps_per_split, gated); \
     }
     if (gated) MID_LAUNCH(bf16_t, true)
     else if (y_dtype == TLI_BF16) MID_LAUNCH(bf16_t, false)
@@ -303,7 +303,7 @@ static int launch_mid_rows(const bf16_t* x, const bf16_t* w, void* y, float* par
 // Four 16-row tiles of x up to 64 rows, eight beyond.
 template <int RT, int WAVES, int DEPTH>
 static int launch_mid(const bf16_t* x, const bf16_t* w, void* y, float* part, int M, int N, int K,
-                      int y_dtype, int gated, int splits, hipStream_t s) {
+                      int y_dtype, GateOut gated, int splits, hipStream_t s) {
     if (M <= 64) return launch_mid_rows<RT, WAVES, DEPTH, 4>(x, w, y, part, M, N, K, y_dtype, gated, splits, s);
     if constexpr (DEPTH <= 3)       // (DEPTH + 2) slices of 32 KiB fit the 160 KiB of LDS
         return launch_mid_rows<RT, WAVES, DEPTH, 8>(x, w, y, part, M, N, K, y_dtype, gated, splits, s);
@@ -402,9 +402,13 @@ extern "C" int tli_gemm_mid_splits_rows(int M, int N, int K, int gated) {
 // splits > 1 (splits as returned by tli_gemm_mid_splits, or forced by the caller); with
 // y null the partial sums [splits][M][N] are left for the consumer to add (tli_gemm_mid_reduce,
 // or tli_add_rmsnorm);
-// cfg 0 picks the launch shape, else DEPTH*100 + RT*10 + WAVES.
+// cfg 0 picks the launch shape, else DEPTH*100 + RT*10 + WAVES.  act, act_scale, y_ld: the output of a gated product
+// (common.h's GateOut; y_ld 0: N/2).
 extern "C" int tli_gemm_mid_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K,
-                                 int y_dtype, int gated, int splits, int cfg, void* stream) {
+                                 int y_dtype, int is_gated, int splits, int cfg, int act, float act_scale, int y_ld,
+                                 void* stream) {
+    const GateOut gated = gate_out(is_gated, act, act_scale, y_ld, N / 2);
+    if (const char* fault = gate_out_fault(gated, N / 2)) return tli_fail("gemm_mid: %s", fault);
     if (M <= 0 || N <= 0) return 0;
     if (M > MID_MAX_ROWS || (gated && M > 128))
         return tli_fail("gemm_mid: %d rows, at most %d (%d for a gated product)", M, MID_MAX_ROWS, 128);
@@ -447,8 +451,8 @@ extern "C" int tli_gemm_mid_reduce(const float* part, void* y, int M, int N, int
     if (M <= 0 || N <= 0) return 0;
     if (!part || !y || splits < 1) return tli_fail("gemm_mid_reduce: bad arguments");
     hipStream_t s = (hipStream_t)stream;
-    if (y_dtype == TLI_BF16) launch_gemm_reduce(part, (bf16_t*)y, M, N, splits, 0, s);
-    else if (y_dtype == TLI_F32) launch_gemm_reduce(part, (float*)y, M, N, splits, 0, s);
+    if (y_dtype == TLI_BF16) launch_gemm_reduce(part, (bf16_t*)y, M, N, splits, GateOut{}, s);
+    else if (y_dtype == TLI_F32) launch_gemm_reduce(part, (float*)y, M, N, splits, GateOut{}, s);
     else return tli_fail("gemm_mid_reduce: bad output dtype %d", y_dtype);
     return tli_check_launch("gemm_mid_reduce");
 }

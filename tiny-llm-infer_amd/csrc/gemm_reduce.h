@@ -7,7 +7,7 @@
 // gate column (j/16)*32 + j%16 and up column 16 further.
 template <typename TO>
 __global__ void gemm_mid_reduce_kernel(const float* __restrict__ part, TO* __restrict__ y, int M, int N,
-                                       int splits, int gated) {
+                                       int splits, GateOut gated) {
     const int n_out = gated ? N / 2 : N;
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= (size_t)M * n_out) return;
@@ -20,7 +20,7 @@ __global__ void gemm_mid_reduce_kernel(const float* __restrict__ part, TO* __res
             g += part[s * plane + (size_t)row * N + gcol];
             u += part[s * plane + (size_t)row * N + gcol + 16];
         }
-        from_f32(y + idx, g / (1.0f + expf(-g)) * u);
+        from_f32(y + (size_t)row * gated.ld + j, gate_unit(g, u, gated));
     } else {
         float v = 0.f;
         for (int s = 0; s < splits; ++s) v += part[s * plane + (size_t)row * N + j];
@@ -32,7 +32,7 @@ __global__ void gemm_mid_reduce_kernel(const float* __restrict__ part, TO* __res
 // 16-byte load a plane and one store.
 template <typename TO>
 __global__ void gemm_mid_reduce4_kernel(const float* __restrict__ part, TO* __restrict__ y, int M, int N,
-                                        int splits, int gated) {
+                                        int splits, GateOut gated) {
     const int n_out = gated ? N / 2 : N, quads = n_out / 4;
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= (size_t)M * quads) return;
@@ -49,7 +49,7 @@ __global__ void gemm_mid_reduce4_kernel(const float* __restrict__ part, TO* __re
             u[0] += b.x; u[1] += b.y; u[2] += b.z; u[3] += b.w;
         }
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o[i] = g[i] / (1.0f + expf(-g[i])) * u[i];
+        for (int i = 0; i < 4; ++i) o[i] = gate_unit(g[i], u[i], gated);
     } else {
         o[0] = o[1] = o[2] = o[3] = 0.f;
         for (int s = 0; s < splits; ++s) {
@@ -57,14 +57,14 @@ __global__ void gemm_mid_reduce4_kernel(const float* __restrict__ part, TO* __re
             o[0] += a.x; o[1] += a.y; o[2] += a.z; o[3] += a.w;
         }
     }
-    store4(y + (size_t)row * n_out + j, o, 4, true);
+    store4(y + (size_t)row * (gated ? gated.ld : n_out) + j, o, 4, true);
 }
 
 // Launches the pass: four columns a thread where the sizes and addresses allow it.
 template <typename TO>
-static inline void launch_gemm_reduce(const float* part, TO* y, int M, int N, int splits, int gated, hipStream_t s) {
+static inline void launch_gemm_reduce(const float* part, TO* y, int M, int N, int splits, GateOut gated, hipStream_t s) {
     const int n_out = gated ? N / 2 : N;
-    if (N % 4 == 0 && n_out % 4 == 0 && !(((uintptr_t)part | (uintptr_t)y) & 15)) {
+    if (N % 4 == 0 && n_out % 4 == 0 && (!gated || gated.ld % 4 == 0) && !(((uintptr_t)part | (uintptr_t)y) & 15)) {
         const size_t total = (size_t)M * (n_out / 4);
         gemm_mid_reduce4_kernel<TO><<<(unsigned)((total + 255) / 256), 256, 0, s>>>(part, y, M, N, splits, gated);
     } else {

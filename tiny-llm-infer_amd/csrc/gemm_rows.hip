@@ -76,7 +76,7 @@ __device__ __forceinline__ void rows_wait_fragments(Pack16r (&a)[RT][4], int j) 
 template <int RT, int WAVES, int MT, int MH, bool GATED, int KG = 1>
 __global__ void __launch_bounds__(WAVES * KG * 64, WAVES * KG == 4 ? 2 : 1)
 gemm_rows_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf16_t* __restrict__ y,
-                 float* __restrict__ part, int M, int N, int K, int splits, int slices_per_split) {
+                 float* __restrict__ part, int M, int N, int K, int splits, int slices_per_split, GateOut out) {
     constexpr int ROWS = MT * 16;
     constexpr int SLICE = ROWS * 128;                        // elements of a slice of x
     constexpr int XI = ROWS / (4 * WAVES);                   // copies a wave issues for a slice (64 x 16 bytes each)
@@ -123,7 +123,7 @@ gemm_rows_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf1
     }
     x += (size_t)row_block * ROWS * K;
     const int n_out = GATED ? N / 2 : N;
-    y += (size_t)row_block * ROWS * n_out;
+    y += (size_t)row_block * ROWS * (GATED ? out.ld : N);
     // with splits > 1 the workgroup walks one of `splits` ranges of k and leaves float32 partial sums
     part += ((size_t)blockIdx.y * M + (size_t)row_block * ROWS) * N;
     M = min(ROWS, M - row_block * ROWS);
@@ -311,10 +311,10 @@ gemm_rows_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf1
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
                     const float g = gate[m][i], u = up[m][i];
-                    o[i] = g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * g)) * u;
+                    o[i] = g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * gate_exponent(g, out.act))) * u * out.scale;
                 }
-                bf16_t* dst = y + (size_t)row * n_out + n0;
-                if (n0 + 3 < n_out && n_out % 4 == 0) {
+                bf16_t* dst = y + (size_t)row * out.ld + n0;
+                if (n0 + 3 < n_out && out.ld % 4 == 0) {
                     *reinterpret_cast<uint2*>(dst) = make_uint2(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]));
                 } else {
 #pragma unroll
@@ -373,7 +373,7 @@ gemm_rows_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf1
 }
 
 template <int RT, int WAVES, int MT, int MH, int KG = 1>
-static int launch_rows(const bf16_t* x, const bf16_t* w, bf16_t* y, float* part, int M, int N, int K, int gated,
+static int launch_rows(const bf16_t* x, const bf16_t* w, bf16_t* y, float* part, int M, int N, int K, GateOut gated,
                        int splits, hipStream_t s) {
     const int n_tiles = (N + 15) / 16, k_steps = (K + 127) / 128;
     const long col_groups = (n_tiles + RT * WAVES - 1) / (RT * WAVES), row_blocks = (M + MT * 16 - 1) / (MT * 16);
@@ -397,7 +397,7 @@ static int launch_rows(const bf16_t* x, const bf16_t* w, bf16_t* y, float* part,
                 return tli_fail("gemm_rows: cannot have %zu bytes of LDS", lds);                           \
             allowed = true;                                                                                \
         }                                                                                                  \
-        kernel<<<grid, WAVES * KG * 64, lds, s>>>(x, w, y, part, M, N, K, splits, slices_per_split);       \
+        kernel<<<grid, WAVES * KG * 64, lds, s>>>(x, w, y, part, M, N, K, splits, slices_per_split, gated); \
     }
     if (gated) ROWS_LAUNCH(true)
     else ROWS_LAUNCH(false)
@@ -475,9 +475,12 @@ static int rows_pick(int M, int N, int K, int splits, int gated) {
 // four waves, 5: 128 x 384 and eight waves (in a gated product the waves of 4 and 5, which hold three
 // column tiles each, exchange the sums of one tile in pairs), 6: 128 x 256
 // by two sets of four waves that take the slices of k in turn; cfg >= 10: the tens for a gated product, the
-// ones for the others (measurements).
+// ones for the others (measurements).  act, act_scale, y_ld: the output of a gated product (common.h's GateOut; y_ld
+// 0: N/2).
 extern "C" int tli_gemm_rows_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K,
-                                  int gated, int splits, int cfg, void* stream) {
+                                  int is_gated, int splits, int cfg, int act, float act_scale, int y_ld, void* stream) {
+    const GateOut gated = gate_out(is_gated, act, act_scale, y_ld, N / 2);
+    if (const char* fault = gate_out_fault(gated, N / 2)) return tli_fail("gemm_rows: %s", fault);
     if (M <= 0 || N <= 0) return 0;
     if (K <= 0 || K % 8) return tli_fail("gemm_rows: K = %d must be a positive multiple of 8", K);
     if (gated && N % 32) return tli_fail("gemm_rows: a gated product needs N %% 32 == 0");

@@ -72,6 +72,7 @@ struct SkinnyFuse {
     const float* norm_w;      // [N] weights of the norm that follows
     bf16_t* xw;               // [M][N] bfloat16(norm_w * resid)
     float* ssq_out;           // [ceil(N/16)][M]
+    GateOut gate;             // of a gated matrix
 };
 
 template <int RT, int MT, int WAVES, typename TO, bool TILED = false, bool GATED = false, int DEPTH = 2,
@@ -279,8 +280,8 @@ gemm_skinny_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, T
             if (row < M) {
                 float o[4];
 #pragma unroll
-                for (int i = 0; i < 4; ++i) o[i] = g[i] / (1.0f + expf(-g[i])) * u[i];
-                store4(y + (size_t)row * n_out + n0, o, n_out - n0, (n_out & 3) == 0);
+                for (int i = 0; i < 4; ++i) o[i] = gate_unit(g[i], u[i], fuse.gate);
+                store4(y + (size_t)row * fuse.gate.ld + n0, o, n_out - n0, (fuse.gate.ld & 3) == 0);
             }
         }
         return;
@@ -325,11 +326,13 @@ gemm_skinny_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, T
 
 template <int RT, int MT, int WAVES>
 static int launch_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N, int K, int y_dtype,
-                         int tiled, hipStream_t s) {
+                         int tiled, const GateOut& gate, hipStream_t s) {
+    SkinnyFuse plain{};
+    plain.gate = gate;
     const int blocks = (N + 16 * RT - 1) / (16 * RT);
     constexpr int D = (MT == 1 && RT <= 2) ? PIPE_DEPTH : 2;    // deep prefetch where the registers allow
     if (tiled == 2) {       // gated: pairs of row tiles, silu(gate)*up written as bfloat16
-        gemm_skinny_kernel<RT, MT, WAVES, bf16_t, true, true, D><<<blocks, WAVES * 64, 0, s>>>(x, w, (bf16_t*)y, M, N, K, SkinnyFuse{});
+        gemm_skinny_kernel<RT, MT, WAVES, bf16_t, true, true, D><<<blocks, WAVES * 64, 0, s>>>(x, w, (bf16_t*)y, M, N, K, plain);
     } else if (tiled) {
         if (y_dtype == TLI_BF16)
             gemm_skinny_kernel<RT, MT, WAVES, bf16_t, true, false, D><<<blocks, WAVES * 64, 0, s>>>(x, w, (bf16_t*)y, M, N, K, SkinnyFuse{});
@@ -346,17 +349,17 @@ static int launch_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N
 
 template <int MT>
 static int pick_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N, int K, int y_dtype,
-                       int tiled, hipStream_t s, int cfg) {
+                       int tiled, const GateOut& gate, hipStream_t s, int cfg) {
     // cfg 0: by shape.  Narrow outputs get one 16-column tile per workgroup so that
     // even N = 4096 gives 256 workgroups; wide outputs share x over two tiles.
     const long tiles = (N + 15) / 16;
     if (cfg == 0) cfg = tiles <= tli_compute_units() ? 18 : (tiles < 4 * tli_compute_units() ? 28 : 24);
     if (tiled == 2 && cfg < 20) cfg = 24;          // gated needs pairs of row tiles
     switch (cfg) {
-        case 14: return launch_skinny<1, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, s);
-        case 18: return launch_skinny<1, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, s);
-        case 24: return launch_skinny<2, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, s);
-        case 28: return launch_skinny<2, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, s);
+        case 14: return launch_skinny<1, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, s);
+        case 18: return launch_skinny<1, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, s);
+        case 24: return launch_skinny<2, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, s);
+        case 28: return launch_skinny<2, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, s);
         default: return tli_fail("gemm_skinny: unknown configuration %d", cfg);
     }
 }
@@ -368,9 +371,12 @@ static int pick_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N, 
 // a wave then reads 1 KiB in a row.  `tiled` = 2: tiled, and the 16-row blocks alternate
 // between a gate matrix and an up matrix (block 2t: gate rows 16t.., block 2t+1: up rows
 // 16t..); N counts both, y is [M, N/2] bfloat16 = silu(x.gate^T) * (x.up^T).  cfg 0 picks the launch shape; other values
-// (row tiles * 10 + waves) force one, for measurements.
+// (row tiles * 10 + waves) force one, for measurements.  act, act_scale, y_ld: the output of a gated product (common.h's
+// GateOut: another activation than the silu, a factor, rows y_ld elements apart; y_ld 0: N/2).
 extern "C" int tli_gemm_skinny_bf16(const void* x, const void* w, void* y, int M, int N, int K,
-                                    int y_dtype, int tiled, int cfg, void* stream) {
+                                    int y_dtype, int tiled, int cfg, int act, float act_scale, int y_ld, void* stream) {
+    const GateOut gate = gate_out(tiled == 2, act, act_scale, y_ld, N / 2);
+    if (const char* fault = gate_out_fault(gate, N / 2)) return tli_fail("gemm_skinny: %s", fault);
     if (M <= 0 || N <= 0) return 0;
     if (M > 64) return tli_fail("gemm_skinny: %d rows, at most 64", M);
     if (K <= 0 || K % 8) return tli_fail("gemm_skinny: K = %d must be a positive multiple of 8", K);
@@ -383,10 +389,10 @@ extern "C" int tli_gemm_skinny_bf16(const void* x, const void* w, void* y, int M
     const bf16_t* xp = (const bf16_t*)x;
     const bf16_t* wp = (const bf16_t*)w;
     switch ((M + 15) / 16) {
-        case 1: return pick_skinny<1>(xp, wp, y, M, N, K, y_dtype, tiled, s, cfg);
-        case 2: return pick_skinny<2>(xp, wp, y, M, N, K, y_dtype, tiled, s, cfg);
-        case 3: return pick_skinny<3>(xp, wp, y, M, N, K, y_dtype, tiled, s, cfg);
-        default: return pick_skinny<4>(xp, wp, y, M, N, K, y_dtype, tiled, s, cfg);
+        case 1: return pick_skinny<1>(xp, wp, y, M, N, K, y_dtype, tiled, gate, s, cfg);
+        case 2: return pick_skinny<2>(xp, wp, y, M, N, K, y_dtype, tiled, gate, s, cfg);
+        case 3: return pick_skinny<3>(xp, wp, y, M, N, K, y_dtype, tiled, gate, s, cfg);
+        default: return pick_skinny<4>(xp, wp, y, M, N, K, y_dtype, tiled, gate, s, cfg);
     }
 }
 
@@ -410,7 +416,10 @@ static int launch_skinny_fused(const bf16_t* x, const bf16_t* w, bf16_t* y, int 
 // SwiGLU of a gated matrix if `gated` (y then [M, N/2]).
 extern "C" int tli_gemm_skinny_fused_bf16(const void* x, const void* w, void* y, int M, int N, int K, int gated,
                                           const float* ssq_in, int parts_in, float eps, float* resid,
-                                          const float* norm_w, void* xw, float* ssq_out, int cfg, void* stream) {
+                                          const float* norm_w, void* xw, float* ssq_out, int cfg, int act, float act_scale,
+                                          int y_ld, void* stream) {
+    const GateOut gate = gate_out(gated, act, act_scale, y_ld, N / 2);
+    if (const char* fault = gate_out_fault(gate, N / 2)) return tli_fail("gemm_skinny: %s", fault);
     if (M <= 0 || N <= 0) return 0;
     if (M > 16) return tli_fail("gemm_skinny with a norm: %d rows, at most 16", M);
     if (K <= 0 || K % 8) return tli_fail("gemm_skinny: K = %d must be a positive multiple of 8", K);
@@ -421,7 +430,7 @@ extern "C" int tli_gemm_skinny_fused_bf16(const void* x, const void* w, void* y,
     if (gated && N % 32) return tli_fail("gemm_skinny: a gated product needs N %% 32 == 0");
     if (((uintptr_t)x | (uintptr_t)w | (uintptr_t)y | (uintptr_t)resid | (uintptr_t)xw) & 15)
         return tli_fail("gemm_skinny: operands must be 16-byte aligned");
-    const SkinnyFuse f{ssq_in, parts_in, eps, resid, norm_w, (bf16_t*)xw, ssq_out};
+    const SkinnyFuse f{ssq_in, parts_in, eps, resid, norm_w, (bf16_t*)xw, ssq_out, gate};
     hipStream_t s = (hipStream_t)stream;
     const bf16_t* xp = (const bf16_t*)x;
     const bf16_t* wp = (const bf16_t*)w;

@@ -19,11 +19,14 @@
 // fetches into registers while the chunk before is walked.  Two more where a portion is long enough to be cut into
 // segments (lightning_carry, lightning_apply: see LT_SEGMENT below).
 //
+// The recurrence serves other layers too (recurrence.h): ROWS variants of its kernels take a factor a row and head in
+// place of one a head.
+//
 // lightning_norm: y = o / sqrt(mean(o^2) + eps) * w * sigmoid(gate) over all heads of a row together.
-#include "common.h"
+#include "recurrence.h"
 
 #define LT_THREADS 256
-#define LT_MAX_DK 256
+#define LT_MAX_DK TLI_RECURRENCE_MAX_DK
 
 __device__ __forceinline__ float lt_silu(float z) { return z / (1.0f + expf(-z)); }
 
@@ -64,7 +67,7 @@ __global__ void lightning_prepare_kernel(const T* __restrict__ proj, int ld, flo
 // have started from; the last sum is the sequence's new state); a third (lightning_apply) adds to every row of segment
 // s >= 1 what the state it should have started from contributes, c^(t + 1) P_s^T q_t for the segment's row t.  The sums are the
 // recurrence's own, in another order.
-#define LT_SEGMENT 256
+#define LT_SEGMENT TLI_RECURRENCE_SEGMENT
 
 struct LtSegment {
     int seq, first, rows, index, count;                  // the sequence; the first row (within the step's rows of the
@@ -93,9 +96,9 @@ __device__ __forceinline__ bool lt_segment_of(int z, const int* __restrict__ row
 }
 
 // L lanes a column (16 or 64), R elements of it a lane, CH rows a chunk
-template <int L, int R, int CH>
+template <int L, int R, int CH, bool ROWS>
 __global__ __launch_bounds__(LT_THREADS) void lightning_recurrence_kernel(
-    const float* __restrict__ qk, const float* __restrict__ vals, int DVP, const float* __restrict__ decay,
+    const float* __restrict__ qk, const float* __restrict__ vals, int DVP, RecurrenceDecay decay, int T,
     float* __restrict__ state, float* __restrict__ out, const int* __restrict__ row_start,
     const int* __restrict__ seq_start, const int* __restrict__ slots, int H, int dk, int dv, int num_seqs, int seg_rows,
     float* __restrict__ carry) {
@@ -107,6 +110,7 @@ __global__ __launch_bounds__(LT_THREADS) void lightning_recurrence_kernel(
     constexpr int VW = R % 4 == 0 ? 4 : R % 2 == 0 ? 2 : 1;   // floats of a piece: what a lane reads or writes at once
     static_assert(PQ * LT_THREADS * 4 == CH * 2 * DKP && PV <= LT_THREADS, "a chunk is shared out evenly");
     __shared__ __align__(16) float rows_s[CH * W];
+    __shared__ float decay_s[ROWS ? CH : 1];
     const int h = blockIdx.y, j0 = blockIdx.x * NC;
     const int tid = threadIdx.x;
     const int sub = tid % L, jl = tid / L;
@@ -120,7 +124,7 @@ __global__ __launch_bounds__(LT_THREADS) void lightning_recurrence_kernel(
     const int seq = seg.seq, n = seg.rows;
     const int r0 = row_start[seq] + seg.first;
     if (n <= 0) return;
-    const float lam = decay[h];
+    const float head_lam = ROWS ? 0.f : decay.head[h];
     // where the state comes from and goes to: the sequence's slot, or the segment's place in `carry`
     const size_t column = ((size_t)h * dv + (j < dv ? j : 0)) * dk;
     float* slot_col = state + (size_t)slots[seq] * H * dv * dk + column;
@@ -157,6 +161,7 @@ __global__ __launch_bounds__(LT_THREADS) void lightning_recurrence_kernel(
     const float* qk_seq = qk + ((size_t)r0 * H + h) * 2 * DKP;
     const float* v_seq = vals + ((size_t)r0 * H + h) * DVP + j0;
     float4 pq[PQ], pv;
+    float pl = 0.f;
     auto fetch = [&](int first) {
 #pragma unroll
         for (int u = 0; u < PQ; ++u) {
@@ -170,6 +175,7 @@ __global__ __launch_bounds__(LT_THREADS) void lightning_recurrence_kernel(
             const int rr = tid / (NC / 4), c4 = tid - rr * (NC / 4);
             if (first + rr < n) pv = *reinterpret_cast<const float4*>(v_seq + (size_t)(first + rr) * H * DVP + c4 * 4);
         }
+        if (ROWS && tid < CH) pl = first + tid < n ? decay.row[(size_t)h * T + r0 + first + tid] : 0.f;
     };
     fetch(0);
     float* o_col = out + (size_t)r0 * H * dv + (size_t)h * dv + j;
@@ -185,6 +191,7 @@ __global__ __launch_bounds__(LT_THREADS) void lightning_recurrence_kernel(
             const int rr = tid / (NC / 4), c4 = tid - rr * (NC / 4);
             *reinterpret_cast<float4*>(rows_s + rr * W + 2 * DKP + c4 * 4) = pv;
         }
+        if (ROWS && tid < CH) decay_s[tid] = pl;
         __syncthreads();
         if (t0 + CH < n) fetch(t0 + CH);
         const int cnt = min(CH, n - t0);
@@ -192,6 +199,7 @@ __global__ __launch_bounds__(LT_THREADS) void lightning_recurrence_kernel(
         for (int t = 0; t < cnt; ++t) {
             const float* row = rows_s + t * W;
             const float v = row[2 * DKP + jl];
+            const float lam = ROWS ? decay_s[t] : head_lam;
             float acc = 0.f;
 #pragma unroll
             for (int r = 0; r < R; ++r) {
@@ -221,7 +229,8 @@ __global__ __launch_bounds__(LT_THREADS) void lightning_recurrence_kernel(
 // The second launch of a step with segments: one thread an element of a sequence's state.  carry[z] holds the end
 // state E of segment z and is left holding the state P that the segment should have started from; the sequence's slot
 // gets its new state.
-__global__ void lightning_carry_kernel(float* __restrict__ carry, float* __restrict__ state, const float* __restrict__ decay,
+template <bool ROWS>
+__global__ void lightning_carry_kernel(float* __restrict__ carry, float* __restrict__ state, RecurrenceDecay decay, int T,
                                        const int* __restrict__ row_start, const int* __restrict__ slots, int num_seqs,
                                        int seg_rows, int H, int dv, int dk) {
     const int seq = blockIdx.y;
@@ -233,14 +242,17 @@ __global__ void lightning_carry_kernel(float* __restrict__ carry, float* __restr
     const int n = row_start[seq + 1] - row_start[seq];
     const int count = max(1, (n + seg_rows - 1) / seg_rows);
     if (count == 1) return;                              // (its one segment wrote the slot itself)
-    const float lam = decay[e / ((size_t)dv * dk)];
-    const float whole = powf(lam, (float)seg_rows), last = powf(lam, (float)(n - (count - 1) * seg_rows));
+    const int h = (int)(e / ((size_t)dv * dk));
+    const float lam = ROWS ? 0.f : decay.head[h];
+    const float whole = ROWS ? 0.f : powf(lam, (float)seg_rows), last = ROWS ? 0.f : powf(lam, (float)(n - (count - 1) * seg_rows));
+    const float* through = ROWS ? decay.log_through + (size_t)h * T + row_start[seq] : nullptr;
     float p = carry[(size_t)z0 * per + e];
     for (int s = 1; s < count; ++s) {
         float* at = carry + (size_t)(z0 + s) * per + e;
         const float end = *at;
         *at = p;
-        p = fmaf(s == count - 1 ? last : whole, p, end);
+        const float kept = ROWS ? expf(through[min((s + 1) * seg_rows, n) - 1]) : s == count - 1 ? last : whole;
+        p = fmaf(kept, p, end);
     }
     state[(size_t)slots[seq] * per + e] = p;
 }
@@ -256,9 +268,9 @@ __global__ void lightning_carry_kernel(float* __restrict__ carry, float* __restr
 // written by the launches before and lie in the cache.
 typedef float lt_f32x4 __attribute__((ext_vector_type(4)));
 
-template <int NT>
+template <int NT, bool ROWS>
 __global__ __launch_bounds__(LT_THREADS) void lightning_apply_kernel(
-    const float* __restrict__ qk, int DKP, const float* __restrict__ decay, float* __restrict__ out,
+    const float* __restrict__ qk, int DKP, RecurrenceDecay decay, int T, float* __restrict__ out,
     const int* __restrict__ row_start, int H, int dk, int dv, int num_seqs, int seg_rows, const float* __restrict__ carry) {
     LtSegment seg;
     if (!lt_segment_of(blockIdx.z, row_start, num_seqs, seg_rows, seg)) return;      // (the grid's slack)
@@ -268,7 +280,7 @@ __global__ __launch_bounds__(LT_THREADS) void lightning_apply_kernel(
     const int h = blockIdx.y, jb = (blockIdx.x / ROW_GROUPS) * 16 * NT;
     const int lane = threadIdx.x % TLI_WAVE, wave = threadIdx.x / TLI_WAVE, r = lane % 16, c = lane / 16;
     const int r0 = row_start[seg.seq] + seg.first, n = seg.rows;
-    const float lam = decay[h];
+    const float lam = ROWS ? 0.f : decay.head[h];
     const float* P = carry + ((size_t)blockIdx.z * H + h) * dv * dk;
     const bool whole = dk % 4 == 0;                      // a lane's four elements of a column exist together, aligned
     const int t0 = (blockIdx.x % ROW_GROUPS) * 64 + wave * 16;
@@ -312,7 +324,7 @@ __global__ __launch_bounds__(LT_THREADS) void lightning_apply_kernel(
         for (int v = 0; v < 4; ++v) {
             const int t = t0 + 4 * c + v;
             if (t >= n) continue;
-            const float power = powf(lam, (float)(t + 1));
+            const float power = ROWS ? expf(decay.log_through[(size_t)h * T + r0 + t]) : powf(lam, (float)(t + 1));
             float* o = out + (size_t)(r0 + t) * H * dv + (size_t)h * dv;
 #pragma unroll
             for (int nt = 0; nt < NT; ++nt) {
@@ -353,45 +365,30 @@ extern "C" long long tli_lightning_scratch_floats(int rows, int seqs, int longes
     return (long long)rows * H * (2LL * (a > b ? a : b) + (dv + 15) / 16 * 16) + segments * H * dv * dk;
 }
 
-// proj: [T, ld] raw projections, q (H dk), k (H dk), v (H dv) first; decay: float32 [H]; state: float32
-// [slots, H, dv, dk]; out: float32 [T, H dv]; row_start [seqs + 1], seq_start, slots [seqs]; scratch: float32,
-// tli_lightning_scratch_floats(T, ...) elements; longest: the most rows that a sequence brings (an upper bound will do);
-// lanes: 16 or 64 lanes a column, or 0 for the launch rule
-extern "C" int tli_lightning_recurrence(const void* proj, int ld, const float* decay, float* state, float* out,
-                                        float* scratch, const int* row_start, const int* seq_start, const int* slots,
-                                        int T, int seqs, int longest, int H, int dk, int dv, int dtype, int lanes,
-                                        void* stream) {
-    if (seqs <= 0 || T <= 0) return 0;
-    if (H <= 0 || dk <= 0 || dv <= 0 || dk > LT_MAX_DK)
-        return tli_fail("lightning: bad sizes (heads %d, keys of %d (at most %d), values of %d)", H, dk, LT_MAX_DK, dv);
-    if (ld < 2 * H * dk + H * dv) return tli_fail("lightning: rows of %d hold fewer than q, k and v", ld);
-    if (H > 65535 || seqs > 65535) return tli_fail("lightning: too many heads or sequences for one launch");
-    if (lanes != 0 && lanes != 16 && lanes != 64) return tli_fail("lightning: 16 or 64 lanes a column, not %d", lanes);
-    if (((uintptr_t)scratch | (uintptr_t)state) & 15) return tli_fail("lightning: scratch and state must be 16-byte aligned");
-    int DKP = 0;
-    lanes = lt_plan(dk, lanes, &DKP);
-    const int DVP = (dv + 15) / 16 * 16;
-    float* qk = scratch;
-    float* vals = qk + (size_t)T * H * 2 * DKP;
-    float* carry = vals + (size_t)T * H * DVP;
-    const int seg = lt_segment_rows(longest);
+RecurrencePlan tli_recurrence_plan(int longest, int dk, int dv, int lanes) {
+    RecurrencePlan p{};
+    p.lanes = lt_plan(dk, lanes, &p.dkp);
+    p.dvp = (dv + 15) / 16 * 16;
+    p.segment = lt_segment_rows(longest);
+    return p;
+}
+
+template <bool ROWS>
+static int lt_run(const RecurrencePlan& plan, float* scratch, const RecurrenceDecay& decay, float* state, float* out,
+                  const int* row_start, const int* seq_start, const int* slots, int T, int seqs, int H, int dk, int dv,
+                  hipStream_t s) {
+    const int lanes = plan.lanes, DKP = plan.dkp, DVP = plan.dvp, seg = plan.segment;
+    const float* qk = scratch;
+    const float* vals = recurrence_values(plan, scratch, T, H);
+    float* carry = scratch + (size_t)T * H * (2 * DKP + DVP);
     const int zs = seg ? T / seg + seqs : seqs;          // (an upper bound of the segments; a workgroup past the last leaves)
-    if (zs > 65535) return tli_fail("lightning: too many segments for one launch");
-    hipStream_t s = (hipStream_t)stream;
-    if (dtype == TLI_F32)
-        hipLaunchKernelGGL((lightning_prepare_kernel<float>), dim3(T, H), dim3(256), 0, s, (const float*)proj, ld, qk, vals, H, dk,
-                           dv, DKP, DVP);
-    else if (dtype == TLI_BF16)
-        hipLaunchKernelGGL((lightning_prepare_kernel<bf16_t>), dim3(T, H), dim3(256), 0, s, (const bf16_t*)proj, ld, qk, vals, H,
-                           dk, dv, DKP, DVP);
-    else
-        return tli_fail("lightning: unknown dtype %d", dtype);
+    if (zs > 65535) return tli_fail("recurrence: too many segments for one launch");
     const int cols = LT_THREADS / lanes;
     const dim3 grid((dv + cols - 1) / cols, H, zs);
     const int R = DKP / lanes;
-#define LT_LAUNCH(L, R, CH)                                                                                         \
-    hipLaunchKernelGGL((lightning_recurrence_kernel<L, R, CH>), grid, dim3(LT_THREADS), 0, s, qk, vals, DVP, decay, \
-                       state, out, row_start, seq_start, slots, H, dk, dv, seqs, seg, carry)
+#define LT_LAUNCH(L, R, CH)                                                                                              \
+    hipLaunchKernelGGL((lightning_recurrence_kernel<L, R, CH, ROWS>), grid, dim3(LT_THREADS), 0, s, qk, vals, DVP, decay, \
+                       T, state, out, row_start, seq_start, slots, H, dk, dv, seqs, seg, carry)
     if (lanes == 64) {
         if (R == 1) LT_LAUNCH(64, 1, 32);
         else if (R == 2) LT_LAUNCH(64, 2, 32);
@@ -404,17 +401,57 @@ extern "C" int tli_lightning_recurrence(const void* proj, int ld, const float* d
 #undef LT_LAUNCH
     if (seg) {
         const size_t per = (size_t)H * dv * dk;
-        hipLaunchKernelGGL(lightning_carry_kernel, dim3((unsigned)((per + 255) / 256), seqs), dim3(256), 0, s, carry, state, decay,
-                           row_start, slots, seqs, seg, H, dv, dk);
+        hipLaunchKernelGGL((lightning_carry_kernel<ROWS>), dim3((unsigned)((per + 255) / 256), seqs), dim3(256), 0, s, carry, state,
+                           decay, T, row_start, slots, seqs, seg, H, dv, dk);
         // (four tiles of 16 columns a wave where the head has them: q is then loaded once for 64 columns)
         if (dv > 32)
-            hipLaunchKernelGGL((lightning_apply_kernel<4>), dim3((dv + 63) / 64 * (LT_SEGMENT / 64), H, zs), dim3(LT_THREADS), 0, s, qk, DKP, decay, out,
-                               row_start, H, dk, dv, seqs, seg, carry);
+            hipLaunchKernelGGL((lightning_apply_kernel<4, ROWS>), dim3((dv + 63) / 64 * (LT_SEGMENT / 64), H, zs), dim3(LT_THREADS), 0, s,
+                               qk, DKP, decay, T, out, row_start, H, dk, dv, seqs, seg, carry);
         else
-            hipLaunchKernelGGL((lightning_apply_kernel<2>), dim3((dv + 31) / 32 * (LT_SEGMENT / 64), H, zs), dim3(LT_THREADS), 0, s, qk, DKP, decay, out,
-                               row_start, H, dk, dv, seqs, seg, carry);
+            hipLaunchKernelGGL((lightning_apply_kernel<2, ROWS>), dim3((dv + 31) / 32 * (LT_SEGMENT / 64), H, zs), dim3(LT_THREADS), 0, s,
+                               qk, DKP, decay, T, out, row_start, H, dk, dv, seqs, seg, carry);
     }
-    return tli_check_launch("lightning_recurrence");
+    return tli_check_launch("recurrence");
+}
+
+int tli_recurrence_run(const RecurrencePlan& plan, float* scratch, const RecurrenceDecay& decay, float* state, float* out,
+                       const int* row_start, const int* seq_start, const int* slots, int T, int seqs, int H, int dk, int dv,
+                       hipStream_t s) {
+    if (H <= 0 || dk <= 0 || dv <= 0 || dk > LT_MAX_DK)
+        return tli_fail("recurrence: bad sizes (heads %d, keys of %d (at most %d), values of %d)", H, dk, LT_MAX_DK, dv);
+    if (H > 65535 || seqs > 65535) return tli_fail("recurrence: too many heads or sequences for one launch");
+    if (((uintptr_t)scratch | (uintptr_t)state) & 15) return tli_fail("recurrence: scratch and state must be 16-byte aligned");
+    if (decay.head) return lt_run<false>(plan, scratch, decay, state, out, row_start, seq_start, slots, T, seqs, H, dk, dv, s);
+    if (!decay.row || (plan.segment && !decay.log_through)) return tli_fail("recurrence: no decays");
+    return lt_run<true>(plan, scratch, decay, state, out, row_start, seq_start, slots, T, seqs, H, dk, dv, s);
+}
+
+// proj: [T, ld] raw projections, q (H dk), k (H dk), v (H dv) first; decay: float32 [H]; state: float32
+// [slots, H, dv, dk]; out: float32 [T, H dv]; row_start [seqs + 1], seq_start, slots [seqs]; scratch: float32,
+// tli_lightning_scratch_floats(T, ...) elements; longest: the most rows that a sequence brings (an upper bound will do);
+// lanes: 16 or 64 lanes a column, or 0 for the launch rule
+extern "C" int tli_lightning_recurrence(const void* proj, int ld, const float* decay, float* state, float* out,
+                                        float* scratch, const int* row_start, const int* seq_start, const int* slots,
+                                        int T, int seqs, int longest, int H, int dk, int dv, int dtype, int lanes,
+                                        void* stream) {
+    if (seqs <= 0 || T <= 0) return 0;
+    if (H <= 0 || H > 65535 || dk <= 0 || dv <= 0 || dk > LT_MAX_DK)
+        return tli_fail("lightning: bad sizes (heads %d, keys of %d (at most %d), values of %d)", H, dk, LT_MAX_DK, dv);
+    if (ld < 2 * H * dk + H * dv) return tli_fail("lightning: rows of %d hold fewer than q, k and v", ld);
+    if (lanes != 0 && lanes != 16 && lanes != 64) return tli_fail("lightning: 16 or 64 lanes a column, not %d", lanes);
+    const RecurrencePlan plan = tli_recurrence_plan(longest, dk, dv, lanes);
+    float* vals = recurrence_values(plan, scratch, T, H);
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == TLI_F32)
+        hipLaunchKernelGGL((lightning_prepare_kernel<float>), dim3(T, H), dim3(256), 0, s, (const float*)proj, ld, scratch, vals, H, dk,
+                           dv, plan.dkp, plan.dvp);
+    else if (dtype == TLI_BF16)
+        hipLaunchKernelGGL((lightning_prepare_kernel<bf16_t>), dim3(T, H), dim3(256), 0, s, (const bf16_t*)proj, ld, scratch, vals, H,
+                           dk, dv, plan.dkp, plan.dvp);
+    else
+        return tli_fail("lightning: unknown dtype %d", dtype);
+    return tli_recurrence_run(plan, scratch, RecurrenceDecay{decay, nullptr, nullptr}, state, out, row_start, seq_start, slots, T,
+                              seqs, H, dk, dv, s);
 }
 
 // one workgroup a row

@@ -2,7 +2,7 @@
 head, and the order in which the blocks run."""
 from __future__ import annotations
 
-from typing import Dict, List, Optional
+from typing import Dict, List, Optional, Tuple
 
 import torch
 
@@ -10,6 +10,12 @@ from ..cache.manager import CacheNeed, StateNeed
 from ..config.base import ConfigError, ModelSpec, PartSpec
 from ..parts.base import BuildEnv, build_part
 from ..weights.loader import TensorDecl, load_tensors, random_tensors, unique_decls
+
+
+def cache_needs_of(mixer) -> Tuple[CacheNeed, ...]:
+    """What a mixer needs of the paged cache: nothing, one need or several."""
+    need = mixer.cache_need()
+    return () if need is None else (need,) if isinstance(need, CacheNeed) else tuple(need)
 
 
 class Model:
@@ -34,19 +40,29 @@ class Model:
     def _check_schedule(self) -> None:
         written = set()
         needs: Dict[int, CacheNeed] = {}
+        self.further: Dict[int, List[int]] = {}      # cache layer -> those of its mixer's further needs
         for i, call in enumerate(self.schedule):
             if not 0 <= call.block < len(self.blocks):
                 raise ConfigError(f"run order entry {i} names block {call.block}, "
                                   f"the model has {len(self.blocks)}")
-            need = self.blocks[call.block].mixer.cache_need()
-            if need is None:
+            wanted = cache_needs_of(self.blocks[call.block].mixer)
+            if not wanted:
                 continue
+            need = wanted[0]
             if call.cache < 0:
                 raise ConfigError(f"run order entry {i}: its mixer needs a cache layer")
             if call.cache in needs and needs[call.cache] != need:
                 raise ConfigError(f"run order entry {i}: cache layer {call.cache} is used with "
                                   f"different sizes")
             needs[call.cache] = need
+            if len(wanted) > 1 and call.cache not in self.further:
+                # a mixer's further needs are cache layers of their own, numbered behind those of the run order
+                at = self.spec.num_cache_layers() + sum(len(v) for v in self.further.values())
+                self.further[call.cache] = list(range(at, at + len(wanted) - 1))
+            for layer, more in zip(self.further.get(call.cache, ()), wanted[1:]):
+                if needs.setdefault(layer, more) != more:
+                    raise ConfigError(f"run order entry {i}: cache layer {call.cache} is used with "
+                                      f"different sizes")
             if call.writes_cache:
                 if call.cache in written:
                     raise ConfigError(f"run order entry {i}: cache layer {call.cache} is written twice")
@@ -57,7 +73,9 @@ class Model:
         self._needs = needs
 
     def cache_needs(self) -> List[Optional[CacheNeed]]:
-        return [self._needs.get(i) for i in range(self.spec.num_cache_layers())]
+        """By cache layer: those the run order names, then those of mixers' further needs."""
+        count = self.spec.num_cache_layers() + sum(len(v) for v in self.further.values())
+        return [self._needs.get(i) for i in range(count)]
 
     def state_needs(self) -> List[Optional[StateNeed]]:
         """Per run-order entry: the fixed-size state its block keeps per request (one need, or

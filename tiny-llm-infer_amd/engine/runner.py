@@ -267,7 +267,7 @@ class ModelRunner:
         groups = []
         for g, gl in enumerate(self.cache.groups):
             groups.append(GroupView(tensors=self.group_tensors[g], tables=dev[lay[f"tables{g}"]].view(seqs, width),
-                                    table_width=width, page_size=page, window=gl.need.window))
+                                    table_width=width, page_size=page, window=gl.need.window, stride=gl.need.stride))
         return StepView(
             num_rows=rows, num_seqs=seqs,
             token_ids=dev[lay["token_ids"]], positions=dev[lay["positions"]],
@@ -288,16 +288,20 @@ class ModelRunner:
         with hold():
             return self._forward(step, num_wanted)
 
+    def _layer_cache(self, step: StepView, cache_layer: int, writes: bool) -> LayerCache:
+        gi = self.cache.group_of_layer[cache_layer]
+        return LayerCache(step.groups[gi], self.cache.groups[gi].local_layer(cache_layer), writes)
+
     def _forward(self, step: StepView, num_wanted: int) -> Optional[torch.Tensor]:
         model = self.model
         resid = model.open_residual(model.embedding.forward(step.token_ids, step.num_rows, step.positions))
         pending = None
         for i, call in enumerate(model.schedule):
             if call.cache >= 0 and call.cache in self.cache.group_of_layer:
-                gi = self.cache.group_of_layer[call.cache]
-                step.cache = LayerCache(step.groups[gi],
-                                        self.cache.groups[gi].local_layer(call.cache),
-                                        call.writes_cache)
+                step.cache = self._layer_cache(step, call.cache, call.writes_cache)
+                further = model.further.get(call.cache)
+                if further:
+                    step.cache.further = [self._layer_cache(step, layer, call.writes_cache) for layer in further]
             else:
                 step.cache = None
             step.state = self.states[i]

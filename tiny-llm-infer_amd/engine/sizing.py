@@ -15,11 +15,12 @@ def _elem_size(dtype, run_dtype) -> int:
 
 def page_bytes(model, page_size: int, windowed=None) -> int:
     """Bytes of one page id across the cache layers (``windowed``: None all of them, False
-    those that keep all keys, True those with a window): every record that the mixers declared."""
+    those that keep all keys, True those with a window): every record that the mixers declared.
+    A layer with one slot for several positions counts with its share of a page."""
     total = 0
     for need in model.cache_needs():
         if need is not None and (windowed is None or (not need.keeps_all) == windowed):
-            total += need_page_bytes(need, page_size, model.env.dtype)
+            total += -(-need_page_bytes(need, page_size, model.env.dtype) // need.stride)
     return total
 
 
@@ -29,13 +30,16 @@ def need_page_bytes(need, page_size: int, run_dtype) -> int:
 
 
 def window_bytes(model, page_size: int, max_batch_tokens: int, max_num_seqs: int) -> int:
-    """What the window groups take: their fixed number of pages, for every layer of the group."""
+    """What the window groups take: their fixed number of pages, for every layer of the group; and
+    the pages that every request has begun in groups with one slot for several positions."""
     from ..cache.manager import window_group_pages
     total = 0
     for need in model.cache_needs():
         if need is not None and not need.keeps_all:
-            pages = window_group_pages(need.reach, page_size, max_num_seqs, max_batch_tokens, need.keep_first)
+            pages = window_group_pages(need.reach, need.page_span(page_size), max_num_seqs, max_batch_tokens, need.keep_first)
             total += pages * need_page_bytes(need, page_size, model.env.dtype)
+        elif need is not None and need.stride > 1:
+            total += max_num_seqs * need_page_bytes(need, page_size, model.env.dtype)
     return total
 
 

@@ -55,6 +55,8 @@ def _dtype_code(dtype: torch.dtype) -> int:
     raise KernelError(f"kernels take float32 or bfloat16 tensors, not {dtype}")
 
 
+# what a product without a gate passes for the activation, the factor and the distance of the outputs' rows
+_NO_GATE = (0, 1.0, 0)
 _LIB = None
 
 
@@ -76,19 +78,19 @@ def load_library():
         "tli_embed": [P, P, P, I, I, I, I, P],
         "tli_feed_tokens": [P, P, P, I, I, P],
         "tli_add_rmsnorm": [P, P, P, P, P, I, I, I, F, I, I, P],
-        "tli_swiglu": [P, P, I, I, I, F, F, P],
+        "tli_swiglu": [P, P, I, I, I, F, F, I, F, I, P],
         "tli_qkv_to_cache": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, F, P, F, P, P, I, I, I, I, I, P],
         "tli_values_to_cache": [P, P, P, P, I, I, P, I, I, I, I, I, I, P],
         "tli_keys_values_to_cache": [P, P, P, P, P, I, I, P, I, I, I, I, I, I, P, F, P, P, I, P],
         "tli_attention_plain": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, P],
         "tli_gemm_plain": [P, P, P, I, I, I, I, I, I, P],
-        "tli_gemm_skinny_bf16": [P, P, P, I, I, I, I, I, I, P],
-        "tli_gemm_skinny_fused_bf16": [P, P, P, I, I, I, I, P, I, F, P, P, P, P, I, P],
-        "tli_gemm_mid_bf16": [P, P, P, P, I, I, I, I, I, I, I, P],
+        "tli_gemm_skinny_bf16": [P, P, P, I, I, I, I, I, I, I, F, I, P],
+        "tli_gemm_skinny_fused_bf16": [P, P, P, I, I, I, I, P, I, F, P, P, P, P, I, I, F, I, P],
+        "tli_gemm_mid_bf16": [P, P, P, P, I, I, I, I, I, I, I, I, F, I, P],
         "tli_gemm_mid_splits": [I, I, I],
         "tli_gemm_mid_splits_rows": [I, I, I, I],
         "tli_gemm_mid_reduce": [P, P, I, I, I, I, P],
-        "tli_gemm_rows_bf16": [P, P, P, P, I, I, I, I, I, I, P],
+        "tli_gemm_rows_bf16": [P, P, P, P, I, I, I, I, I, I, I, F, I, P],
         "tli_gemm_rows_splits": [I, I, I],
         "tli_attention_decode_bf16": [P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, I, I, I, P],
         "tli_qkv_attention_decode_bf16": [P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, F, P, F, P, P, I,
@@ -131,6 +133,12 @@ def load_library():
         "tli_add_bias": [P, P, I, I, I, P],
         "tli_lightning_recurrence": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
         "tli_lightning_norm": [P, P, I, P, P, I, I, F, I, P],
+        "tli_retention": [P, I, P, P, P, P, P, P, P, P, P, P, I, I, I, F, I, I, I, I, I, I, I, I, P],
+        "tli_mlstm": [P, I, P, ctypes.c_longlong, ctypes.c_longlong, P, F, F, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
+        "tli_head_norm_gate": [P, P, P, P, I, P, I, I, I, I, F, I, F, I, P],
+        "tli_pooled_prepare": [P, I, P, P, P, P, P, P, P, P, I, P, I, I, I, I, I, I, I, I, P, P, F, P, P, I, I, I, P, P, P, I, I, I, I, I, P],
+        "tli_attention_pooled_plain": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
+        "tli_attention_pooled_mfma_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
         "tli_sample": [P, I, I, P, P, P, P, P, P],
         "tli_sample_scratch_bytes": [I],
         "tli_random_normal": [P, ctypes.c_longlong, ctypes.c_uint32, ctypes.c_uint32, ctypes.c_uint32, P, F, F, I, P],
@@ -441,7 +449,7 @@ class HipOps:
                     m1 = min(M, m0 + self.SKINNY_ROWS)
                     self._call(self.lib.tli_gemm_skinny_bf16, x[m0:m1].data_ptr(), wp.data_ptr(),
                                y[m0:m1].data_ptr(), m1 - m0, N, K, _dtype_code(out_dtype),
-                               0 if tiled is None else 1, self.skinny_cfg, self._stream())
+                               0 if tiled is None else 1, self.skinny_cfg, *_NO_GATE, self._stream())
                 return y
             if tiled is not None and out_dtype == torch.bfloat16 and self._rows_kernel_wins(x, matrix, tiled, M, N, K, 0):
                 return self._linear_rows(x, tiled, y, M, N, K, 0, deferred or sums_only)
@@ -468,11 +476,11 @@ class HipOps:
         xw = torch.empty((M, N), dtype=torch.bfloat16, device=self.device)
         ssq = torch.empty(((N + 15) // 16, M), dtype=torch.float32, device=self.device)
         self._call(self.lib.tli_gemm_skinny_fused_bf16, x.data_ptr(), m.tiled.data_ptr(), None, M, N, K, 0,
-                   None, 0, 0.0, resid.data_ptr(), weight.data_ptr(), xw.data_ptr(), ssq.data_ptr(), 0,
+                   None, 0, 0.0, resid.data_ptr(), weight.data_ptr(), xw.data_ptr(), ssq.data_ptr(), 0, *_NO_GATE,
                    self._stream())
         return NormedRows(xw, ssq, eps)
 
-    def _linear_normed(self, x: NormedRows, m, tiled, gated: int, out_dtype=None):
+    def _linear_normed(self, x: NormedRows, m, tiled, gated: int, out_dtype=None, act: int = 0, scale: float = 1.0, into=None):
         """y = normed rows . W^T with the rows' factor applied to the outputs."""
         M, K = x.xw.shape
         if tiled is None:
@@ -483,22 +491,25 @@ class HipOps:
         if _shape_of(m)[1] != K:
             raise KernelError(f"linear: input has {K} columns, the matrix {_shape_of(m)[1]}")
         N = 2 * m.inter if gated else rows_out
-        y = torch.empty((M, m.inter if gated else N), dtype=torch.bfloat16, device=self.device)
-        self._call(self.lib.tli_gemm_skinny_fused_bf16, x.xw.data_ptr(), tiled.data_ptr(), y.data_ptr(), M, N, K,
-                   gated, x.ssq.data_ptr(), x.ssq.shape[0], x.eps, None, None, None, None, 0, self._stream())
+        y, y_at, ld = self._rows_into(into, M, m.inter if gated else N, torch.bfloat16)
+        self._call(self.lib.tli_gemm_skinny_fused_bf16, x.xw.data_ptr(), tiled.data_ptr(), y_at, M, N, K,
+                   gated, x.ssq.data_ptr(), x.ssq.shape[0], x.eps, None, None, None, None, 0, act, float(scale), ld,
+                   self._stream())
         return y
 
-    def _linear_mid(self, x, tiled, y, M, N, K, gated, deferred=False):
+    def _linear_mid(self, x, tiled, y, M, N, K, gated, deferred=False, gate=None):
         """17..128 rows (without a gate: up to 256): the kernel that shares x through LDS, k cut into
         ranges when the output alone gives too few workgroups.  ``deferred``: the partial sums of the
-        ranges are left for the consumer to add, which saves the pass that adds them."""
+        ranges are left for the consumer to add, which saves the pass that adds them.  ``gate``: (address of
+        the output, activation, factor, distance of its rows) of a gated product."""
         splits = self.mid_splits or self.lib.tli_gemm_mid_splits_rows(M, N, K, gated)
         part = None
         if splits > 1:
             part = torch.empty((splits, M, N), dtype=torch.float32, device=self.device)
         leave = deferred and splits > 1 and not gated and y.dtype == torch.bfloat16
-        self._call(self.lib.tli_gemm_mid_bf16, x.data_ptr(), tiled.data_ptr(), None if leave else y.data_ptr(),
-                   _ptr(part), M, N, K, _dtype_code(y.dtype), gated, splits, self.mid_cfg, self._stream())
+        y_at, *gate = gate or (y.data_ptr(), *_NO_GATE)
+        self._call(self.lib.tli_gemm_mid_bf16, x.data_ptr(), tiled.data_ptr(), None if leave else y_at,
+                   _ptr(part), M, N, K, _dtype_code(y.dtype), gated, splits, self.mid_cfg, *gate, self._stream())
         return DeferredSum(part, y.dtype) if leave else y
 
     def _rows_kernel_wins(self, x, matrix, tiled, M, N, K, gated) -> bool:
@@ -552,17 +563,18 @@ class HipOps:
         self.measured[key] = won
         return won
 
-    def _linear_rows(self, x, tiled, y, M, N, K, gated, deferred=False):
+    def _linear_rows(self, x, tiled, y, M, N, K, gated, deferred=False, gate=None):
         """Any number of rows from the decode layout; k cut into ranges when the output
         alone gives too few workgroups.  ``deferred``: the partial sums of the ranges are
-        left for the consumer to add."""
+        left for the consumer to add.  ``gate`` as in ``_linear_mid``."""
         splits = self.rows_splits or self.lib.tli_gemm_rows_splits(M, N, K)
         part = None
         if splits > 1:
             part = torch.empty((splits, M, N), dtype=torch.float32, device=self.device)
         leave = deferred and splits > 1 and not gated
-        self._call(self.lib.tli_gemm_rows_bf16, x.data_ptr(), tiled.data_ptr(), None if leave else y.data_ptr(),
-                   _ptr(part), M, N, K, gated, splits, self.rows_cfg, self._stream())
+        y_at, *gate = gate or (y.data_ptr(), *_NO_GATE)
+        self._call(self.lib.tli_gemm_rows_bf16, x.data_ptr(), tiled.data_ptr(), None if leave else y_at,
+                   _ptr(part), M, N, K, gated, splits, self.rows_cfg, *gate, self._stream())
         return DeferredSum(part, y.dtype) if leave else y
 
     def linear_plain(self, x: torch.Tensor, w: torch.Tensor, out_dtype: Optional[torch.dtype] = None):
@@ -577,40 +589,63 @@ class HipOps:
                    _dtype_code(x.dtype), _dtype_code(w.dtype), _dtype_code(out_dtype), self._stream())
         return y
 
-    def linear_swiglu(self, x: torch.Tensor, m) -> torch.Tensor:
-        """silu(x gate^T) * (x up^T) for a ``GatedMatrix``.  Few rows: one pass of
+    GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+
+    def check_gate_activation(self, name: str) -> None:
+        if name not in self.GATE_ACTIVATIONS:
+            raise KernelError(f"gate activation '{name}' is not known; known: {', '.join(sorted(self.GATE_ACTIVATIONS))}")
+
+    def _rows_into(self, into, rows: int, cols: int, dtype):
+        """(tensor, address, distance of its rows) of ``rows`` x ``cols`` outputs: a new tensor, or, for ``into`` =
+        (tensor, column), the columns from there on of the rows of that tensor, which other outputs share."""
+        if into is None:
+            y = torch.empty((rows, cols), dtype=dtype, device=self.device)
+            return y, y.data_ptr(), cols
+        y, at = into
+        self._want(y, "shared rows of outputs", dtype)
+        if y.dim() != 2 or y.shape[0] != rows or at < 0 or at % 8 or at + cols > y.shape[1] or y.shape[1] % 8:
+            raise KernelError(f"{cols} columns from {at} on (a multiple of 8) do not fit shared rows of shape {tuple(y.shape)}")
+        return y, y.data_ptr() + at * y.element_size(), y.shape[1]
+
+    def linear_swiglu(self, x: torch.Tensor, m, activation: str = "silu", scale: float = 1.0, into=None) -> torch.Tensor:
+        """act(x gate^T) * (x up^T) * scale for a ``GatedMatrix``.  Few rows: one pass of
         the weight-streaming kernel over the interleaved layout, the activation in
-        its epilogue.  Otherwise the stacked product, then the activation."""
+        its epilogue.  Otherwise the stacked product, then the activation.  ``into`` (a tensor and a
+        column of it): the outputs go there, beside what else its rows hold."""
+        act = self.GATE_ACTIVATIONS[activation]
         if isinstance(x, NormedRows):
-            return self._linear_normed(x, m, getattr(m, "gated", None), 1)
+            return self._linear_normed(x, m, getattr(m, "gated", None), 1, act=act, scale=scale, into=into)
         M, K = x.shape
         gated = getattr(m, "gated", None) if not self.plain_products else None
         if gated is not None and 0 < M <= self.MID_ROWS_TO and x.dtype == torch.bfloat16:
             self._want(x, "linear input", torch.bfloat16, (M, _shape_of(m)[1]))
-            y = torch.empty((M, m.inter), dtype=x.dtype, device=self.device)
+            y, y_at, ld = self._rows_into(into, M, m.inter, x.dtype)
             if M >= self.MID_ROWS_FROM:
-                return self._linear_mid(x, gated, y, M, 2 * m.inter, K, 1)
-            self._call(self.lib.tli_gemm_skinny_bf16, x.data_ptr(), gated.data_ptr(), y.data_ptr(), M,
-                       2 * m.inter, K, BF16, 2, self.skinny_cfg if self.skinny_cfg >= 20 else 0, self._stream())
+                return self._linear_mid(x, gated, y, M, 2 * m.inter, K, 1, gate=(y_at, act, float(scale), ld))
+            self._call(self.lib.tli_gemm_skinny_bf16, x.data_ptr(), gated.data_ptr(), y_at, M,
+                       2 * m.inter, K, BF16, 2, self.skinny_cfg if self.skinny_cfg >= 20 else 0, act, float(scale), ld,
+                       self._stream())
             return y
         if (gated is not None and x.dtype == torch.bfloat16 and K % 8 == 0
                 and self._rows_kernel_wins(x, m, gated, M, 2 * m.inter, K, 1)):
             self._want(x, "linear input", torch.bfloat16, (M, _shape_of(m)[1]))
-            y = torch.empty((M, m.inter), dtype=x.dtype, device=self.device)
-            return self._linear_rows(x, gated, y, M, 2 * m.inter, K, 1)
-        return self.swiglu(self.linear(x, m))
+            y, y_at, ld = self._rows_into(into, M, m.inter, x.dtype)
+            return self._linear_rows(x, gated, y, M, 2 * m.inter, K, 1, gate=(y_at, act, float(scale), ld))
+        return self.swiglu(self.linear(x, m), activation=activation, scale=scale, into=into)
 
-    def swiglu(self, gu: torch.Tensor, limit: float = 0.0, slope: float = 1.0) -> torch.Tensor:
-        """From gate and up sums side by side [rows, 2 n] to the hidden units [rows, n]: silu(g) * u, or with a
+    def swiglu(self, gu: torch.Tensor, limit: float = 0.0, slope: float = 1.0, activation: str = "silu", scale: float = 1.0,
+               into=None) -> torch.Tensor:
+        """From gate and up sums side by side [rows, 2 n] to the hidden units [rows, n]: act(g) * u * scale, or with a
         positive ``limit`` the limited form g' * sigmoid(slope * g') * (u' + 1), g' = min(g, limit), u' = clamp(u,
-        -limit, limit)."""
+        -limit, limit).  ``into`` as in ``linear_swiglu``."""
         rows, two = gu.shape
         if two % 2:
             raise KernelError("swiglu input must hold gate and up side by side")
         self._want(gu, "swiglu input")
-        out = torch.empty((rows, two // 2), dtype=gu.dtype, device=self.device)
-        self._call(self.lib.tli_swiglu, gu.data_ptr(), out.data_ptr(), rows, two // 2,
-                   _dtype_code(gu.dtype), float(limit), float(slope), self._stream())
+        out, out_at, ld = self._rows_into(into, rows, two // 2, gu.dtype)
+        self._call(self.lib.tli_swiglu, gu.data_ptr(), out_at, rows, two // 2,
+                   _dtype_code(gu.dtype), float(limit), float(slope), self.GATE_ACTIVATIONS[activation], float(scale), ld,
+                   self._stream())
         return out
 
     def qkv_to_cache(self, qkv, step, cache, heads, kv_heads, head_dim, q_norm, k_norm, rotary, queries=True):
@@ -1130,7 +1165,7 @@ class HipOps:
         for n0 in range(0, N, self.SKINNY_ROWS):
             n1 = min(N, n0 + self.SKINNY_ROWS)
             self._call(self.lib.tli_gemm_skinny_bf16, w_rows[n0:n1].data_ptr(), x.data_ptr(), y[n0:n1].data_ptr(), n1 - n0, M, K,
-                       F32, 0, 0, self._stream())
+                       F32, 0, 0, *_NO_GATE, self._stream())
         return y, True
 
     def delta_state_shape(self, heads: int, dk: int, dv: int):
@@ -1575,6 +1610,161 @@ class HipOps:
         self._call(self.lib.tli_lightning_norm, o.data_ptr(), proj.data_ptr() + gate_at * proj.element_size(), proj.shape[1],
                    weight.data_ptr(), out.data_ptr(), T, n, float(eps), _dtype_code(out_dtype), self._stream())
         return out
+
+    # ---- attention over a window and pooled blocks --------------------------------------------------------
+    def _pairs(self, rotary, step):
+        """(cos, sin, turned elements, pairing code, positions) of a ``RotaryTables`` or None, for kernels that turn
+        either kind of pairs."""
+        if rotary is None:
+            return None, None, 0, 0, 0
+        codes = {"half": 0, "interleaved": 1}
+        if rotary[3] not in codes:
+            raise KernelError(f"the pairing '{rotary[3]}' of a rotation is not known")
+        cos, sin, rd = self._rotary(rotary[:3], step)
+        return cos, sin, rd, codes[rotary[3]], cos.shape[0]
+
+    def pooled_window_attention(self, proj, at, step, cache, heads, kv_heads, key_dim, value_dim, bias, q_weight, k_weight,
+                                eps, rotary, scale, sinks, window, pool, out, out_at, out_scale):
+        """From the raw projections ``proj[:, at:]`` (q (heads key_dim) | k (kv_heads key_dim) | v (kv_heads value_dim))
+        to the heads' outputs times ``out_scale`` in ``out[:, out_at : out_at + heads value_dim]``: biases, RMS norms of q
+        and of k over all their elements (weights float32 or None), rotation of either pairing, keys and values into
+        the cache (records "k", "v"), the means of every ``pool`` positions' keys and values into ``cache.further[0]``, and
+        attention over the window's tokens and the blocks before it with ``sinks`` (float32 [heads] or None)."""
+        T = step.num_rows
+        self.check_sized_attention(heads, kv_heads, key_dim, value_dim)
+        qn, kn, vn = heads * key_dim, kv_heads * key_dim, kv_heads * value_dim
+        self._want(proj, "projections", out.dtype)
+        if proj.dim() != 2 or proj.shape[0] != T or at < 0 or proj.shape[1] < at + qn + kn + vn:
+            raise KernelError(f"the projections have shape {tuple(proj.shape)}, expected [{T}, >= {at + qn + kn + vn}]")
+        for w, n, what in ((bias, qn + kn + vn, "projections' bias"), (q_weight, qn, "norm weight of q"),
+                           (k_weight, kn, "norm weight of k"), (sinks, heads, "sinks")):
+            if w is not None:
+                self._want(w, what, torch.float32, (n,))
+        if cache is None or not cache.writes or len(cache.further) != 1:
+            raise KernelError("this attention writes its keys and their means into cache layers of its own")
+        if window <= 0 or pool <= 0:
+            raise KernelError("a window and blocks of at least one position each")
+        blocks = cache.further[0]
+        kc, vc, g = cache.record("k"), cache.record("v"), cache.group
+        bk, bv, bg = blocks.record("k"), blocks.record("v"), blocks.group
+        for k, v, gr, what in ((kc, vc, g, "cache"), (bk, bv, bg, "cache of blocks")):
+            self._want(k, f"key {what}", proj.dtype, (k.shape[0], kv_heads, gr.page_size, key_dim))
+            self._want(v, f"value {what}", proj.dtype, (k.shape[0], kv_heads, value_dim, gr.page_size))
+        if bg.page_size != g.page_size or bg.stride != pool or g.stride != 1:
+            raise KernelError(f"the cache of blocks has one slot for {bg.stride} positions, the blocks have {pool}")
+        self._check_tables(g, step)
+        self._want(bg.tables, "block tables of the blocks", torch.int32, (step.num_seqs, bg.table_width))
+        if -(-step.max_seq_len // (bg.page_size * pool)) > bg.table_width:
+            raise KernelError("a block table is narrower than its sequence needs")
+        _, out_ptr, out_ld = self._rows_into((out, out_at), T, heads * value_dim, proj.dtype)
+        cos, sin, dims, pairing, npos = self._pairs(rotary, step)
+        if dims > key_dim:
+            raise KernelError(f"{dims} turned elements do not fit a head of {key_dim}")
+        q = torch.empty((T, heads, key_dim), dtype=proj.dtype, device=self.device)
+        single = 1 if step.max_rows_per_seq == 1 and step.num_seqs == T else 0
+        pooled = (bk.data_ptr(), bv.data_ptr(), bg.tables.data_ptr(), bg.table_width, bk.shape[0], pool)
+        self._call(self.lib.tli_pooled_prepare, proj.data_ptr() + at * proj.element_size(), proj.shape[1], _ptr(bias), q.data_ptr(),
+                   kc.data_ptr(), vc.data_ptr(), step.positions.data_ptr(), step.seq_of_row.data_ptr(), step.row_start.data_ptr(),
+                   step.seq_start.data_ptr(), step.num_seqs, g.tables.data_ptr(), g.table_width, g.page_size, kc.shape[0], T,
+                   heads, kv_heads, key_dim, value_dim, _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(cos), _ptr(sin), dims,
+                   pairing, npos, *pooled, single, _dtype_code(proj.dtype), self._stream())
+        if (proj.dtype == torch.bfloat16 and not self.force_plain
+                and self.lib.tli_attention_sized_mfma_takes(key_dim, value_dim, g.page_size, 1)):
+            starts = step.h_row_start
+            tiles = T if single else sum((starts[i + 1] - starts[i] + 15) // 16 for i in range(step.num_seqs))
+            self._call(self.lib.tli_attention_pooled_mfma_bf16, q.data_ptr(), out_ptr, kc.data_ptr(), vc.data_ptr(),
+                       step.row_start.data_ptr(), step.seq_start.data_ptr(), step.num_seqs, tiles, g.tables.data_ptr(),
+                       g.table_width, g.page_size, kc.shape[0], heads, kv_heads, key_dim, value_dim, float(scale), int(window),
+                       *pooled, single, _ptr(sinks), out_ld, float(out_scale), self._stream())
+            return
+        self._call(self.lib.tli_attention_pooled_plain, q.data_ptr(), out_ptr, kc.data_ptr(), vc.data_ptr(),
+                   step.positions.data_ptr(), step.seq_of_row.data_ptr(), g.tables.data_ptr(), g.table_width, g.page_size,
+                   kc.shape[0], T, heads, kv_heads, key_dim, value_dim, float(scale), int(window), *pooled,
+                   _dtype_code(proj.dtype), _ptr(sinks), out_ld, float(out_scale), self._stream())
+
+    # ---- retention, mLSTM --------------------------------------------------------------------------------
+    def _recurrent_inputs(self, proj, at, state, shape, step, heads, dk, dv):
+        T = step.num_rows
+        self.check_lightning_sizes(heads, dk, dv)
+        need = at + 2 * heads * dk + heads * dv
+        self._want(proj, "projections")
+        if proj.dim() != 2 or proj.shape[0] != T or at < 0 or proj.shape[1] < need:
+            raise KernelError(f"the projections have shape {tuple(proj.shape)}, expected [{T}, >= {need}]")
+        self._want(state, "recurrent state", torch.float32, (state.shape[0],) + tuple(shape))
+        if max(step.h_slots, default=0) >= state.shape[0]:
+            raise KernelError("a sequence's slot lies outside the state")
+
+    def _recurrence_scratch(self, step, heads, dk, dv, more=0):
+        n = int(self.lib.tli_lightning_scratch_floats(step.num_rows, step.num_seqs, int(step.max_rows_per_seq), heads, dk, dv))
+        return torch.empty((n + more,), dtype=torch.float32, device=self.device), n
+
+    def retention(self, proj, at, decay, state, step, heads, dk, dv, rotary, k_scale):
+        """From the raw projections ``proj[:, at:]`` (q (H dk) | k (H dk) | v (H dv)) to the heads' outputs of the
+        recurrence S <- decay_h S + k v^T, o = S^T q, float32 [T, H, dv], with q and k turned (``rotary``, of either
+        pairing, or None) and k times ``k_scale``.  ``state``: float32 [slots, H, dv, dk], read (unless a sequence starts at
+        position 0) and replaced."""
+        T = step.num_rows
+        self._recurrent_inputs(proj, at, state, (heads, dv, dk), step, heads, dk, dv)
+        self._want(decay, "decays", torch.float32, (heads,))
+        cos, sin, dims, pairing, npos = self._pairs(rotary, step)
+        if dims > dk:
+            raise KernelError(f"{dims} turned elements do not fit a head of {dk}")
+        out = torch.empty((T, heads, dv), dtype=torch.float32, device=self.device)
+        scratch, _ = self._recurrence_scratch(step, heads, dk, dv)
+        self._call(self.lib.tli_retention, proj.data_ptr() + at * proj.element_size(), proj.shape[1], decay.data_ptr(),
+                   state.data_ptr(), out.data_ptr(), scratch.data_ptr(), step.positions.data_ptr(), step.row_start.data_ptr(),
+                   step.seq_start.data_ptr(), step.slots.data_ptr(), _ptr(cos), _ptr(sin), dims, pairing, npos, float(k_scale),
+                   T, step.num_seqs, int(step.max_rows_per_seq), heads, dk, dv, _dtype_code(proj.dtype),
+                   int(self.lightning_lanes), self._stream())
+        return out
+
+    def mlstm_state_shape(self, heads: int, dk: int, dv: int):
+        """The shape of one request's S beside its n: a head's matrix is kept transposed, n is its column dv."""
+        return (heads, dv + 1, dk)
+
+    def mlstm(self, proj, at, gates, gates_transposed, gate_bias, cap, state, m_state, step, heads, dk, dv, q_scale):
+        """From the raw projections ``proj[:, at:]`` (q (H dk) | k (H dk) | v (H dv)) and the gates' products ``gates``
+        (float32 [T, 2 H]: input gates, then forget gates; [2 H, T] with ``gates_transposed``) to the memory's outputs:
+        (o, floors), o float32 [T, H, dv + 1] the heads' S^T q and, behind them, n . q, floors float32 [H, T] the
+        exp(-m).  ``state``: float32 [slots, *mlstm_state_shape]; ``m_state``: float32 [slots, H]."""
+        T = step.num_rows
+        self._recurrent_inputs(proj, at, state, self.mlstm_state_shape(heads, dk, dv), step, heads, dk, dv)
+        self._want(m_state, "running maxima", torch.float32, (state.shape[0], heads))
+        self._want(gates, "gate products", torch.float32, (2 * heads, T) if gates_transposed else (T, 2 * heads))
+        self._want(gate_bias, "gate biases", torch.float32, (2 * heads,))
+        z_row, z_col = (1, T) if gates_transposed else (2 * heads, 1)
+        single = 1 if step.max_rows_per_seq == 1 and step.num_seqs == T else 0
+        out = torch.empty((T, heads, dv + 1), dtype=torch.float32, device=self.device)
+        floors = torch.empty((heads, T), dtype=torch.float32, device=self.device)
+        scratch, n = self._recurrence_scratch(step, heads, dk, dv + 1, more=3 * heads * T)
+        self._call(self.lib.tli_mlstm, proj.data_ptr() + at * proj.element_size(), proj.shape[1], gates.data_ptr(), z_row, z_col,
+                   gate_bias.data_ptr(), float(cap), float(q_scale), m_state.data_ptr(), state.data_ptr(), out.data_ptr(),
+                   floors.data_ptr(), scratch.data_ptr(), scratch.data_ptr() + 4 * n, step.row_start.data_ptr(),
+                   step.seq_start.data_ptr(), step.slots.data_ptr(), T, step.num_seqs, int(step.max_rows_per_seq), single,
+                   heads, dk, dv, _dtype_code(proj.dtype), int(self.lightning_lanes), self._stream())
+        return out, floors
+
+    OUTPUT_GATES = {"silu": 0, "sigmoid": 1}
+
+    def head_norm_gate(self, o, floors, weight, proj, gate_at, heads, dv, eps, gate, scale, out, out_at):
+        """x = o of a head, float32 [T, H, dv]; with ``floors`` (float32 [H, T]; ``o`` is then [T, H, dv + 1]) divided by
+        max(|o[dv]|, floor) + 1e-6; then x / sqrt(mean(x^2) + eps) * weight * gate(proj[:, gate_at:]) * scale in
+        ``out[:, out_at : out_at + H dv]``.  ``weight``: float32 [H dv] or None; ``gate``: "silu" or "sigmoid"."""
+        T = o.shape[0]
+        self._want(o, "heads' outputs", torch.float32, (T, heads, dv + (1 if floors is not None else 0)))
+        if floors is not None:
+            self._want(floors, "normalisers' floors", torch.float32, (heads, T))
+        if weight is not None:
+            self._want(weight, "norm weight", torch.float32, (heads * dv,))
+        self._want(proj, "projections", out.dtype)
+        if proj.shape[0] != T or gate_at < 0 or proj.shape[1] < gate_at + heads * dv:
+            raise KernelError("the gate lies outside the projections")
+        if gate not in self.OUTPUT_GATES:
+            raise KernelError(f"gate '{gate}' is not known; known: {', '.join(sorted(self.OUTPUT_GATES))}")
+        _, out_ptr, out_ld = self._rows_into((out, out_at), T, heads * dv, proj.dtype)
+        self._call(self.lib.tli_head_norm_gate, o.data_ptr(), _ptr(floors), _ptr(weight),
+                   proj.data_ptr() + gate_at * proj.element_size(), proj.shape[1], out_ptr, out_ld, T, heads, dv, float(eps),
+                   self.OUTPUT_GATES[gate], float(scale), _dtype_code(proj.dtype), self._stream())
 
     def sample(self, logits: torch.Tensor, temperatures: Optional[torch.Tensor] = None,
                seeds: Optional[torch.Tensor] = None, top_p: Optional[torch.Tensor] = None) -> torch.Tensor:

@@ -4,3 +4,4 @@ from . import sinepel  # noqa: F401
 from . import kapanex  # noqa: F401
 from . import gimipel  # noqa: F401
 from . import defosun  # noqa: F401
+from . import kosusun  # noqa: F401

@@ -41,8 +41,9 @@ class GroupView:
     tensors: Dict[str, torch.Tensor]   # record name -> [layers in group, pages, *page shape of the record]
     tables: torch.Tensor          # int32 [sequences in step, table width], -1 where no page
     table_width: int
-    page_size: int
+    page_size: int                # slots of a page
     window: Optional[int]
+    stride: int = 1               # positions that a slot stands for
 
 
 @dataclass
@@ -51,6 +52,7 @@ class LayerCache:
     group: GroupView
     layer: int                    # index inside the group's tensors
     writes: bool                  # False: keys/values were written by another call of this step
+    further: List["LayerCache"] = field(default_factory=list)    # of the mixer's further needs, in their order
 
     def record(self, name: str) -> torch.Tensor:
         """This layer's tensor of the record ``name``: [pages, *page shape]."""
@@ -177,7 +179,9 @@ class Mixer(Part):
     # before it may then leave its scalar factor to that product (``lazy`` norms)
     takes_normed_rows = False
 
-    def cache_need(self) -> Optional[CacheNeed]:
+    def cache_need(self):
+        """None, a ``CacheNeed``, or a tuple of them: the first one's layer is ``step.cache``, the
+        others' are ``step.cache.further``."""
         return None
 
     def state_need(self) -> Optional[StateNeed]:

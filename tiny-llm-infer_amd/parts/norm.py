@@ -2,7 +2,9 @@
 (kernels/src/rmsnorm_kernel_cpu.cpp:27-43).  The weight is a plain multiplier; a
 norm whose spec names no weight has none (all ones).  ``weight_offset`` c: the checkpoint stores
 the multiplier less c (a weight kept around zero is ``weight_offset`` 1), added in float32 when
-the weight is loaded.
+the weight is loaded.  ``output_scale`` s: what the norm gives is s times that (a constant that a
+design puts behind the product which follows, such as a factor of the logits), taken into the
+float32 weight likewise.
 The residual stream is float32; the norm adds what the previous part owes the
 residual before it normalises, so the residual sum is never rounded.
 
@@ -29,6 +31,7 @@ class RMSNorm(Norm):
         self.eps = float(spec.params["eps"])
         self.weight_name = spec.names.get("weight")             # None: a norm without weights
         self.offset = float(spec.params.get("weight_offset", 0.0))
+        self.output_scale = float(spec.params.get("output_scale", 1.0))
         self.weight: Optional[torch.Tensor] = None
 
     def tensors(self) -> List[TensorDecl]:
@@ -44,6 +47,8 @@ class RMSNorm(Norm):
             self.weight = weights[self.weight_name].to(torch.float32).contiguous()
             if self.offset != 0.0:
                 self.weight = (self.weight + self.offset).contiguous()
+        if self.output_scale != 1.0:
+            self.weight = (self.weight * self.output_scale).contiguous()
 
     def as_rms(self):
         return self.weight, self.eps
