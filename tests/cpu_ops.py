@@ -360,8 +360,17 @@ class CpuOps:
         y = x.to(torch.float32) @ w.to(torch.float32).t()
         return y.to(out_dtype or x.dtype)
 
-    def linear_swiglu(self, x, m):
-        return self.swiglu(self.linear(x, m))
+    def check_gate_activation(self, name):
+        assert name in ("silu", "gelu_tanh")
+
+    def linear_swiglu(self, x, m, activation="silu", scale=1.0, into=None):
+        if into is None:
+            return self.swiglu(self.linear(x, m))
+        gu = self.linear(x, m, out_dtype=torch.float32)
+        n = gu.shape[1] // 2
+        out, at = into
+        out[:, at:at + n] = (self.activation(gu[:, :n], activation) * gu[:, n:] * scale).to(out.dtype)
+        return out
 
     @staticmethod
     def _gated(g, u, limit, slope):
@@ -450,6 +459,124 @@ class CpuOps:
         n = o.shape[1]
         g = proj[:, gate_at:gate_at + n].to(torch.float32)
         return (o * torch.rsqrt((o * o).mean(-1, keepdim=True) + eps) * weight * torch.sigmoid(g)).to(out_dtype)
+
+    # ---- attention over a window and pooled blocks, retention, mLSTM ----------------------
+    @staticmethod
+    def _turned(x, rotary, pos):
+        """x [T, heads, d] turned, pairs of either kind."""
+        if rotary is None:
+            return x
+        cos, sin, rd, pairing = rotary
+        c, s = cos[pos][:, None, :], sin[pos][:, None, :]
+        a, b = (x[..., 0:rd:2], x[..., 1:rd:2]) if pairing == "interleaved" else (x[..., :rd // 2], x[..., rd // 2:rd])
+        u, v = a * c - b * s, b * c + a * s
+        if pairing == "interleaved":
+            return torch.cat([torch.stack([u, v], dim=-1).flatten(-2), x[..., rd:]], dim=-1)
+        return torch.cat([u, v, x[..., rd:]], dim=-1)
+
+    def pooled_window_attention(self, proj, at, step, cache, heads, kv_heads, key_dim, value_dim, bias, q_weight, k_weight,
+                                eps, rotary, scale, sinks, window, pool, out, out_at, out_scale):
+        T = step.num_rows
+        qn, kn, vn = heads * key_dim, kv_heads * key_dim, kv_heads * value_dim
+        x = proj[:, at:at + qn + kn + vn].to(torch.float32)
+        if bias is not None:
+            x = x + bias
+        unit = lambda t, w: t if w is None else t * torch.rsqrt((t * t).mean(-1, keepdim=True) + eps) * w
+        pos, seq = step.positions.long(), step.seq_of_row.long()
+        q = self._turned(unit(x[:, :qn], q_weight).reshape(T, heads, key_dim), rotary, pos).to(proj.dtype).to(torch.float32)
+        k = self._turned(unit(x[:, qn:qn + kn], k_weight).reshape(T, kv_heads, key_dim), rotary, pos)
+        v = x[:, qn + kn:].reshape(T, kv_heads, value_dim)
+        page, tables = cache.group.page_size, cache.group.tables
+        blocks = cache.further[0]
+        btables = blocks.group.tables
+        kc, vc, bk, bv = cache.record("k"), cache.record("v"), blocks.record("k"), blocks.record("v")
+
+        def held(tab, s, idx):
+            pages = tab[s, idx // page].long()
+            assert (pages >= 0).all(), "a page that is not held"
+            return pages
+        for r in range(T):                                          # tokens, and the blocks that they end
+            p = int(pos[r])
+            pg = held(tables, int(seq[r]), torch.tensor(p))
+            kc[pg, :, p % page] = k[r].to(kc.dtype)
+            vc[pg, :, :, p % page] = v[r].to(vc.dtype)
+            if (p + 1) % pool == 0:
+                idx = torch.arange(p + 1 - pool, p + 1)
+                pg = held(tables, int(seq[r]), idx)
+                b = p // pool
+                to = held(btables, int(seq[r]), torch.tensor(b))
+                bk[to, :, b % page] = kc[pg, :, idx % page].to(torch.float32).mean(0).to(bk.dtype)
+                bv[to, :, :, b % page] = vc[pg, :, :, idx % page].to(torch.float32).mean(0).to(bv.dtype)
+        mul = heads // kv_heads
+        for r in range(T):
+            p = int(pos[r])
+            idx = torch.arange(max(0, p - window + 1), p + 1)
+            pg = held(tables, int(seq[r]), idx)
+            bidx = torch.arange(max(0, (p - window + 1) // pool) if p >= window - 1 else 0)
+            bp = held(btables, int(seq[r]), bidx)
+            kk = torch.cat([kc[pg, :, idx % page], bk[bp, :, bidx % page]]).to(torch.float32)
+            vv = torch.cat([vc[pg, :, :, idx % page], bv[bp, :, :, bidx % page]]).to(torch.float32)
+            for h in range(heads):
+                sc = (kk[:, h // mul] @ q[r, h]) * scale
+                if sinks is not None:
+                    sc = torch.cat([sc, sinks[h:h + 1]])
+                w = torch.softmax(sc, dim=0)[:len(kk)]
+                o = (w @ vv[:, h // mul]) * out_scale
+                out[r, out_at + h * value_dim:out_at + (h + 1) * value_dim] = o.to(out.dtype)
+
+    def _qkv_heads(self, proj, at, heads, dk, dv):
+        x, T = proj.to(torch.float32), proj.shape[0]
+        q, k = (x[:, at + i * heads * dk:at + (i + 1) * heads * dk].reshape(T, heads, dk) for i in (0, 1))
+        return q, k, x[:, at + 2 * heads * dk:at + 2 * heads * dk + heads * dv].reshape(T, heads, dv)
+
+    def retention(self, proj, at, decay, state, step, heads, dk, dv, rotary, k_scale):
+        q, k, v = self._qkv_heads(proj, at, heads, dk, dv)
+        pos = step.positions.long()
+        q, k = self._turned(q, rotary, pos), self._turned(k, rotary, pos) * k_scale
+        out = torch.zeros(step.num_rows, heads, dv)
+        for i in range(step.num_seqs):
+            slot = step.h_slots[i]
+            S = state[slot].clone() if step.h_seq_start[i] > 0 else torch.zeros(heads, dv, dk)
+            for t in range(step.h_row_start[i], step.h_row_start[i + 1]):
+                S = decay[:, None, None] * S + v[t][:, :, None] * k[t][:, None, :]
+                out[t] = torch.einsum("hvk,hk->hv", S, q[t])
+            state[slot] = S
+        return out
+
+    def mlstm_state_shape(self, heads, dk, dv):
+        return (heads, dv + 1, dk)
+
+    def mlstm(self, proj, at, gates, gates_transposed, gate_bias, cap, state, m_state, step, heads, dk, dv, q_scale):
+        q, k, v = self._qkv_heads(proj, at, heads, dk, dv)
+        q = q * q_scale
+        z = cap * torch.tanh(((gates.t() if gates_transposed else gates) + gate_bias) / cap)
+        li, lf = z[:, :heads], torch.nn.functional.logsigmoid(z[:, heads:])
+        out, floors = torch.zeros(step.num_rows, heads, dv + 1), torch.zeros(heads, step.num_rows)
+        for i in range(step.num_seqs):
+            slot, fresh = step.h_slots[i], step.h_seq_start[i] == 0
+            S = torch.zeros(heads, dv + 1, dk) if fresh else state[slot].clone()
+            m = torch.zeros(heads) if fresh else m_state[slot].clone()
+            for t in range(step.h_row_start[i], step.h_row_start[i + 1]):
+                new = torch.maximum(lf[t] + m, li[t])
+                ones = torch.cat([v[t], torch.ones(heads, 1)], dim=-1)
+                S = torch.exp(lf[t] + m - new)[:, None, None] * S + torch.exp(li[t] - new)[:, None, None] * ones[:, :, None] * k[t][:, None, :]
+                m = new
+                out[t] = torch.einsum("hvk,hk->hv", S, q[t])
+                floors[:, t] = torch.exp(-m)
+            state[slot], m_state[slot] = S, m
+        return out, floors
+
+    def head_norm_gate(self, o, floors, weight, proj, gate_at, heads, dv, eps, gate, scale, out, out_at):
+        T = o.shape[0]
+        x = o
+        if floors is not None:
+            x = o[..., :dv] / (torch.maximum(o[..., dv].abs(), floors.t()) + 1e-6)[..., None]
+        x = (x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps)).reshape(T, heads * dv)
+        if weight is not None:
+            x = x * weight
+        g = proj[:, gate_at:gate_at + heads * dv].to(torch.float32)
+        x = x * torch.sigmoid(g) * (g if gate == "silu" else 1.0) * scale
+        out[:, out_at:out_at + heads * dv] = x.to(out.dtype)
 
     def qkv_to_cache(self, qkv, step, cache, heads, kv_heads, head_dim, q_norm, k_norm, rotary):
         T = step.num_rows
