@@ -66,14 +66,14 @@ DESIGN_SIZES = {
 
 
 def compare_designs(args):
-    """Prefill and decode of the Sinepel design (or, with --design-names, of others: Kapanex, Gimipel, Defosun) beside the Qwen3
+    """Prefill and decode of the Sinepel design (or, with --design-names, of others: Kapanex, Gimipel, Defosun, Kosusun) beside the Qwen3
     dense decoder at equal layer sizes
     (random bfloat16 weights, 4 layers unless --layers says otherwise), through the step function:
     one prompt of --prefill-tokens in one step, and decode steps of --batch and 64 requests at
     --prompt-len tokens of context.  One JSON line."""
     import torch
 
-    from tiny_llm_infer_amd.config import DefosunConfig, GimipelConfig, KapanexConfig, Qwen3Config, SinepelConfig
+    from tiny_llm_infer_amd.config import DefosunConfig, GimipelConfig, KapanexConfig, KosusunConfig, Qwen3Config, SinepelConfig
     from tiny_llm_infer_amd.engine.loading import random_model
     from tiny_llm_infer_amd.engine.runner import ModelRunner, StepEntry
     import random
@@ -144,7 +144,19 @@ def compare_designs(args):
         defosun = DefosunConfig.from_dict({
             "architecture": "Defosun", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "streams": 4, "max_positions": context,
             "layers": [{"type": dmixers[i % 3][0], "mixer": dmixers[i % 3][1], "mlp": dmixers[i % 3][2]} for i in range(layers)]})
-        known = {"sinepel": ("Sinepel", sinepel), "kapanex": ("Kapanex", kapanex), "gimipel": ("Gimipel", gimipel),
+        # Kosusun: an attention over a window of 1,024 and blocks of 16 beside a retention (both with heads as Qwen3's, a
+        # state of dim x dim a head), and an mLSTM (the same heads and state), in turn, each with the dense feed-forward
+        rot = {"dims": dim, "base": 1e6}
+        two = {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                        "mask": {"size": 1024, "pool": 16}, "rot": rot},
+               "right": {"heads": heads, "dim": dim, "vdim": dim, "rot": rot,
+                         "decay": [1.0 - 2.0 ** (-1 - 8 * h / heads) for h in range(heads)]}, "left_scale": 0.7, "right_scale": 0.7}
+        kmixers = [("parallel", two), ("mlstm", {"heads": heads, "dim": dim, "vdim": dim, "gate_cap": 15.0})]
+        kosusun = KosusunConfig.from_dict({
+            "architecture": "Kosusun", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "max_positions": context,
+            "embedding": {"scale": 1.0}, "residual_mult": 1.0, "logit_scale": 1.0,
+            "layers": [{"type": kmixers[i % 2][0], "mixer": kmixers[i % 2][1], "mlp": {"kind": "dense", "ff": ff}} for i in range(layers)]})
+        known = {"kosusun": ("Kosusun", kosusun), "sinepel": ("Sinepel", sinepel), "kapanex": ("Kapanex", kapanex), "gimipel": ("Gimipel", gimipel),
                  "defosun": ("Defosun", defosun), "qwen3": ("Qwen3ForCausalLM", qwen)}
         names = [n for n in args.design_names.split(",") if n]
         if any(n not in known for n in names):
@@ -226,7 +238,7 @@ def main():
                     help="instead of the default workload: the Sinepel design beside the Qwen3 dense decoder at equal layer "
                          f"sizes, prefill and decode; a list of {','.join(DESIGN_SIZES)} or 'all'")
     ap.add_argument("--design-names", default="sinepel,qwen3",
-                    help="with --designs: which designs are run at every size (sinepel, kapanex, gimipel, defosun, qwen3)")
+                    help="with --designs: which designs are run at every size (sinepel, kapanex, gimipel, defosun, kosusun, qwen3)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py runs on one GPU only; --gpus {args.gpus} is not supported (single-GPU engine)")
