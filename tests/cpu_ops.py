@@ -529,29 +529,30 @@ class CpuOps:
         q, k = (x[:, at + i * heads * dk:at + (i + 1) * heads * dk].reshape(T, heads, dk) for i in (0, 1))
         return q, k, x[:, at + 2 * heads * dk:at + 2 * heads * dk + heads * dv].reshape(T, heads, dv)
 
-    def retention(self, proj, at, decay, state, step, heads, dk, dv, rotary, k_scale):
+    def retention(self, proj, at, decay, state, step, heads, dk, dv, rotary, k_scale, eps, scale, out, out_at):
         q, k, v = self._qkv_heads(proj, at, heads, dk, dv)
         pos = step.positions.long()
         q, k = self._turned(q, rotary, pos), self._turned(k, rotary, pos) * k_scale
-        out = torch.zeros(step.num_rows, heads, dv)
+        o = torch.zeros(step.num_rows, heads, dv)
         for i in range(step.num_seqs):
             slot = step.h_slots[i]
             S = state[slot].clone() if step.h_seq_start[i] > 0 else torch.zeros(heads, dv, dk)
             for t in range(step.h_row_start[i], step.h_row_start[i + 1]):
                 S = decay[:, None, None] * S + v[t][:, :, None] * k[t][:, None, :]
-                out[t] = torch.einsum("hvk,hk->hv", S, q[t])
+                o[t] = torch.einsum("hvk,hk->hv", S, q[t])
             state[slot] = S
-        return out
+        self.head_norm_gate(o, None, None, proj, at + 2 * heads * dk + heads * dv, heads, dv, eps, "silu", scale, out, out_at)
 
     def mlstm_state_shape(self, heads, dk, dv):
         return (heads, dv + 1, dk)
 
-    def mlstm(self, proj, at, gates, gates_transposed, gate_bias, cap, state, m_state, step, heads, dk, dv, q_scale):
+    def mlstm(self, proj, at, x, w_gates, gate_bias, cap, state, m_state, step, heads, dk, dv, q_scale, weight, eps, scale, out,
+              out_at):
         q, k, v = self._qkv_heads(proj, at, heads, dk, dv)
         q = q * q_scale
-        z = cap * torch.tanh(((gates.t() if gates_transposed else gates) + gate_bias) / cap)
+        z = cap * torch.tanh((x.to(torch.float32) @ w_gates.to(torch.float32).t() + gate_bias) / cap)
         li, lf = z[:, :heads], torch.nn.functional.logsigmoid(z[:, heads:])
-        out, floors = torch.zeros(step.num_rows, heads, dv + 1), torch.zeros(heads, step.num_rows)
+        o, floors = torch.zeros(step.num_rows, heads, dv + 1), torch.zeros(heads, step.num_rows)
         for i in range(step.num_seqs):
             slot, fresh = step.h_slots[i], step.h_seq_start[i] == 0
             S = torch.zeros(heads, dv + 1, dk) if fresh else state[slot].clone()
@@ -561,10 +562,10 @@ class CpuOps:
                 ones = torch.cat([v[t], torch.ones(heads, 1)], dim=-1)
                 S = torch.exp(lf[t] + m - new)[:, None, None] * S + torch.exp(li[t] - new)[:, None, None] * ones[:, :, None] * k[t][:, None, :]
                 m = new
-                out[t] = torch.einsum("hvk,hk->hv", S, q[t])
+                o[t] = torch.einsum("hvk,hk->hv", S, q[t])
                 floors[:, t] = torch.exp(-m)
             state[slot], m_state[slot] = S, m
-        return out, floors
+        self.head_norm_gate(o, floors, weight, proj, at + 2 * heads * dk + heads * dv, heads, dv, eps, "sigmoid", scale, out, out_at)
 
     def head_norm_gate(self, o, floors, weight, proj, gate_at, heads, dv, eps, gate, scale, out, out_at):
         T = o.shape[0]

@@ -287,7 +287,7 @@ RECURRENT = [(2, 16, 24), (3, 20, 12), (1, 40, 20), (4, 64, 32), (2, 128, 128), 
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("lengths, cuts", [([61, 97, 45], [1, 43, 2, 16, 33, 7]), ([900, 30, 301], [700, 390, 1, 2])])
+@pytest.mark.parametrize("lengths, cuts", [([61, 97, 45], [1, 43, 2, 16, 33, 7]), ([900, 30, 301], [700, 390, 1, 2]), ([24, 20, 3], [1])])
 @pytest.mark.parametrize("heads, dk, dv", RECURRENT)
 def test_retention_in_portions_and_slots_that_are_used_again(ops, dtype, heads, dk, dv, lengths, cuts):
     """Sequences side by side in portions down to one row, also long ones that are walked in segments; then
@@ -316,9 +316,10 @@ def test_retention_in_portions_and_slots_that_are_used_again(ops, dtype, heads, 
         got = [[] for _ in lengths]
         for starts, counts, live in _portions(lengths, cuts):
             rows = torch.cat([torch.zeros(sum(counts), 3, dtype=dt), torch.cat([proj[i][s:s + c] for i, s, c in zip(live, starts, counts)])], dim=1).cuda()
-            o = ops.retention(rows, 3, decay.cuda(), state, _view(starts, counts, [slots[i] for i in live]), heads, dk, dv, part.rotary(), dk ** -0.5)
-            y = torch.zeros((len(rows), (heads * dv + 15) // 8 * 8), dtype=dt, device="cuda")
-            ops.head_norm_gate(o, None, None, rows, 3 + 2 * heads * dk + heads * dv, heads, dv, 1e-5, "silu", 0.7, y, 8)
+            y = torch.full((len(rows), (heads * dv + 15) // 8 * 8), 4.0, dtype=dt, device="cuda")
+            ops.retention(rows, 3, decay.cuda(), state, _view(starts, counts, [slots[i] for i in live]), heads, dk, dv, part.rotary(), dk ** -0.5,
+                          1e-5, 0.7, y, 8)
+            assert (y[:, :8] == 4.0).all() and (y[:, 8 + heads * dv:] == 4.0).all()
             r = 0
             for i, c in zip(live, counts):
                 got[i].append(y[r:r + c, 8:8 + heads * dv].cpu())
@@ -329,7 +330,7 @@ def test_retention_in_portions_and_slots_that_are_used_again(ops, dtype, heads, 
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("lengths, cuts", [([61, 97, 45], [1, 43, 2, 16, 33, 7]), ([900, 30, 301], [700, 390, 1, 2])])
+@pytest.mark.parametrize("lengths, cuts", [([61, 97, 45], [1, 43, 2, 16, 33, 7]), ([900, 30, 301], [700, 390, 1, 2]), ([24, 20, 3], [1])])
 @pytest.mark.parametrize("heads, dk, dv", RECURRENT)
 def test_matrix_memory_in_portions_and_slots_that_are_used_again(ops, dtype, heads, dk, dv, lengths, cuts):
     """As the retention's test; gates that open and close, so that the running maximum is taken over again and again, and
@@ -341,6 +342,8 @@ def test_matrix_memory_in_portions_and_slots_that_are_used_again(ops, dtype, hea
     m = {"heads": heads, "dim": dk, "vdim": dv, "gate_cap": cap}
     wide = 2 * heads * dk + 2 * heads * dv
     eye = torch.eye(wide + 2 * heads, dtype=F64)
+    n = 4 * heads + (8 if dk % 8 == 0 else 3)                        # the layer's input, which only the gates read here
+    w_gates = (torch.randn(2 * heads, n, generator=g) * 2 * n ** -0.5).to(dt)
     bias = torch.randn(2 * heads, generator=g)
     bias[heads:] += 3.0
     bias[heads] = 40.0
@@ -352,24 +355,26 @@ def test_matrix_memory_in_portions_and_slots_that_are_used_again(ops, dtype, hea
     maxima = torch.full((3, heads), 50.0, device="cuda")
     for slots in ([0, 1, 2], [2, 0, 1]):
         proj = [(torch.randn(n, wide, generator=g)).to(dt) for n in lengths]
-        z = [torch.randn(n, 2 * heads, generator=g) * 2.0 for n in lengths]
+        x = [torch.randn(c, n, generator=g).to(dt) for c in lengths]
         for p in proj:
             p[:, heads * dk:2 * heads * dk] += p[:, :heads * dk]
         got = [[] for _ in lengths]
-        for k, (starts, counts, live) in enumerate(_portions(lengths, cuts)):
+        for k, (starts, counts, live) in enumerate(_portions(lengths, cuts + [1])):
             rows = torch.cat([torch.zeros(sum(counts), 5, dtype=dt), torch.cat([proj[i][s:s + c] for i, s, c in zip(live, starts, counts)])], dim=1).cuda()
-            gates = torch.cat([z[i][s:s + c] for i, s, c in zip(live, starts, counts)]).cuda()
-            flip = k % 2 == 1                                                                    # both layouts of the gates' products
-            o, floors = ops.mlstm(rows, 5, gates.t().contiguous() if flip else gates, flip, bias.cuda(), cap, state, maxima,
-                                  _view(starts, counts, [slots[i] for i in live]), heads, dk, dv, dk ** -0.5)
-            y = torch.zeros((len(rows), (heads * dv + 7) // 8 * 8), dtype=dt, device="cuda")
-            ops.head_norm_gate(o, floors, weight.cuda(), rows, 5 + at[3], heads, dv, 1e-5, "sigmoid", 1.0, y, 0)
+            inputs = torch.cat([x[i][s:s + c] for i, s, c in zip(live, starts, counts)]).cuda()
+            if k % 3 == 2 and dtype == "bfloat16":                                               # rows that still owe a factor of 1/2, in three parts
+                from tiny_llm_infer_amd.kernels.ops import NormedRows
+                inputs = NormedRows((inputs.float() * 2).to(dt), torch.full((3, len(rows)), n * 3.9 / 3, device="cuda"), 0.1)
+            y = torch.full((len(rows), (heads * dv + 7) // 8 * 8), 4.0, dtype=dt, device="cuda")
+            ops.mlstm(rows, 5, inputs, w_gates.cuda(), bias.cuda(), cap, state, maxima, _view(starts, counts, [slots[i] for i in live]), heads, dk, dv,
+                      dk ** -0.5, weight.cuda(), 1e-5, 1.3, y, 0)
+            assert (y[:, heads * dv:] == 4.0).all()
             r = 0
             for i, c in zip(live, counts):
                 got[i].append(y[r:r + c, :heads * dv].cpu())
                 r += c
         for i in range(len(lengths)):
-            want = plain_kosusun.mlstm(torch.cat([proj[i].double(), z[i].double()], dim=1), m, names, "", 1e-5)
+            want = 1.3 * plain_kosusun.mlstm(torch.cat([proj[i].double(), x[i].double() @ w_gates.double().T], dim=1), m, names, "", 1e-5)
             _close(torch.cat(got[i]), want, 5e-5 if dtype == "float32" else 1.5e-2, f"sequence {i} in slot {slots[i]}")
 
 

@@ -17,11 +17,9 @@
 // mlstm_prepare: a workgroup a (row, head) leaves q, k and v in float32 for the recurrence.  In a step of single rows
 // (`single`) it makes the gates itself and there is no scan.
 #include "recurrence.h"
+#include "row_gates.h"
 
 #define ML_THREADS TLI_RECURRENCE_SEGMENT
-
-__device__ __forceinline__ float ml_capped(float z, float cap) { return cap * tanhf(z / cap); }
-__device__ __forceinline__ float ml_log_sigmoid(float u) { return fminf(u, 0.f) - log1pf(expf(-fabsf(u))); }
 
 struct MlGates {
     const float* z;          // logits: head h's input gate of row r at z[r z_row + h z_col], its forget gate H columns on
@@ -29,9 +27,10 @@ struct MlGates {
     const float* bias;       // [2 H]
     float cap;
     int H;
-    __device__ __forceinline__ float input(int r, int h) const { return ml_capped(z[r * z_row + h * z_col] + bias[h], cap); }
-    __device__ __forceinline__ float forget(int r, int h) const {
-        return ml_log_sigmoid(ml_capped(z[r * z_row + (H + h) * z_col] + bias[H + h], cap));
+    RowFactor factor;        // of the rows that the logits were made from
+    __device__ __forceinline__ float input(int r, int h, float f) const { return gate_capped(z[r * z_row + h * z_col] * f + bias[h], cap); }
+    __device__ __forceinline__ float forget(int r, int h, float f) const {
+        return gate_log_sigmoid(gate_capped(z[r * z_row + (H + h) * z_col] * f + bias[H + h], cap));
     }
 };
 
@@ -50,8 +49,9 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_scan_kernel(MlGates gates, f
     for (int first = 0; first < n; first += ML_THREADS) {
         const int r = r0 + first + tid;
         const bool live = first + tid < n;
-        const float f = live ? gates.forget(r, h) : 0.f;
-        const float i = live ? gates.input(r, h) : -INFINITY;          // (a row past the end leaves m alone)
+        const float owed = live ? gates.factor.of(r) : 1.f;
+        const float f = live ? gates.forget(r, h, owed) : 0.f;
+        const float i = live ? gates.input(r, h, owed) : -INFINITY;          // (a row past the end leaves m alone)
         float F = f, M = i;                                            // the map of this row and those before it in the wave
 #pragma unroll
         for (int off = 1; off < TLI_WAVE; off <<= 1) {
@@ -102,7 +102,8 @@ __global__ void mlstm_prepare_kernel(const T* __restrict__ proj, int ld, float q
     if (single) {                                                      // row r is sequence r
         float* slot = m_state + (size_t)slots[row] * H + h;
         const float m0 = seq_start[row] != 0 ? *slot : 0.f;
-        const float f = gates.forget((int)row, h), i = gates.input((int)row, h);
+        const float owed = gates.factor.of((int)row);
+        const float f = gates.forget((int)row, h, owed), i = gates.input((int)row, h, owed);
         const float m = fmaxf(f + m0, i);
         take = expf(i - m);
         __syncthreads();                                               // m0 is read by all before it is replaced
@@ -130,11 +131,13 @@ __global__ void mlstm_prepare_kernel(const T* __restrict__ proj, int ld, float q
     }
 }
 
-// proj: [T, ld], q (H dk), k (H dk), v (H dv) first; z, z_row, z_col, bias, cap: the gates (MlGates); m_state: float32
+// proj: [T, ld], q (H dk), k (H dk), v (H dv) first; z, z_row, z_col, bias, cap: the gates (MlGates; ssq: [parts][T] sums
+// of squares of rows of x_size elements whose factor the logits still owe, or null); m_state: float32
 // [slots, H]; state: float32 [slots, H, dv + 1, dk]; out: float32 [T, H, dv + 1]; floors: float32 [H][T] (written);
 // scratch: tli_lightning_scratch_floats(T, seqs, longest, H, dk, dv + 1) and 3 H T floats behind it at `rows_scratch`;
 // longest: the most rows that a sequence brings; single: every sequence brings one row
-extern "C" int tli_mlstm(const void* proj, int ld, const float* z, long long z_row, long long z_col, const float* bias, float cap,
+extern "C" int tli_mlstm(const void* proj, int ld, const float* z, long long z_row, long long z_col, const float* ssq, int parts,
+                         int x_size, float x_eps, const float* bias, float cap,
                          float q_scale, float* m_state, float* state, float* out, float* floors, float* scratch,
                          float* rows_scratch, const int* row_start, const int* seq_start, const int* slots, int T, int seqs,
                          int longest, int single, int H, int dk, int dv, int dtype, int lanes, void* stream) {
@@ -150,7 +153,8 @@ extern "C" int tli_mlstm(const void* proj, int ld, const float* z, long long z_r
     float* keep = rows_scratch;
     float* take = keep + (size_t)H * T;
     float* through = take + (size_t)H * T;
-    const MlGates gates{z, z_row, z_col, bias, cap, H};
+    if (ssq && (parts <= 0 || x_size <= 0)) return tli_fail("mlstm: bad sums of squares");
+    const MlGates gates{z, z_row, z_col, bias, cap, H, RowFactor{ssq, ssq ? parts : 0, T, 1.0f / (float)(x_size > 0 ? x_size : 1), x_eps}};
     hipStream_t s = (hipStream_t)stream;
     if (!single)
         mlstm_scan_kernel<<<dim3(H, seqs), ML_THREADS, 0, s>>>(gates, m_state, keep, take, floors, through, row_start, seq_start, slots, T);

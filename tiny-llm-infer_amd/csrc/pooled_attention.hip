@@ -11,7 +11,7 @@
 #include "common.h"
 #include "pooled.h"
 
-#define PN_THREADS 256
+#define PN_THREADS 512
 
 // the mean of element (key: d of kv head g; value likewise) over the block's positions, read from the tokens' pages
 template <typename T, bool VALUE>
@@ -28,99 +28,171 @@ __device__ __forceinline__ float block_mean(const T* __restrict__ cache, const i
     return sum / (float)pool;
 }
 
+// element e of a block's means of kv head g: e < key_dim the key's, then the value's
 template <typename T>
-__device__ __forceinline__ void store_block_means(const T* __restrict__ k_cache, const T* __restrict__ v_cache,
-                                                  const int* __restrict__ table, int page_size, int num_pages, int kv_heads,
-                                                  int key_dim, int value_dim, int g, int block, const PooledKeys& pooled,
-                                                  const int* __restrict__ pooled_table, int first_thread, int threads) {
+__device__ __forceinline__ void store_block_mean(const T* __restrict__ k_cache, const T* __restrict__ v_cache,
+                                                 const int* __restrict__ table, int page_size, int num_pages, int kv_heads,
+                                                 int key_dim, int value_dim, int g, int e, int block, const PooledKeys& pooled,
+                                                 const int* __restrict__ pooled_table) {
     const int page = pooled_table[block / page_size], slot = block % page_size;
     if (page < 0 || page >= pooled.pages) return;
-    T* k_dst = (T*)pooled.k + (((size_t)page * kv_heads + g) * page_size + slot) * key_dim;
-    T* v_dst = (T*)pooled.v + ((size_t)page * kv_heads + g) * page_size * value_dim + slot;
-    for (int e = first_thread; e < key_dim + value_dim; e += threads) {
-        T m;
-        if (e < key_dim) {
-            from_f32(&m, block_mean<T, false>(k_cache, table, page_size, num_pages, kv_heads, g, key_dim, e, block * pooled.pool, pooled.pool));
-            k_dst[e] = cache_value(m);
-        } else {
-            const int d = e - key_dim;
-            from_f32(&m, block_mean<T, true>(v_cache, table, page_size, num_pages, kv_heads, g, value_dim, d, block * pooled.pool, pooled.pool));
-            v_dst[(size_t)d * page_size] = cache_value(m);
-        }
+    const size_t head = ((size_t)page * kv_heads + g) * page_size;
+    T m;
+    if (e < key_dim) {
+        from_f32(&m, block_mean<T, false>(k_cache, table, page_size, num_pages, kv_heads, g, key_dim, e, block * pooled.pool, pooled.pool));
+        ((T*)pooled.k)[(head + slot) * key_dim + e] = cache_value(m);
+    } else {
+        const int d = e - key_dim;
+        from_f32(&m, block_mean<T, true>(v_cache, table, page_size, num_pages, kv_heads, g, value_dim, d, block * pooled.pool, pooled.pool));
+        ((T*)pooled.v)[head * value_dim + (size_t)d * page_size + slot] = cache_value(m);
     }
 }
 
-template <typename T>
+// N consecutive elements at once: 8 where sizes and addresses allow 16-byte accesses of bfloat16, else 1
+template <int N, typename T>
+__device__ __forceinline__ void pn_load(const T* p, float (&v)[N]) {
+    if constexpr (N == 8) {
+        const uint4 w = *reinterpret_cast<const uint4*>(p);
+        const uint32_t u[4] = {w.x, w.y, w.z, w.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[2 * i] = bf16_to_f32((bf16_t)(u[i] & 0xffffu)), v[2 * i + 1] = bf16_to_f32((bf16_t)(u[i] >> 16));
+    } else {
+        v[0] = to_f32(p[0]);
+    }
+}
+template <int N>
+__device__ __forceinline__ void pn_load_f32(const float* p, float (&v)[N]) {
+    if constexpr (N == 8) {
+        const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+        v[0] = a.x, v[1] = a.y, v[2] = a.z, v[3] = a.w, v[4] = b.x, v[5] = b.y, v[6] = b.z, v[7] = b.w;
+    } else {
+        v[0] = p[0];
+    }
+}
+template <int N, bool CACHE, typename T>
+__device__ __forceinline__ void pn_store(T* p, const float (&v)[N]) {
+    T o[N];
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+        from_f32(o + i, v[i]);
+        if (CACHE) o[i] = cache_value(o[i]);
+    }
+    if constexpr (N == 8)
+        *reinterpret_cast<uint4*>(p) = make_uint4(o[0] | (uint32_t)o[1] << 16, o[2] | (uint32_t)o[3] << 16, o[4] | (uint32_t)o[5] << 16,
+                                                  o[6] | (uint32_t)o[7] << 16);
+    else
+        p[0] = o[0];
+}
+
+// N: elements a thread takes at once (8: every size in eights, operands 16-byte aligned)
+template <typename T, int N>
 __global__ __launch_bounds__(PN_THREADS) void projection_norm_prepare_kernel(
     const T* __restrict__ proj, int ld, const float* __restrict__ bias, T* __restrict__ q_out, T* k_cache, T* v_cache,
     const int* __restrict__ positions, const int* __restrict__ seq_of_row, const int* __restrict__ tables, int table_width,
     int page_size, int num_pages, int heads, int kv_heads, int key_dim, int value_dim, const float* __restrict__ q_weight,
     const float* __restrict__ k_weight, float eps, const float* __restrict__ cos_table, const float* __restrict__ sin_table,
     int dims, int pairing, int table_positions, PooledKeys pooled, int single) {
-    extern __shared__ float pn_row[];                    // q and k of the row, all heads
+    extern __shared__ __align__(16) float pn_row[];      // q and k of the row, all heads, times their norm's weights
     __shared__ float red[16];
     const int row = blockIdx.x, tid = threadIdx.x;
-    const int qn = heads * key_dim, kn = kv_heads * key_dim;
+    const int qn = heads * key_dim, kn = kv_heads * key_dim, vn = kv_heads * value_dim;
     const T* src = proj + (size_t)row * ld;
-    float ssq = 0.f, ssk = 0.f;
-    for (int i = tid; i < qn + kn; i += PN_THREADS) {
-        const float x = to_f32(src[i]) + (bias ? bias[i] : 0.f);
-        pn_row[i] = x;
-        if (i < qn) ssq = fmaf(x, x, ssq);
-        else ssk = fmaf(x, x, ssk);
-    }
-    const float q_factor = q_weight ? 1.0f / sqrtf(block_sum(ssq, red) / (float)qn + eps) : 1.f;
-    const float k_factor = k_weight ? 1.0f / sqrtf(block_sum(ssk, red) / (float)kn + eps) : 1.f;
-    __syncthreads();
     const int pos = positions[row];
     const int* table = tables + (size_t)seq_of_row[row] * table_width;
     const int page = table[pos / page_size], slot = pos % page_size;
     const bool kept = page >= 0 && page < num_pages;
+    float ssq = 0.f, ssk = 0.f;
+    for (int i = tid * N; i < qn + kn; i += PN_THREADS * N) {
+        float x[N], w[N];
+        pn_load<N>(src + i, x);
+        if (bias) {
+            pn_load_f32<N>(bias + i, w);
+#pragma unroll
+            for (int j = 0; j < N; ++j) x[j] += w[j];
+        }
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < N; ++j) ss = fmaf(x[j], x[j], ss);
+        const bool is_q = i < qn;
+        const float* weight = is_q ? q_weight : k_weight;
+        (is_q ? ssq : ssk) += ss;
+        if (weight) {
+            pn_load_f32<N>(weight + (is_q ? i : i - qn), w);
+#pragma unroll
+            for (int j = 0; j < N; ++j) x[j] *= w[j];
+        }
+#pragma unroll
+        for (int j = 0; j < N; ++j) pn_row[i + j] = x[j];
+    }
+    if (kept)
+        for (int i = tid * N; i < vn; i += PN_THREADS * N) {
+            float x[N], w[N];
+            pn_load<N>(src + qn + kn + i, x);
+            if (bias) {
+                pn_load_f32<N>(bias + qn + kn + i, w);
+#pragma unroll
+                for (int j = 0; j < N; ++j) x[j] += w[j];
+            }
+#pragma unroll
+            for (int j = 0; j < N; ++j) {
+                T v;
+                from_f32(&v, x[j]);
+                v_cache[((size_t)page * vn + i + j) * page_size + slot] = cache_value(v);      // (kv head, dim) is i + j
+            }
+        }
+    // (the sums of q and of k in one exchange)
+    {
+        const float a = wave_sum(ssq), b = wave_sum(ssk);
+        if (tid % TLI_WAVE == 0) red[tid / TLI_WAVE] = a, red[8 + tid / TLI_WAVE] = b;
+    }
+    __syncthreads();                                     // (pn_row as well)
+    float q_factor = 1.f, k_factor = 1.f;
+    {
+        float a = 0.f, b = 0.f;
+#pragma unroll
+        for (int w = 0; w < PN_THREADS / TLI_WAVE; ++w) a += red[w], b += red[8 + w];
+        if (q_weight) q_factor = 1.0f / sqrtf(a / (float)qn + eps);
+        if (k_weight) k_factor = 1.0f / sqrtf(b / (float)kn + eps);
+    }
     const int half = dims / 2;
     const bool turn = cos_table && pos >= 0 && pos < table_positions;
     const float* cos_row = turn ? cos_table + (size_t)pos * half : nullptr;
     const float* sin_row = turn ? sin_table + (size_t)pos * half : nullptr;
-    for (int i = tid; i < qn + kn; i += PN_THREADS) {
+    for (int i = tid * N; i < qn + kn; i += PN_THREADS * N) {
         const bool is_q = i < qn;
-        const float* w = is_q ? q_weight : k_weight;
-        const int base = is_q ? 0 : qn;
+        const int base = is_q ? 0 : qn, d0 = (i - base) % key_dim;
         const float factor = is_q ? q_factor : k_factor;
-        auto normed = [&](int j) { return w ? pn_row[j] * factor * w[j - base] : pn_row[j]; };
-        const int d = (i - base) % key_dim;
-        float x = normed(i);
-        if (turn && d < dims) {
-            const bool second = pairing ? (d & 1) : d >= half;
-            const int pair = pairing ? d / 2 : second ? d - half : d;
-            const float other = normed(pairing ? (second ? i - 1 : i + 1) : second ? i - half : i + half);
-            x = second ? rotate_second_half(x, other, cos_row[pair], sin_row[pair])
-                       : rotate_first_half(x, other, cos_row[pair], sin_row[pair]);
+        float x[N];
+#pragma unroll
+        for (int j = 0; j < N; ++j) {
+            const int d = d0 + j;
+            x[j] = pn_row[i + j] * factor;
+            if (turn && d < dims) {
+                const bool second = pairing ? (d & 1) : d >= half;
+                const int pair = pairing ? d / 2 : second ? d - half : d;
+                const int at = i + j;
+                const float other = pn_row[pairing ? (second ? at - 1 : at + 1) : second ? at - half : at + half] * factor;
+                x[j] = second ? rotate_second_half(x[j], other, cos_row[pair], sin_row[pair])
+                              : rotate_first_half(x[j], other, cos_row[pair], sin_row[pair]);
+            }
         }
-        if (is_q) {
-            from_f32(q_out + (size_t)row * qn + i, x);
-        } else if (kept) {
-            T k;
-            from_f32(&k, x);
-            k_cache[(((size_t)page * kv_heads + (i - qn) / key_dim) * page_size + slot) * key_dim + d] = cache_value(k);
-        }
+        if (is_q) pn_store<N, false>(q_out + (size_t)row * qn + i, x);
+        else if (kept) pn_store<N, true>(k_cache + (((size_t)page * kv_heads + (i - qn) / key_dim) * page_size + slot) * key_dim + d0, x);
     }
-    const int vn = kv_heads * value_dim;
-    if (kept)
-        for (int i = tid; i < vn; i += PN_THREADS) {
-            T v;
-            from_f32(&v, to_f32(src[qn + kn + i]) + (bias ? bias[qn + kn + i] : 0.f));
-            v_cache[((size_t)page * vn + i) * page_size + slot] = cache_value(v);      // (kv head, dim) is i
-        }
     if (single && pooled.pool > 0 && (pos + 1) % pooled.pool == 0) {
         __syncthreads();                                 // the row's own key and value are in their page
         const int* pooled_table = pooled.tables + (size_t)seq_of_row[row] * pooled.width;
-        for (int g = 0; g < kv_heads; ++g)
-            store_block_means<T>(k_cache, v_cache, table, page_size, num_pages, kv_heads, key_dim, value_dim, g, pos / pooled.pool,
-                                 pooled, pooled_table, tid, PN_THREADS);
+        const int each = key_dim + value_dim;
+        for (int u = tid; u < kv_heads * each; u += PN_THREADS)
+            store_block_mean<T>(k_cache, v_cache, table, page_size, num_pages, kv_heads, key_dim, value_dim, u / each, u % each,
+                                pos / pooled.pool, pooled, pooled_table);
     }
 }
 
+#define PB_THREADS 256
+
 template <typename T>
-__global__ __launch_bounds__(PN_THREADS) void pool_blocks_kernel(
+__global__ __launch_bounds__(PB_THREADS) void pool_blocks_kernel(
     const T* __restrict__ k_cache, const T* __restrict__ v_cache, const int* __restrict__ row_start,
     const int* __restrict__ seq_start, int num_seqs, const int* __restrict__ tables, int table_width, int page_size, int num_pages,
     int kv_heads, int key_dim, int value_dim, PooledKeys pooled) {
@@ -135,8 +207,9 @@ __global__ __launch_bounds__(PN_THREADS) void pool_blocks_kernel(
         block -= count;
     }
     if (seq >= num_seqs) return;                         // (the grid's slack)
-    store_block_means<T>(k_cache, v_cache, tables + (size_t)seq * table_width, page_size, num_pages, kv_heads, key_dim, value_dim,
-                         blockIdx.y, block, pooled, pooled.tables + (size_t)seq * pooled.width, threadIdx.x, blockDim.x);
+    for (int e = threadIdx.x; e < key_dim + value_dim; e += blockDim.x)
+        store_block_mean<T>(k_cache, v_cache, tables + (size_t)seq * table_width, page_size, num_pages, kv_heads, key_dim, value_dim,
+                            blockIdx.y, e, block, pooled, pooled.tables + (size_t)seq * pooled.width);
 }
 
 // proj: [rows, ld], q (heads key_dim) | k (kv_heads key_dim) | v (kv_heads value_dim) first; bias: float32 over these or
@@ -161,9 +234,9 @@ extern "C" int tli_pooled_prepare(const void* proj, int ld, const float* bias, v
     if (lds > 150 * 1024) return tli_fail("pooled_prepare: q and k of %zu bytes do not fit LDS", lds);
     const PooledKeys pooled{pooled_k, pooled_v, pooled_tables, pooled_width, pooled_pages, pool};
     hipStream_t s = (hipStream_t)stream;
-#define PN_RUN(T)                                                                                                              \
+#define PN_RUN(T, N)                                                                                                           \
     {                                                                                                                          \
-        auto kernel = projection_norm_prepare_kernel<T>;                                                                       \
+        auto kernel = projection_norm_prepare_kernel<T, N>;                                                                    \
         static bool allowed = false;                                                                                           \
         if (lds > 65536 && !allowed) {                                                                                         \
             if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024) != hipSuccess) \
@@ -175,12 +248,15 @@ extern "C" int tli_pooled_prepare(const void* proj, int ld, const float* bias, v
                                              value_dim, q_weight, k_weight, eps, cos_table, sin_table, dims, pairing,          \
                                              table_positions, pooled, single);                                                 \
         if (pool > 0 && !single)                                                                                               \
-            pool_blocks_kernel<T><<<dim3(rows / pool + num_seqs, kv_heads), PN_THREADS, 0, s>>>(                               \
+            pool_blocks_kernel<T><<<dim3(rows / pool + num_seqs, kv_heads), PB_THREADS, 0, s>>>(                               \
                 (const T*)k_cache, (const T*)v_cache, row_start, seq_start, num_seqs, tables, table_width, page_size,          \
                 num_pages, kv_heads, key_dim, value_dim, pooled);                                                              \
     }
-    if (dtype == TLI_F32) PN_RUN(float)
-    else if (dtype == TLI_BF16) PN_RUN(bf16_t)
+    const bool eights = ld % 8 == 0 && key_dim % 8 == 0 && value_dim % 8 == 0 &&
+                        !(((uintptr_t)proj | (uintptr_t)bias | (uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)q_weight | (uintptr_t)k_weight) & 15);
+    if (dtype == TLI_F32) PN_RUN(float, 1)
+    else if (dtype == TLI_BF16 && eights) PN_RUN(bf16_t, 8)
+    else if (dtype == TLI_BF16) PN_RUN(bf16_t, 1)
     else return tli_fail("pooled_prepare: unknown dtype %d", dtype);
 #undef PN_RUN
     return tli_check_launch("pooled_prepare");

@@ -134,7 +134,9 @@ def load_library():
         "tli_lightning_recurrence": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
         "tli_lightning_norm": [P, P, I, P, P, I, I, F, I, P],
         "tli_retention": [P, I, P, P, P, P, P, P, P, P, P, P, I, I, I, F, I, I, I, I, I, I, I, I, P],
-        "tli_mlstm": [P, I, P, ctypes.c_longlong, ctypes.c_longlong, P, F, F, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
+        "tli_retention_step": [P, I, P, P, P, I, P, P, P, P, P, I, I, I, F, F, F, I, I, I, I, I, P],
+        "tli_mlstm_step": [P, I, P, P, I, P, I, F, P, F, F, P, P, P, P, I, P, P, F, F, I, I, I, I, I, P],
+        "tli_mlstm": [P, I, P, ctypes.c_longlong, ctypes.c_longlong, P, I, I, F, P, F, F, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
         "tli_head_norm_gate": [P, P, P, P, I, P, I, I, I, I, F, I, F, I, P],
         "tli_pooled_prepare": [P, I, P, P, P, P, P, P, P, P, I, P, I, I, I, I, I, I, I, I, P, P, F, P, P, I, I, I, P, P, P, I, I, I, I, I, P],
         "tli_attention_pooled_plain": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
@@ -1698,51 +1700,84 @@ class HipOps:
         n = int(self.lib.tli_lightning_scratch_floats(step.num_rows, step.num_seqs, int(step.max_rows_per_seq), heads, dk, dv))
         return torch.empty((n + more,), dtype=torch.float32, device=self.device), n
 
-    def retention(self, proj, at, decay, state, step, heads, dk, dv, rotary, k_scale):
-        """From the raw projections ``proj[:, at:]`` (q (H dk) | k (H dk) | v (H dv)) to the heads' outputs of the
-        recurrence S <- decay_h S + k v^T, o = S^T q, float32 [T, H, dv], with q and k turned (``rotary``, of either
-        pairing, or None) and k times ``k_scale``.  ``state``: float32 [slots, H, dv, dk], read (unless a sequence starts at
-        position 0) and replaced."""
+    def _single_rows(self, step) -> bool:
+        """Whether every sequence of the step brings one row, and such a step may run through kernels of its own."""
+        return step.max_rows_per_seq == 1 and step.num_seqs == step.num_rows and not self.unfused_decode
+
+    def retention(self, proj, at, decay, state, step, heads, dk, dv, rotary, k_scale, eps, scale, out, out_at):
+        """From the raw projections ``proj[:, at:]`` (q (H dk) | k (H dk) | v (H dv) | gate (H dv)) to the layer's rows in
+        ``out[:, out_at : out_at + H dv]``: the recurrence S <- decay_h S + k v^T, o = S^T q with q and k turned
+        (``rotary``, of either pairing, or None) and k times ``k_scale``, then o / sqrt(mean(o^2) + eps) * silu(gate) * scale
+        head by head.  ``state``: float32 [slots, H, dv, dk], read (unless a sequence starts at position 0) and replaced."""
         T = step.num_rows
         self._recurrent_inputs(proj, at, state, (heads, dv, dk), step, heads, dk, dv)
         self._want(decay, "decays", torch.float32, (heads,))
         cos, sin, dims, pairing, npos = self._pairs(rotary, step)
         if dims > dk:
             raise KernelError(f"{dims} turned elements do not fit a head of {dk}")
-        out = torch.empty((T, heads, dv), dtype=torch.float32, device=self.device)
+        _, out_ptr, out_ld = self._rows_into((out, out_at), T, heads * dv, proj.dtype)
+        proj_ptr = proj.data_ptr() + at * proj.element_size()
+        if self._single_rows(step):
+            self._call(self.lib.tli_retention_step, proj_ptr, proj.shape[1], decay.data_ptr(), state.data_ptr(), out_ptr, out_ld,
+                       step.positions.data_ptr(), step.seq_start.data_ptr(), step.slots.data_ptr(), _ptr(cos), _ptr(sin), dims,
+                       pairing, npos, float(k_scale), float(eps), float(scale), T, heads, dk, dv, _dtype_code(proj.dtype),
+                       self._stream())
+            return
+        o = torch.empty((T, heads, dv), dtype=torch.float32, device=self.device)
         scratch, _ = self._recurrence_scratch(step, heads, dk, dv)
-        self._call(self.lib.tli_retention, proj.data_ptr() + at * proj.element_size(), proj.shape[1], decay.data_ptr(),
-                   state.data_ptr(), out.data_ptr(), scratch.data_ptr(), step.positions.data_ptr(), step.row_start.data_ptr(),
+        self._call(self.lib.tli_retention, proj_ptr, proj.shape[1], decay.data_ptr(),
+                   state.data_ptr(), o.data_ptr(), scratch.data_ptr(), step.positions.data_ptr(), step.row_start.data_ptr(),
                    step.seq_start.data_ptr(), step.slots.data_ptr(), _ptr(cos), _ptr(sin), dims, pairing, npos, float(k_scale),
                    T, step.num_seqs, int(step.max_rows_per_seq), heads, dk, dv, _dtype_code(proj.dtype),
                    int(self.lightning_lanes), self._stream())
-        return out
+        self.head_norm_gate(o, None, None, proj, at + 2 * heads * dk + heads * dv, heads, dv, eps, "silu", scale, out, out_at)
 
     def mlstm_state_shape(self, heads: int, dk: int, dv: int):
         """The shape of one request's S beside its n: a head's matrix is kept transposed, n is its column dv."""
         return (heads, dv + 1, dk)
 
-    def mlstm(self, proj, at, gates, gates_transposed, gate_bias, cap, state, m_state, step, heads, dk, dv, q_scale):
-        """From the raw projections ``proj[:, at:]`` (q (H dk) | k (H dk) | v (H dv)) and the gates' products ``gates``
-        (float32 [T, 2 H]: input gates, then forget gates; [2 H, T] with ``gates_transposed``) to the memory's outputs:
-        (o, floors), o float32 [T, H, dv + 1] the heads' S^T q and, behind them, n . q, floors float32 [H, T] the
-        exp(-m).  ``state``: float32 [slots, *mlstm_state_shape]; ``m_state``: float32 [slots, H]."""
+    def mlstm(self, proj, at, x, w_gates, gate_bias, cap, state, m_state, step, heads, dk, dv, q_scale, weight, eps, scale, out,
+              out_at):
+        """From the raw projections ``proj[:, at:]`` (q (H dk) | k (H dk) | v (H dv) | gate (H dv)) and the layer's input
+        ``x`` (a tensor or ``NormedRows``) to the layer's rows in ``out[:, out_at : out_at + H dv]``: the gates' logits x
+        w_gates^T + gate_bias (``w_gates`` [2 H, n]: input gates, then forget gates; float32 sums), the matrix memory, and
+        o / sqrt(mean(o^2) + eps) * weight * sigmoid(gate) * scale head by head.  ``state``: float32 [slots,
+        *mlstm_state_shape]; ``m_state``: float32 [slots, H]."""
         T = step.num_rows
         self._recurrent_inputs(proj, at, state, self.mlstm_state_shape(heads, dk, dv), step, heads, dk, dv)
         self._want(m_state, "running maxima", torch.float32, (state.shape[0], heads))
-        self._want(gates, "gate products", torch.float32, (2 * heads, T) if gates_transposed else (T, 2 * heads))
         self._want(gate_bias, "gate biases", torch.float32, (2 * heads,))
-        z_row, z_col = (1, T) if gates_transposed else (2 * heads, 1)
+        self._want(weight, "norm weight", torch.float32, (heads * dv,))
+        rows, ssq, x_eps = (x.xw, x.ssq, x.eps) if isinstance(x, NormedRows) else (x, None, 0.0)
+        n = rows.shape[1]
+        self._want(rows, "layer input", proj.dtype, (T, n))
+        self._want(w_gates, "gate rows", proj.dtype, (2 * heads, n))
+        parts = 0 if ssq is None else ssq.shape[0]
+        if ssq is not None:
+            self._want(ssq, "sums of squares", torch.float32, (parts, T))
+        _, out_ptr, out_ld = self._rows_into((out, out_at), T, heads * dv, proj.dtype)
+        gate_at = at + 2 * heads * dk + heads * dv
+        if proj.shape[1] < gate_at + heads * dv:
+            raise KernelError("the gate lies outside the projections")
+        proj_ptr = proj.data_ptr() + at * proj.element_size()
+        if self._single_rows(step):
+            self._call(self.lib.tli_mlstm_step, proj_ptr, proj.shape[1], rows.data_ptr(), w_gates.data_ptr(), n, _ptr(ssq), parts,
+                       float(x_eps), gate_bias.data_ptr(), float(cap), float(q_scale), weight.data_ptr(), m_state.data_ptr(),
+                       state.data_ptr(), out_ptr, out_ld, step.seq_start.data_ptr(), step.slots.data_ptr(), float(eps),
+                       float(scale), T, heads, dk, dv, _dtype_code(proj.dtype), self._stream())
+            return
+        gates, transposed = self.small_product(rows, w_gates)
+        z_row, z_col = (1, T) if transposed else (2 * heads, 1)
         single = 1 if step.max_rows_per_seq == 1 and step.num_seqs == T else 0
-        out = torch.empty((T, heads, dv + 1), dtype=torch.float32, device=self.device)
+        o = torch.empty((T, heads, dv + 1), dtype=torch.float32, device=self.device)
         floors = torch.empty((heads, T), dtype=torch.float32, device=self.device)
-        scratch, n = self._recurrence_scratch(step, heads, dk, dv + 1, more=3 * heads * T)
-        self._call(self.lib.tli_mlstm, proj.data_ptr() + at * proj.element_size(), proj.shape[1], gates.data_ptr(), z_row, z_col,
-                   gate_bias.data_ptr(), float(cap), float(q_scale), m_state.data_ptr(), state.data_ptr(), out.data_ptr(),
-                   floors.data_ptr(), scratch.data_ptr(), scratch.data_ptr() + 4 * n, step.row_start.data_ptr(),
+        scratch, size = self._recurrence_scratch(step, heads, dk, dv + 1, more=3 * heads * T)
+        self._call(self.lib.tli_mlstm, proj_ptr, proj.shape[1], gates.data_ptr(), z_row, z_col, _ptr(ssq), parts, n, float(x_eps),
+                   gate_bias.data_ptr(), float(cap), float(q_scale), m_state.data_ptr(), state.data_ptr(), o.data_ptr(),
+                   floors.data_ptr(), scratch.data_ptr(), scratch.data_ptr() + 4 * size, step.row_start.data_ptr(),
                    step.seq_start.data_ptr(), step.slots.data_ptr(), T, step.num_seqs, int(step.max_rows_per_seq), single,
                    heads, dk, dv, _dtype_code(proj.dtype), int(self.lightning_lanes), self._stream())
-        return out, floors
+        self.head_norm_gate(o, floors, weight, proj, gate_at, heads, dv, eps, "sigmoid", scale, out, out_at)
 
     OUTPUT_GATES = {"silu": 0, "sigmoid": 1}
 

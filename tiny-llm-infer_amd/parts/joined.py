@@ -60,7 +60,7 @@ class SplitMixer(Mixer):
     the order of their projections, with the rows of each), ``output`` (the role of the last matrix),
     ``rows_width``, ``load_between`` and ``between``."""
     replayable = True
-    between_reads_x = False          # ``between`` uses x itself, so x must be a tensor of normed rows
+    between_reads_x = False          # ``between`` needs x as a tensor of normed rows (not as rows that owe their factor)
 
     def inputs(self) -> List[Tuple[str, int]]:
         raise NotImplementedError

@@ -27,8 +27,6 @@ from .joined import SplitMixer
 
 
 class MatrixLSTM(SplitMixer):
-    between_reads_x = True           # the gates' logits are a small product of their own, in float32
-
     def __init__(self, spec):
         super().__init__(spec)
         p = spec.params
@@ -72,12 +70,8 @@ class MatrixLSTM(SplitMixer):
         return rows * (2 * qk + 2 * v + 2 * (4 * qk + 2 * v) + 2 * v + v + 8 * self.heads)
 
     def between(self, x, proj, at, step: StepView, out, out_at, scale) -> None:
-        ops = self.env.ops
-        gates, transposed = ops.small_product(x, self.w_gates)
-        o, floors = ops.mlstm(proj, at, gates, transposed, self.gate_bias, self.cap, step.state["S"], step.state["m"], step,
-                              self.heads, self.dk, self.dv, 1.0 / math.sqrt(self.dk))
-        gate_at = at + 2 * self.heads * self.dk + self.heads * self.dv
-        ops.head_norm_gate(o, floors, self.norm, proj, gate_at, self.heads, self.dv, self.eps, "sigmoid", scale, out, out_at)
+        self.env.ops.mlstm(proj, at, x, self.w_gates, self.gate_bias, self.cap, step.state["S"], step.state["m"], step,
+                           self.heads, self.dk, self.dv, 1.0 / math.sqrt(self.dk), self.norm, self.eps, scale, out, out_at)
 
 
 register_part("mixer", "mlstm", MatrixLSTM)

@@ -71,10 +71,8 @@ class Retention(SplitMixer):
         return rows * (2 * qk + 2 * v + 2 * (4 * qk + 2 * v) + 2 * v + v)
 
     def between(self, x, proj, at, step: StepView, out, out_at, scale) -> None:
-        ops = self.env.ops
-        o = ops.retention(proj, at, self.decay, step.state, step, self.heads, self.dk, self.dv, self.rotary, 1.0 / math.sqrt(self.dk))
-        gate_at = at + 2 * self.heads * self.dk + self.heads * self.dv
-        ops.head_norm_gate(o, None, None, proj, gate_at, self.heads, self.dv, self.eps, "silu", scale, out, out_at)
+        self.env.ops.retention(proj, at, self.decay, step.state, step, self.heads, self.dk, self.dv, self.rotary,
+                               1.0 / math.sqrt(self.dk), self.eps, scale, out, out_at)
 
 
 register_part("mixer", "retention", Retention)
