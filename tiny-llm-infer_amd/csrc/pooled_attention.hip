@@ -84,14 +84,15 @@ __device__ __forceinline__ void pn_store(T* p, const float (&v)[N]) {
         p[0] = o[0];
 }
 
-// N: elements a thread takes at once (8: every size in eights, operands 16-byte aligned)
-template <typename T, int N>
+// any sizes
+template <typename T>
 __global__ __launch_bounds__(PN_THREADS) void projection_norm_prepare_kernel(
     const T* __restrict__ proj, int ld, const float* __restrict__ bias, T* __restrict__ q_out, T* k_cache, T* v_cache,
     const int* __restrict__ positions, const int* __restrict__ seq_of_row, const int* __restrict__ tables, int table_width,
     int page_size, int num_pages, int heads, int kv_heads, int key_dim, int value_dim, const float* __restrict__ q_weight,
     const float* __restrict__ k_weight, float eps, const float* __restrict__ cos_table, const float* __restrict__ sin_table,
     int dims, int pairing, int table_positions, PooledKeys pooled, int single) {
+    constexpr int N = 1;
     extern __shared__ __align__(16) float pn_row[];      // q and k of the row, all heads, times their norm's weights
     __shared__ float red[16];
     const int row = blockIdx.x, tid = threadIdx.x;
@@ -189,6 +190,129 @@ __global__ __launch_bounds__(PN_THREADS) void projection_norm_prepare_kernel(
     }
 }
 
+// Sizes in eights, bfloat16: a thread takes pieces of 8 elements (16 bytes) of the row q | k | v, up to KEEP of them,
+// and asks for all it needs before it waits for anything: projections, biases, weights, and (neighbours: the partner
+// is in the piece) the rotation's cosines and sines.
+template <int KEEP>
+__global__ __launch_bounds__(PN_THREADS) void projection_norm_prepare8_kernel(
+    const bf16_t* __restrict__ proj, int ld, const float* __restrict__ bias, bf16_t* __restrict__ q_out, bf16_t* k_cache,
+    bf16_t* v_cache, const int* __restrict__ positions, const int* __restrict__ seq_of_row, const int* __restrict__ tables,
+    int table_width, int page_size, int num_pages, int heads, int kv_heads, int key_dim, int value_dim,
+    const float* __restrict__ q_weight, const float* __restrict__ k_weight, float eps, const float* __restrict__ cos_table,
+    const float* __restrict__ sin_table, int dims, int pairing, int table_positions, PooledKeys pooled, int single) {
+    extern __shared__ __align__(16) float pn_row[];      // pairing 0: q and k of the row times their norm's weights
+    __shared__ float red[16];
+    const int row = blockIdx.x, tid = threadIdx.x;
+    const int qn = heads * key_dim, kn = kv_heads * key_dim, vn = kv_heads * value_dim, all = qn + kn + vn;
+    const bf16_t* src = proj + (size_t)row * ld;
+    const int pos = positions[row];
+    const int* table = tables + (size_t)seq_of_row[row] * table_width;
+    const int half = dims / 2;
+    const bool turn = cos_table && pos >= 0 && pos < table_positions;
+    const float* cos_row = turn ? cos_table + (size_t)pos * half : nullptr;
+    const float* sin_row = turn ? sin_table + (size_t)pos * half : nullptr;
+    float x[KEEP][8];
+    float cs[KEEP][4], sn[KEEP][4];
+    int dim0[KEEP];
+    float ssq = 0.f, ssk = 0.f;
+#pragma unroll
+    for (int u = 0; u < KEEP; ++u) {
+        const int i = (tid + u * PN_THREADS) * 8;
+        dim0[u] = i < qn + kn ? (i < qn ? i : i - qn) % key_dim : 0;
+        if (i >= all) continue;
+        pn_load<8>(src + i, x[u]);
+        if (bias) {
+            float w[8];
+            pn_load_f32<8>(bias + i, w);
+#pragma unroll
+            for (int j = 0; j < 8; ++j) x[u][j] += w[j];
+        }
+        if (i >= qn + kn) continue;
+        if (turn && pairing && dim0[u] < dims) {
+            const float4 c = *reinterpret_cast<const float4*>(cos_row + dim0[u] / 2), s = *reinterpret_cast<const float4*>(sin_row + dim0[u] / 2);
+            cs[u][0] = c.x, cs[u][1] = c.y, cs[u][2] = c.z, cs[u][3] = c.w;
+            sn[u][0] = s.x, sn[u][1] = s.y, sn[u][2] = s.z, sn[u][3] = s.w;
+        }
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) ss = fmaf(x[u][j], x[u][j], ss);
+        (i < qn ? ssq : ssk) += ss;
+        const float* weight = i < qn ? q_weight : k_weight;
+        if (weight) {
+            float w[8];
+            pn_load_f32<8>(weight + (i < qn ? i : i - qn), w);
+#pragma unroll
+            for (int j = 0; j < 8; ++j) x[u][j] *= w[j];
+        }
+        if (!pairing) {
+            *reinterpret_cast<float4*>(pn_row + i) = make_float4(x[u][0], x[u][1], x[u][2], x[u][3]);
+            *reinterpret_cast<float4*>(pn_row + i + 4) = make_float4(x[u][4], x[u][5], x[u][6], x[u][7]);
+        }
+    }
+    const int page = table[pos / page_size], slot = pos % page_size;
+    const bool kept = page >= 0 && page < num_pages;
+    {
+        const float a = wave_sum(ssq), b = wave_sum(ssk);
+        if (tid % TLI_WAVE == 0) red[tid / TLI_WAVE] = a, red[8 + tid / TLI_WAVE] = b;
+    }
+    __syncthreads();                                     // (pn_row as well)
+    float q_factor = 1.f, k_factor = 1.f;
+    {
+        float a = 0.f, b = 0.f;
+#pragma unroll
+        for (int w = 0; w < PN_THREADS / TLI_WAVE; ++w) a += red[w], b += red[8 + w];
+        if (q_weight) q_factor = 1.0f / sqrtf(a / (float)qn + eps);
+        if (k_weight) k_factor = 1.0f / sqrtf(b / (float)kn + eps);
+    }
+#pragma unroll
+    for (int u = 0; u < KEEP; ++u) {
+        const int i = (tid + u * PN_THREADS) * 8;
+        if (i >= all) continue;
+        if (i >= qn + kn) {
+            if (kept) {
+                const int e = i - qn - kn;                             // (kv head, dim) is e + j
+#pragma unroll
+                for (int j = 0; j < 8; ++j) v_cache[((size_t)page * vn + e + j) * page_size + slot] = cache_value(f32_to_bf16(x[u][j]));
+            }
+            continue;
+        }
+        const float factor = i < qn ? q_factor : k_factor;
+        const int d0 = dim0[u];
+        float y[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) y[j] = x[u][j] * factor;
+        if (turn && d0 < dims) {
+            if (pairing) {
+#pragma unroll
+                for (int p = 0; p < 4; ++p) {
+                    const float a = y[2 * p], b = y[2 * p + 1];
+                    y[2 * p] = rotate_first_half(a, b, cs[u][p], sn[u][p]);
+                    y[2 * p + 1] = rotate_second_half(b, a, cs[u][p], sn[u][p]);
+                }
+            } else {
+                const bool second = d0 >= half;                        // (half is in eights: a piece lies in one of them)
+                float other[8], c[8], s[8];
+                pn_load_f32<8>(pn_row + (second ? i - half : i + half), other);
+                pn_load_f32<8>(cos_row + (second ? d0 - half : d0), c);
+                pn_load_f32<8>(sin_row + (second ? d0 - half : d0), s);
+#pragma unroll
+                for (int j = 0; j < 8; ++j)
+                    y[j] = second ? rotate_second_half(y[j], other[j] * factor, c[j], s[j]) : rotate_first_half(y[j], other[j] * factor, c[j], s[j]);
+            }
+        }
+        if (i < qn) pn_store<8, false>(q_out + (size_t)row * qn + i, y);
+        else if (kept) pn_store<8, true>(k_cache + (((size_t)page * kv_heads + (i - qn) / key_dim) * page_size + slot) * key_dim + d0, y);
+    }
+    if (single && pooled.pool > 0 && (pos + 1) % pooled.pool == 0) {
+        __syncthreads();                                 // the row's own key and value are in their page
+        const int* pooled_table = pooled.tables + (size_t)seq_of_row[row] * pooled.width;
+        const int each = key_dim + value_dim;
+        for (int u = tid; u < kv_heads * each; u += PN_THREADS)
+            store_block_mean<bf16_t>(k_cache, v_cache, table, page_size, num_pages, kv_heads, key_dim, value_dim, u / each, u % each,
+                                     pos / pooled.pool, pooled, pooled_table);
+    }
+}
+
 #define PB_THREADS 256
 
 template <typename T>
@@ -234,9 +358,9 @@ extern "C" int tli_pooled_prepare(const void* proj, int ld, const float* bias, v
     if (lds > 150 * 1024) return tli_fail("pooled_prepare: q and k of %zu bytes do not fit LDS", lds);
     const PooledKeys pooled{pooled_k, pooled_v, pooled_tables, pooled_width, pooled_pages, pool};
     hipStream_t s = (hipStream_t)stream;
-#define PN_RUN(T, N)                                                                                                           \
+#define PN_RUN(T, KERNEL)                                                                                                           \
     {                                                                                                                          \
-        auto kernel = projection_norm_prepare_kernel<T, N>;                                                                    \
+        auto kernel = KERNEL;                                                                                                  \
         static bool allowed = false;                                                                                           \
         if (lds > 65536 && !allowed) {                                                                                         \
             if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024) != hipSuccess) \
@@ -252,11 +376,15 @@ extern "C" int tli_pooled_prepare(const void* proj, int ld, const float* bias, v
                 (const T*)k_cache, (const T*)v_cache, row_start, seq_start, num_seqs, tables, table_width, page_size,          \
                 num_pages, kv_heads, key_dim, value_dim, pooled);                                                              \
     }
-    const bool eights = ld % 8 == 0 && key_dim % 8 == 0 && value_dim % 8 == 0 &&
-                        !(((uintptr_t)proj | (uintptr_t)bias | (uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)q_weight | (uintptr_t)k_weight) & 15);
-    if (dtype == TLI_F32) PN_RUN(float, 1)
-    else if (dtype == TLI_BF16 && eights) PN_RUN(bf16_t, 8)
-    else if (dtype == TLI_BF16) PN_RUN(bf16_t, 1)
+    const int pieces = ((heads + kv_heads) * key_dim + kv_heads * value_dim) / 8;
+    const bool eights = ld % 8 == 0 && key_dim % 8 == 0 && value_dim % 8 == 0 && pieces <= 8 * PN_THREADS &&
+                        (!cos_table || dims % (pairing ? 8 : 16) == 0) &&
+                        !(((uintptr_t)proj | (uintptr_t)bias | (uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)q_weight |
+                           (uintptr_t)k_weight | (uintptr_t)cos_table | (uintptr_t)sin_table) & 15);
+    if (dtype == TLI_F32) PN_RUN(float, projection_norm_prepare_kernel<float>)
+    else if (dtype == TLI_BF16 && eights && pieces <= 2 * PN_THREADS) PN_RUN(bf16_t, projection_norm_prepare8_kernel<2>)
+    else if (dtype == TLI_BF16 && eights) PN_RUN(bf16_t, projection_norm_prepare8_kernel<8>)
+    else if (dtype == TLI_BF16) PN_RUN(bf16_t, projection_norm_prepare_kernel<bf16_t>)
     else return tli_fail("pooled_prepare: unknown dtype %d", dtype);
 #undef PN_RUN
     return tli_check_launch("pooled_prepare");

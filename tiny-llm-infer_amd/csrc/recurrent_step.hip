@@ -91,35 +91,54 @@ __global__ __launch_bounds__(RS_THREADS) void recurrent_step_kernel(StepRows a, 
     const bool fresh = a.seq_start[row] == 0;
     float* S_head = a.state + ((size_t)slot * H + h) * OV * dk;
     const bool whole = dk == DKP && dk % 4 == 0;
-    float S[GROUPS][R];
-    auto load = [&](int j0) {
+    float S[GROUPS][R], n[MEMORY ? R : 1];               // n: the mLSTM's normaliser, column dv, with the first 16 lanes
+    auto load_column = [&](int j, auto& c) {
 #pragma unroll
-        for (int g = 0; g < GROUPS; ++g) {
-            const int j = j0 + g * NC + jl;
+        for (int r = 0; r < R; ++r) c[r] = 0.f;
+        if (fresh) return;
+        const float* col = S_head + (size_t)j * dk;
+        if (whole) {
 #pragma unroll
-            for (int r = 0; r < R; ++r) S[g][r] = 0.f;
-            if (fresh || j >= OV) continue;
-            const float* col = S_head + (size_t)j * dk;
-            if (whole) {
-#pragma unroll
-                for (int r = 0; r < R; r += VW) {
-                    if constexpr (VW == 4) {
-                        const float4 v = *reinterpret_cast<const float4*>(col + at(r));
-                        S[g][r] = v.x, S[g][r + 1] = v.y, S[g][r + 2] = v.z, S[g][r + 3] = v.w;
-                    } else if constexpr (VW == 2) {
-                        const float2 v = *reinterpret_cast<const float2*>(col + at(r));
-                        S[g][r] = v.x, S[g][r + 1] = v.y;
-                    } else {
-                        S[g][r] = col[at(r)];
-                    }
+            for (int r = 0; r < R; r += VW) {
+                if constexpr (VW == 4) {
+                    const float4 v = *reinterpret_cast<const float4*>(col + at(r));
+                    c[r] = v.x, c[r + 1] = v.y, c[r + 2] = v.z, c[r + 3] = v.w;
+                } else if constexpr (VW == 2) {
+                    const float2 v = *reinterpret_cast<const float2*>(col + at(r));
+                    c[r] = v.x, c[r + 1] = v.y;
+                } else {
+                    c[r] = col[at(r)];
                 }
-            } else {
-#pragma unroll
-                for (int r = 0; r < R; ++r)
-                    if (at(r) < dk) S[g][r] = col[at(r)];
             }
+        } else {
+#pragma unroll
+            for (int r = 0; r < R; ++r)
+                if (at(r) < dk) c[r] = col[at(r)];
         }
     };
+    auto store_column = [&](int j, const auto& c) {
+        float* col = S_head + (size_t)j * dk;
+        if (whole) {
+#pragma unroll
+            for (int r = 0; r < R; r += VW) {
+                if constexpr (VW == 4) *reinterpret_cast<float4*>(col + at(r)) = make_float4(c[r], c[r + 1], c[r + 2], c[r + 3]);
+                else if constexpr (VW == 2) *reinterpret_cast<float2*>(col + at(r)) = make_float2(c[r], c[r + 1]);
+                else col[at(r)] = c[r];
+            }
+        } else {
+#pragma unroll
+            for (int r = 0; r < R; ++r)
+                if (at(r) < dk) col[at(r)] = c[r];
+        }
+    };
+    auto load = [&](int j0) {
+#pragma unroll
+        for (int g = 0; g < GROUPS; ++g)
+            if (j0 + g * NC + jl < dv) load_column(j0 + g * NC + jl, S[g]);
+    };
+    if constexpr (MEMORY) {
+        if (jl == 0) load_column(dv, n);
+    }
     load(0);
     const T* src = (const T*)a.proj + (size_t)row * a.ld;
     const T* q_src = src + (size_t)h * dk;
@@ -197,35 +216,26 @@ __global__ __launch_bounds__(RS_THREADS) void recurrent_step_kernel(StepRows a, 
     float q[R], k[R];
 #pragma unroll
     for (int r = 0; r < R; ++r) q[r] = q_s[at(r)], k[r] = k_s[at(r)];
-    for (int j0 = 0; j0 < OV; j0 += GROUPS * NC) {
+    auto walk = [&](int j, auto& c) {                    // (all 16 lanes of a column come here together, or none)
+        const float v = v_s[j];
+        float acc = 0.f;
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            c[r] = fmaf(keep, c[r], k[r] * v);
+            acc = fmaf(c[r], q[r], acc);
+        }
+        acc = rs_sum16(acc);
+        if (sub == 0) o_s[j] = acc;
+        store_column(j, c);
+    };
+    if constexpr (MEMORY) {
+        if (jl == 0) walk(dv, n);
+    }
+    for (int j0 = 0; j0 < dv; j0 += GROUPS * NC) {
         if (j0 > 0) load(j0);
 #pragma unroll
-        for (int g = 0; g < GROUPS; ++g) {
-            const int j = j0 + g * NC + jl;
-            const float v = j < OV ? v_s[j] : 0.f;
-            float acc = 0.f;
-#pragma unroll
-            for (int r = 0; r < R; ++r) {
-                S[g][r] = fmaf(keep, S[g][r], k[r] * v);
-                acc = fmaf(S[g][r], q[r], acc);
-            }
-            acc = rs_sum16(acc);
-            if (j >= OV) continue;
-            if (sub == 0) o_s[j] = acc;
-            float* col = S_head + (size_t)j * dk;
-            if (whole) {
-#pragma unroll
-                for (int r = 0; r < R; r += VW) {
-                    if constexpr (VW == 4) *reinterpret_cast<float4*>(col + at(r)) = make_float4(S[g][r], S[g][r + 1], S[g][r + 2], S[g][r + 3]);
-                    else if constexpr (VW == 2) *reinterpret_cast<float2*>(col + at(r)) = make_float2(S[g][r], S[g][r + 1]);
-                    else col[at(r)] = S[g][r];
-                }
-            } else {
-#pragma unroll
-                for (int r = 0; r < R; ++r)
-                    if (at(r) < dk) col[at(r)] = S[g][r];
-            }
-        }
+        for (int g = 0; g < GROUPS; ++g)
+            if (j0 + g * NC + jl < dv) walk(j0 + g * NC + jl, S[g]);
     }
     __syncthreads();
     const float by = MEMORY ? 1.f / (fmaxf(fabsf(o_s[dv]), floor_) + 1e-6f) : 1.f;
