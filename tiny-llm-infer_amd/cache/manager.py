@@ -185,6 +185,8 @@ class RequestCache:
     prefix_hash: int = 0                              # chained hash of those pages
     tables: List[PageTable] = field(default_factory=list)    # per group: block -> page or -1
     reserved_tokens: int = 0                          # positions [0, reserved) are covered
+    tabled_tokens: int = 0                            # positions up to here have an entry in every group's table
+    passed: List[int] = field(default_factory=list)   # per group: the blocks before this one have been given back
 
 
 def _blocks(tokens: int, page: int) -> int:
@@ -266,7 +268,8 @@ class CacheManager:
                 self.groups.append(g)
             g.cache_layers.append(layer)
             self.group_of_layer[layer] = g.index
-        self._alike = all(g.need.keeps_all and g.need.stride == 1 for g in self.groups)    # every group's table grows alike
+        self._spans = [self.span(g) for g in self.groups]
+        self._none_needed = [0] * len(self.groups)                  # (never written)
         self._free_slots = list(range(max_requests - 1, -1, -1))   # pop() gives the lowest
         self._live: Dict[Hashable, RequestCache] = {}
         self.pages_taken_total = 0
@@ -301,7 +304,7 @@ class CacheManager:
         if not self._free_slots:
             raise CacheFull("no state slot is free")
         slot = self._free_slots.pop()
-        rc = RequestCache(key=key, slot=slot, tables=[PageTable() for _ in self.groups])
+        rc = RequestCache(key=key, slot=slot, tables=[PageTable() for _ in self.groups], passed=[0] * len(self.groups))
         self._live[key] = rc
         return rc
 
@@ -361,6 +364,7 @@ class CacheManager:
                 rc.tables[gi].append(page)
         rc.num_tokens = n * self.page_size
         rc.reserved_tokens = rc.num_tokens
+        self._count_tables(rc)
         rc.hashed_blocks = n
         rc.prefix_hash = 0
         for b in range(n):
@@ -396,6 +400,9 @@ class CacheManager:
         """The positions that a page of the group covers."""
         return g.need.page_span(self.page_size)
 
+    def _count_tables(self, rc: RequestCache) -> None:
+        rc.tabled_tokens = min((len(table) * span for table, span in zip(rc.tables, self._spans)), default=1 << 60)
+
     def _kept_blocks(self, g: GroupLayout) -> int:
         """The leading blocks of a request that a window group never gives back: those of the first
         positions that every later row still reads."""
@@ -405,9 +412,8 @@ class CacheManager:
         """Per group, pages that must be taken so that the request can run the
         tokens at positions [num_tokens, new_total)."""
         rc = self._live[key]
-        if self._alike:                       # (every step of every request comes through here: the short way)
-            nb = _blocks(new_total, self.page_size)
-            return [max(0, nb - len(table)) for table in rc.tables]
+        if new_total <= rc.tabled_tokens:     # (every step of every request comes through here: the short way)
+            return self._none_needed
         out = []
         for gi, g in enumerate(self.groups):
             # every block from the first one a query at num_tokens reads up to the table's end is
@@ -460,6 +466,7 @@ class CacheManager:
                 table, nb = rc.tables[gi], _blocks(total, self.span(g))
                 while len(table) < nb:
                     table.append(self._take(gi))
+        self._count_tables(rc)
 
     def reserve(self, key: Hashable, new_total: int) -> None:
         """Take pages so that positions up to ``new_total`` can be written and
@@ -468,11 +475,11 @@ class CacheManager:
         rc = self._live[key]
         if new_total < rc.num_tokens:
             raise ValueError("a request cannot shrink")
-        needs = self.pages_needed(key, new_total)
-        if not any(needs) and self._alike:                # a token that goes into a page already held
+        if new_total <= rc.tabled_tokens:                 # a token that goes into pages already held
             if new_total > rc.reserved_tokens:
                 rc.reserved_tokens = new_total
             return
+        needs = self.pages_needed(key, new_total)
         if any(n > g.pool.free_count for n, g in zip(needs, self.groups)):
             raise CacheFull(f"not enough free pages to hold {new_total} tokens of {key!r}")
         for gi, g in enumerate(self.groups):
@@ -484,6 +491,7 @@ class CacheManager:
             for b in range(max(first, held), nb):
                 table.append(self._take(gi))
         rc.reserved_tokens = max(rc.reserved_tokens, new_total)
+        self._count_tables(rc)
 
     def advance(self, key: Hashable, new_total: int) -> None:
         """Record that the tokens up to ``new_total`` are now in the cache and
@@ -497,8 +505,11 @@ class CacheManager:
             if g.need.keeps_all:
                 continue
             table = rc.tables[gi]
-            first = min(self._first_needed_block(g, new_total), len(table))
-            for b in range(self._kept_blocks(g), first):
+            first = min(g.need.first_read(new_total) // self._spans[gi], len(table))
+            if first <= rc.passed[gi]:
+                continue
+            start, rc.passed[gi] = rc.passed[gi], first
+            for b in range(max(start, self._kept_blocks(g)), first):
                 if table[b] >= 0:
                     g.pool.release(table[b])
                     self.pages_returned_total += 1
