@@ -283,17 +283,21 @@ def test_norms_over_the_projection_rotation_and_bias(ops, dtype, heads, kv_heads
 
 
 # --------------------------------------------------------------- the recurrences, alone ---
-RECURRENT = [(2, 16, 24), (3, 20, 12), (1, 40, 20), (4, 64, 32), (2, 128, 128), (1, 200, 50), (5, 8, 7), (1, 256, 16)]
+RECURRENT = [(2, 16, 24), (3, 20, 12), (1, 40, 20), (4, 64, 32), (2, 128, 128), (1, 200, 50), (5, 8, 7), (1, 256, 16), (2, 64, 64), (3, 48, 112), (2, 96, 16)]
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("lengths, cuts", [([61, 97, 45], [1, 43, 2, 16, 33, 7]), ([900, 30, 301], [700, 390, 1, 2]), ([24, 20, 3], [1])])
 @pytest.mark.parametrize("heads, dk, dv", RECURRENT)
-def test_retention_in_portions_and_slots_that_are_used_again(ops, dtype, heads, dk, dv, lengths, cuts):
+@pytest.mark.parametrize("chunks", [True, False], ids=["chunks", "rows"])
+def test_retention_in_portions_and_slots_that_are_used_again(ops, dtype, heads, dk, dv, lengths, cuts, chunks, monkeypatch):
     """Sequences side by side in portions down to one row, also long ones that are walked in segments; then
     others in the same slots, which are never cleared."""
     from tiny_llm_infer_amd.parts.base import BuildEnv, build_part
     from tiny_llm_infer_amd.config.base import PartSpec
+    if chunks and (dtype == "float32" or dk % 16 or dv % 16 or max(dk, dv) > 128):
+        pytest.skip("these rows do not go through chunks")
+    monkeypatch.setattr(ops, "recurrence_in_chunks", chunks)
     if max(lengths) > 500 and (dk > 128 or heads > 2):
         lengths = [min(n, 480) for n in lengths]
     g = torch.Generator().manual_seed(dk * dv)
@@ -315,9 +319,10 @@ def test_retention_in_portions_and_slots_that_are_used_again(ops, dtype, heads, 
             p[:, heads * dk:2 * heads * dk] += p[:, :heads * dk]                                 # (no output that is all rounding)
         got = [[] for _ in lengths]
         for starts, counts, live in _portions(lengths, cuts):
-            rows = torch.cat([torch.zeros(sum(counts), 3, dtype=dt), torch.cat([proj[i][s:s + c] for i, s, c in zip(live, starts, counts)])], dim=1).cuda()
+            pad = 8 if chunks else 3
+            rows = torch.cat([torch.zeros(sum(counts), pad, dtype=dt), torch.cat([proj[i][s:s + c] for i, s, c in zip(live, starts, counts)])], dim=1).cuda()
             y = torch.full((len(rows), (heads * dv + 15) // 8 * 8), 4.0, dtype=dt, device="cuda")
-            ops.retention(rows, 3, decay.cuda(), state, _view(starts, counts, [slots[i] for i in live]), heads, dk, dv, part.rotary(), dk ** -0.5,
+            ops.retention(rows, pad, decay.cuda(), state, _view(starts, counts, [slots[i] for i in live]), heads, dk, dv, part.rotary(), dk ** -0.5,
                           1e-5, 0.7, y, 8)
             assert (y[:, :8] == 4.0).all() and (y[:, 8 + heads * dv:] == 4.0).all()
             r = 0
@@ -332,9 +337,13 @@ def test_retention_in_portions_and_slots_that_are_used_again(ops, dtype, heads, 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("lengths, cuts", [([61, 97, 45], [1, 43, 2, 16, 33, 7]), ([900, 30, 301], [700, 390, 1, 2]), ([24, 20, 3], [1])])
 @pytest.mark.parametrize("heads, dk, dv", RECURRENT)
-def test_matrix_memory_in_portions_and_slots_that_are_used_again(ops, dtype, heads, dk, dv, lengths, cuts):
+@pytest.mark.parametrize("chunks", [True, False], ids=["chunks", "rows"])
+def test_matrix_memory_in_portions_and_slots_that_are_used_again(ops, dtype, heads, dk, dv, lengths, cuts, chunks, monkeypatch):
     """As the retention's test; gates that open and close, so that the running maximum is taken over again and again, and
     a head whose forget gate is open throughout."""
+    if chunks and (dtype == "float32" or dk % 16 or dv % 16 or max(dk, dv) > 128):
+        pytest.skip("these rows do not go through chunks")
+    monkeypatch.setattr(ops, "recurrence_in_chunks", chunks)
     if max(lengths) > 500 and (dk > 128 or heads > 2):
         lengths = [min(n, 480) for n in lengths]
     g = torch.Generator().manual_seed(dk + dv)
@@ -360,13 +369,14 @@ def test_matrix_memory_in_portions_and_slots_that_are_used_again(ops, dtype, hea
             p[:, heads * dk:2 * heads * dk] += p[:, :heads * dk]
         got = [[] for _ in lengths]
         for k, (starts, counts, live) in enumerate(_portions(lengths, cuts + [1])):
-            rows = torch.cat([torch.zeros(sum(counts), 5, dtype=dt), torch.cat([proj[i][s:s + c] for i, s, c in zip(live, starts, counts)])], dim=1).cuda()
+            pad = 8 if chunks else 5
+            rows = torch.cat([torch.zeros(sum(counts), pad, dtype=dt), torch.cat([proj[i][s:s + c] for i, s, c in zip(live, starts, counts)])], dim=1).cuda()
             inputs = torch.cat([x[i][s:s + c] for i, s, c in zip(live, starts, counts)]).cuda()
             if k % 3 == 2 and dtype == "bfloat16":                                               # rows that still owe a factor of 1/2, in three parts
                 from tiny_llm_infer_amd.kernels.ops import NormedRows
                 inputs = NormedRows((inputs.float() * 2).to(dt), torch.full((3, len(rows)), n * 3.9 / 3, device="cuda"), 0.1)
             y = torch.full((len(rows), (heads * dv + 7) // 8 * 8), 4.0, dtype=dt, device="cuda")
-            ops.mlstm(rows, 5, inputs, w_gates.cuda(), bias.cuda(), cap, state, maxima, _view(starts, counts, [slots[i] for i in live]), heads, dk, dv,
+            ops.mlstm(rows, pad, inputs, w_gates.cuda(), bias.cuda(), cap, state, maxima, _view(starts, counts, [slots[i] for i in live]), heads, dk, dv,
                       dk ** -0.5, weight.cuda(), 1e-5, 1.3, y, 0)
             assert (y[:, heads * dv:] == 4.0).all()
             r = 0

@@ -1,0 +1,453 @@
+// Portions of prompts through the recurrent layers whose heads are normed one by one (retention.hip, mlstm.hip), bfloat16
+// rows, head sizes in sixteens up to 128: the recurrence S_t = a_t S_(t-1) + w_t k_t v_t^T, o_t = S_t^T q_t in chunks of 64
+// rows.  With A_t the product of a from the chunk's first row to t and P the state before the chunk,
+//   o_t = A_t P^T q_t + sum over s <= t of (A_t / A_s) w_s (q_t . k_s) v_s,        P' = A_end P + sum_s (A_end / A_s) w_s k_s v_s^T
+// (the mLSTM's normaliser n is one more column of S whose value is 1), which are products of matrices.  All of them are
+// float32 on v_mfma_f32_16x16x4_f32, which takes float32 as it is: nothing of the recurrence is rounded to bfloat16.
+//
+// chunk_states: a workgroup a (32 elements of k, 64 of v; head; sequence) walks the sequence's chunks, its part of S in
+//   the accumulators of the products, and leaves P of every chunk in scratch; the last S goes to the sequence's slot.
+// chunk_outputs: a workgroup a (chunk; head), a wave 16 rows: the two terms of o from P, K and V in LDS (P first, then K
+//   and V in its place), the scores and their weights in registers (transposed, S^T = K Q^T, so that they are already the
+//   second operand of the product with V), then the head's norm and its gate.
+//
+// The matrix instruction's operands: A: lane l has row l % 16, k = l / 16; B: k = l / 16, column l % 16; sums: rows 4 (l / 16) ..
+// + 3 of column l % 16.  Of 16 consecutive k, lane group c takes 4 c .. 4 c + 3 in four instructions, so that a lane's
+// operands are four consecutive elements.
+#include "chunked.h"
+
+#define CK_ROWS TLI_CHUNK_ROWS
+#define CK_THREADS 256
+
+typedef float ck_f32x4 __attribute__((ext_vector_type(4)));
+
+struct ChunkRows {                                       // what both kinds read and write
+    const bf16_t* proj;                                  // [T, ld]: q (H dk) | k (H dk) | v (H dv) | gate (H dv)
+    int ld;
+    float* state;                                        // [slots][H][OV][dk], OV = dv, or dv + 1 with a normaliser
+    float* before;                                       // scratch [chunks][H][OV][dk]: S before every chunk
+    const int* row_start;
+    const int* seq_start;
+    const int* slots;
+    int T, seqs, H, dk, dv;
+};
+
+struct ChunkRotation {                                   // of q and k, and the factors behind it
+    const int* positions;
+    const float* cos_table;                              // [table_positions, dims / 2] or null
+    const float* sin_table;
+    int dims, pairing, table_positions;
+    float q_scale, k_scale;
+};
+
+struct ChunkDecay {
+    const float* head;                                   // [H]: one factor a head and w = 1; or null, and then, [H][T]:
+    const float* through;                                // log A_t
+    const float* take;                                   // w_t
+};
+
+// N consecutive elements from dim d on of a head's q or k at `head`, in float32, turned, not scaled.  N is 4 or 8 and a
+// piece lies on one side of every border (dims and half of it are multiples of N, for neighbours dims is).
+template <int N>
+__device__ __forceinline__ void ck_load(const bf16_t* p, float (&v)[N]) {
+    uint32_t u[N / 2];
+    if constexpr (N == 8) {
+        const uint4 w = *reinterpret_cast<const uint4*>(p);
+        u[0] = w.x, u[1] = w.y, u[2] = w.z, u[3] = w.w;
+    } else {
+        const uint2 w = *reinterpret_cast<const uint2*>(p);
+        u[0] = w.x, u[1] = w.y;
+    }
+#pragma unroll
+    for (int i = 0; i < N / 2; ++i) v[2 * i] = bf16_to_f32((bf16_t)(u[i] & 0xffffu)), v[2 * i + 1] = bf16_to_f32((bf16_t)(u[i] >> 16));
+}
+template <int N>
+__device__ __forceinline__ void ck_turned(const bf16_t* head, int d, const ChunkRotation& rot, int pos, float (&x)[N]) {
+    ck_load<N>(head + d, x);
+    if (!rot.cos_table || d >= rot.dims || pos >= rot.table_positions) return;
+    const int half = rot.dims / 2;
+    const float* cos_row = rot.cos_table + (size_t)pos * half;
+    const float* sin_row = rot.sin_table + (size_t)pos * half;
+    if (rot.pairing) {
+#pragma unroll
+        for (int p = 0; p < N / 2; ++p) {
+            const float c = cos_row[d / 2 + p], s = sin_row[d / 2 + p], a = x[2 * p], b = x[2 * p + 1];
+            x[2 * p] = rotate_first_half(a, b, c, s);
+            x[2 * p + 1] = rotate_second_half(b, a, c, s);
+        }
+    } else {
+        const bool second = d >= half;
+        float other[N];
+        ck_load<N>(head + (second ? d - half : d + half), other);
+        const float* c = cos_row + (second ? d - half : d);
+        const float* s = sin_row + (second ? d - half : d);
+#pragma unroll
+        for (int i = 0; i < N; i += 4) {
+            const float4 cc = *reinterpret_cast<const float4*>(c + i), ss = *reinterpret_cast<const float4*>(s + i);
+            const float cv[4] = {cc.x, cc.y, cc.z, cc.w}, sv[4] = {ss.x, ss.y, ss.z, ss.w};
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+                x[i + j] = second ? rotate_second_half(x[i + j], other[i + j], cv[j], sv[j])
+                                  : rotate_first_half(x[i + j], other[i + j], cv[j], sv[j]);
+        }
+    }
+}
+
+__device__ __forceinline__ int ck_chunks(int rows) { return (rows + CK_ROWS - 1) / CK_ROWS; }
+
+#define CK_KDIMS 32          // of k a workgroup of chunk_states
+#define CK_VDIMS 64          // of v
+#define CK_KLD (CK_ROWS + 4)
+
+template <bool MEMORY>
+__global__ __launch_bounds__(CK_THREADS) void chunk_states_kernel(ChunkRows a, ChunkRotation rot, ChunkDecay decay) {
+    __shared__ __align__(16) float kt[2][CK_KDIMS][CK_KLD];            // the chunk's weighted keys, transposed
+    const int tid = threadIdx.x, lane = tid % TLI_WAVE, wave = tid / TLI_WAVE, col = lane % 16, grp = lane / 16;
+    const int dk = a.dk, dv = a.dv, H = a.H, OV = dv + (MEMORY ? 1 : 0);
+    const int k_slices = (dk + CK_KDIMS - 1) / CK_KDIMS;
+    const int dk0 = (blockIdx.x % k_slices) * CK_KDIMS, dv0 = (blockIdx.x / k_slices) * CK_VDIMS;
+    const int h = blockIdx.y, seq = blockIdx.z;
+    const int r0 = a.row_start[seq], n = a.row_start[seq + 1] - r0;
+    if (n <= 0) return;
+    int z0 = 0;
+    for (int i = 0; i < seq; ++i) z0 += ck_chunks(a.row_start[i + 1] - a.row_start[i]);
+    const int chunks = ck_chunks(n);
+    const int j = dv0 + wave * 16 + col;                               // this lane's column of S
+    const bool mine = dv0 + wave * 16 < dv;
+    const bool norm_too = MEMORY && dv0 == 0 && wave == 0;             // this wave keeps n of these elements of k as well
+    const bool tile1 = dk0 + 16 < dk;                                  // (dk in sixteens)
+    float* slot = a.state + ((size_t)a.slots[seq] * H + h) * OV * dk;
+    const bool fresh = a.seq_start[seq] == 0;
+    ck_f32x4 S[2];
+    float nk[2] = {0.f, 0.f};
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+        S[t] = (ck_f32x4){0.f, 0.f, 0.f, 0.f};
+        if (fresh || (t == 1 && !tile1)) continue;
+        if (mine) S[t] = *reinterpret_cast<const ck_f32x4*>(slot + (size_t)j * dk + dk0 + 16 * t + 4 * grp);
+        if (norm_too) nk[t] = slot[(size_t)dv * dk + dk0 + 16 * t + col];
+    }
+    const bf16_t* k_head = a.proj + (size_t)r0 * a.ld + (size_t)(H + h) * dk;
+    const bf16_t* v_head = a.proj + (size_t)r0 * a.ld + (size_t)2 * H * dk + (size_t)h * dv + (mine ? j : 0);
+    const int kr = tid / 4, kd = dk0 + (tid % 4) * 8;                  // this thread's row and piece of the chunk's keys
+    const float lam = MEMORY ? 0.f : decay.head[h];
+    const float* through = MEMORY ? decay.through + (size_t)h * a.T + r0 : nullptr;
+    const float* takes = MEMORY ? decay.take + (size_t)h * a.T + r0 : nullptr;
+    float x[8], w = 0.f;
+    bf16_t v[16];
+    auto fetch = [&](int z) {
+        const int first = z * CK_ROWS, count = min(CK_ROWS, n - first);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] = 0.f;
+        w = 0.f;
+        if (kr < count && kd < dk) {
+            const int pos = rot.cos_table ? rot.positions[r0 + first + kr] : 0;
+            ck_turned<8>(k_head + (size_t)(first + kr) * a.ld, kd, rot, pos, x);
+            if constexpr (MEMORY) w = expf(through[first + count - 1] - through[first + kr]) * takes[first + kr];
+            else w = powf(lam, (float)(count - 1 - kr)) * rot.k_scale;
+        }
+#pragma unroll
+        for (int s = 0; s < 4; ++s)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) v[4 * s + i] = v_head[(size_t)(first + min(16 * s + 4 * grp + i, count - 1)) * a.ld];
+    };
+    fetch(0);
+    for (int z = 0; z < chunks; ++z) {
+        const int first = z * CK_ROWS, count = min(CK_ROWS, n - first);
+        float(*k_lds)[CK_KLD] = kt[z & 1];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) k_lds[kd - dk0 + e][kr] = x[e] * w;
+        float vf[16];
+#pragma unroll
+        for (int i = 0; i < 16; ++i) vf[i] = bf16_to_f32(v[i]);
+        __syncthreads();                                               // (the buffer's last readers passed the barrier before)
+        if (z + 1 < chunks) fetch(z + 1);
+        float* P = a.before + ((size_t)(z0 + z) * H + h) * OV * dk;
+        const float g = MEMORY ? expf(through[first + count - 1]) : powf(lam, (float)count);
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+            if (t == 1 && !tile1) continue;
+            if (mine) *reinterpret_cast<ck_f32x4*>(P + (size_t)j * dk + dk0 + 16 * t + 4 * grp) = S[t];
+            if (norm_too && grp == 0) P[(size_t)dv * dk + dk0 + 16 * t + col] = nk[t];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) S[t][i] *= g;
+        }
+        float sum[2] = {0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+            if (16 * s >= count) continue;
+#pragma unroll
+            for (int t = 0; t < 2; ++t) {
+                const ck_f32x4 kk = *reinterpret_cast<const ck_f32x4*>(&k_lds[16 * t + col][16 * s + 4 * grp]);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[i], vf[4 * s + i], S[t], 0, 0, 0);
+                if (MEMORY) sum[t] += (kk[0] + kk[1]) + (kk[2] + kk[3]);
+            }
+        }
+        if (norm_too) {
+#pragma unroll
+            for (int t = 0; t < 2; ++t) nk[t] = fmaf(g, nk[t], quad_rows_sum(sum[t]));
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+        if (t == 1 && !tile1) continue;
+        if (mine) *reinterpret_cast<ck_f32x4*>(slot + (size_t)j * dk + dk0 + 16 * t + 4 * grp) = S[t];
+        if (norm_too && grp == 0) slot[(size_t)dv * dk + dk0 + 16 * t + col] = nk[t];
+    }
+}
+
+struct ChunkOutput {
+    bf16_t* out;                                         // rows out_ld elements apart, H dv of each
+    int out_ld;
+    const float* weight;                                 // [H dv] or null
+    const float* floors;                                 // [H][T]: exp(-m), with a normaliser
+    float eps, scale;
+};
+
+static inline size_t ck_lds_floats(int dk, int dv) {
+    const size_t state = (size_t)dv * (dk + 4), rows = (size_t)CK_ROWS * (dk + 4 + dv + 4);
+    return state > rows ? state : rows;
+}
+
+// MEMORY: with a normaliser and the logistic gate; else the silu gate.  NK, NV: sixteens of a head (EXACT), or their
+// bound: sixteens past a head's are multiplied all the same, q's as zeros and v's into sums that nobody reads, from
+// addresses of the head's last, so that no matrix instruction stands behind a condition
+template <bool MEMORY, int NK, int NV, bool EXACT>
+__global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows a, ChunkRotation rot, ChunkDecay decay, ChunkOutput out) {
+    extern __shared__ __align__(16) float ck_lds[];
+    __shared__ float log_s[CK_ROWS], take_s[CK_ROWS];                  // mLSTM: log A and w; else the powers of the decay
+    const int tid = threadIdx.x, lane = tid % TLI_WAVE, wave = __builtin_amdgcn_readfirstlane(tid / TLI_WAVE), col = lane % 16, grp = lane / 16;
+    const int nk = EXACT ? NK : a.dk / 16, nv = EXACT ? NV : a.dv / 16;
+    const int dk = nk * 16, dv = nv * 16, H = a.H, OV = dv + (MEMORY ? 1 : 0), KLD = dk + 4, VLD = dv + 4;
+    const int h = blockIdx.y;
+    int z = blockIdx.x, seq = 0, n = 0;
+    for (; seq < a.seqs; ++seq) {
+        n = a.row_start[seq + 1] - a.row_start[seq];
+        const int c = ck_chunks(n);
+        if (z < c) break;
+        z -= c;
+    }
+    if (seq >= a.seqs) return;                                         // (the grid's slack)
+    const int r0 = a.row_start[seq] + z * CK_ROWS, count = min(CK_ROWS, n - z * CK_ROWS);
+    const bool from_nothing = z == 0 && a.seq_start[seq] == 0;
+    const float* P = a.before + ((size_t)blockIdx.x * H + h) * OV * dk;
+    const bf16_t* rows = a.proj + (size_t)r0 * a.ld;
+    const float lam = MEMORY ? 0.f : decay.head[h];
+    const int i = 16 * wave + col;                                     // this lane's row of the chunk
+    const int row = min(i, count - 1);
+    const bool works = 16 * wave < count;                              // (the same for the whole wave)
+
+    if (!from_nothing) {                                               // P, [dv][dk]
+        const int pieces = dv * dk / 4, per = dk / 4;
+        for (int p = tid; p < pieces; p += CK_THREADS)
+            *reinterpret_cast<float4*>(ck_lds + (p / per) * KLD + (p % per) * 4) = *reinterpret_cast<const float4*>(P + (size_t)p * 4);
+    }
+    if (tid < CK_ROWS) {
+        if constexpr (MEMORY) {
+            const bool live = tid < count;
+            log_s[tid] = live ? decay.through[(size_t)h * a.T + r0 + tid] : 0.f;
+            take_s[tid] = live ? decay.take[(size_t)h * a.T + r0 + tid] : 0.f;
+        } else {
+            log_s[tid] = powf(lam, (float)tid);                        // lam^0 .. lam^63
+        }
+    }
+    auto k_tile = [&](int b) { return EXACT ? b : min(b, nk - 1); };
+    auto v_tile = [&](int t) { return EXACT ? t : min(t, nv - 1); };
+    float q[NK][4];
+#pragma unroll
+    for (int b = 0; b < NK; ++b) {
+        ck_turned<4>(rows + (size_t)row * a.ld + (size_t)h * dk, 16 * k_tile(b) + 4 * grp, rot, rot.cos_table ? rot.positions[r0 + row] : 0, q[b]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) q[b][e] = b < nk ? q[b][e] * rot.q_scale : 0.f;
+    }
+    ck_f32x4 acc[NV];
+#pragma unroll
+    for (int t = 0; t < NV; ++t) acc[t] = (ck_f32x4){0.f, 0.f, 0.f, 0.f};
+    float nq = 0.f;                                                    // n . q of this lane's row, this lane group's share
+    __syncthreads();
+    if (!from_nothing && works) {
+        const float g = MEMORY ? expf(log_s[row]) : log_s[row] * lam;  // A of the row
+#pragma unroll
+        for (int b = 0; b < NK; ++b) {
+            if constexpr (MEMORY) {
+                const float4 nn = *reinterpret_cast<const float4*>(P + (size_t)dv * dk + 16 * k_tile(b) + 4 * grp);
+                nq += q[b][0] * nn.x + q[b][1] * nn.y + q[b][2] * nn.z + q[b][3] * nn.w;
+            }
+            ck_f32x4 p[NV];
+#pragma unroll
+            for (int t = 0; t < NV; ++t)
+                p[t] = *reinterpret_cast<const ck_f32x4*>(ck_lds + (16 * v_tile(t) + col) * KLD + 16 * k_tile(b) + 4 * grp);
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+#pragma unroll
+                for (int t = 0; t < NV; ++t)
+                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[t][e], q[b][e], acc[t], 0, 0, 0);
+        }
+        nq *= g;
+#pragma unroll
+        for (int t = 0; t < NV; ++t)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) acc[t][e] *= g;
+    }
+    __syncthreads();                                                   // P has been read
+    float* k_s = ck_lds;                                               // [row][dk + 4]
+    float* v_s = ck_lds + CK_ROWS * KLD;                               // [row][dv + 4]
+    for (int p = tid; p < count * (dk / 8); p += CK_THREADS) {
+        const int r = p / (dk / 8), d = (p % (dk / 8)) * 8;
+        float x[8];
+        ck_turned<8>(rows + (size_t)r * a.ld + (size_t)(H + h) * dk, d, rot, rot.cos_table ? rot.positions[r0 + r] : 0, x);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) k_s[r * KLD + d + e] = x[e] * rot.k_scale;
+    }
+    for (int p = tid; p < count * (dv / 8); p += CK_THREADS) {
+        const int r = p / (dv / 8), d = (p % (dv / 8)) * 8;
+        float x[8];
+        ck_load<8>(rows + (size_t)r * a.ld + (size_t)2 * H * dk + (size_t)h * dv + d, x);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v_s[r * VLD + d + e] = x[e];
+    }
+    __syncthreads();
+    if (!works) return;
+    const float my_log = MEMORY ? log_s[row] : 0.f;
+    for (int jt = 0; jt <= wave; ++jt) {
+        // (rows of K and V past the chunk's last are what was in LDS before: their scores are set to 0, and their
+        // values are read from the last row)
+        ck_f32x4 s[2] = {(ck_f32x4){0.f, 0.f, 0.f, 0.f}, (ck_f32x4){0.f, 0.f, 0.f, 0.f}};
+        const float* k_row = k_s + min(16 * jt + col, count - 1) * KLD + 4 * grp;
+#pragma unroll
+        for (int b = 0; b < NK; ++b) {
+            const ck_f32x4 kk = *reinterpret_cast<const ck_f32x4*>(k_row + 16 * k_tile(b));
+#pragma unroll
+            for (int e = 0; e < 4; ++e) s[e & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[e], q[b][e], s[e & 1], 0, 0, 0);
+        }
+        float p[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {                                  // row 16 jt + 4 grp + e of K against this lane's row
+            const int j = 16 * jt + 4 * grp + e;
+            float w = 0.f;
+            if (j <= i && j < count) w = MEMORY ? expf(my_log - log_s[j]) * take_s[j] : log_s[i - j];
+            p[e] = (s[0][e] + s[1][e]) * w;
+            if (MEMORY) nq += p[e];
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const float* v_row = v_s + min(16 * jt + 4 * grp + e, count - 1) * VLD + col;
+#pragma unroll
+            for (int t = 0; t < NV; ++t)
+                acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(v_row[16 * v_tile(t)], p[e], acc[t], 0, 0, 0);
+        }
+    }
+    // the head's norm and gate: this lane has elements 16 t + 4 grp .. + 3 of its row
+    float by = 1.f;
+    if constexpr (MEMORY) by = 1.f / (fmaxf(fabsf(quad_rows_sum(nq)), out.floors[(size_t)h * a.T + r0 + row]) + 1e-6f);
+    float ss = 0.f;
+#pragma unroll
+    for (int t = 0; t < NV; ++t)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            acc[t][e] *= by;
+            if (t < nv) ss = fmaf(acc[t][e], acc[t][e], ss);
+        }
+    const float factor = out.scale / sqrtf(quad_rows_sum(ss) / (float)dv + out.eps);
+    if (i >= count) return;
+    const bf16_t* gate = rows + (size_t)i * a.ld + (size_t)H * (2 * dk + dv) + (size_t)h * dv;
+    bf16_t* dst = out.out + (size_t)(r0 + i) * out.out_ld + (size_t)h * dv;
+#pragma unroll
+    for (int t = 0; t < NV; ++t) {
+        if (t >= nv) continue;
+        const int d = 16 * t + 4 * grp;
+        float g[4], y[4];
+        ck_load<4>(gate + d, g);
+        float wt[4] = {1.f, 1.f, 1.f, 1.f};
+        if (out.weight) {
+            const float4 w4 = *reinterpret_cast<const float4*>(out.weight + (size_t)h * dv + d);
+            wt[0] = w4.x, wt[1] = w4.y, wt[2] = w4.z, wt[3] = w4.w;
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y[e] = acc[t][e] * factor * wt[e] * ((MEMORY ? 1.f : g[e]) / (1.f + expf(-g[e])));
+        *reinterpret_cast<uint2*>(dst + d) = make_uint2(pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3]));
+    }
+}
+
+// Whether rows of these sizes go through here (else the shared recurrence serves): dims turned elements (0: none).
+extern "C" int tli_chunked_takes(int dk, int dv, int dims, int pairing) {
+    if (dk % 16 || dv % 16 || dk < 16 || dv < 16 || dk > 128 || dv > 128) return 0;
+    return dims % (pairing ? 8 : 16) == 0;
+}
+
+// float32 elements of scratch for T rows in `seqs` sequences; OV: dv, or dv + 1 with a normaliser
+extern "C" long long tli_chunked_scratch_floats(int T, int seqs, int H, int dk, int OV) {
+    return ((long long)T / CK_ROWS + seqs) * H * OV * dk;
+}
+
+template <bool MEMORY>
+static int run_chunked(const ChunkRows& a, const ChunkRotation& rot, const ChunkDecay& decay, const ChunkOutput& out, hipStream_t s) {
+    const int zs = a.T / CK_ROWS + a.seqs;               // (an upper bound of the chunks; a workgroup past the last leaves)
+    if (a.H > 65535 || a.seqs > 65535) return tli_fail("chunked recurrence: too many heads or sequences for one launch");
+    if (a.ld % 8 || a.ld < 2 * a.H * (a.dk + a.dv)) return tli_fail("chunked recurrence: rows of %d elements", a.ld);
+    if (out.out_ld % 4 || out.out_ld < a.H * a.dv) return tli_fail("chunked recurrence: output rows of %d elements", out.out_ld);
+    if ((((uintptr_t)a.proj | (uintptr_t)a.state | (uintptr_t)a.before | (uintptr_t)out.weight | (uintptr_t)rot.cos_table | (uintptr_t)rot.sin_table) & 15) ||
+        ((uintptr_t)out.out & 7))
+        return tli_fail("chunked recurrence: operands must be 16-byte aligned");
+    const int slices = ((a.dk + CK_KDIMS - 1) / CK_KDIMS) * ((a.dv + CK_VDIMS - 1) / CK_VDIMS);
+    chunk_states_kernel<MEMORY><<<dim3(slices, a.H, a.seqs), CK_THREADS, 0, s>>>(a, rot, decay);
+    const size_t lds = ck_lds_floats(a.dk, a.dv) * sizeof(float);
+    const dim3 grid(zs, a.H);
+#define CK_RUN(NK, NV, EXACT)                                                                                               \
+    {                                                                                                                       \
+        auto kernel = chunk_outputs_kernel<MEMORY, NK, NV, EXACT>;                                                          \
+        static bool allowed = false;                                                                                        \
+        if (lds > 60 * 1024 && !allowed) {                                                                                  \
+            if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 72 * 1024) !=          \
+                hipSuccess)                                                                                                 \
+                return tli_fail("chunked recurrence: cannot have %zu bytes of LDS", lds);                                   \
+            allowed = true;                                                                                                 \
+        }                                                                                                                   \
+        kernel<<<grid, CK_THREADS, lds, s>>>(a, rot, decay, out);                                                           \
+    }
+    if (a.dk == 128 && a.dv == 128) CK_RUN(8, 8, true)
+    else if (a.dk == 64 && a.dv == 64) CK_RUN(4, 4, true)
+    else if (a.dk <= 32 && a.dv <= 32) CK_RUN(2, 2, false)
+    else if (a.dk <= 64 && a.dv <= 64) CK_RUN(4, 4, false)
+    else CK_RUN(8, 8, false)
+#undef CK_RUN
+    return tli_check_launch("chunked recurrence");
+}
+
+// bfloat16 rows; the arguments as for tli_retention_step (recurrent_step.hip), row_start [seqs + 1], seq_start, slots
+// [seqs]; scratch: tli_chunked_scratch_floats(T, seqs, H, dk, dv) floats
+extern "C" int tli_retention_chunked_bf16(const void* proj, int ld, const float* decay, float* state, void* out, int out_ld,
+                                          float* scratch, const int* positions, const int* row_start, const int* seq_start,
+                                          const int* slots, const float* cos_table, const float* sin_table, int dims, int pairing,
+                                          int table_positions, float k_scale, float eps, float scale, int T, int seqs, int H, int dk,
+                                          int dv, void* stream) {
+    if (T <= 0 || seqs <= 0) return 0;
+    if (H <= 0 || !tli_chunked_takes(dk, dv, cos_table ? dims : 0, pairing) || (cos_table && (dims <= 0 || dims > dk)))
+        return tli_fail("retention in chunks: heads of %d and %d with %d turned elements", dk, dv, dims);
+    const ChunkRows a{(const bf16_t*)proj, ld, state, scratch, row_start, seq_start, slots, T, seqs, H, dk, dv};
+    return run_chunked<false>(a, ChunkRotation{positions, cos_table, sin_table, dims, pairing, table_positions, 1.0f, k_scale},
+                              ChunkDecay{decay, nullptr, nullptr}, ChunkOutput{(bf16_t*)out, out_ld, nullptr, nullptr, eps, scale},
+                              (hipStream_t)stream);
+}
+
+// bfloat16 rows; the arguments as for tli_mlstm (mlstm.hip) and tli_mlstm_step; scratch: tli_chunked_scratch_floats(T, seqs,
+// H, dk, dv + 1) floats, rows_scratch: 4 H T floats
+extern "C" int tli_mlstm_chunked_bf16(const void* proj, int ld, const float* z, long long z_row, long long z_col, const float* ssq,
+                                      int parts, int x_size, float x_eps, const float* bias, float cap, float q_scale,
+                                      const float* weight, float* m_state, float* state, void* out, int out_ld, float* scratch,
+                                      float* rows_scratch, const int* row_start, const int* seq_start, const int* slots, float eps,
+                                      float scale, int T, int seqs, int H, int dk, int dv, void* stream) {
+    if (T <= 0 || seqs <= 0) return 0;
+    if (H <= 0 || H > 65535 || seqs > 65535 || !tli_chunked_takes(dk, dv, 0, 0)) return tli_fail("mlstm in chunks: heads of %d and %d", dk, dv);
+    if (!(cap > 0.f)) return tli_fail("mlstm: the gates' cap must be positive");
+    if (ssq && (parts <= 0 || x_size <= 0)) return tli_fail("mlstm: bad sums of squares");
+    hipStream_t s = (hipStream_t)stream;
+    const size_t per = (size_t)H * T;
+    float *keep = rows_scratch, *take = keep + per, *through = take + per, *floors = through + per;
+    const MlGates gates{z, z_row, z_col, bias, cap, H, RowFactor{ssq, ssq ? parts : 0, T, 1.0f / (float)(x_size > 0 ? x_size : 1), x_eps}};
+    if (tli_mlstm_scan(gates, m_state, keep, take, floors, through, CK_ROWS, row_start, seq_start, slots, T, seqs, s)) return 1;
+    const ChunkRows a{(const bf16_t*)proj, ld, state, scratch, row_start, seq_start, slots, T, seqs, H, dk, dv};
+    return run_chunked<true>(a, ChunkRotation{nullptr, nullptr, nullptr, 0, 0, 0, q_scale, 1.0f}, ChunkDecay{nullptr, through, take},
+                             ChunkOutput{(bf16_t*)out, out_ld, weight, floors, eps, scale}, s);
+}

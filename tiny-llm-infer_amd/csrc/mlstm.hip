@@ -16,28 +16,14 @@
 // are made from the same m.
 // mlstm_prepare: a workgroup a (row, head) leaves q, k and v in float32 for the recurrence.  In a step of single rows
 // (`single`) it makes the gates itself and there is no scan.
-#include "recurrence.h"
-#include "row_gates.h"
+#include "chunked.h"
 
 #define ML_THREADS TLI_RECURRENCE_SEGMENT
 
-struct MlGates {
-    const float* z;          // logits: head h's input gate of row r at z[r z_row + h z_col], its forget gate H columns on
-    long long z_row, z_col;
-    const float* bias;       // [2 H]
-    float cap;
-    int H;
-    RowFactor factor;        // of the rows that the logits were made from
-    __device__ __forceinline__ float input(int r, int h, float f) const { return gate_capped(z[r * z_row + h * z_col] * f + bias[h], cap); }
-    __device__ __forceinline__ float forget(int r, int h, float f) const {
-        return gate_log_sigmoid(gate_capped(z[r * z_row + (H + h) * z_col] * f + bias[H + h], cap));
-    }
-};
-
-// keep, take, floors, through: [H][T]: a_t; exp(i_t - m_t); exp(-m_t); log of the product of a from the 256 rows' first
+// (its results: chunked.h)
 __global__ __launch_bounds__(ML_THREADS) void mlstm_scan_kernel(MlGates gates, float* __restrict__ m_state,
                                                                 float* __restrict__ keep, float* __restrict__ take,
-                                                                float* __restrict__ floors, float* __restrict__ through,
+                                                                float* __restrict__ floors, float* __restrict__ through, int unit,
                                                                 const int* __restrict__ row_start, const int* __restrict__ seq_start,
                                                                 const int* __restrict__ slots, int T) {
     __shared__ float wave_f[ML_THREADS / TLI_WAVE], wave_m[ML_THREADS / TLI_WAVE];
@@ -66,6 +52,7 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_scan_kernel(MlGates gates, f
             wave_m[wave] = M;
         }
         __syncthreads();
+        const float F_wave = F;                                        // from the wave's first row on
         float Fw = 0.f, Mw = -INFINITY;                                // the waves before
         for (int w = 0; w < wave; ++w) {
             Mw = fmaxf(Mw + wave_f[w], wave_m[w]);
@@ -82,12 +69,22 @@ __global__ __launch_bounds__(ML_THREADS) void mlstm_scan_kernel(MlGates gates, f
             keep[at] = expf(f + m_of[tid] - m);
             take[at] = expf(i - m);
             floors[at] = expf(-m);
-            through[at] = F + m0 - m;
+            through[at] = unit == TLI_WAVE ? F_wave + m_of[wave * TLI_WAVE] - m : F + m0 - m;
         }
         m0 = m_of[min(n - first, ML_THREADS)];
         __syncthreads();
     }
     if (tid == 0 && n > 0) *slot = m0;
+}
+
+static_assert(TLI_CHUNK_ROWS == TLI_WAVE, "a chunk's rows are a wave of the scan");
+
+int tli_mlstm_scan(const MlGates& gates, float* m_state, float* keep, float* take, float* floors, float* through, int unit,
+                   const int* row_start, const int* seq_start, const int* slots, int T, int seqs, hipStream_t s) {
+    if (unit != TLI_CHUNK_ROWS && unit != TLI_RECURRENCE_SEGMENT) return tli_fail("mlstm_scan: units of %d rows", unit);
+    mlstm_scan_kernel<<<dim3(gates.H, seqs), ML_THREADS, 0, s>>>(gates, m_state, keep, take, floors, through, unit, row_start,
+                                                                 seq_start, slots, T);
+    return tli_check_launch("mlstm_scan");
 }
 
 template <typename T>
@@ -156,8 +153,8 @@ extern "C" int tli_mlstm(const void* proj, int ld, const float* z, long long z_r
     if (ssq && (parts <= 0 || x_size <= 0)) return tli_fail("mlstm: bad sums of squares");
     const MlGates gates{z, z_row, z_col, bias, cap, H, RowFactor{ssq, ssq ? parts : 0, T, 1.0f / (float)(x_size > 0 ? x_size : 1), x_eps}};
     hipStream_t s = (hipStream_t)stream;
-    if (!single)
-        mlstm_scan_kernel<<<dim3(H, seqs), ML_THREADS, 0, s>>>(gates, m_state, keep, take, floors, through, row_start, seq_start, slots, T);
+    if (!single && tli_mlstm_scan(gates, m_state, keep, take, floors, through, TLI_RECURRENCE_SEGMENT, row_start, seq_start, slots, T, seqs, s))
+        return 1;
     if (dtype == TLI_F32)
         mlstm_prepare_kernel<float><<<dim3(T, H), 256, 0, s>>>((const float*)proj, ld, q_scale, scratch, vals, gates, m_state, keep, take,
                                                                floors, seq_start, slots, T, single, dk, dv, plan.dkp, plan.dvp);

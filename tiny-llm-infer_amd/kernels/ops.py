@@ -136,6 +136,9 @@ def load_library():
         "tli_retention": [P, I, P, P, P, P, P, P, P, P, P, P, I, I, I, F, I, I, I, I, I, I, I, I, P],
         "tli_retention_step": [P, I, P, P, P, I, P, P, P, P, P, I, I, I, F, F, F, I, I, I, I, I, P],
         "tli_mlstm_step": [P, I, P, P, I, P, I, F, P, F, F, P, P, P, P, I, P, P, F, F, I, I, I, I, I, P],
+        "tli_chunked_takes": [I, I, I, I],
+        "tli_retention_chunked_bf16": [P, I, P, P, P, I, P, P, P, P, P, P, P, I, I, I, F, F, F, I, I, I, I, I, P],
+        "tli_mlstm_chunked_bf16": [P, I, P, ctypes.c_longlong, ctypes.c_longlong, P, I, I, F, P, F, F, P, P, P, P, I, P, P, P, P, P, F, F, I, I, I, I, I, P],
         "tli_mlstm": [P, I, P, ctypes.c_longlong, ctypes.c_longlong, P, I, I, F, P, F, F, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
         "tli_head_norm_gate": [P, P, P, P, I, P, I, I, I, I, F, I, F, I, P],
         "tli_pooled_prepare": [P, I, P, P, P, P, P, P, P, P, I, P, I, I, I, I, I, I, I, I, P, P, F, P, P, I, I, I, P, P, P, I, I, I, I, I, P],
@@ -151,6 +154,8 @@ def load_library():
         fn.restype = c_int
     lib.tli_lightning_scratch_floats.argtypes = [I, I, I, I, I, I]
     lib.tli_lightning_scratch_floats.restype = ctypes.c_longlong
+    lib.tli_chunked_scratch_floats.argtypes = [I, I, I, I, I]
+    lib.tli_chunked_scratch_floats.restype = ctypes.c_longlong
     lib.tli_sample_uniform.argtypes = [ctypes.c_uint32, ctypes.c_uint32, ctypes.c_uint32]
     lib.tli_sample_uniform.restype = c_float
     _LIB = lib
@@ -238,6 +243,7 @@ class HipOps:
         self.sinks_in_prefill = os.environ.get("TLI_SINKS_IN_PREFILL", "1") != "0"   # measurements, tests: False sends portions of prompts with sinks through sized_attention too
         self.lightning_lanes = int(os.environ.get("TLI_LIGHTNING_LANES", "0"))   # measurements, tests: 16 or 64 lanes a column of the lightning recurrence's state (0: the launch rule)
         self.rows_splits = 0
+        self.recurrence_in_chunks = True    # measurements, tests: False sends the portions of prompts of retention and mLSTM through the recurrence row by row
 
     @property
     def keep_row_major(self) -> bool:
@@ -1704,6 +1710,16 @@ class HipOps:
         """Whether every sequence of the step brings one row, and such a step may run through kernels of its own."""
         return step.max_rows_per_seq == 1 and step.num_seqs == step.num_rows and not self.unfused_decode
 
+    def _in_chunks(self, proj, at, dk, dv, dims=0, pairing=0) -> bool:
+        """Whether rows go through the recurrence in chunks (csrc/chunked.hip), else row by row."""
+        return (self.recurrence_in_chunks and proj.dtype == torch.bfloat16 and not self.force_plain
+                and (proj.data_ptr() + 2 * at) % 16 == 0 and proj.shape[1] % 8 == 0
+                and bool(self.lib.tli_chunked_takes(dk, dv, dims, pairing)))
+
+    def _chunked_scratch(self, step, heads, dk, columns, more=0):
+        n = int(self.lib.tli_chunked_scratch_floats(step.num_rows, step.num_seqs, heads, dk, columns))
+        return torch.empty((n + more,), dtype=torch.float32, device=self.device), n
+
     def retention(self, proj, at, decay, state, step, heads, dk, dv, rotary, k_scale, eps, scale, out, out_at):
         """From the raw projections ``proj[:, at:]`` (q (H dk) | k (H dk) | v (H dv) | gate (H dv)) to the layer's rows in
         ``out[:, out_at : out_at + H dv]``: the recurrence S <- decay_h S + k v^T, o = S^T q with q and k turned
@@ -1722,6 +1738,13 @@ class HipOps:
                        step.positions.data_ptr(), step.seq_start.data_ptr(), step.slots.data_ptr(), _ptr(cos), _ptr(sin), dims,
                        pairing, npos, float(k_scale), float(eps), float(scale), T, heads, dk, dv, _dtype_code(proj.dtype),
                        self._stream())
+            return
+        if self._in_chunks(proj, at, dk, dv, dims, pairing):
+            scratch, _ = self._chunked_scratch(step, heads, dk, dv)
+            self._call(self.lib.tli_retention_chunked_bf16, proj_ptr, proj.shape[1], decay.data_ptr(), state.data_ptr(), out_ptr, out_ld,
+                       scratch.data_ptr(), step.positions.data_ptr(), step.row_start.data_ptr(), step.seq_start.data_ptr(),
+                       step.slots.data_ptr(), _ptr(cos), _ptr(sin), dims, pairing, npos, float(k_scale), float(eps), float(scale),
+                       T, step.num_seqs, heads, dk, dv, self._stream())
             return
         o = torch.empty((T, heads, dv), dtype=torch.float32, device=self.device)
         scratch, _ = self._recurrence_scratch(step, heads, dk, dv)
@@ -1768,6 +1791,14 @@ class HipOps:
             return
         gates, transposed = self.small_product(rows, w_gates)
         z_row, z_col = (1, T) if transposed else (2 * heads, 1)
+        if self._in_chunks(proj, at, dk, dv):
+            scratch, size = self._chunked_scratch(step, heads, dk, dv + 1, more=4 * heads * T)
+            self._call(self.lib.tli_mlstm_chunked_bf16, proj_ptr, proj.shape[1], gates.data_ptr(), z_row, z_col, _ptr(ssq), parts, n,
+                       float(x_eps), gate_bias.data_ptr(), float(cap), float(q_scale), weight.data_ptr(), m_state.data_ptr(),
+                       state.data_ptr(), out_ptr, out_ld, scratch.data_ptr(), scratch.data_ptr() + 4 * size,
+                       step.row_start.data_ptr(), step.seq_start.data_ptr(), step.slots.data_ptr(), float(eps), float(scale), T,
+                       step.num_seqs, heads, dk, dv, self._stream())
+            return
         single = 1 if step.max_rows_per_seq == 1 and step.num_seqs == T else 0
         o = torch.empty((T, heads, dv + 1), dtype=torch.float32, device=self.device)
         floors = torch.empty((heads, T), dtype=torch.float32, device=self.device)

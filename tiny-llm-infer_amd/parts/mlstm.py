@@ -67,7 +67,7 @@ class MatrixLSTM(SplitMixer):
 
     def workspace_elems(self, rows: int) -> int:
         qk, v = self.heads * self.dk, self.heads * self.dv
-        return rows * (2 * qk + 2 * v + 2 * (4 * qk + 2 * v) + 2 * v + v + 8 * self.heads)
+        return rows * (2 * qk + 2 * v + max(2 * (4 * qk + 2 * v) + 2 * v + v, qk * (self.dv + 1) // 32) + 8 * self.heads)
 
     def between(self, x, proj, at, step: StepView, out, out_at, scale) -> None:
         self.env.ops.mlstm(proj, at, x, self.w_gates, self.gate_bias, self.cap, step.state["S"], step.state["m"], step,

@@ -66,9 +66,9 @@ class Retention(SplitMixer):
         return StateNeed(tuple(self.env.ops.lightning_state_shape(self.heads, self.dk, self.dv)), torch.float32)
 
     def workspace_elems(self, rows: int) -> int:
-        # the projections, then q, k, v (padded at worst to twice their size) and o in float32
+        # the projections, then q, k, v (padded at worst to twice their size) and o in float32, or the states before chunks of rows
         qk, v = self.heads * self.dk, self.heads * self.dv
-        return rows * (2 * qk + 2 * v + 2 * (4 * qk + 2 * v) + 2 * v + v)
+        return rows * (2 * qk + 2 * v + max(2 * (4 * qk + 2 * v) + 2 * v + v, qk * self.dv // 32))
 
     def between(self, x, proj, at, step: StepView, out, out_at, scale) -> None:
         self.env.ops.retention(proj, at, self.decay, step.state, step, self.heads, self.dk, self.dv, self.rotary,
