@@ -5,7 +5,7 @@
 // (the mLSTM's normaliser n is one more column of S whose value is 1), which are products of matrices.  All of them are
 // float32 on v_mfma_f32_16x16x4_f32, which takes float32 as it is: nothing of the recurrence is rounded to bfloat16.
 //
-// chunk_states: a workgroup a (32 elements of k, 64 of v; head; sequence) walks the sequence's chunks, its part of S in
+// chunk_states: a workgroup a (two pairs of pieces of k, 32 elements; 64 of v; head; sequence) walks the sequence's chunks, its part of S in
 //   the accumulators of the products, and leaves P of every chunk in scratch; the last S goes to the sequence's slot.
 // chunk_outputs: a workgroup a (chunk; head), a wave 16 rows: the two terms of o from P, K and V in LDS (P first, then K
 //   and V in its place), the scores and their weights in registers (transposed, S^T = K Q^T, so that they are already the
@@ -33,7 +33,6 @@ struct ChunkRows {                                       // what both kinds read
 };
 
 struct ChunkRotation {                                   // of q and k, and the factors behind it
-    const int* positions;
     const float* cos_table;                              // [table_positions, dims / 2] or null
     const float* sin_table;
     int dims, pairing, table_positions;
@@ -60,6 +59,11 @@ __device__ __forceinline__ void ck_load(const bf16_t* p, float (&v)[N]) {
     }
 #pragma unroll
     for (int i = 0; i < N / 2; ++i) v[2 * i] = bf16_to_f32((bf16_t)(u[i] & 0xffffu)), v[2 * i + 1] = bf16_to_f32((bf16_t)(u[i] >> 16));
+}
+__device__ __forceinline__ void ck_widen(const uint4& w, float (&v)[8]) {
+    const uint32_t u[4] = {w.x, w.y, w.z, w.w};
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[2 * i] = bf16_to_f32((bf16_t)(u[i] & 0xffffu)), v[2 * i + 1] = bf16_to_f32((bf16_t)(u[i] >> 16));
 }
 template <int N>
 __device__ __forceinline__ void ck_turned(const bf16_t* head, int d, const ChunkRotation& rot, int pos, float (&x)[N]) {
@@ -93,107 +97,204 @@ __device__ __forceinline__ void ck_turned(const bf16_t* head, int d, const Chunk
     }
 }
 
+// Two pieces of 8 elements of a row of K and the rotation's entries for them, as they are loaded: asked for early, made
+// into float32 where they are needed.  Pieces that turn together (halves) are one pair; of the others, and of
+// neighbours, two pieces side by side are.
+struct KeyPair {
+    uint4 raw[2];
+    float4 c[2], s[2];       // halves: 8 of each; neighbours: 4 for each piece
+};
+__device__ __forceinline__ void ck_pair_dims(int u, const ChunkRotation& rot, int& d1, int& d2) {
+    const int together = rot.cos_table && !rot.pairing ? rot.dims / 16 : 0;      // pairs of pieces of the two halves
+    if (u < together) {
+        d1 = 8 * u;
+        d2 = d1 + rot.dims / 2;
+    } else {
+        d1 = (rot.cos_table && !rot.pairing ? rot.dims : 0) + 16 * (u - together);
+        d2 = d1 + 8;
+    }
+}
+__device__ __forceinline__ void ck_pair_fetch(const bf16_t* head, int u, const ChunkRotation& rot, int pos, KeyPair& k) {
+    int d1, d2;
+    ck_pair_dims(u, rot, d1, d2);
+    k.raw[0] = *reinterpret_cast<const uint4*>(head + d1);
+    k.raw[1] = *reinterpret_cast<const uint4*>(head + d2);
+    if (rot.cos_table && d1 < rot.dims) {
+        const int half = rot.dims / 2;
+        const float* c = rot.cos_table + (size_t)min(pos, rot.table_positions - 1) * half + (rot.pairing ? d1 / 2 : d1);
+        const float* s = rot.sin_table + (size_t)min(pos, rot.table_positions - 1) * half + (rot.pairing ? d1 / 2 : d1);
+        // (neighbours: the second piece may lie past the turned elements; its entries are then not used)
+        const int second = rot.pairing && d2 >= rot.dims ? 0 : 4;
+        k.c[0] = *reinterpret_cast<const float4*>(c), k.c[1] = *reinterpret_cast<const float4*>(c + second);
+        k.s[0] = *reinterpret_cast<const float4*>(s), k.s[1] = *reinterpret_cast<const float4*>(s + second);
+    }
+}
+__device__ __forceinline__ void ck_pair_turn(const KeyPair& k, int u, const ChunkRotation& rot, int& d1, int& d2, float (&x)[8], float (&y)[8]) {
+    ck_pair_dims(u, rot, d1, d2);
+    ck_widen(k.raw[0], x);
+    ck_widen(k.raw[1], y);
+    if (!rot.cos_table || d1 >= rot.dims) return;
+    const float c[8] = {k.c[0].x, k.c[0].y, k.c[0].z, k.c[0].w, k.c[1].x, k.c[1].y, k.c[1].z, k.c[1].w};
+    const float s[8] = {k.s[0].x, k.s[0].y, k.s[0].z, k.s[0].w, k.s[1].x, k.s[1].y, k.s[1].z, k.s[1].w};
+    if (rot.pairing) {
+#pragma unroll
+        for (int p = 0; p < 4; ++p) {
+            const float a = x[2 * p], b = x[2 * p + 1];
+            x[2 * p] = rotate_first_half(a, b, c[p], s[p]);
+            x[2 * p + 1] = rotate_second_half(b, a, c[p], s[p]);
+            if (d2 < rot.dims) {
+                const float e = y[2 * p], f = y[2 * p + 1];
+                y[2 * p] = rotate_first_half(e, f, c[4 + p], s[4 + p]);
+                y[2 * p + 1] = rotate_second_half(f, e, c[4 + p], s[4 + p]);
+            }
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const float a = x[i], b = y[i];
+            x[i] = rotate_first_half(a, b, c[i], s[i]);
+            y[i] = rotate_second_half(b, a, c[i], s[i]);
+        }
+    }
+}
+
 __device__ __forceinline__ int ck_chunks(int rows) { return (rows + CK_ROWS - 1) / CK_ROWS; }
 
-#define CK_KDIMS 32          // of k a workgroup of chunk_states
-#define CK_VDIMS 64          // of v
+#define CK_PAIRS 2           // pairs of pieces of k (16 elements each) a workgroup of chunk_states
+#define CK_VDIMS 64          // elements of v
 #define CK_KLD (CK_ROWS + 4)
 
 template <bool MEMORY>
 __global__ __launch_bounds__(CK_THREADS) void chunk_states_kernel(ChunkRows a, ChunkRotation rot, ChunkDecay decay) {
-    __shared__ __align__(16) float kt[2][CK_KDIMS][CK_KLD];            // the chunk's weighted keys, transposed
+    __shared__ __align__(16) float kt[2][CK_PAIRS * 16][CK_KLD];       // the chunk's weighted keys, transposed
     const int tid = threadIdx.x, lane = tid % TLI_WAVE, wave = tid / TLI_WAVE, col = lane % 16, grp = lane / 16;
     const int dk = a.dk, dv = a.dv, H = a.H, OV = dv + (MEMORY ? 1 : 0);
-    const int k_slices = (dk + CK_KDIMS - 1) / CK_KDIMS;
-    const int dk0 = (blockIdx.x % k_slices) * CK_KDIMS, dv0 = (blockIdx.x / k_slices) * CK_VDIMS;
+    const int pairs = dk / 16, k_slices = (pairs + CK_PAIRS - 1) / CK_PAIRS;
+    const int u0 = (blockIdx.x % k_slices) * CK_PAIRS, dv0 = (blockIdx.x / k_slices) * CK_VDIMS;
     const int h = blockIdx.y, seq = blockIdx.z;
     const int r0 = a.row_start[seq], n = a.row_start[seq + 1] - r0;
     if (n <= 0) return;
     int z0 = 0;
     for (int i = 0; i < seq; ++i) z0 += ck_chunks(a.row_start[i + 1] - a.row_start[i]);
-    const int chunks = ck_chunks(n);
+    const int chunks = ck_chunks(n), pos0 = a.seq_start[seq];
     const int j = dv0 + wave * 16 + col;                               // this lane's column of S
     const bool mine = dv0 + wave * 16 < dv;
     const bool norm_too = MEMORY && dv0 == 0 && wave == 0;             // this wave keeps n of these elements of k as well
-    const bool tile1 = dk0 + 16 < dk;                                  // (dk in sixteens)
-    float* slot = a.state + ((size_t)a.slots[seq] * H + h) * OV * dk;
-    const bool fresh = a.seq_start[seq] == 0;
-    ck_f32x4 S[2];
-    float nk[2] = {0.f, 0.f};
+    const int tiles = min(CK_PAIRS, pairs - u0);                       // of 16 elements of k: tile t's rows of kt are pair u0 + t's pieces
+    // element of k that row r (0..15) of a tile's is, and the first of the four consecutive ones from row 4 grp on
+    int dim_col[CK_PAIRS], dim_grp[CK_PAIRS];
 #pragma unroll
-    for (int t = 0; t < 2; ++t) {
+    for (int t = 0; t < CK_PAIRS; ++t) {
+        int d1, d2;
+        ck_pair_dims(min(u0 + t, pairs - 1), rot, d1, d2);
+        dim_col[t] = col < 8 ? d1 + col : d2 + col - 8;
+        dim_grp[t] = grp < 2 ? d1 + 4 * grp : d2 + 4 * grp - 8;
+    }
+    float* slot = a.state + ((size_t)a.slots[seq] * H + h) * OV * dk;
+    const bool fresh = pos0 == 0;
+    ck_f32x4 S[CK_PAIRS];
+    float nk[CK_PAIRS];
+#pragma unroll
+    for (int t = 0; t < CK_PAIRS; ++t) {
         S[t] = (ck_f32x4){0.f, 0.f, 0.f, 0.f};
-        if (fresh || (t == 1 && !tile1)) continue;
-        if (mine) S[t] = *reinterpret_cast<const ck_f32x4*>(slot + (size_t)j * dk + dk0 + 16 * t + 4 * grp);
-        if (norm_too) nk[t] = slot[(size_t)dv * dk + dk0 + 16 * t + col];
+        nk[t] = 0.f;
+        if (fresh || t >= tiles) continue;
+        if (mine) S[t] = *reinterpret_cast<const ck_f32x4*>(slot + (size_t)j * dk + dim_grp[t]);
+        if (norm_too) nk[t] = slot[(size_t)dv * dk + dim_col[t]];
     }
     const bf16_t* k_head = a.proj + (size_t)r0 * a.ld + (size_t)(H + h) * dk;
     const bf16_t* v_head = a.proj + (size_t)r0 * a.ld + (size_t)2 * H * dk + (size_t)h * dv + (mine ? j : 0);
-    const int kr = tid / 4, kd = dk0 + (tid % 4) * 8;                  // this thread's row and piece of the chunk's keys
+    // half of the threads bring a chunk's keys (a pair of pieces each), the two halves every second chunk
+    const int kr = (tid / CK_PAIRS) % CK_ROWS, ku = tid % CK_PAIRS, k_turn = tid / (CK_PAIRS * CK_ROWS);
+    const bool k_mine = ku < tiles;
     const float lam = MEMORY ? 0.f : decay.head[h];
     const float* through = MEMORY ? decay.through + (size_t)h * a.T + r0 : nullptr;
     const float* takes = MEMORY ? decay.take + (size_t)h * a.T + r0 : nullptr;
-    float x[8], w = 0.f;
-    bf16_t v[16];
-    auto fetch = [&](int z) {
+    KeyPair kp;
+    float w_end = 0.f, w_row = 0.f, w_take = 0.f;
+    auto fetch_keys = [&](int z) {
+        const int first = z * CK_ROWS, last = min(first + CK_ROWS, n) - 1, r = min(first + kr, last);
+        if (k_mine) ck_pair_fetch(k_head + (size_t)r * a.ld, u0 + ku, rot, pos0 + r, kp);
+        if (MEMORY) w_end = through[last], w_row = through[r], w_take = takes[r];
+    };
+    auto store_keys = [&](int z) {
         const int first = z * CK_ROWS, count = min(CK_ROWS, n - first);
+        float x[8], y[8], w = 0.f;
+        int d1, d2;
+        ck_pair_turn(kp, u0 + ku, rot, d1, d2, x, y);
+        if (kr < count) w = MEMORY ? expf(w_end - w_row) * w_take : powf(lam, (float)(count - 1 - kr)) * rot.k_scale;
+        if (!k_mine) return;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) x[e] = 0.f;
-        w = 0.f;
-        if (kr < count && kd < dk) {
-            const int pos = rot.cos_table ? rot.positions[r0 + first + kr] : 0;
-            ck_turned<8>(k_head + (size_t)(first + kr) * a.ld, kd, rot, pos, x);
-            if constexpr (MEMORY) w = expf(through[first + count - 1] - through[first + kr]) * takes[first + kr];
-            else w = powf(lam, (float)(count - 1 - kr)) * rot.k_scale;
+        for (int e = 0; e < 8; ++e) {
+            kt[z & 1][16 * ku + e][kr] = x[e] * w;
+            kt[z & 1][16 * ku + 8 + e][kr] = y[e] * w;
         }
+    };
+    auto fetch_values = [&](int z, bf16_t (&v)[16]) {
+        const int first = z * CK_ROWS, last = min(first + CK_ROWS, n) - 1;
 #pragma unroll
         for (int s = 0; s < 4; ++s)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) v[4 * s + i] = v_head[(size_t)(first + min(16 * s + 4 * grp + i, count - 1)) * a.ld];
+            for (int i = 0; i < 4; ++i) v[4 * s + i] = v_head[(size_t)min(first + 16 * s + 4 * grp + i, last) * a.ld];
     };
-    fetch(0);
-    for (int z = 0; z < chunks; ++z) {
+    auto walk = [&](int z, const bf16_t (&v)[16]) {
         const int first = z * CK_ROWS, count = min(CK_ROWS, n - first);
-        float(*k_lds)[CK_KLD] = kt[z & 1];
-#pragma unroll
-        for (int e = 0; e < 8; ++e) k_lds[kd - dk0 + e][kr] = x[e] * w;
-        float vf[16];
-#pragma unroll
-        for (int i = 0; i < 16; ++i) vf[i] = bf16_to_f32(v[i]);
-        __syncthreads();                                               // (the buffer's last readers passed the barrier before)
-        if (z + 1 < chunks) fetch(z + 1);
         float* P = a.before + ((size_t)(z0 + z) * H + h) * OV * dk;
         const float g = MEMORY ? expf(through[first + count - 1]) : powf(lam, (float)count);
 #pragma unroll
-        for (int t = 0; t < 2; ++t) {
-            if (t == 1 && !tile1) continue;
-            if (mine) *reinterpret_cast<ck_f32x4*>(P + (size_t)j * dk + dk0 + 16 * t + 4 * grp) = S[t];
-            if (norm_too && grp == 0) P[(size_t)dv * dk + dk0 + 16 * t + col] = nk[t];
+        for (int t = 0; t < CK_PAIRS; ++t) {
+            if (t < tiles) {
+                if (mine) *reinterpret_cast<ck_f32x4*>(P + (size_t)j * dk + dim_grp[t]) = S[t];
+                if (norm_too && grp == 0) P[(size_t)dv * dk + dim_col[t]] = nk[t];
+            }
 #pragma unroll
             for (int i = 0; i < 4; ++i) S[t][i] *= g;
         }
-        float sum[2] = {0.f, 0.f};
+        float sum[CK_PAIRS] = {};
 #pragma unroll
         for (int s = 0; s < 4; ++s) {
-            if (16 * s >= count) continue;
 #pragma unroll
-            for (int t = 0; t < 2; ++t) {
-                const ck_f32x4 kk = *reinterpret_cast<const ck_f32x4*>(&k_lds[16 * t + col][16 * s + 4 * grp]);
+            for (int t = 0; t < CK_PAIRS; ++t) {
+                const ck_f32x4 kk = *reinterpret_cast<const ck_f32x4*>(&kt[z & 1][16 * t + col][16 * s + 4 * grp]);
 #pragma unroll
-                for (int i = 0; i < 4; ++i) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[i], vf[4 * s + i], S[t], 0, 0, 0);
+                for (int i = 0; i < 4; ++i) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[i], bf16_to_f32(v[4 * s + i]), S[t], 0, 0, 0);
                 if (MEMORY) sum[t] += (kk[0] + kk[1]) + (kk[2] + kk[3]);
             }
         }
         if (norm_too) {
 #pragma unroll
-            for (int t = 0; t < 2; ++t) nk[t] = fmaf(g, nk[t], quad_rows_sum(sum[t]));
+            for (int t = 0; t < CK_PAIRS; ++t) nk[t] = fmaf(g, nk[t], quad_rows_sum(sum[t]));
         }
+    };
+    // A chunk's keys are asked for two chunks ahead, each half of the threads having one chunk's on the way, its values
+    // one ahead.  (A tile without elements of k, t >= tiles, multiplies what LDS holds and is not stored.)
+    bf16_t v0[16], v1[16];
+    if (k_turn < chunks) fetch_keys(k_turn);
+    fetch_values(0, v0);
+    if (k_turn == 0) {
+        store_keys(0);
+        if (2 < chunks) fetch_keys(2);
+    }
+    __syncthreads();
+    for (int z = 0; z < chunks; ++z) {
+        // chunk z is in kt[z & 1]; the other buffer was last read before the barrier
+        if (z + 1 < chunks) {
+            if (z & 1) fetch_values(z + 1, v0);
+            else fetch_values(z + 1, v1);
+            if (k_turn == ((z + 1) & 1)) {
+                store_keys(z + 1);
+                if (z + 3 < chunks) fetch_keys(z + 3);
+            }
+        }
+        if (z & 1) walk(z, v1);
+        else walk(z, v0);
+        __syncthreads();
     }
 #pragma unroll
-    for (int t = 0; t < 2; ++t) {
-        if (t == 1 && !tile1) continue;
-        if (mine) *reinterpret_cast<ck_f32x4*>(slot + (size_t)j * dk + dk0 + 16 * t + 4 * grp) = S[t];
-        if (norm_too && grp == 0) slot[(size_t)dv * dk + dk0 + 16 * t + col] = nk[t];
+    for (int t = 0; t < CK_PAIRS; ++t) {
+        if (t >= tiles) continue;
+        if (mine) *reinterpret_cast<ck_f32x4*>(slot + (size_t)j * dk + dim_grp[t]) = S[t];
+        if (norm_too && grp == 0) slot[(size_t)dv * dk + dim_col[t]] = nk[t];
     }
 }
 
@@ -234,14 +335,37 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
     const float* P = a.before + ((size_t)blockIdx.x * H + h) * OV * dk;
     const bf16_t* rows = a.proj + (size_t)r0 * a.ld;
     const float lam = MEMORY ? 0.f : decay.head[h];
-    const int i = 16 * wave + col;                                     // this lane's row of the chunk
-    const int row = min(i, count - 1);
-    const bool works = 16 * wave < count;                              // (the same for the whole wave)
+    // a wave's tile of 16 rows: the later a tile, the more scores it has, so every second round of workgroups deals them out
+    // the other way round
+    const int rt = ((blockIdx.y * gridDim.x + blockIdx.x) >> 8) & 1 ? CK_ROWS / 16 - 1 - wave : wave;
+    const int i = 16 * rt + col;                                       // this lane's row of the chunk
+    const int row = min(i, count - 1), pos0 = a.seq_start[seq] + z * CK_ROWS;
+    const bool works = 16 * rt < count;                                // (the same for the whole wave)
 
-    if (!from_nothing) {                                               // P, [dv][dk]
-        const int pieces = dv * dk / 4, per = dk / 4;
-        for (int p = tid; p < pieces; p += CK_THREADS)
-            *reinterpret_cast<float4*>(ck_lds + (p / per) * KLD + (p % per) * 4) = *reinterpret_cast<const float4*>(P + (size_t)p * 4);
+    // everything that the workgroup reads is asked for at once: P, q, K and V (K's and V's stay in registers until P's place
+    // in LDS is free)
+    constexpr int PP = (NK * NV * 16 * 16 / 4 + CK_THREADS - 1) / CK_THREADS, KP = (CK_ROWS * NK + CK_THREADS - 1) / CK_THREADS;
+    constexpr int VP = (CK_ROWS * NV * 2 + CK_THREADS - 1) / CK_THREADS;
+    const int p_row = dk / 4, p_all = dv * p_row;
+    float4 pr[PP];
+    if (!from_nothing) {
+#pragma unroll
+        for (int u = 0; u < PP; ++u) {
+            const int p = tid + u * CK_THREADS;
+            pr[u] = *reinterpret_cast<const float4*>(P + (size_t)min(p, p_all - 1) * 4);
+        }
+    }
+    KeyPair kp[KP];
+    uint4 vr[VP];
+#pragma unroll
+    for (int u = 0; u < KP; ++u) {
+        const int p = min(tid + u * CK_THREADS, count * nk - 1), r = p / nk;
+        ck_pair_fetch(rows + (size_t)r * a.ld + (size_t)(H + h) * dk, p - r * nk, rot, pos0 + r, kp[u]);
+    }
+#pragma unroll
+    for (int u = 0; u < VP; ++u) {
+        const int p = min(tid + u * CK_THREADS, count * nv * 2 - 1), r = p / (nv * 2);
+        vr[u] = *reinterpret_cast<const uint4*>(rows + (size_t)r * a.ld + (size_t)2 * H * dk + (size_t)h * dv + (p - r * nv * 2) * 8);
     }
     if (tid < CK_ROWS) {
         if constexpr (MEMORY) {
@@ -257,7 +381,7 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
     float q[NK][4];
 #pragma unroll
     for (int b = 0; b < NK; ++b) {
-        ck_turned<4>(rows + (size_t)row * a.ld + (size_t)h * dk, 16 * k_tile(b) + 4 * grp, rot, rot.cos_table ? rot.positions[r0 + row] : 0, q[b]);
+        ck_turned<4>(rows + (size_t)row * a.ld + (size_t)h * dk, 16 * k_tile(b) + 4 * grp, rot, pos0 + row, q[b]);
 #pragma unroll
         for (int e = 0; e < 4; ++e) q[b][e] = b < nk ? q[b][e] * rot.q_scale : 0.f;
     }
@@ -265,6 +389,13 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
 #pragma unroll
     for (int t = 0; t < NV; ++t) acc[t] = (ck_f32x4){0.f, 0.f, 0.f, 0.f};
     float nq = 0.f;                                                    // n . q of this lane's row, this lane group's share
+    if (!from_nothing) {                                               // P, [dv][dk]
+#pragma unroll
+        for (int u = 0; u < PP; ++u) {
+            const int p = tid + u * CK_THREADS;
+            if (p < p_all) *reinterpret_cast<float4*>(ck_lds + (p / p_row) * KLD + (p % p_row) * 4) = pr[u];
+        }
+    }
     __syncthreads();
     if (!from_nothing && works) {
         const float g = MEMORY ? expf(log_s[row]) : log_s[row] * lam;  // A of the row
@@ -293,24 +424,33 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
     __syncthreads();                                                   // P has been read
     float* k_s = ck_lds;                                               // [row][dk + 4]
     float* v_s = ck_lds + CK_ROWS * KLD;                               // [row][dv + 4]
-    for (int p = tid; p < count * (dk / 8); p += CK_THREADS) {
-        const int r = p / (dk / 8), d = (p % (dk / 8)) * 8;
-        float x[8];
-        ck_turned<8>(rows + (size_t)r * a.ld + (size_t)(H + h) * dk, d, rot, rot.cos_table ? rot.positions[r0 + r] : 0, x);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) k_s[r * KLD + d + e] = x[e] * rot.k_scale;
+    for (int u = 0; u < KP; ++u) {
+        const int p = tid + u * CK_THREADS, r = p / nk;
+        if (p >= count * nk) continue;
+        float x[8], y[8];
+        int d1, d2;
+        ck_pair_turn(kp[u], p - r * nk, rot, d1, d2, x, y);
+        float* dst = k_s + r * KLD;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) dst[d1 + e] = x[e] * rot.k_scale;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) dst[d2 + e] = y[e] * rot.k_scale;
     }
-    for (int p = tid; p < count * (dv / 8); p += CK_THREADS) {
-        const int r = p / (dv / 8), d = (p % (dv / 8)) * 8;
-        float x[8];
-        ck_load<8>(rows + (size_t)r * a.ld + (size_t)2 * H * dk + (size_t)h * dv + d, x);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) v_s[r * VLD + d + e] = x[e];
+    for (int u = 0; u < VP; ++u) {
+        const int p = tid + u * CK_THREADS, r = p / (nv * 2);
+        if (p >= count * nv * 2) continue;
+        float x[8];
+        ck_widen(vr[u], x);
+        float* dst = v_s + r * VLD + (p - r * nv * 2) * 8;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) dst[e] = x[e];
     }
     __syncthreads();
     if (!works) return;
     const float my_log = MEMORY ? log_s[row] : 0.f;
-    for (int jt = 0; jt <= wave; ++jt) {
+    for (int jt = 0; jt <= rt; ++jt) {
         // (rows of K and V past the chunk's last are what was in LDS before: their scores are set to 0, and their
         // values are read from the last row)
         ck_f32x4 s[2] = {(ck_f32x4){0.f, 0.f, 0.f, 0.f}, (ck_f32x4){0.f, 0.f, 0.f, 0.f}};
@@ -390,7 +530,7 @@ static int run_chunked(const ChunkRows& a, const ChunkRotation& rot, const Chunk
     if ((((uintptr_t)a.proj | (uintptr_t)a.state | (uintptr_t)a.before | (uintptr_t)out.weight | (uintptr_t)rot.cos_table | (uintptr_t)rot.sin_table) & 15) ||
         ((uintptr_t)out.out & 7))
         return tli_fail("chunked recurrence: operands must be 16-byte aligned");
-    const int slices = ((a.dk + CK_KDIMS - 1) / CK_KDIMS) * ((a.dv + CK_VDIMS - 1) / CK_VDIMS);
+    const int slices = ((a.dk / 16 + CK_PAIRS - 1) / CK_PAIRS) * ((a.dv + CK_VDIMS - 1) / CK_VDIMS);
     chunk_states_kernel<MEMORY><<<dim3(slices, a.H, a.seqs), CK_THREADS, 0, s>>>(a, rot, decay);
     const size_t lds = ck_lds_floats(a.dk, a.dv) * sizeof(float);
     const dim3 grid(zs, a.H);
@@ -418,7 +558,7 @@ static int run_chunked(const ChunkRows& a, const ChunkRotation& rot, const Chunk
 // bfloat16 rows; the arguments as for tli_retention_step (recurrent_step.hip), row_start [seqs + 1], seq_start, slots
 // [seqs]; scratch: tli_chunked_scratch_floats(T, seqs, H, dk, dv) floats
 extern "C" int tli_retention_chunked_bf16(const void* proj, int ld, const float* decay, float* state, void* out, int out_ld,
-                                          float* scratch, const int* positions, const int* row_start, const int* seq_start,
+                                          float* scratch, const int* row_start, const int* seq_start,
                                           const int* slots, const float* cos_table, const float* sin_table, int dims, int pairing,
                                           int table_positions, float k_scale, float eps, float scale, int T, int seqs, int H, int dk,
                                           int dv, void* stream) {
@@ -426,7 +566,7 @@ extern "C" int tli_retention_chunked_bf16(const void* proj, int ld, const float*
     if (H <= 0 || !tli_chunked_takes(dk, dv, cos_table ? dims : 0, pairing) || (cos_table && (dims <= 0 || dims > dk)))
         return tli_fail("retention in chunks: heads of %d and %d with %d turned elements", dk, dv, dims);
     const ChunkRows a{(const bf16_t*)proj, ld, state, scratch, row_start, seq_start, slots, T, seqs, H, dk, dv};
-    return run_chunked<false>(a, ChunkRotation{positions, cos_table, sin_table, dims, pairing, table_positions, 1.0f, k_scale},
+    return run_chunked<false>(a, ChunkRotation{cos_table, sin_table, dims, pairing, table_positions, 1.0f, k_scale},
                               ChunkDecay{decay, nullptr, nullptr}, ChunkOutput{(bf16_t*)out, out_ld, nullptr, nullptr, eps, scale},
                               (hipStream_t)stream);
 }
@@ -448,6 +588,6 @@ extern "C" int tli_mlstm_chunked_bf16(const void* proj, int ld, const float* z, 
     const MlGates gates{z, z_row, z_col, bias, cap, H, RowFactor{ssq, ssq ? parts : 0, T, 1.0f / (float)(x_size > 0 ? x_size : 1), x_eps}};
     if (tli_mlstm_scan(gates, m_state, keep, take, floors, through, CK_ROWS, row_start, seq_start, slots, T, seqs, s)) return 1;
     const ChunkRows a{(const bf16_t*)proj, ld, state, scratch, row_start, seq_start, slots, T, seqs, H, dk, dv};
-    return run_chunked<true>(a, ChunkRotation{nullptr, nullptr, nullptr, 0, 0, 0, q_scale, 1.0f}, ChunkDecay{nullptr, through, take},
+    return run_chunked<true>(a, ChunkRotation{nullptr, nullptr, 0, 0, 0, q_scale, 1.0f}, ChunkDecay{nullptr, through, take},
                              ChunkOutput{(bf16_t*)out, out_ld, weight, floors, eps, scale}, s);
 }

@@ -137,7 +137,7 @@ def load_library():
         "tli_retention_step": [P, I, P, P, P, I, P, P, P, P, P, I, I, I, F, F, F, I, I, I, I, I, P],
         "tli_mlstm_step": [P, I, P, P, I, P, I, F, P, F, F, P, P, P, P, I, P, P, F, F, I, I, I, I, I, P],
         "tli_chunked_takes": [I, I, I, I],
-        "tli_retention_chunked_bf16": [P, I, P, P, P, I, P, P, P, P, P, P, P, I, I, I, F, F, F, I, I, I, I, I, P],
+        "tli_retention_chunked_bf16": [P, I, P, P, P, I, P, P, P, P, P, P, I, I, I, F, F, F, I, I, I, I, I, P],
         "tli_mlstm_chunked_bf16": [P, I, P, ctypes.c_longlong, ctypes.c_longlong, P, I, I, F, P, F, F, P, P, P, P, I, P, P, P, P, P, F, F, I, I, I, I, I, P],
         "tli_mlstm": [P, I, P, ctypes.c_longlong, ctypes.c_longlong, P, I, I, F, P, F, F, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
         "tli_head_norm_gate": [P, P, P, P, I, P, I, I, I, I, F, I, F, I, P],
@@ -1742,7 +1742,7 @@ class HipOps:
         if self._in_chunks(proj, at, dk, dv, dims, pairing):
             scratch, _ = self._chunked_scratch(step, heads, dk, dv)
             self._call(self.lib.tli_retention_chunked_bf16, proj_ptr, proj.shape[1], decay.data_ptr(), state.data_ptr(), out_ptr, out_ld,
-                       scratch.data_ptr(), step.positions.data_ptr(), step.row_start.data_ptr(), step.seq_start.data_ptr(),
+                       scratch.data_ptr(), step.row_start.data_ptr(), step.seq_start.data_ptr(),
                        step.slots.data_ptr(), _ptr(cos), _ptr(sin), dims, pairing, npos, float(k_scale), float(eps), float(scale),
                        T, step.num_seqs, heads, dk, dv, self._stream())
             return
