@@ -45,54 +45,63 @@ struct ChunkDecay {
     const float* take;                                   // w_t
 };
 
-// N consecutive elements from dim d on of a head's q or k at `head`, in float32, turned, not scaled.  N is 4 or 8 and a
-// piece lies on one side of every border (dims and half of it are multiples of N, for neighbours dims is).
-template <int N>
-__device__ __forceinline__ void ck_load(const bf16_t* p, float (&v)[N]) {
-    uint32_t u[N / 2];
-    if constexpr (N == 8) {
-        const uint4 w = *reinterpret_cast<const uint4*>(p);
-        u[0] = w.x, u[1] = w.y, u[2] = w.z, u[3] = w.w;
-    } else {
-        const uint2 w = *reinterpret_cast<const uint2*>(p);
-        u[0] = w.x, u[1] = w.y;
-    }
-#pragma unroll
-    for (int i = 0; i < N / 2; ++i) v[2 * i] = bf16_to_f32((bf16_t)(u[i] & 0xffffu)), v[2 * i + 1] = bf16_to_f32((bf16_t)(u[i] >> 16));
+// How q and k turn: not at all, pair i being (i, i + dims/2), or (2i, 2i + 1).  Pieces of 4 or 8 elements lie on one side of
+// every border (dims and half of it are multiples of 8, for neighbours dims is).  Elements past the turned ones turn by
+// an angle of 0, so that no load stands behind a condition.
+enum { ROT_NONE = 0, ROT_HALVES = 1, ROT_NEIGHBOURS = 2 };
+
+__device__ __forceinline__ void ck_widen(const uint2& w, float (&v)[4]) {
+    v[0] = bf16_to_f32((bf16_t)(w.x & 0xffffu)), v[1] = bf16_to_f32((bf16_t)(w.x >> 16));
+    v[2] = bf16_to_f32((bf16_t)(w.y & 0xffffu)), v[3] = bf16_to_f32((bf16_t)(w.y >> 16));
 }
 __device__ __forceinline__ void ck_widen(const uint4& w, float (&v)[8]) {
     const uint32_t u[4] = {w.x, w.y, w.z, w.w};
 #pragma unroll
     for (int i = 0; i < 4; ++i) v[2 * i] = bf16_to_f32((bf16_t)(u[i] & 0xffffu)), v[2 * i + 1] = bf16_to_f32((bf16_t)(u[i] >> 16));
 }
-template <int N>
-__device__ __forceinline__ void ck_turned(const bf16_t* head, int d, const ChunkRotation& rot, int pos, float (&x)[N]) {
-    ck_load<N>(head + d, x);
-    if (!rot.cos_table || d >= rot.dims || pos >= rot.table_positions) return;
+
+// Four elements of a row of q from dim d on and what turns them, as they are loaded.
+struct QueryPiece {
+    uint2 raw, other;        // halves: the partners
+    float4 c, s;             // halves: of four pairs; neighbours: of two
+};
+template <int ROT>
+__device__ __forceinline__ void ck_query_fetch(const bf16_t* head, int d, const ChunkRotation& rot, int pos, QueryPiece& q) {
+    q.raw = *reinterpret_cast<const uint2*>(head + d);
+    if constexpr (ROT == ROT_NONE) return;
     const int half = rot.dims / 2;
-    const float* cos_row = rot.cos_table + (size_t)pos * half;
-    const float* sin_row = rot.sin_table + (size_t)pos * half;
-    if (rot.pairing) {
-#pragma unroll
-        for (int p = 0; p < N / 2; ++p) {
-            const float c = cos_row[d / 2 + p], s = sin_row[d / 2 + p], a = x[2 * p], b = x[2 * p + 1];
-            x[2 * p] = rotate_first_half(a, b, c, s);
-            x[2 * p + 1] = rotate_second_half(b, a, c, s);
-        }
+    const bool in = d < rot.dims, second = d >= half;
+    if (ROT == ROT_HALVES) {
+        q.other = *reinterpret_cast<const uint2*>(head + (!in ? d : second ? d - half : d + half));
+        const size_t at = (size_t)pos * half + (!in ? 0 : second ? d - half : d);
+        q.c = *reinterpret_cast<const float4*>(rot.cos_table + at);
+        q.s = *reinterpret_cast<const float4*>(rot.sin_table + at);
     } else {
-        const bool second = d >= half;
-        float other[N];
-        ck_load<N>(head + (second ? d - half : d + half), other);
-        const float* c = cos_row + (second ? d - half : d);
-        const float* s = sin_row + (second ? d - half : d);
+        const size_t at = (size_t)pos * half + (in ? d / 2 : 0);
+        const float2 c = *reinterpret_cast<const float2*>(rot.cos_table + at), s = *reinterpret_cast<const float2*>(rot.sin_table + at);
+        q.c = make_float4(c.x, c.y, 0.f, 0.f);
+        q.s = make_float4(s.x, s.y, 0.f, 0.f);
+    }
+}
+template <int ROT>
+__device__ __forceinline__ void ck_query_turn(const QueryPiece& q, int d, const ChunkRotation& rot, float (&x)[4]) {
+    ck_widen(q.raw, x);
+    if constexpr (ROT == ROT_NONE) return;
+    if (d >= rot.dims) return;
+    const float c[4] = {q.c.x, q.c.y, q.c.z, q.c.w}, s[4] = {q.s.x, q.s.y, q.s.z, q.s.w};
+    if (ROT == ROT_HALVES) {
+        float other[4];
+        ck_widen(q.other, other);
+        const bool second = d >= rot.dims / 2;
 #pragma unroll
-        for (int i = 0; i < N; i += 4) {
-            const float4 cc = *reinterpret_cast<const float4*>(c + i), ss = *reinterpret_cast<const float4*>(s + i);
-            const float cv[4] = {cc.x, cc.y, cc.z, cc.w}, sv[4] = {ss.x, ss.y, ss.z, ss.w};
+        for (int i = 0; i < 4; ++i)
+            x[i] = second ? rotate_second_half(x[i], other[i], c[i], s[i]) : rotate_first_half(x[i], other[i], c[i], s[i]);
+    } else {
 #pragma unroll
-            for (int j = 0; j < 4; ++j)
-                x[i + j] = second ? rotate_second_half(x[i + j], other[i + j], cv[j], sv[j])
-                                  : rotate_first_half(x[i + j], other[i + j], cv[j], sv[j]);
+        for (int p = 0; p < 2; ++p) {
+            const float a = x[2 * p], b = x[2 * p + 1];
+            x[2 * p] = rotate_first_half(a, b, c[p], s[p]);
+            x[2 * p + 1] = rotate_second_half(b, a, c[p], s[p]);
         }
     }
 }
@@ -102,58 +111,67 @@ __device__ __forceinline__ void ck_turned(const bf16_t* head, int d, const Chunk
 // neighbours, two pieces side by side are.
 struct KeyPair {
     uint4 raw[2];
-    float4 c[2], s[2];       // halves: 8 of each; neighbours: 4 for each piece
+    float4 c[2], s[2];       // halves: of eight pairs; neighbours: of four for each piece
 };
+template <int ROT>
 __device__ __forceinline__ void ck_pair_dims(int u, const ChunkRotation& rot, int& d1, int& d2) {
-    const int together = rot.cos_table && !rot.pairing ? rot.dims / 16 : 0;      // pairs of pieces of the two halves
-    if (u < together) {
-        d1 = 8 * u;
-        d2 = d1 + rot.dims / 2;
-    } else {
-        d1 = (rot.cos_table && !rot.pairing ? rot.dims : 0) + 16 * (u - together);
-        d2 = d1 + 8;
-    }
+    const int together = ROT == ROT_HALVES ? rot.dims / 16 : 0;        // pairs of pieces of the two halves
+    d1 = u < together ? 8 * u : (ROT == ROT_HALVES ? rot.dims : 0) + 16 * (u - together);
+    d2 = u < together ? d1 + rot.dims / 2 : d1 + 8;
 }
-__device__ __forceinline__ void ck_pair_fetch(const bf16_t* head, int u, const ChunkRotation& rot, int pos, KeyPair& k) {
+template <int ROT>
+__device__ __forceinline__ void ck_pair_fetch(const bf16_t* head, int u, const ChunkRotation& rot, KeyPair& k) {
     int d1, d2;
-    ck_pair_dims(u, rot, d1, d2);
+    ck_pair_dims<ROT>(u, rot, d1, d2);
     k.raw[0] = *reinterpret_cast<const uint4*>(head + d1);
     k.raw[1] = *reinterpret_cast<const uint4*>(head + d2);
-    if (rot.cos_table && d1 < rot.dims) {
-        const int half = rot.dims / 2;
-        const float* c = rot.cos_table + (size_t)min(pos, rot.table_positions - 1) * half + (rot.pairing ? d1 / 2 : d1);
-        const float* s = rot.sin_table + (size_t)min(pos, rot.table_positions - 1) * half + (rot.pairing ? d1 / 2 : d1);
-        // (neighbours: the second piece may lie past the turned elements; its entries are then not used)
-        const int second = rot.pairing && d2 >= rot.dims ? 0 : 4;
-        k.c[0] = *reinterpret_cast<const float4*>(c), k.c[1] = *reinterpret_cast<const float4*>(c + second);
-        k.s[0] = *reinterpret_cast<const float4*>(s), k.s[1] = *reinterpret_cast<const float4*>(s + second);
-    }
 }
+template <int ROT>
+__device__ __forceinline__ void ck_pair_angles(int u, const ChunkRotation& rot, int pos, KeyPair& k) {
+    if constexpr (ROT == ROT_NONE) return;
+    int d1, d2;
+    ck_pair_dims<ROT>(u, rot, d1, d2);
+    const size_t row = (size_t)pos * (rot.dims / 2);
+    size_t first = row, second = row;
+    if (ROT == ROT_HALVES) {
+        first += d1 < rot.dims ? d1 : 0;
+        second = first + 4;
+    } else {
+        first += d1 < rot.dims ? d1 / 2 : 0;
+        second += d2 < rot.dims ? d2 / 2 : 0;
+    }
+    k.c[0] = *reinterpret_cast<const float4*>(rot.cos_table + first), k.c[1] = *reinterpret_cast<const float4*>(rot.cos_table + second);
+    k.s[0] = *reinterpret_cast<const float4*>(rot.sin_table + first), k.s[1] = *reinterpret_cast<const float4*>(rot.sin_table + second);
+}
+template <int ROT>
 __device__ __forceinline__ void ck_pair_turn(const KeyPair& k, int u, const ChunkRotation& rot, int& d1, int& d2, float (&x)[8], float (&y)[8]) {
-    ck_pair_dims(u, rot, d1, d2);
+    ck_pair_dims<ROT>(u, rot, d1, d2);
     ck_widen(k.raw[0], x);
     ck_widen(k.raw[1], y);
-    if (!rot.cos_table || d1 >= rot.dims) return;
+    if constexpr (ROT == ROT_NONE) return;
     const float c[8] = {k.c[0].x, k.c[0].y, k.c[0].z, k.c[0].w, k.c[1].x, k.c[1].y, k.c[1].z, k.c[1].w};
     const float s[8] = {k.s[0].x, k.s[0].y, k.s[0].z, k.s[0].w, k.s[1].x, k.s[1].y, k.s[1].z, k.s[1].w};
-    if (rot.pairing) {
-#pragma unroll
-        for (int p = 0; p < 4; ++p) {
-            const float a = x[2 * p], b = x[2 * p + 1];
-            x[2 * p] = rotate_first_half(a, b, c[p], s[p]);
-            x[2 * p + 1] = rotate_second_half(b, a, c[p], s[p]);
-            if (d2 < rot.dims) {
-                const float e = y[2 * p], f = y[2 * p + 1];
-                y[2 * p] = rotate_first_half(e, f, c[4 + p], s[4 + p]);
-                y[2 * p + 1] = rotate_second_half(f, e, c[4 + p], s[4 + p]);
-            }
-        }
-    } else {
+    if (ROT == ROT_HALVES) {
+        if (d1 >= rot.dims) return;
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
             const float a = x[i], b = y[i];
             x[i] = rotate_first_half(a, b, c[i], s[i]);
             y[i] = rotate_second_half(b, a, c[i], s[i]);
+        }
+    } else {
+#pragma unroll
+        for (int p = 0; p < 4; ++p) {
+            if (d1 < rot.dims) {
+                const float a = x[2 * p], b = x[2 * p + 1];
+                x[2 * p] = rotate_first_half(a, b, c[p], s[p]);
+                x[2 * p + 1] = rotate_second_half(b, a, c[p], s[p]);
+            }
+            if (d2 < rot.dims) {
+                const float a = y[2 * p], b = y[2 * p + 1];
+                y[2 * p] = rotate_first_half(a, b, c[4 + p], s[4 + p]);
+                y[2 * p + 1] = rotate_second_half(b, a, c[4 + p], s[4 + p]);
+            }
         }
     }
 }
@@ -164,7 +182,7 @@ __device__ __forceinline__ int ck_chunks(int rows) { return (rows + CK_ROWS - 1)
 #define CK_VDIMS 64          // elements of v
 #define CK_KLD (CK_ROWS + 4)
 
-template <bool MEMORY>
+template <bool MEMORY, int ROT>
 __global__ __launch_bounds__(CK_THREADS) void chunk_states_kernel(ChunkRows a, ChunkRotation rot, ChunkDecay decay) {
     __shared__ __align__(16) float kt[2][CK_PAIRS * 16][CK_KLD];       // the chunk's weighted keys, transposed
     const int tid = threadIdx.x, lane = tid % TLI_WAVE, wave = tid / TLI_WAVE, col = lane % 16, grp = lane / 16;
@@ -186,7 +204,7 @@ __global__ __launch_bounds__(CK_THREADS) void chunk_states_kernel(ChunkRows a, C
 #pragma unroll
     for (int t = 0; t < CK_PAIRS; ++t) {
         int d1, d2;
-        ck_pair_dims(min(u0 + t, pairs - 1), rot, d1, d2);
+        ck_pair_dims<ROT>(min(u0 + t, pairs - 1), rot, d1, d2);
         dim_col[t] = col < 8 ? d1 + col : d2 + col - 8;
         dim_grp[t] = grp < 2 ? d1 + 4 * grp : d2 + 4 * grp - 8;
     }
@@ -203,26 +221,32 @@ __global__ __launch_bounds__(CK_THREADS) void chunk_states_kernel(ChunkRows a, C
         if (norm_too) nk[t] = slot[(size_t)dv * dk + dim_col[t]];
     }
     const bf16_t* k_head = a.proj + (size_t)r0 * a.ld + (size_t)(H + h) * dk;
-    const bf16_t* v_head = a.proj + (size_t)r0 * a.ld + (size_t)2 * H * dk + (size_t)h * dv + (mine ? j : 0);
+    const bf16_t* v_head = a.proj + (size_t)r0 * a.ld + (size_t)2 * H * dk + (size_t)h * dv;      // (the same for all lanes)
+    const uint32_t v_lane = (uint32_t)(4 * grp) * a.ld + (mine ? j : 0);
     // half of the threads bring a chunk's keys (a pair of pieces each), the two halves every second chunk
     const int kr = (tid / CK_PAIRS) % CK_ROWS, ku = tid % CK_PAIRS, k_turn = tid / (CK_PAIRS * CK_ROWS);
     const bool k_mine = ku < tiles;
     const float lam = MEMORY ? 0.f : decay.head[h];
     const float* through = MEMORY ? decay.through + (size_t)h * a.T + r0 : nullptr;
     const float* takes = MEMORY ? decay.take + (size_t)h * a.T + r0 : nullptr;
+    const float whole = MEMORY ? 0.f : powf(lam, (float)CK_ROWS), w_whole = MEMORY ? 0.f : powf(lam, (float)(CK_ROWS - 1 - kr)) * rot.k_scale;
+    const int tail = n - (chunks - 1) * CK_ROWS;                       // rows of the last chunk
     KeyPair kp;
     float w_end = 0.f, w_row = 0.f, w_take = 0.f;
     auto fetch_keys = [&](int z) {
         const int first = z * CK_ROWS, last = min(first + CK_ROWS, n) - 1, r = min(first + kr, last);
-        if (k_mine) ck_pair_fetch(k_head + (size_t)r * a.ld, u0 + ku, rot, pos0 + r, kp);
+        const int u = u0 + min(ku, tiles - 1);
+        ck_pair_fetch<ROT>(k_head + (size_t)r * a.ld, u, rot, kp);
+        ck_pair_angles<ROT>(u, rot, pos0 + r, kp);
         if (MEMORY) w_end = through[last], w_row = through[r], w_take = takes[r];
     };
     auto store_keys = [&](int z) {
-        const int first = z * CK_ROWS, count = min(CK_ROWS, n - first);
-        float x[8], y[8], w = 0.f;
+        float x[8], y[8], w = w_whole;
         int d1, d2;
-        ck_pair_turn(kp, u0 + ku, rot, d1, d2, x, y);
-        if (kr < count) w = MEMORY ? expf(w_end - w_row) * w_take : powf(lam, (float)(count - 1 - kr)) * rot.k_scale;
+        ck_pair_turn<ROT>(kp, u0 + ku, rot, d1, d2, x, y);
+        if (MEMORY) w = expf(w_end - w_row) * w_take;
+        else if (z == chunks - 1 && tail < CK_ROWS) w = powf(lam, (float)max(tail - 1 - kr, 0)) * rot.k_scale;
+        if (z == chunks - 1 && kr >= tail) w = 0.f;
         if (!k_mine) return;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
@@ -230,17 +254,25 @@ __global__ __launch_bounds__(CK_THREADS) void chunk_states_kernel(ChunkRows a, C
             kt[z & 1][16 * ku + 8 + e][kr] = y[e] * w;
         }
     };
-    auto fetch_values = [&](int z, bf16_t (&v)[16]) {
-        const int first = z * CK_ROWS, last = min(first + CK_ROWS, n) - 1;
+    auto fetch_values = [&](int z, bf16_t (&v)[16], float& end) {
+        const int first = z * CK_ROWS;
+        if (MEMORY) end = through[min(first + CK_ROWS, n) - 1];
+        const bf16_t* base = v_head + (size_t)first * a.ld;
+        if (z < chunks - 1 || tail == CK_ROWS) {
 #pragma unroll
-        for (int s = 0; s < 4; ++s)
+            for (int s = 0; s < 4; ++s)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) v[4 * s + i] = v_head[(size_t)min(first + 16 * s + 4 * grp + i, last) * a.ld];
+                for (int i = 0; i < 4; ++i) v[4 * s + i] = (base + (size_t)(16 * s + i) * a.ld)[v_lane];
+        } else {
+#pragma unroll
+            for (int s = 0; s < 4; ++s)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) v[4 * s + i] = base[(size_t)min(16 * s + 4 * grp + i, tail - 1) * a.ld + (mine ? j : 0)];
+        }
     };
-    auto walk = [&](int z, const bf16_t (&v)[16]) {
-        const int first = z * CK_ROWS, count = min(CK_ROWS, n - first);
+    auto walk = [&](int z, const bf16_t (&v)[16], float end) {
         float* P = a.before + ((size_t)(z0 + z) * H + h) * OV * dk;
-        const float g = MEMORY ? expf(through[first + count - 1]) : powf(lam, (float)count);
+        const float g = MEMORY ? expf(end) : z == chunks - 1 && tail < CK_ROWS ? powf(lam, (float)tail) : whole;
 #pragma unroll
         for (int t = 0; t < CK_PAIRS; ++t) {
             if (t < tiles) {
@@ -269,8 +301,9 @@ __global__ __launch_bounds__(CK_THREADS) void chunk_states_kernel(ChunkRows a, C
     // A chunk's keys are asked for two chunks ahead, each half of the threads having one chunk's on the way, its values
     // one ahead.  (A tile without elements of k, t >= tiles, multiplies what LDS holds and is not stored.)
     bf16_t v0[16], v1[16];
+    float end0 = 0.f, end1 = 0.f;                        // the last log A of the chunks whose values are in v0 and v1
     if (k_turn < chunks) fetch_keys(k_turn);
-    fetch_values(0, v0);
+    fetch_values(0, v0, end0);
     if (k_turn == 0) {
         store_keys(0);
         if (2 < chunks) fetch_keys(2);
@@ -279,15 +312,15 @@ __global__ __launch_bounds__(CK_THREADS) void chunk_states_kernel(ChunkRows a, C
     for (int z = 0; z < chunks; ++z) {
         // chunk z is in kt[z & 1]; the other buffer was last read before the barrier
         if (z + 1 < chunks) {
-            if (z & 1) fetch_values(z + 1, v0);
-            else fetch_values(z + 1, v1);
+            if (z & 1) fetch_values(z + 1, v0, end0);
+            else fetch_values(z + 1, v1, end1);
             if (k_turn == ((z + 1) & 1)) {
                 store_keys(z + 1);
                 if (z + 3 < chunks) fetch_keys(z + 3);
             }
         }
-        if (z & 1) walk(z, v1);
-        else walk(z, v0);
+        if (z & 1) walk(z, v1, end1);
+        else walk(z, v0, end0);
         __syncthreads();
     }
 #pragma unroll
@@ -314,7 +347,7 @@ static inline size_t ck_lds_floats(int dk, int dv) {
 // MEMORY: with a normaliser and the logistic gate; else the silu gate.  NK, NV: sixteens of a head (EXACT), or their
 // bound: sixteens past a head's are multiplied all the same, q's as zeros and v's into sums that nobody reads, from
 // addresses of the head's last, so that no matrix instruction stands behind a condition
-template <bool MEMORY, int NK, int NV, bool EXACT>
+template <bool MEMORY, int ROT, int NK, int NV, bool EXACT>
 __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows a, ChunkRotation rot, ChunkDecay decay, ChunkOutput out) {
     extern __shared__ __align__(16) float ck_lds[];
     __shared__ float log_s[CK_ROWS], take_s[CK_ROWS];                  // mLSTM: log A and w; else the powers of the decay
@@ -360,7 +393,7 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
 #pragma unroll
     for (int u = 0; u < KP; ++u) {
         const int p = min(tid + u * CK_THREADS, count * nk - 1), r = p / nk;
-        ck_pair_fetch(rows + (size_t)r * a.ld + (size_t)(H + h) * dk, p - r * nk, rot, pos0 + r, kp[u]);
+        ck_pair_fetch<ROT>(rows + (size_t)r * a.ld + (size_t)(H + h) * dk, p - r * nk, rot, kp[u]);
     }
 #pragma unroll
     for (int u = 0; u < VP; ++u) {
@@ -379,11 +412,17 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
     auto k_tile = [&](int b) { return EXACT ? b : min(b, nk - 1); };
     auto v_tile = [&](int t) { return EXACT ? t : min(t, nv - 1); };
     float q[NK][4];
+    {
+        QueryPiece piece[NK];
+        const bf16_t* q_row = rows + (size_t)row * a.ld + (size_t)h * dk;
 #pragma unroll
-    for (int b = 0; b < NK; ++b) {
-        ck_turned<4>(rows + (size_t)row * a.ld + (size_t)h * dk, 16 * k_tile(b) + 4 * grp, rot, pos0 + row, q[b]);
+        for (int b = 0; b < NK; ++b) ck_query_fetch<ROT>(q_row, 16 * k_tile(b) + 4 * grp, rot, pos0 + row, piece[b]);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) q[b][e] = b < nk ? q[b][e] * rot.q_scale : 0.f;
+        for (int b = 0; b < NK; ++b) {
+            ck_query_turn<ROT>(piece[b], 16 * k_tile(b) + 4 * grp, rot, q[b]);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) q[b][e] = b < nk ? q[b][e] * rot.q_scale : 0.f;
+        }
     }
     ck_f32x4 acc[NV];
 #pragma unroll
@@ -395,6 +434,11 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
             const int p = tid + u * CK_THREADS;
             if (p < p_all) *reinterpret_cast<float4*>(ck_lds + (p / p_row) * KLD + (p % p_row) * 4) = pr[u];
         }
+    }
+#pragma unroll
+    for (int u = 0; u < KP; ++u) {                                     // (while the products with P run)
+        const int p = min(tid + u * CK_THREADS, count * nk - 1), r = p / nk;
+        ck_pair_angles<ROT>(p - r * nk, rot, pos0 + r, kp[u]);
     }
     __syncthreads();
     if (!from_nothing && works) {
@@ -430,7 +474,7 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
         if (p >= count * nk) continue;
         float x[8], y[8];
         int d1, d2;
-        ck_pair_turn(kp[u], p - r * nk, rot, d1, d2, x, y);
+        ck_pair_turn<ROT>(kp[u], p - r * nk, rot, d1, d2, x, y);
         float* dst = k_s + r * KLD;
 #pragma unroll
         for (int e = 0; e < 8; ++e) dst[d1 + e] = x[e] * rot.k_scale;
@@ -498,7 +542,7 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
         if (t >= nv) continue;
         const int d = 16 * t + 4 * grp;
         float g[4], y[4];
-        ck_load<4>(gate + d, g);
+        ck_widen(*reinterpret_cast<const uint2*>(gate + d), g);
         float wt[4] = {1.f, 1.f, 1.f, 1.f};
         if (out.weight) {
             const float4 w4 = *reinterpret_cast<const float4*>(out.weight + (size_t)h * dv + d);
@@ -531,12 +575,12 @@ static int run_chunked(const ChunkRows& a, const ChunkRotation& rot, const Chunk
         ((uintptr_t)out.out & 7))
         return tli_fail("chunked recurrence: operands must be 16-byte aligned");
     const int slices = ((a.dk / 16 + CK_PAIRS - 1) / CK_PAIRS) * ((a.dv + CK_VDIMS - 1) / CK_VDIMS);
-    chunk_states_kernel<MEMORY><<<dim3(slices, a.H, a.seqs), CK_THREADS, 0, s>>>(a, rot, decay);
+    const dim3 states_grid(slices, a.H, a.seqs);
     const size_t lds = ck_lds_floats(a.dk, a.dv) * sizeof(float);
     const dim3 grid(zs, a.H);
-#define CK_RUN(NK, NV, EXACT)                                                                                               \
+#define CK_RUN(ROT, NK, NV, EXACT)                                                                                          \
     {                                                                                                                       \
-        auto kernel = chunk_outputs_kernel<MEMORY, NK, NV, EXACT>;                                                          \
+        auto kernel = chunk_outputs_kernel<MEMORY, ROT, NK, NV, EXACT>;                                                     \
         static bool allowed = false;                                                                                        \
         if (lds > 60 * 1024 && !allowed) {                                                                                  \
             if (hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 72 * 1024) !=          \
@@ -546,11 +590,20 @@ static int run_chunked(const ChunkRows& a, const ChunkRotation& rot, const Chunk
         }                                                                                                                   \
         kernel<<<grid, CK_THREADS, lds, s>>>(a, rot, decay, out);                                                           \
     }
-    if (a.dk == 128 && a.dv == 128) CK_RUN(8, 8, true)
-    else if (a.dk == 64 && a.dv == 64) CK_RUN(4, 4, true)
-    else if (a.dk <= 32 && a.dv <= 32) CK_RUN(2, 2, false)
-    else if (a.dk <= 64 && a.dv <= 64) CK_RUN(4, 4, false)
-    else CK_RUN(8, 8, false)
+#define CK_SIZES(ROT)                                                                                                       \
+    {                                                                                                                       \
+        chunk_states_kernel<MEMORY, ROT><<<states_grid, CK_THREADS, 0, s>>>(a, rot, decay);                                 \
+        if (a.dk == 128 && a.dv == 128) CK_RUN(ROT, 8, 8, true)                                                             \
+        else if (a.dk == 64 && a.dv == 64) CK_RUN(ROT, 4, 4, true)                                                          \
+        else if (a.dk <= 32 && a.dv <= 32) CK_RUN(ROT, 2, 2, false)                                                         \
+        else if (a.dk <= 64 && a.dv <= 64) CK_RUN(ROT, 4, 4, false)                                                         \
+        else CK_RUN(ROT, 8, 8, false)                                                                                       \
+    }
+    if constexpr (MEMORY) CK_SIZES(ROT_NONE)
+    else if (!rot.cos_table) CK_SIZES(ROT_NONE)
+    else if (rot.pairing) CK_SIZES(ROT_NEIGHBOURS)
+    else CK_SIZES(ROT_HALVES)
+#undef CK_SIZES
 #undef CK_RUN
     return tli_check_launch("chunked recurrence");
 }
