@@ -164,15 +164,19 @@ def _attend(ops, q, k, v, scale, window, pool, sinks, page, cuts, out_scale=1.0,
 
 SIZES = [  # heads, kv heads, key size, value size, window, pool, page
     (4, 2, 16, 32, 20, 4, 16), (6, 2, 64, 64, 33, 12, 16), (4, 1, 128, 128, 40, 16, 32), (3, 3, 20, 12, 7, 10, 8),
-    (2, 1, 48, 80, 16, 1, 16), (34, 2, 16, 16, 1, 3, 16), (2, 2, 256, 144, 25, 5, 64), (1, 1, 7, 5, 30, 8, 4), (18, 1, 288, 64, 50, 7, 16),
+    (2, 1, 48, 80, 16, 1, 16), (6, 3, 64, 64, 20, 6, 8), (3, 1, 128, 128, 70, 2, 64), (8, 1, 64, 64, 1, 1, 16), (34, 2, 16, 16, 1, 3, 16), (2, 2, 256, 144, 25, 5, 64), (1, 1, 7, 5, 30, 8, 4), (18, 1, 288, 64, 50, 7, 16),
 ]
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("sizes", SIZES, ids=lambda s: "-".join(map(str, s)))
-def test_window_and_blocks_in_portions(ops, dtype, sizes):
+@pytest.mark.parametrize("own", [True, False], ids=["own", "sized"])
+def test_window_and_blocks_in_portions(ops, dtype, sizes, own, monkeypatch):
     """Sequences of unequal lengths side by side, in portions of 1 to 70 rows and row by row."""
     H, G, d, e, window, pool, page = sizes
+    if not own and (dtype == "float32" or not ops.lib.tli_pooled_prefill_takes(d, e, page, 200, window, pool)):
+        pytest.skip("no prefill kernel of their own")
+    monkeypatch.setattr(ops, "pooled_prefill", own)
     g = torch.Generator().manual_seed(d + e)
     lengths = [150, 1, 67, pool + window]
     dt = DTYPES[dtype]

@@ -645,9 +645,7 @@ static int run_sized_mfma(
         // (sizes with a kernel of their own: heads of 64 and 128 with values of 64 to 256 in float32, for the
         // attention with two maps; a latent vector of 512 beside a turned part of 64)
         if (pooled.pool > 0) {
-            if (nk == 8 && nv == 8) AST_RUN(8, 8, false, bf16_t, true, 4, true)
-            else if (nk == 4 && nv == 4) AST_RUN(4, 4, false, bf16_t, true, 4, true)
-            else if (nk <= 8 && nv <= 8) AST_RUN(8, 8, false, bf16_t, false, 4, true)
+            if (nk <= 8 && nv <= 8) AST_RUN(8, 8, false, bf16_t, false, 4, true)
             else if (nk <= 16 && nv <= 16) AST_RUN(16, 16, false, bf16_t, false, 4, true)
             else AST_RUN(40, 32, false, bf16_t, false, 4, true)
         } else if (v_cache && out_f32 && nk == 4 && nv == 4) AST_ONE(4, 4, false, float, true, 4)

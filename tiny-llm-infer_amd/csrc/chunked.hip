@@ -20,6 +20,7 @@
 #define CK_THREADS 256
 
 typedef float ck_f32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t ck_u32x4 __attribute__((ext_vector_type(4)));
 
 struct ChunkRows {                                       // what both kinds read and write
     const bf16_t* proj;                                  // [T, ld]: q (H dk) | k (H dk) | v (H dv) | gate (H dv)
@@ -380,16 +381,16 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
     constexpr int PP = (NK * NV * 16 * 16 / 4 + CK_THREADS - 1) / CK_THREADS, KP = (CK_ROWS * NK + CK_THREADS - 1) / CK_THREADS;
     constexpr int VP = (CK_ROWS * NV * 2 + CK_THREADS - 1) / CK_THREADS;
     const int p_row = dk / 4, p_all = dv * p_row;
-    float4 pr[PP];
+    ck_f32x4 pr[PP];                                                   // (a native vector type: an array of float4 would go to memory)
     if (!from_nothing) {
 #pragma unroll
         for (int u = 0; u < PP; ++u) {
             const int p = tid + u * CK_THREADS;
-            pr[u] = *reinterpret_cast<const float4*>(P + (size_t)min(p, p_all - 1) * 4);
+            pr[u] = *reinterpret_cast<const ck_f32x4*>(P + (size_t)min(p, p_all - 1) * 4);
         }
     }
     KeyPair kp[KP];
-    uint4 vr[VP];
+    ck_u32x4 vr[VP];
 #pragma unroll
     for (int u = 0; u < KP; ++u) {
         const int p = min(tid + u * CK_THREADS, count * nk - 1), r = p / nk;
@@ -398,7 +399,7 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
 #pragma unroll
     for (int u = 0; u < VP; ++u) {
         const int p = min(tid + u * CK_THREADS, count * nv * 2 - 1), r = p / (nv * 2);
-        vr[u] = *reinterpret_cast<const uint4*>(rows + (size_t)r * a.ld + (size_t)2 * H * dk + (size_t)h * dv + (p - r * nv * 2) * 8);
+        vr[u] = *reinterpret_cast<const ck_u32x4*>(rows + (size_t)r * a.ld + (size_t)2 * H * dk + (size_t)h * dv + (p - r * nv * 2) * 8);
     }
     if (tid < CK_ROWS) {
         if constexpr (MEMORY) {
@@ -432,7 +433,7 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
 #pragma unroll
         for (int u = 0; u < PP; ++u) {
             const int p = tid + u * CK_THREADS;
-            if (p < p_all) *reinterpret_cast<float4*>(ck_lds + (p / p_row) * KLD + (p % p_row) * 4) = pr[u];
+            if (p < p_all) *reinterpret_cast<ck_f32x4*>(ck_lds + (p / p_row) * KLD + (p % p_row) * 4) = pr[u];
         }
     }
 #pragma unroll
@@ -486,7 +487,7 @@ __global__ __launch_bounds__(CK_THREADS, 2) void chunk_outputs_kernel(ChunkRows 
         const int p = tid + u * CK_THREADS, r = p / (nv * 2);
         if (p >= count * nv * 2) continue;
         float x[8];
-        ck_widen(vr[u], x);
+        ck_widen(make_uint4(vr[u][0], vr[u][1], vr[u][2], vr[u][3]), x);
         float* dst = v_s + r * VLD + (p - r * nv * 2) * 8;
 #pragma unroll
         for (int e = 0; e < 8; ++e) dst[e] = x[e];

@@ -143,6 +143,8 @@ def load_library():
         "tli_head_norm_gate": [P, P, P, P, I, P, I, I, I, I, F, I, F, I, P],
         "tli_pooled_prepare": [P, I, P, P, P, P, P, P, P, P, I, P, I, I, I, I, I, I, I, I, P, P, F, P, P, I, I, I, P, P, P, I, I, I, I, I, P],
         "tli_attention_pooled_plain": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
+        "tli_pooled_prefill_takes": [I, I, I, I, I, I],
+        "tli_pooled_prefill_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
         "tli_attention_pooled_mfma_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
         "tli_sample": [P, I, I, P, P, P, P, P, P],
         "tli_sample_scratch_bytes": [I],
@@ -243,6 +245,7 @@ class HipOps:
         self.sinks_in_prefill = os.environ.get("TLI_SINKS_IN_PREFILL", "1") != "0"   # measurements, tests: False sends portions of prompts with sinks through sized_attention too
         self.lightning_lanes = int(os.environ.get("TLI_LIGHTNING_LANES", "0"))   # measurements, tests: 16 or 64 lanes a column of the lightning recurrence's state (0: the launch rule)
         self.rows_splits = 0
+        self.pooled_prefill = True       # measurements, tests: False sends portions of prompts over windows and pooled blocks through the kernels for sizes of their own
         self.recurrence_in_chunks = True    # measurements, tests: False sends the portions of prompts of retention and mLSTM through the recurrence row by row
 
     @property
@@ -1676,9 +1679,17 @@ class HipOps:
                    step.seq_start.data_ptr(), step.num_seqs, g.tables.data_ptr(), g.table_width, g.page_size, kc.shape[0], T,
                    heads, kv_heads, key_dim, value_dim, _ptr(q_weight), _ptr(k_weight), float(eps), _ptr(cos), _ptr(sin), dims,
                    pairing, npos, *pooled, single, _dtype_code(proj.dtype), self._stream())
+        starts = step.h_row_start
+        if (proj.dtype == torch.bfloat16 and not self.force_plain and not single and self.pooled_prefill
+                and self.lib.tli_pooled_prefill_takes(key_dim, value_dim, g.page_size, int(step.max_seq_len), int(window), pool)):
+            tiles = sum((starts[i + 1] - starts[i] + 31) // 32 for i in range(step.num_seqs))
+            self._call(self.lib.tli_pooled_prefill_bf16, q.data_ptr(), out_ptr, kc.data_ptr(), vc.data_ptr(),
+                       step.row_start.data_ptr(), step.seq_start.data_ptr(), step.num_seqs, tiles, g.tables.data_ptr(),
+                       g.table_width, g.page_size, kc.shape[0], heads, kv_heads, key_dim, value_dim, float(scale), int(window),
+                       *pooled, int(step.max_seq_len), _ptr(sinks), out_ld, float(out_scale), self._stream())
+            return
         if (proj.dtype == torch.bfloat16 and not self.force_plain
                 and self.lib.tli_attention_sized_mfma_takes(key_dim, value_dim, g.page_size, 1)):
-            starts = step.h_row_start
             tiles = T if single else sum((starts[i + 1] - starts[i] + 15) // 16 for i in range(step.num_seqs))
             self._call(self.lib.tli_attention_pooled_mfma_bf16, q.data_ptr(), out_ptr, kc.data_ptr(), vc.data_ptr(),
                        step.row_start.data_ptr(), step.seq_start.data_ptr(), step.num_seqs, tiles, g.tables.data_ptr(),
