@@ -13,7 +13,7 @@ import torch
 import plain_kosusun
 from cpu_ops import CpuOps
 from helpers import collect, max_error, random_prompt, trace_mixed, trace_portions, trace_prefill_then_decode, trace_whole
-from kosusun_helpers import (SMALL, _config, _layer, _parallel, _retention, _rot, _window, make_weights, plain_greedy, plain_logits,
+from kosusun_helpers import (SMALL, _config, _layer, _mlstm, _parallel, _retention, _rot, _window, make_weights, plain_greedy, plain_logits,
                              write_folder)
 from tiny_llm_infer_amd.cache.manager import PAGE, CacheFull, CacheManager, CacheNeed, CacheRecord
 from tiny_llm_infer_amd.config import ConfigError, KosusunConfig
@@ -251,6 +251,27 @@ def test_greedy_generation_matches_plain(folders, name):
     assert [r.token_ids for r in got] == want
     eng.runner.cache.check()
     assert eng.runner.cache.free_pages() == eng.runner.cache.pages_per_group()
+
+
+def test_a_model_that_keeps_state_only(tmp_path):
+    """mLSTM layers alone: no group of pages at all, requests live by their slots."""
+    cfg = _config(97, 40, [_layer("mlstm", _mlstm(2, 12, 9, 7.0), 33), _layer("mlstm", _mlstm(3, 8, 16, 12.0), None)], mult=0.7)
+    folder = write_folder(str(tmp_path / "state"), cfg, make_weights(cfg, 2))
+    reqs = {f"r{i}": random_prompt(97, n, i) for i, n in enumerate((40, 3, 65, 21, 30))}
+    want = plain_logits(folder, reqs)
+    for steps in (trace_whole(reqs), trace_portions(reqs, seed=3), trace_mixed(reqs, max_tokens=256, seed=9)):
+        runner = _runner(folder, 16, 256)
+        assert not runner.cache.groups
+        got = collect(steps, _replay(runner, steps))
+        for rid in reqs:
+            err, row, scale = max_error(got[rid], want[rid])
+            assert err <= 2e-5 * scale, (rid, err, row)
+        assert not runner.cache.live()
+    prompts = [random_prompt(97, n, 40 + n) for n in (5, 17, 9)]
+    eng = LLMEngine.from_folder(folder, dtype="float32", device="cpu", max_model_len=64, page_size=16, num_kv_blocks=0, max_num_seqs=2,
+                                max_num_batched_tokens=24, ops=CpuOps())
+    got = eng.generate(prompts, SamplingParams(max_tokens=6, ignore_eos=True))
+    assert [r.token_ids for r in got] == [plain_greedy(folder, p, 6) for p in prompts]
 
 
 def test_a_request_that_the_blocks_pages_cannot_hold_is_refused(folders):
