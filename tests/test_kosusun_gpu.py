@@ -189,6 +189,13 @@ def test_window_and_blocks_in_portions(ops, dtype, sizes, own, monkeypatch):
         got = _attend(ops, q, k, v, d ** -0.5, window, pool, sinks, page, cuts, out_scale=0.5)
         for i, n in enumerate(lengths):
             _close(got[i], 0.5 * want[i], 1e-5 if dtype == "float32" else 2e-2, f"sequence {i} in portions of {cuts}")
+    if dtype == "bfloat16" and ops.lib.tli_attention_sized_mfma_takes(d, e, page, 1):
+        for splits in (2, 5, 64):                       # a row's keys shared out over workgroups, some of which have none
+            monkeypatch.setattr(ops, "pooled_splits", splits)
+            got = _attend(ops, q, k, v, d ** -0.5, window, pool, sinks, page, [1], out_scale=0.5)
+            for i, n in enumerate(lengths):
+                _close(got[i], 0.5 * want[i], 2e-2, f"sequence {i} row by row in {splits} splits")
+        monkeypatch.setattr(ops, "pooled_splits", None)
     got = _attend(ops, q, k, v, d ** -0.5, window, pool, None, page, [29, 64])
     for i in range(len(lengths)):
         bare = plain_kosusun.windowed_attention(q[i].double(), k[i].double(), v[i].double(), d ** -0.5, window, pool, None)
@@ -198,7 +205,7 @@ def test_window_and_blocks_in_portions(ops, dtype, sizes, own, monkeypatch):
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("sizes", [(4, 2, 16, 32, 20, 4, 16), (4, 2, 64, 64, 37, 12, 16), (2, 1, 128, 128, 40, 16, 32), (2, 1, 20, 12, 7, 10, 8)],
                          ids=lambda s: "-".join(map(str, s)))
-def test_one_key_at_every_edge(ops, dtype, sizes):
+def test_one_key_at_every_edge(ops, dtype, sizes, monkeypatch):
     """One key answers the last row's query far above all others.  It stands just inside and just outside the window
     (there in no block that is seen, or in the last one that is), in the first and last position of blocks, at the
     borders of pages, at position 0 and hundreds back; in a prompt, at the end of a portion of two, and decoded alone.
@@ -226,7 +233,8 @@ def test_one_key_at_every_edge(ops, dtype, sizes):
             want = _last_row(q, kk, v, window, pool)
             for other in (window - 1, window + 1):
                 told += float((_last_row(q, kk, v, other, pool) - want).abs().max()) > 0.1 * float(want.abs().max())
-            for cuts in ([n], [n - 2, 2], [n - 1, 1]):
+            for cuts, splits in (([n], None), ([n - 2, 2], None), ([n - 1, 1], None), ([n - 1, 1], 3)):
+                monkeypatch.setattr(ops, "pooled_splits", splits)
                 got = _attend(ops, [q], [kk], [v], 1.0, window, pool, None, page, cuts)[0][i]
                 _close(got, want, 1e-5 if dtype == "float32" else 2e-2, f"{n} rows in {cuts}, the key at {at} (window from {edge}, {seen} blocks)")
     assert told >= 4
@@ -243,13 +251,14 @@ def _last_row(q, k, v, window, pool):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_a_sink_that_takes_most_of_the_weight(ops, dtype):
+def test_a_sink_that_takes_most_of_the_weight(ops, dtype, monkeypatch):
     g = torch.Generator().manual_seed(5)
     dt = DTYPES[dtype]
     q, k, v = ((torch.randn(90, h, 16, generator=g)).to(dt) for h in (3, 1, 1))
     for sinks in (torch.tensor([9.0, -30.0, 2.0]), torch.tensor([80.0, 5.0, 0.0])):
         want = plain_kosusun.windowed_attention(q.double(), k.double(), v.double(), 0.25, 24, 6, sinks)
-        for cuts in ([90], [30, 1]):
+        for cuts, splits in (([90], None), ([30, 1], None), ([30, 1], 4)):
+            monkeypatch.setattr(ops, "pooled_splits", splits)
             _close(_attend(ops, [q], [k], [v], 0.25, 24, 6, sinks, 16, cuts)[0], want, 1e-5 if dtype == "float32" else 2e-2, f"{sinks} {cuts}")
 
 

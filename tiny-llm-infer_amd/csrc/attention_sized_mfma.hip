@@ -72,7 +72,7 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
     const bf16_t* __restrict__ v_cache, const int* __restrict__ row_start, const int* __restrict__ seq_start,
     int num_seqs, const int* __restrict__ tables, int table_width, int page_size, int num_pages, int heads,
     int kv_heads, int maps, int nk_arg, int nv_arg, float scale, int window, int keep_first, int grouped, int col_groups,
-    const float* __restrict__ sinks, PooledKeys pooled, int out_ld, float out_scale) {
+    const float* __restrict__ sinks, PooledKeys pooled, int out_ld, float out_scale, float* __restrict__ parts) {
     const int nk = EXACT ? NKM : nk_arg, nv = EXACT ? NVM : nv_arg;
     const int DK = nk * 16, DV = nv * 16, LD = DK + ASM_PAD;
     const int pieces = 2 * nk;                                          // 16-byte pieces of one key
@@ -185,8 +185,11 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
             }
         }
     };
-    if (wave < n_tiles) fetch(wave);
-    for (int it = wave; it < n_tiles; it += ASM_WAVES) {
+    // with splits (gridDim.z of them) the waves of all the workgroups of one (row, key head) take turns at its tiles
+    const int stride = POOLED ? ASM_WAVES * (int)gridDim.z : ASM_WAVES;
+    const int first = POOLED ? ASM_WAVES * (int)blockIdx.z + wave : wave;
+    if (first < n_tiles) fetch(first);
+    for (int it = first; it < n_tiles; it += stride) {
         const int k0 = tile_key(it);
         {
             int ck = key_first, cp = piece_first;
@@ -202,7 +205,7 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
                 }
             }
         }
-        if (it + ASM_WAVES < n_tiles) fetch(it + ASM_WAVES);
+        if (it + stride < n_tiles) fetch(it + stride);
         const bool block = is_block(it);
         // the values of this tile's keys from their own cache: dim 16 j + col of the keys k0 + 4 grp + i
         SFrag4 vf[VKEY ? 1 : NVM];
@@ -315,6 +318,14 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
     float inv = lt > 0.f ? 1.0f / lt : 0.f;
     if (sinks) inv = asm_sink_factor(sinks[unit], mt, lt);
     inv *= out_scale;
+    float* part = nullptr;
+    if (POOLED && parts) {                              // the sums as they are, with m and l behind them
+        part = parts + (((size_t)(row0 + my) * units + unit) * gridDim.z + blockIdx.z) * (DV + 4);
+        if (grp == 0) {
+            part[DV] = mt;
+            part[DV + 1] = lt;
+        }
+    }
     TO* o_row = out + (size_t)(row0 + my) * out_ld + (size_t)unit * DV;
 #pragma unroll
     for (int j = 0; j < NVM; ++j) {
@@ -328,8 +339,43 @@ __global__ __launch_bounds__(64 * ASM_WAVES) void attention_sized_mfma_kernel(
 #pragma unroll
                 for (int i = 0; i < 4; ++i) a[i] += t[i] * fw[w];
             }
-            asm_store4(o_row + j * 16 + grp * 4, a, inv);
+            if (POOLED && part)
+                asm_store4(part + j * 16 + grp * 4, a, 1.0f);
+            else
+                asm_store4(o_row + j * 16 + grp * 4, a, inv);
         }
+    }
+}
+
+// The splits of a (row, head) put together: a wave each, a lane value elements 4 lane .. + 3 (and every 256 further on).
+__global__ __launch_bounds__(256) void attention_parts_merge_kernel(
+    const float* __restrict__ parts, int splits, int pairs, int heads, int DV, const float* __restrict__ sinks,
+    bf16_t* __restrict__ out, int out_ld, float out_scale) {
+    const int lane = threadIdx.x % 64, pair = blockIdx.x * 4 + threadIdx.x / 64;
+    if (pair >= pairs) return;
+    const int row = pair / heads, head = pair - row * heads;
+    const float* mine = parts + (size_t)pair * splits * (DV + 4);
+    // lane s has split s's m and l (at most 64 splits)
+    const bool have = lane < splits;
+    const float m = have ? mine[(size_t)lane * (DV + 4) + DV] : -INFINITY;
+    const float mt = wave_max(m);
+    const float f = (m == -INFINITY) ? 0.f : __expf(m - mt);
+    const float l = wave_sum(have ? mine[(size_t)lane * (DV + 4) + DV + 1] * f : 0.f);
+    float inv = l > 0.f ? 1.0f / l : 0.f;
+    if (sinks) inv = asm_sink_factor(sinks[head], mt, l);
+    inv *= out_scale;
+    for (int d0 = 0; d0 < DV; d0 += 256) {              // (every lane stays in for the exchanges)
+        const int d = d0 + lane * 4;
+        f32x4 a = (f32x4){0.f, 0.f, 0.f, 0.f};
+        for (int s = 0; s < splits; ++s) {
+            const float fs = __shfl(f, s);
+            if (d < DV) {
+                const f32x4 t = *reinterpret_cast<const f32x4*>(mine + (size_t)s * (DV + 4) + d);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) a[i] += t[i] * fs;
+            }
+        }
+        if (d < DV) asm_store4(out + (size_t)row * out_ld + (size_t)head * DV + d, a, inv);
     }
 }
 
@@ -592,7 +638,7 @@ static int run_sized_mfma(
     const void* q, void* out, const void* k_cache, const void* v_cache, const int* row_start, const int* seq_start,
     int num_seqs, int tiles, const int* tables, int table_width, int page_size, int num_pages, int heads, int kv_heads,
     int maps, int key_dim, int value_dim, float scale, int window, int keep_first, int grouped, int out_f32,
-    const float* sinks, const PooledKeys& pooled, int out_ld, float out_scale, void* stream) {
+    const float* sinks, const PooledKeys& pooled, int out_ld, float out_scale, int splits, float* parts, void* stream) {
     if (num_seqs <= 0 || tiles <= 0) return 0;
     if (!tli_attention_sized_mfma_takes(key_dim, value_dim, page_size, v_cache != nullptr))
         return tli_fail("attention: the matrix-core kernel does not take keys of %d and values of %d in pages of %d", key_dim,
@@ -664,7 +710,7 @@ static int run_sized_mfma(
 #undef AST_RUN
         return tli_check_launch("attention_sized_shared");
     }
-    const dim3 grid(tiles, (unsigned)gy);
+    const dim3 grid(tiles, (unsigned)gy, (unsigned)splits);
     const size_t bytes = asm_lds_bytes(key_dim, value_dim);
 #define ASM_ARGS (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, row_start, seq_start, num_seqs, tables, \
         table_width, page_size, num_pages, heads, kv_heads, maps, nk, nv, scale, window, keep_first, grouped, col_groups
@@ -683,7 +729,7 @@ static int run_sized_mfma(
                                                    (const bf16_t*)v_cache, row_start, seq_start, num_seqs, tables,         \
                                                    table_width, page_size, num_pages, heads, kv_heads, maps, nk, nv,       \
                                                    scale, window, keep_first, grouped, col_groups, sinks, pooled, out_ld,  \
-                                                   out_scale);                                                             \
+                                                   out_scale, splits > 1 ? parts : nullptr);                                                             \
     }
 #define ASM_SIZES(VKEY, TO)                                                   \
     if (nk <= 8 && nv <= 8) ASM_ONE(8, 8, VKEY, TO, false)                    \
@@ -719,20 +765,30 @@ extern "C" int tli_attention_sized_mfma_bf16(
     const float* sinks, void* stream) {
     return run_sized_mfma(q, out, k_cache, v_cache, row_start, seq_start, num_seqs, tiles, tables, table_width, page_size,
                           num_pages, heads, kv_heads, maps, key_dim, value_dim, scale, window, keep_first, grouped, out_f32, sinks,
-                          PooledKeys{}, heads * maps * value_dim, 1.0f, stream);
+                          PooledKeys{}, heads * maps * value_dim, 1.0f, 1, nullptr, stream);
 }
 
 // The same over a window and the pooled blocks before it (pooled.h; their caches hold kv_heads heads): one map, values of
-// their own, bfloat16 output rows out_ld elements apart (a multiple of 4) and times out_scale.
+// their own, bfloat16 output rows out_ld elements apart (a multiple of 4) and times out_scale.  With `grouped` the keys
+// of a row may be shared out over 2 to 64 splits, whose sums go to `parts` (float32, 16-byte aligned:
+// [rows, heads, splits, value_dim + 4]) and are put together by a second launch; `tiles` is then the number of rows.
 extern "C" int tli_attention_pooled_mfma_bf16(
     const void* q, void* out, const void* k_cache, const void* v_cache, const int* row_start, const int* seq_start,
     int num_seqs, int tiles, const int* tables, int table_width, int page_size, int num_pages, int heads, int kv_heads,
     int key_dim, int value_dim, float scale, int window, const void* pooled_k, const void* pooled_v, const int* pooled_tables,
-    int pooled_width, int pooled_pages, int pool, int grouped, const float* sinks, int out_ld, float out_scale, void* stream) {
+    int pooled_width, int pooled_pages, int pool, int grouped, const float* sinks, int out_ld, float out_scale, int splits,
+    float* parts, void* stream) {
     if (window <= 0 || pool <= 0 || pooled_width <= 0 || pooled_pages <= 0 || !v_cache)
         return tli_fail("attention: blocks of %d beside a window of %d", pool, window);
     if (((uintptr_t)pooled_k | (uintptr_t)pooled_v) & 15) return tli_fail("attention: operands must be 16-byte aligned");
-    return run_sized_mfma(q, out, k_cache, v_cache, row_start, seq_start, num_seqs, tiles, tables, table_width, page_size,
+    if (splits < 1 || splits > 64 || (splits > 1 && (!grouped || !parts || ((uintptr_t)parts & 15))))
+        return tli_fail("attention: %d splits", splits);
+    const int rc = run_sized_mfma(q, out, k_cache, v_cache, row_start, seq_start, num_seqs, tiles, tables, table_width, page_size,
                           num_pages, heads, kv_heads, 1, key_dim, value_dim, scale, window, 0, grouped, 0, sinks,
-                          PooledKeys{pooled_k, pooled_v, pooled_tables, pooled_width, pooled_pages, pool}, out_ld, out_scale, stream);
+                          PooledKeys{pooled_k, pooled_v, pooled_tables, pooled_width, pooled_pages, pool}, out_ld, out_scale, splits, parts, stream);
+    if (rc || splits == 1 || num_seqs <= 0 || tiles <= 0) return rc;
+    const int pairs = tiles * heads;
+    attention_parts_merge_kernel<<<(pairs + 3) / 4, 256, 0, (hipStream_t)stream>>>(parts, splits, pairs, heads, value_dim, sinks,
+                                                                                   (bf16_t*)out, out_ld, out_scale);
+    return tli_check_launch("attention_parts_merge");
 }

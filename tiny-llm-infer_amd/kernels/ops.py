@@ -145,7 +145,7 @@ def load_library():
         "tli_attention_pooled_plain": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
         "tli_pooled_prefill_takes": [I, I, I, I, I, I],
         "tli_pooled_prefill_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
-        "tli_attention_pooled_mfma_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
+        "tli_attention_pooled_mfma_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, I, P, P],
         "tli_sample": [P, I, I, P, P, P, P, P, P],
         "tli_sample_scratch_bytes": [I],
         "tli_random_normal": [P, ctypes.c_longlong, ctypes.c_uint32, ctypes.c_uint32, ctypes.c_uint32, P, F, F, I, P],
@@ -246,6 +246,7 @@ class HipOps:
         self.lightning_lanes = int(os.environ.get("TLI_LIGHTNING_LANES", "0"))   # measurements, tests: 16 or 64 lanes a column of the lightning recurrence's state (0: the launch rule)
         self.rows_splits = 0
         self.pooled_prefill = True       # measurements, tests: False sends portions of prompts over windows and pooled blocks through the kernels for sizes of their own
+        self.pooled_splits = None        # measurements, tests: into how many splits a decoding row's keys over windows and pooled blocks go (None: the rule)
         self.recurrence_in_chunks = True    # measurements, tests: False sends the portions of prompts of retention and mLSTM through the recurrence row by row
 
     @property
@@ -1691,15 +1692,34 @@ class HipOps:
         if (proj.dtype == torch.bfloat16 and not self.force_plain
                 and self.lib.tli_attention_sized_mfma_takes(key_dim, value_dim, g.page_size, 1)):
             tiles = T if single else sum((starts[i + 1] - starts[i] + 15) // 16 for i in range(step.num_seqs))
+            splits, parts = self._pooled_splits(T, step.reach, heads, kv_heads, value_dim, window, pool) if single else (1, None)
             self._call(self.lib.tli_attention_pooled_mfma_bf16, q.data_ptr(), out_ptr, kc.data_ptr(), vc.data_ptr(),
                        step.row_start.data_ptr(), step.seq_start.data_ptr(), step.num_seqs, tiles, g.tables.data_ptr(),
                        g.table_width, g.page_size, kc.shape[0], heads, kv_heads, key_dim, value_dim, float(scale), int(window),
-                       *pooled, single, _ptr(sinks), out_ld, float(out_scale), self._stream())
+                       *pooled, single, _ptr(sinks), out_ld, float(out_scale), splits, _ptr(parts), self._stream())
             return
         self._call(self.lib.tli_attention_pooled_plain, q.data_ptr(), out_ptr, kc.data_ptr(), vc.data_ptr(),
                    step.positions.data_ptr(), step.seq_of_row.data_ptr(), g.tables.data_ptr(), g.table_width, g.page_size,
                    kc.shape[0], T, heads, kv_heads, key_dim, value_dim, float(scale), int(window), *pooled,
                    _dtype_code(proj.dtype), _ptr(sinks), out_ld, float(out_scale), self._stream())
+
+    POOLED_WORKGROUPS = 768          # a split of decoding rows over windows and blocks: the workgroups aimed at,
+    POOLED_SPLIT_KEYS = 128          # and the fewest keys of a split (two rounds of tiles of 16 over four waves)
+
+    def _pooled_splits(self, T, reach, heads, kv_heads, value_dim, window, pool):
+        """Over how many workgroups the keys of one (row, key head) that decodes are shared out, and the room for
+        their sums; ``reach``: a power of two that the longest sequence fits.  A wave's tiles follow one another, each
+        with its wait for memory (3 us), so a split pays for its merge where workgroups are few.  Measured at heads of
+        128 on 8 key heads, 1,060 keys, a whole step of 4 layers (2 of them with this attention): 8 rows in 1, 2, 4, 8
+        splits 0.585, 0.550, 0.532, 0.509 ms, 64 rows in 1, 2, 3, 4 splits 1.046, 1.006, 1.038, 1.009; at 700 keys 64
+        rows 0.972, 0.989 and 0.984 in 1, 2 and 4; below 256 keys the same in 1 and 2."""
+        keys = min(reach, window + 15) + max(0, reach - window) // pool
+        groups = T * kv_heads * ((heads // kv_heads + 15) // 16)
+        most = keys // self.POOLED_SPLIT_KEYS if keys >= 4 * self.POOLED_SPLIT_KEYS else 1
+        splits = self.pooled_splits or min(self.POOLED_WORKGROUPS // groups, most, 64)
+        if splits <= 1:
+            return 1, None
+        return splits, torch.empty((T * heads * splits * (value_dim + 4),), dtype=torch.float32, device=self.device)
 
     # ---- retention, mLSTM --------------------------------------------------------------------------------
     def _recurrent_inputs(self, proj, at, state, shape, step, heads, dk, dv):
