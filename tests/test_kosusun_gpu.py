@@ -251,6 +251,18 @@ def _last_row(q, k, v, window, pool):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_blocks_of_more_sequences_than_a_wave_has_lanes(ops, dtype):
+    g = torch.Generator().manual_seed(8)
+    lengths = [1 + (7 * i) % 23 for i in range(150)]
+    q, k, v = ([torch.randn(n, h, 16, generator=g).to(DTYPES[dtype]) for n in lengths] for h in (2, 1, 1))
+    for cuts in ([30], [3, 9, 2]):
+        got = _attend(ops, q, k, v, 0.25, 5, 3, None, 16, cuts)
+        for i in range(len(lengths)):
+            want = plain_kosusun.windowed_attention(q[i].double(), k[i].double(), v[i].double(), 0.25, 5, 3, None)
+            _close(got[i], want, 1e-5 if dtype == "float32" else 2e-2, f"sequence {i} in portions of {cuts}")
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_a_sink_that_takes_most_of_the_weight(ops, dtype, monkeypatch):
     g = torch.Generator().manual_seed(5)
     dt = DTYPES[dtype]

@@ -12,18 +12,34 @@
 #include "pooled.h"
 
 #define PN_THREADS 512
+#define PB_AHEAD 8             // positions of a block whose loads are under way together
 
 // the mean of element (key: d of kv head g; value likewise) over the block's positions, read from the tokens' pages
 template <typename T, bool VALUE>
 __device__ __forceinline__ float block_mean(const T* __restrict__ cache, const int* __restrict__ table, int page_size, int num_pages,
                                             int kv_heads, int g, int dim, int d, int first, int pool) {
     float sum = 0.f;
-    for (int j = 0; j < pool; ++j) {
-        const int pos = first + j, slot = pos % page_size;
-        const int page = table[pos / page_size];
-        if (page < 0 || page >= num_pages) continue;
-        const size_t head = ((size_t)page * kv_heads + g) * page_size * dim;
-        sum += to_f32(VALUE ? cache[head + (size_t)d * page_size + slot] : cache[head + (size_t)slot * dim + d]);
+    int at = first / page_size, slot = first - at * page_size;
+    for (int j0 = 0; j0 < pool; j0 += PB_AHEAD) {        // every load of eight positions is issued before one is used
+        int page[PB_AHEAD], where[PB_AHEAD];
+        float v[PB_AHEAD];
+#pragma unroll
+        for (int j = 0; j < PB_AHEAD; ++j) {
+            page[j] = table[at];
+            where[j] = slot;
+            if (j0 + j + 1 < pool) ++slot;               // (past the block's end: its last position again, not added)
+            if (slot == page_size) slot = 0, ++at;
+        }
+#pragma unroll
+        for (int j = 0; j < PB_AHEAD; ++j) {
+            const bool have = page[j] >= 0 && page[j] < num_pages;
+            const size_t head = ((size_t)(have ? page[j] : 0) * kv_heads + g) * page_size * dim;
+            v[j] = to_f32(VALUE ? cache[head + (size_t)d * page_size + where[j]] : cache[head + (size_t)where[j] * dim + d]);
+        }
+#pragma unroll
+        for (int j = 0; j < PB_AHEAD; ++j) asm volatile("" : "+v"(v[j]));       // (not loaded under the conditions below)
+#pragma unroll
+        for (int j = 0; j < PB_AHEAD; ++j) sum += page[j] >= 0 && page[j] < num_pages && j0 + j < pool ? v[j] : 0.f;
     }
     return sum / (float)pool;
 }
@@ -320,17 +336,33 @@ __global__ __launch_bounds__(PB_THREADS) void pool_blocks_kernel(
     const T* __restrict__ k_cache, const T* __restrict__ v_cache, const int* __restrict__ row_start,
     const int* __restrict__ seq_start, int num_seqs, const int* __restrict__ tables, int table_width, int page_size, int num_pages,
     int kv_heads, int key_dim, int value_dim, PooledKeys pooled) {
-    int block = blockIdx.x, seq = 0;
-    for (; seq < num_seqs; ++seq) {
-        const int start = seq_start[seq], end = start + row_start[seq + 1] - row_start[seq];
-        const int first = start / pooled.pool, count = end / pooled.pool - first;      // blocks that end within the step
-        if (block < count) {
-            block += first;
-            break;
+    // which sequence's: 64 sequences at a time, a lane each
+    const int lane = threadIdx.x % 64;
+    int block = blockIdx.x, seq = -1;
+    for (int base = 0; base < num_seqs && seq < 0; base += 64) {
+        int first = 0, count = 0;
+        if (base + lane < num_seqs) {
+            const int start = seq_start[base + lane], end = start + row_start[base + lane + 1] - row_start[base + lane];
+            first = start / pooled.pool;
+            count = end / pooled.pool - first;           // blocks that end within the step
         }
-        block -= count;
+        int upto = count;
+        for (int off = 1; off < 64; off *= 2) {
+            const int before = __shfl_up(upto, off);
+            if (lane >= off) upto += before;
+        }
+        const unsigned long long beyond = __ballot(block < upto);
+        if (beyond) {
+            const int at = __ffsll(beyond) - 1;
+            block += __shfl(first - (upto - count), at);
+            seq = base + at;
+        } else {
+            block -= __shfl(upto, 63);
+        }
     }
-    if (seq >= num_seqs) return;                         // (the grid's slack)
+    if (seq < 0) return;                                 // (the grid's slack)
+    seq = __builtin_amdgcn_readfirstlane(seq);
+    block = __builtin_amdgcn_readfirstlane(block);
     for (int e = threadIdx.x; e < key_dim + value_dim; e += blockDim.x)
         store_block_mean<T>(k_cache, v_cache, tables + (size_t)seq * table_width, page_size, num_pages, kv_heads, key_dim, value_dim,
                             blockIdx.y, e, block, pooled, pooled.tables + (size_t)seq * pooled.width);
