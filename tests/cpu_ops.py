@@ -31,19 +31,24 @@ class CpuOps:
         return cap * torch.tanh(logits / cap)
 
     def check_activation(self, name):
-        assert name in ("relu2", "relu", "silu", "gelu_tanh")
+        assert name in ("relu2", "relu", "silu", "gelu_tanh", "gelu")
 
     def activation(self, x, name):
-        z = x.to(torch.float32)
+        return self._act(x.to(torch.float32), name).to(x.dtype)
+
+    @staticmethod
+    def _act(z, name):
         if name == "relu2":
             y = torch.relu(z) ** 2
         elif name == "relu":
             y = torch.relu(z)
         elif name == "silu":
             y = z / (1 + torch.exp(-z))
+        elif name == "gelu":
+            y = 0.5 * z * (1 + torch.erf(z * 0.7071067811865476))
         else:
             y = 0.5 * z * (1 + torch.tanh(0.7978845608028654 * (z + 0.044715 * z ** 3)))
-        return y.to(x.dtype)
+        return y
 
     # ---- several residual streams ------------------------------------------------
     def check_streams(self, streams, width):
@@ -206,7 +211,7 @@ class CpuOps:
     def check_expert_sizes(self, experts, top, groups, keep, hidden, inter):
         pass
 
-    def pack_experts(self, w_gate_up, w_down):
+    def pack_experts(self, w_gate_up, w_down, gated=True):
         return None
 
     def check_router(self, score, group_score):
@@ -230,7 +235,8 @@ class CpuOps:
         w = w / (w.sum(-1, keepdim=True) + 1e-20) * scale if normalize else w * scale
         return ids.to(torch.int32), w, (torch.sigmoid(z[:, experts]) if has_shared else None)
 
-    def apply_experts(self, x, ids, weights, w_gate_up, w_down, packed, shared, shared_gate, limit=0.0, slope=1.0):
+    def apply_experts(self, x, ids, weights, w_gate_up, w_down, packed, shared, shared_gate, limit=0.0, slope=1.0,
+                      activation=None, weight_on_input=False):
         T, n = x.shape
         E = w_gate_up.shape[0]
         ff = w_gate_up.shape[1] // 2
@@ -243,6 +249,10 @@ class CpuOps:
                     out[t] += weights[t, j] * xf[t]
                     continue
                 gu = w_gate_up[e].to(torch.float32) @ xf[t]
+                if activation is not None:
+                    a = self._act(gu * (weights[t, j] if weight_on_input else 1.0), activation).to(x.dtype).to(torch.float32)
+                    out[t] += (1.0 if weight_on_input else weights[t, j]) * (w_down[e].to(torch.float32) @ a)
+                    continue
                 a = self._gated(gu[:ff], gu[ff:], limit, slope).to(x.dtype).to(torch.float32)
                 out[t] += weights[t, j] * (w_down[e].to(torch.float32) @ a)
         if shared is not None:
@@ -257,6 +267,67 @@ class CpuOps:
         yf = y.to(torch.float32)
         resid += weight * yf * torch.rsqrt((yf * yf).mean(dim=-1, keepdim=True) + eps)
         return resid if out_dtype == torch.float32 else resid.to(out_dtype)
+
+    def norm_add_norm(self, resid, y, w_out, eps_out, w_in, eps_in, out_dtype, rows=None, num_rows=None):
+        x = resid
+        if y is not None:
+            yf = y.to(torch.float32)
+            x = resid + w_out * yf * torch.rsqrt((yf * yf).mean(dim=-1, keepdim=True) + eps_out)
+            if rows is None:
+                resid.copy_(x)
+        if rows is not None:
+            x = x[rows[:num_rows].long()]
+        return (w_in * x * torch.rsqrt((x * x).mean(dim=-1, keepdim=True) + eps_in)).to(out_dtype)
+
+    def norm_add_norm_mixes(self, resid, y, w_out, eps_out, w_in, eps_in, out_dtype, mixes, step):
+        if step.max_rows_per_seq != 1 or step.num_seqs != step.num_rows:
+            return None
+        h = self.norm_add_norm(resid, y, w_out, eps_out, w_in, eps_in, out_dtype)
+        return self.token_mixes(h, mixes[0], mixes[1], step)
+
+    def token_mixes(self, h, mu, kept, step):
+        out = torch.empty((mu.shape[0],) + tuple(h.shape), dtype=h.dtype)
+        hf = h.to(torch.float32)
+        for i in range(step.num_seqs):
+            r0, r1 = step.h_row_start[i], step.h_row_start[i + 1]
+            slot = step.h_slots[i]
+            first = kept[slot].to(torch.float32) if step.h_seq_start[i] > 0 else torch.zeros(h.shape[1])
+            prev = torch.cat([first[None], hf[r0:r1 - 1]], dim=0)
+            for m in range(mu.shape[0]):
+                out[m, r0:r1] = (hf[r0:r1] + (prev - hf[r0:r1]) * mu[m]).to(h.dtype)
+            kept[slot] = h[r1 - 1]
+        return out
+
+    def token_gate(self, z, table, at, token_ids, activation):
+        own = table[token_ids[:z.shape[0]].long(), at:at + z.shape[1]].to(torch.float32)
+        return (self._act(z.to(torch.float32), activation) * own).to(z.dtype)
+
+    def check_wkv_sizes(self, heads, dk, dv, rank):
+        pass
+
+    def wkv_state_shape(self, heads, dk, dv):
+        return (heads, dv, dk)
+
+    def linear_groups(self, xs, groups):
+        return (torch.cat([self.linear(x, m) for x, m in zip(xs, groups.each)], dim=1),) + self.small_product(xs[len(groups.each)], groups.few)
+
+    def wkv(self, proj, z, transposed, w2, w0, u, state, step, heads, dk, dv, weight, eps, out_dtype):
+        T = step.num_rows
+        r, k, v = self._qkv_heads(proj, 0, heads, dk, dv)
+        z = z.t() if transposed else z
+        d = torch.exp(-torch.exp(torch.tanh(z) @ w2.to(torch.float32).t() + w0)).reshape(T, heads, dk)
+        o = torch.zeros(T, heads, dv)
+        for i in range(step.num_seqs):
+            slot = step.h_slots[i]
+            S = state[slot].clone() if step.h_seq_start[i] > 0 else torch.zeros(heads, dv, dk)
+            for t in range(step.h_row_start[i], step.h_row_start[i + 1]):
+                kv = v[t][:, :, None] * k[t][:, None, :]
+                o[t] = torch.einsum("hvk,hk->hv", S + u[:, None, :] * kv, r[t])
+                S = d[t][:, None, :] * S + kv
+            state[slot] = S
+        out = torch.empty(T, heads * dv, dtype=out_dtype)
+        self.head_norm_gate(o, None, weight, proj, 2 * heads * dk + heads * dv, heads, dv, eps, "silu", 1.0, out, 0)
+        return out
 
     def check_sized_attention(self, heads, kv_heads, key_dim, value_dim):
         pass
@@ -303,10 +374,13 @@ class CpuOps:
                 out[r, h] = o * torch.rsqrt((o * o).mean() + norm_eps) * after * gate[r, h]
         return out.reshape(T, heads * vdim).to(proj.dtype)
 
-    def latent_attention(self, proj, step, cache, heads, dim, rot, rank, vdim, norm_weight, norm_eps, rotary, scale,
-                         w_qk, w_v, sinks=None):
+    def norm_rows(self, proj, at, n, weight, eps):
+        x = proj[:, at:at + n].to(torch.float32)
+        return (weight * x * torch.rsqrt((x * x).mean(dim=-1, keepdim=True) + eps)).to(proj.dtype)
+
+    def latent_attention(self, query, q_at, own, step, cache, heads, dim, rot, rank, vdim, rotary, scale, w_qk, w_v, window=None,
+                         sinks=None, gate=None):
         T = step.num_rows
-        x = proj.to(torch.float32)
         cos, sin, rd = rotary
         half = rd // 2
         pos, seq = step.positions.long(), step.seq_of_row.long()
@@ -314,21 +388,24 @@ class CpuOps:
         def turn(t, c, s):
             a, b, rest = t[..., :half], t[..., half:rd], t[..., rd:]
             return torch.cat([a * c - b * s, b * c + a * s, rest], dim=-1)
-        q = x[:, :heads * (dim + rot)].reshape(T, heads, dim + rot)
-        down = x[:, heads * (dim + rot):]
-        c = down[:, :rank]
-        c = norm_weight * c * torch.rsqrt((c * c).mean(dim=-1, keepdim=True) + norm_eps)
-        entry = torch.cat([c, turn(down[:, rank:], cos[pos], sin[pos])], dim=-1)
+        q = query[:, q_at:q_at + heads * (dim + rot)].to(torch.float32).reshape(T, heads, dim + rot)
         page, tables = cache.group.page_size, cache.group.tables
-        pages = tables[seq, pos // page].long()
-        assert (pages >= 0).all(), "a row writes to a page that is not held"
         kc = cache.record("latent")
-        kc[pages, pos % page] = entry.to(kc.dtype)
-        q_lat = torch.einsum("thd,hnd->thn", q[..., :dim].to(proj.dtype).to(torch.float32), w_qk.to(torch.float32))
-        qk = torch.cat([q_lat, turn(q[..., dim:], cos[pos][:, None], sin[pos][:, None])], dim=-1).to(proj.dtype).to(torch.float32)
+        assert cache.writes == (own is not None)
+        if own is not None:
+            proj, at, norm_weight, norm_eps = own
+            down = proj[:, at:at + rank + rot].to(torch.float32)
+            c = down[:, :rank]
+            c = norm_weight * c * torch.rsqrt((c * c).mean(dim=-1, keepdim=True) + norm_eps)
+            entry = torch.cat([c, turn(down[:, rank:], cos[pos], sin[pos])], dim=-1)
+            pages = tables[seq, pos // page].long()
+            assert (pages >= 0).all(), "a row writes to a page that is not held"
+            kc[pages, pos % page] = entry.to(kc.dtype)
+        q_lat = torch.einsum("thd,hnd->thn", q[..., :dim], w_qk.to(torch.float32))
+        qk = torch.cat([q_lat, turn(q[..., dim:], cos[pos][:, None], sin[pos][:, None])], dim=-1).to(query.dtype).to(torch.float32)
         o = torch.zeros(T, heads, rank)
         for r in range(T):
-            idx = torch.arange(0, int(pos[r]) + 1)
+            idx = self._seen(int(pos[r]), window, 0)
             pg = tables[int(seq[r]), idx // page].long()
             assert (pg >= 0).all(), "a row reads a page that is not held"
             kk = kc[pg, idx % page].to(torch.float32)               # [n, rank + rot]
@@ -337,8 +414,12 @@ class CpuOps:
                 sc = torch.cat([sc, sinks[:, None]], dim=-1)
             w = torch.softmax(sc, dim=-1)[:, :len(idx)]
             o[r] = w @ kk[:, :rank]
-        o = o.to(proj.dtype).to(torch.float32)
-        return torch.einsum("thn,hen->the", o, w_v.to(torch.float32)).reshape(T, heads * vdim).to(proj.dtype)
+        o = o.to(query.dtype).to(torch.float32)
+        out = torch.einsum("thn,hen->the", o, w_v.to(torch.float32))
+        if gate is not None:
+            z, z_at = gate
+            out = out * torch.sigmoid(z[:, z_at:z_at + heads].to(torch.float32))[..., None]
+        return out.reshape(T, heads * vdim).to(query.dtype)
 
     def add_rmsnorm(self, resid, delta, weight, eps, out_dtype, rows=None, num_rows=None, lazy=False):
         if rows is None:

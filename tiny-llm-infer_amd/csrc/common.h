@@ -84,6 +84,28 @@ __device__ __forceinline__ float gated_unit(float g, float u, float limit, float
     return g / (1.0f + expf(-slope * g)) * (u + 1.0f);
 }
 
+// Activations of a feed-forward without a gate, element by element in float32:
+// 0 relu(z)^2, 1 relu(z), 2 z / (1 + exp(-z)), 3 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), 4 0.5 z (1 + erf(z / sqrt(2)))
+#define TLI_ACT_KINDS 5
+__device__ __forceinline__ float act_of(float z, int kind) {
+    switch (kind) {
+        case 0: { const float r = fmaxf(z, 0.f); return r * r; }
+        case 1: return fmaxf(z, 0.f);
+        case 2: return z / (1.0f + expf(-z));
+        case 3: return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+        default: return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
+    }
+}
+
+// What the hidden units of a routed expert are made of its sums.  kind < 0: gate and up matrices, gated_unit.  Else an up
+// matrix alone: act_of(w u, kind), w the pair's weight where it belongs on the expert's input (W (w x) = w (W x)), or 1.
+struct ExpertUnit {
+    int kind;
+    float limit, slope;
+    const float* weights;        // of the pairs, or null
+    __device__ __forceinline__ float of_pair(int pair) const { return weights ? weights[pair] : 1.0f; }
+};
+
 // The output of a gated product: act(g) * u * scale from the sums g and u of a gate row and an up row, act the silu
 // (`act` 0) or the tanh form of gelu (1), rows `ld` elements apart.  (tanh form: 0.5 z (1 + tanh(t / 2)) with
 // t = 2 sqrt(2 / pi) (z + 0.044715 z^3), which is z / (1 + exp(-t)); silu is the same with t = z.)

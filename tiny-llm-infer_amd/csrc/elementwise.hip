@@ -354,18 +354,6 @@ extern "C" int tli_embed_scaled(const void* table, const int* ids, const void* p
     return tli_check_launch("embed_scaled");
 }
 
-// Activations of a feed-forward without a gate, element by element in float32:
-// 0 relu(z)^2, 1 relu(z), 2 z / (1 + exp(-z)), 3 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))
-#define TLI_ACT_KINDS 4
-__device__ __forceinline__ float act_of(float z, int kind) {
-    switch (kind) {
-        case 0: { const float r = fmaxf(z, 0.f); return r * r; }
-        case 1: return fmaxf(z, 0.f);
-        case 2: return z / (1.0f + expf(-z));
-        default: return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-    }
-}
-
 template <typename T>
 __global__ void activation_kernel(const T* __restrict__ x, T* __restrict__ out, size_t total, int kind) {
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -412,7 +400,8 @@ extern "C" int tli_activation(const void* x, void* out, long long total, int kin
             case 0: activation_vec_kernel<0><<<blocks, 256, 0, s>>>(xi, xo, groups); break;
             case 1: activation_vec_kernel<1><<<blocks, 256, 0, s>>>(xi, xo, groups); break;
             case 2: activation_vec_kernel<2><<<blocks, 256, 0, s>>>(xi, xo, groups); break;
-            default: activation_vec_kernel<3><<<blocks, 256, 0, s>>>(xi, xo, groups); break;
+            case 3: activation_vec_kernel<3><<<blocks, 256, 0, s>>>(xi, xo, groups); break;
+            default: activation_vec_kernel<4><<<blocks, 256, 0, s>>>(xi, xo, groups); break;
         }
     }
     else if (dtype == TLI_BF16)
@@ -433,4 +422,35 @@ extern "C" int tli_softcap(float* z, long long total, float cap, void* stream) {
     if (!(cap > 0.f)) return tli_fail("softcap: the cap must be positive");
     softcap_kernel<<<(unsigned)(((size_t)total + 255) / 256), 256, 0, (hipStream_t)stream>>>(z, (size_t)total, cap);
     return tli_check_launch("softcap");
+}
+
+// What a token's own vector is multiplied by:  out[t, i] = act(z[t, i]) * table[id[t], at + i], i < dim, in float32 and
+// rounded once.  A workgroup takes 256 elements.
+template <typename T>
+__global__ void token_gate_kernel(const T* __restrict__ z, const T* __restrict__ table, const int* __restrict__ ids,
+                                  T* __restrict__ out, size_t total, int dim, int width, int at, int vocab, int kind) {
+    const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= total) return;
+    const size_t row = idx / dim;
+    const int i = (int)(idx % dim);
+    int id = ids[row];
+    if (id < 0 || id >= vocab) id = 0;          // the host rejects such ids before the launch
+    from_f32(out + idx, act_of(to_f32(z[idx]), kind) * to_f32(table[(size_t)id * width + at + i]));
+}
+
+extern "C" int tli_token_gate(const void* z, const void* table, const int* ids, void* out, int rows, int dim, int width, int at,
+                              int vocab, int kind, int dtype, void* stream) {
+    if (rows <= 0) return 0;
+    if (dim <= 0 || at < 0 || at + dim > width || vocab <= 0) return tli_fail("token_gate: bad sizes");
+    if (kind < 0 || kind >= TLI_ACT_KINDS) return tli_fail("token_gate: unknown activation %d", kind);
+    hipStream_t s = (hipStream_t)stream;
+    const size_t n = (size_t)rows * dim;
+    const unsigned blocks = (unsigned)((n + 255) / 256);
+    if (dtype == TLI_F32)
+        token_gate_kernel<float><<<blocks, 256, 0, s>>>((const float*)z, (const float*)table, ids, (float*)out, n, dim, width, at, vocab, kind);
+    else if (dtype == TLI_BF16)
+        token_gate_kernel<bf16_t><<<blocks, 256, 0, s>>>((const bf16_t*)z, (const bf16_t*)table, ids, (bf16_t*)out, n, dim, width, at, vocab, kind);
+    else
+        return tli_fail("token_gate: unknown dtype %d", dtype);
+    return tli_check_launch("token_gate");
 }

@@ -1,26 +1,36 @@
 // Attention over a latent vector a position: what stands before and behind the attention itself.
 //
-// prepare:        from the raw projections of a row (q of `heads` heads of dim + rot elements, then the latent
+// prepare:        from the raw projections of a row (q of `heads` heads of dim + rot elements; the latent
 //                 vector of `rank` elements and one key part of `rot` elements) the cache entry of the position,
 //                 [RMS norm of the latent vector with its weight | the key part, turned], and the queries' own
 //                 turned parts, written behind the place where their `rank` elements in the latent space go.
 //                 The first rot_dims elements of a part are turned in pairs (i, i + rot_dims / 2).  One workgroup
-//                 a row; float32 arithmetic.
+//                 a row; float32 arithmetic.  Without a latent vector (a layer that reads another's) the queries only.
 // head_products:  y[t, h, :] = W[h] x[t, h, :] for a matrix a head (float32 sums), with strides so that inputs
-//                 and outputs may lie inside wider rows.  Plain: any sizes and both types.
+//                 and outputs may lie inside wider rows; times sigmoid(gate[t, h]) where gates are given.  Plain: any
+//                 sizes and both types.
 #include "common.h"
 
 #define LP_THREADS 256
 
+// One number a row and head that the head's output is multiplied by: the logistic function of logits that lie `ld`
+// elements a row apart, or 1 without them.
+template <typename T>
+struct HeadGate {
+    const T* z;
+    int ld;
+    __device__ __forceinline__ float of(int t, int h) const { return z ? 1.0f / (1.0f + expf(-to_f32(z[(size_t)t * ld + h]))) : 1.0f; }
+};
+
 template <typename T>
 __global__ __launch_bounds__(LP_THREADS) void latent_prepare_kernel(
-    const T* __restrict__ proj, int ld, T* __restrict__ q_out, T* __restrict__ cache, const int* __restrict__ positions,
+    const T* __restrict__ q_in, int q_ld, const T* __restrict__ down_in, int down_ld, T* __restrict__ q_out, T* __restrict__ cache, const int* __restrict__ positions,
     const int* __restrict__ seq_of_row, const int* __restrict__ tables, int table_width, int page_size, int num_pages,
     int heads, int dim, int rot, int rank, int rot_dims, const float* __restrict__ norm_weight, float eps,
     const float* __restrict__ cos_t, const float* __restrict__ sin_t) {
     __shared__ float red[16];
     const int row = blockIdx.x, tid = threadIdx.x;
-    const T* src = proj + (size_t)row * ld;
+    const T* src = q_in + (size_t)row * q_ld;
     const int pos = positions[row];
     const int half = rot_dims / 2;
     const float* cs = cos_t + (size_t)pos * half;
@@ -35,8 +45,9 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prepare_kernel(
         else if (d < rot_dims) v = rotate_second_half(v, to_f32(part[d - half]), cs[d - half], sn[d - half]);
         from_f32(q_out + ((size_t)row * heads + h) * key + rank + d, v);
     }
+    if (!down_in) return;
     const int page = tables[(size_t)seq_of_row[row] * table_width + pos / page_size];
-    const T* down = src + (size_t)heads * (dim + rot);
+    const T* down = down_in + (size_t)row * down_ld;
     float ssq = 0.f;
     for (int d = tid; d < rank; d += LP_THREADS) {
         const float a = to_f32(down[d]);
@@ -64,7 +75,7 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prepare_kernel(
 template <typename T>
 __global__ __launch_bounds__(256) void head_products_plain_kernel(const T* __restrict__ x, long long x_row, long long x_head,
                                                                   const T* __restrict__ w, T* __restrict__ y, long long y_row,
-                                                                  long long y_head, int N, int K) {
+                                                                  long long y_head, int N, int K, HeadGate<T> gate) {
     extern __shared__ float xs[];
     const int t = blockIdx.x, h = blockIdx.y;
     const T* xr = x + (size_t)t * x_row + (size_t)h * x_head;
@@ -76,28 +87,29 @@ __global__ __launch_bounds__(256) void head_products_plain_kernel(const T* __res
         float a = 0.f;
         for (int k = lane; k < K; k += TLI_WAVE) a = fmaf(xs[k], to_f32(wr[k]), a);
         a = wave_sum(a);
-        if (lane == 0) from_f32(y + (size_t)t * y_row + (size_t)h * y_head + n, a);
+        if (lane == 0) from_f32(y + (size_t)t * y_row + (size_t)h * y_head + n, a * gate.of(t, h));
     }
 }
 
-// proj [rows, ld]: q (heads * (dim + rot)) | latent (rank) | key part (rot);  q_out [rows, heads, rank + rot] (only
+// q_in: rows q_ld elements apart, heads * (dim + rot) of each;  down_in: rows down_ld apart, latent (rank) | key part (rot),
+// or null;  q_out [rows, heads, rank + rot] (only
 // the last rot of every head are written);  cache [pages][slot][rank + rot];  cos_t, sin_t [positions, rot_dims / 2]
-extern "C" int tli_latent_prepare(const void* proj, int ld, void* q_out, void* cache, const int* positions,
+extern "C" int tli_latent_prepare(const void* q_in, int q_ld, const void* down_in, int down_ld, void* q_out, void* cache, const int* positions,
                                   const int* seq_of_row, const int* tables, int table_width, int page_size, int num_pages,
                                   int rows, int heads, int dim, int rot, int rank, int rot_dims, const float* norm_weight,
                                   float eps, const float* cos_t, const float* sin_t, int dtype, void* stream) {
     if (rows <= 0) return 0;
     if (heads <= 0 || dim <= 0 || rot <= 0 || rank <= 0 || rot_dims <= 0 || rot_dims % 2 || rot_dims > rot ||
-        ld < heads * (dim + rot) + rank + rot)
+        !q_in || q_ld < heads * (dim + rot) || (down_in && (down_ld < rank + rot || !norm_weight)))
         return tli_fail("latent_prepare: bad sizes");
     if (page_size <= 0 || table_width <= 0 || num_pages <= 0) return tli_fail("latent_prepare: bad cache geometry");
     hipStream_t s = (hipStream_t)stream;
     if (dtype == TLI_F32)
-        latent_prepare_kernel<float><<<rows, LP_THREADS, 0, s>>>((const float*)proj, ld, (float*)q_out, (float*)cache, positions,
+        latent_prepare_kernel<float><<<rows, LP_THREADS, 0, s>>>((const float*)q_in, q_ld, (const float*)down_in, down_ld, (float*)q_out, (float*)cache, positions,
                                                                  seq_of_row, tables, table_width, page_size, num_pages, heads, dim,
                                                                  rot, rank, rot_dims, norm_weight, eps, cos_t, sin_t);
     else if (dtype == TLI_BF16)
-        latent_prepare_kernel<bf16_t><<<rows, LP_THREADS, 0, s>>>((const bf16_t*)proj, ld, (bf16_t*)q_out, (bf16_t*)cache, positions,
+        latent_prepare_kernel<bf16_t><<<rows, LP_THREADS, 0, s>>>((const bf16_t*)q_in, q_ld, (const bf16_t*)down_in, down_ld, (bf16_t*)q_out, (bf16_t*)cache, positions,
                                                                   seq_of_row, tables, table_width, page_size, num_pages, heads, dim,
                                                                   rot, rank, rot_dims, norm_weight, eps, cos_t, sin_t);
     else
@@ -105,19 +117,20 @@ extern "C" int tli_latent_prepare(const void* proj, int ld, void* q_out, void* c
     return tli_check_launch("latent_prepare");
 }
 
-// y[t, h, n] = sum_k x[t, h, k] w[h, n, k];  x at x + t * x_row + h * x_head (elements), y likewise;  w [heads, N, K]
+// y[t, h, n] = sum_k x[t, h, k] w[h, n, k] (times sigmoid(gate[t * gate_ld + h]), if given);  x at x + t * x_row + h * x_head (elements), y likewise;  w [heads, N, K]
 extern "C" int tli_head_products_plain(const void* x, long long x_row, long long x_head, const void* w, void* y, long long y_row,
-                                       long long y_head, int rows, int heads, int N, int K, int dtype, void* stream) {
+                                       long long y_head, int rows, int heads, int N, int K, const void* gate, int gate_ld,
+                                       int dtype, void* stream) {
     if (rows <= 0) return 0;
     if (heads <= 0 || heads > 65535 || N <= 0 || K <= 0 || K > 12288) return tli_fail("head_products: bad sizes");
     hipStream_t s = (hipStream_t)stream;
     const dim3 grid(rows, heads);
     if (dtype == TLI_F32)
         head_products_plain_kernel<float><<<grid, 256, (size_t)K * 4, s>>>((const float*)x, x_row, x_head, (const float*)w, (float*)y,
-                                                                           y_row, y_head, N, K);
+                                                                           y_row, y_head, N, K, HeadGate<float>{(const float*)gate, gate_ld});
     else if (dtype == TLI_BF16)
         head_products_plain_kernel<bf16_t><<<grid, 256, (size_t)K * 4, s>>>((const bf16_t*)x, x_row, x_head, (const bf16_t*)w, (bf16_t*)y,
-                                                                            y_row, y_head, N, K);
+                                                                            y_row, y_head, N, K, HeadGate<bf16_t>{(const bf16_t*)gate, gate_ld});
     else
         return tli_fail("head_products: unknown dtype %d", dtype);
     return tli_check_launch("head_products_plain");
@@ -143,7 +156,7 @@ union HpFrag {
 template <int KM, bool EXACT, int RT>
 __global__ __launch_bounds__(256) void head_products_mfma_kernel(const bf16_t* __restrict__ x, long long x_row, long long x_head,
                                                                  const bf16_t* __restrict__ w, bf16_t* __restrict__ y,
-                                                                 long long y_row, long long y_head, int T, int N, int K) {
+                                                                 long long y_row, long long y_head, int T, int N, int K, HeadGate<bf16_t> gate) {
     const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
     const int col = lane % 16, grp = lane / 16;
     const int t0 = (blockIdx.x * 4 + wave) * 16 * RT, h = blockIdx.y;
@@ -160,6 +173,9 @@ __global__ __launch_bounds__(256) void head_products_mfma_kernel(const bf16_t* _
             if (j < nk) xf[r][j].u = *reinterpret_cast<const uint2*>(xr + j * 16 + grp * 4);
         }
     }
+    float by[RT];
+#pragma unroll
+    for (int r = 0; r < RT; ++r) by[r] = gate.of(min(t0 + r * 16 + col, T - 1), h);
     // (few rows: the blocks of outputs are shared out over blockIdx.z, an even number each)
     const int per_z = (((N / 16 + gridDim.z - 1) / gridDim.z) + 1) & ~1;
     const int nblocks = min(N / 16, (int)(blockIdx.z + 1) * per_z);
@@ -189,12 +205,12 @@ __global__ __launch_bounds__(256) void head_products_mfma_kernel(const bf16_t* _
             if (t < T) {
                 bf16_t* yr = y + (size_t)t * y_row + (size_t)h * y_head + grp * 4 + nb * 16;
                 uint2 st;
-                st.x = pack_bf16x2(acc0[r][0], acc0[r][1]);
-                st.y = pack_bf16x2(acc0[r][2], acc0[r][3]);
+                st.x = pack_bf16x2(acc0[r][0] * by[r], acc0[r][1] * by[r]);
+                st.y = pack_bf16x2(acc0[r][2] * by[r], acc0[r][3] * by[r]);
                 *reinterpret_cast<uint2*>(yr) = st;
                 if (two) {
-                    st.x = pack_bf16x2(acc1[r][0], acc1[r][1]);
-                    st.y = pack_bf16x2(acc1[r][2], acc1[r][3]);
+                    st.x = pack_bf16x2(acc1[r][0] * by[r], acc1[r][1] * by[r]);
+                    st.y = pack_bf16x2(acc1[r][2] * by[r], acc1[r][3] * by[r]);
                     *reinterpret_cast<uint2*>(yr + 16) = st;
                 }
             }
@@ -210,7 +226,7 @@ __global__ __launch_bounds__(256) void head_products_mfma_kernel(const bf16_t* _
 template <int KM, int RT>
 __global__ __launch_bounds__(256) void head_products_lds_kernel(const bf16_t* __restrict__ x, long long x_row, long long x_head,
                                                                 const bf16_t* __restrict__ w, bf16_t* __restrict__ y,
-                                                                long long y_row, long long y_head, int T, int N) {
+                                                                long long y_row, long long y_head, int T, int N, HeadGate<bf16_t> gate) {
     constexpr int K = KM * 16, LDW = K + 8, NB = 32 / KM, ROWS = NB * 16, PIECES = K / 8;
     __shared__ __align__(16) bf16_t wt[2][ROWS * LDW];
     const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64;
@@ -224,6 +240,9 @@ __global__ __launch_bounds__(256) void head_products_lds_kernel(const bf16_t* __
 #pragma unroll
         for (int j = 0; j < KM; ++j) xf[r][j].u = *reinterpret_cast<const uint2*>(xr + j * 16 + grp * 4);
     }
+    float by[RT];
+#pragma unroll
+    for (int r = 0; r < RT; ++r) by[r] = gate.of(min(t0 + r * 16 + col, T - 1), h);
     const bf16_t* wh = w + (size_t)h * N * K;
     const int chunks = (N + ROWS - 1) / ROWS;
     uint4 next[4];                                                      // ROWS * PIECES = 1024 pieces of 16 bytes a chunk
@@ -275,8 +294,8 @@ __global__ __launch_bounds__(256) void head_products_lds_kernel(const bf16_t* __
                     const int t = t0 + r * 16 + col;
                     if (t < T) {
                         uint2 st;
-                        st.x = pack_bf16x2(even[r][0] + odd[r][0], even[r][1] + odd[r][1]);
-                        st.y = pack_bf16x2(even[r][2] + odd[r][2], even[r][3] + odd[r][3]);
+                        st.x = pack_bf16x2((even[r][0] + odd[r][0]) * by[r], (even[r][1] + odd[r][1]) * by[r]);
+                        st.y = pack_bf16x2((even[r][2] + odd[r][2]) * by[r], (even[r][3] + odd[r][3]) * by[r]);
                         *reinterpret_cast<uint2*>(y + (size_t)t * y_row + (size_t)h * y_head + n0 + grp * 4) = st;
                     }
                 }
@@ -293,17 +312,19 @@ extern "C" int tli_head_products_mfma_takes(int N, int K, long long x_row, long 
 }
 
 extern "C" int tli_head_products_mfma_bf16(const void* x, long long x_row, long long x_head, const void* w, void* y,
-                                           long long y_row, long long y_head, int rows, int heads, int N, int K, void* stream) {
+                                           long long y_row, long long y_head, int rows, int heads, int N, int K,
+                                           const void* gate_z, int gate_ld, void* stream) {
     if (rows <= 0) return 0;
     if (heads <= 0 || heads > 65535 || !tli_head_products_mfma_takes(N, K, x_row, x_head, y_row, y_head))
         return tli_fail("head_products: the matrix-core kernel takes sizes in sixteens (k up to 640), not %d x %d", N, K);
     if ((((uintptr_t)x | (uintptr_t)w | (uintptr_t)y) & 7)) return tli_fail("head_products: operands must be 8-byte aligned");
+    const HeadGate<bf16_t> gate{(const bf16_t*)gate_z, gate_ld};
     if (rows >= 1024 && (K == 64 || K == 128 || K == 256 || K == 512)) {
         const dim3 lgrid((rows + 127) / 128, heads);
         hipStream_t ls = (hipStream_t)stream;
 #define HP_LDS(KM)                                                                                                       \
     head_products_lds_kernel<KM, 2><<<lgrid, 256, 0, ls>>>((const bf16_t*)x, x_row, x_head, (const bf16_t*)w, (bf16_t*)y, \
-                                                           y_row, y_head, rows, N)
+                                                           y_row, y_head, rows, N, gate)
         if (K == 64) HP_LDS(4);
         else if (K == 128) HP_LDS(8);
         else if (K == 256) HP_LDS(16);
@@ -320,7 +341,7 @@ extern "C" int tli_head_products_mfma_bf16(const void* x, long long x_row, long 
     hipStream_t s = (hipStream_t)stream;
 #define HP_ONE(KM, EXACT, RT)                                                                                              \
     head_products_mfma_kernel<KM, EXACT, RT><<<grid, 256, 0, s>>>((const bf16_t*)x, x_row, x_head, (const bf16_t*)w, (bf16_t*)y, \
-                                                                  y_row, y_head, rows, N, K)
+                                                                  y_row, y_head, rows, N, K, gate)
     if (K == 64) { if (rt == 4) HP_ONE(4, true, 4); else HP_ONE(4, true, 1); }
     else if (K == 128) { if (rt == 4) HP_ONE(8, true, 4); else HP_ONE(8, true, 1); }
     else if (K == 256) { if (rt == 2) HP_ONE(16, true, 2); else HP_ONE(16, true, 1); }

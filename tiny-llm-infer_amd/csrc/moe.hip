@@ -10,7 +10,8 @@
 //          a shared expert: sigmoid of it.  Ids from `experts` on (see the kernels below) are experts that
 //          hand their input on: they have no matrices.
 // hidden:  for the pair (row, chosen expert e): a_f = silu(x . Wg_e[f]) * (x . Wu_e[f]), or the limited form of
-//          common.h's gated_unit (limit > 0)
+//          common.h's gated_unit (limit > 0); or, of experts without a gate, a_f = act(x . Wu_e[f]), the weight
+//          multiplied in before the activation where it belongs on the expert's input (common.h's ExpertUnit)
 // down:    y_c = sum_j weight_j (a_j . Wd_e(j)[c])  (+ shared gate * shared_c), summed in the order of
 //          the choice, so that a row's result does not depend on what else is in the step.
 //
@@ -92,7 +93,7 @@ __global__ void moe_route_kernel(const float* __restrict__ z, long long z_row, l
 // one workgroup a pair; a wave takes every (waves)th hidden unit, its lanes share out k
 template <typename T>
 __global__ void moe_hidden_kernel(const T* __restrict__ x, const int* __restrict__ ids, const T* __restrict__ w_gu,
-                                  T* __restrict__ hid, int top, int D, int ff, int E, float limit, float slope) {
+                                  T* __restrict__ hid, int top, int D, int ff, int E, ExpertUnit unit) {
     extern __shared__ float xs[];                  // the pair's input row
     const int pair = blockIdx.x;
     const int t = pair / top;
@@ -101,6 +102,17 @@ __global__ void moe_hidden_kernel(const T* __restrict__ x, const int* __restrict
     for (int i = threadIdx.x; i < D; i += blockDim.x) xs[i] = to_f32(x[(size_t)t * D + i]);
     __syncthreads();
     const int lane = threadIdx.x % TLI_WAVE, wave = threadIdx.x / TLI_WAVE, waves = blockDim.x / TLI_WAVE;
+    if (unit.kind >= 0) {                          // an up matrix alone
+        const float by = unit.of_pair(pair);
+        for (int f = wave; f < ff; f += waves) {
+            const T* u = w_gu + ((size_t)e * ff + f) * D;
+            float b = 0.f;
+            for (int i = lane; i < D; i += TLI_WAVE) b = fmaf(xs[i], to_f32(u[i]), b);
+            b = wave_sum(b);
+            if (lane == 0) from_f32(hid + (size_t)pair * ff + f, act_of(by * b, unit.kind));
+        }
+        return;
+    }
     const T* wg = w_gu + (size_t)e * 2 * ff * D;
     const T* wu = wg + (size_t)ff * D;
     for (int f = wave; f < ff; f += waves) {
@@ -113,7 +125,7 @@ __global__ void moe_hidden_kernel(const T* __restrict__ x, const int* __restrict
         }
         a = wave_sum(a);
         b = wave_sum(b);
-        if (lane == 0) from_f32(hid + (size_t)pair * ff + f, gated_unit(a, b, limit, slope));
+        if (lane == 0) from_f32(hid + (size_t)pair * ff + f, gated_unit(a, b, unit.limit, unit.slope));
     }
 }
 
@@ -135,13 +147,13 @@ __global__ void moe_down_kernel(const T* __restrict__ hid, const int* __restrict
         for (int j = 0; j < top; ++j) {
             const int e = ids[(size_t)t * top + j];
             if (e < 0 || e >= E) {                 // hands its input on
-                y = fmaf(weights[(size_t)t * top + j], to_f32(x[(size_t)t * D + c]), y);
+                y = fmaf(weights ? weights[(size_t)t * top + j] : 1.0f, to_f32(x[(size_t)t * D + c]), y);
                 continue;
             }
             const T* w = w_down + ((size_t)e * D + c) * ff;
             float a = 0.f;
             for (int i = lane; i < ff; i += TLI_WAVE) a = fmaf(hs[(size_t)j * ff + i], to_f32(w[i]), a);
-            y = fmaf(weights[(size_t)t * top + j], wave_sum(a), y);
+            y = fmaf(weights ? weights[(size_t)t * top + j] : 1.0f, wave_sum(a), y);
         }
         if (shared) y = fmaf(shared_gate ? shared_gate[t] : 1.0f, to_f32(shared[(size_t)t * D + c]), y);
         if (lane == 0) from_f32(out + (size_t)t * D + c, y);
@@ -165,13 +177,18 @@ extern "C" int tli_moe_route(const float* z, long long z_row, long long z_col, i
     return tli_check_launch("moe_route");
 }
 
-// x [T, D]; ids, weights [T, top]; w_gu [E, 2 ff, D] (an expert's gate rows, then its up rows);
+// x [T, D]; ids, weights [T, top]; w_gu [E, 2 ff, D] (an expert's gate rows, then its up rows), or [E, ff, D] (up rows)
+// where act >= 0 names an activation; weight_on_input: see ExpertUnit;
 // w_down [E, D, ff]; hid [T * top, ff] is scratch; shared [T, D] or null (shared_gate null: added as it is); out [T, D];
 // an id outside 0..E-1 is an expert that hands its input on; limit, slope: the activation (gated_unit)
 extern "C" int tli_moe_experts(const void* x, const int* ids, const float* weights, const void* w_gu,
                                const void* w_down, void* hid, const void* shared, const float* shared_gate, void* out,
-                               int T, int top, int D, int ff, int E, int dtype, float limit, float slope, void* stream) {
+                               int T, int top, int D, int ff, int E, int dtype, float limit, float slope, int act,
+                               int weight_on_input, void* stream) {
     if (T <= 0) return 0;
+    if (act >= TLI_ACT_KINDS || (act < 0 && weight_on_input)) return tli_fail("moe_experts: bad activation");
+    const ExpertUnit unit{act, limit, slope, weight_on_input ? weights : nullptr};
+    if (weight_on_input) weights = nullptr;
     if (top <= 0 || D <= 0 || ff <= 0) return tli_fail("moe_experts: bad sizes");
     if ((size_t)D * 4 > 64 * 1024 || (size_t)top * ff * 4 > 64 * 1024)
         return tli_fail("moe_experts: a row of %d or %d x %d hidden units does not fit the workgroup's memory", D, top, ff);
@@ -181,12 +198,12 @@ extern "C" int tli_moe_experts(const void* x, const int* ids, const float* weigh
     const dim3 dgrid((D + cols - 1) / cols, T);
     if (dtype == TLI_F32) {
         hipLaunchKernelGGL((moe_hidden_kernel<float>), dim3(T * top), dim3(256), (size_t)D * 4, s, (const float*)x, ids,
-                           (const float*)w_gu, (float*)hid, top, D, ff, E, limit, slope);
+                           (const float*)w_gu, (float*)hid, top, D, ff, E, unit);
         hipLaunchKernelGGL((moe_down_kernel<float>), dgrid, dim3(256), (size_t)top * ff * 4, s, (const float*)hid, ids,
                            weights, (const float*)w_down, (const float*)shared, shared_gate, (float*)out, top, D, ff, cols, E, (const float*)x);
     } else if (dtype == TLI_BF16) {
         hipLaunchKernelGGL((moe_hidden_kernel<bf16_t>), dim3(T * top), dim3(256), (size_t)D * 4, s, (const bf16_t*)x, ids,
-                           (const bf16_t*)w_gu, (bf16_t*)hid, top, D, ff, E, limit, slope);
+                           (const bf16_t*)w_gu, (bf16_t*)hid, top, D, ff, E, unit);
         hipLaunchKernelGGL((moe_down_kernel<bf16_t>), dgrid, dim3(256), (size_t)top * ff * 4, s, (const bf16_t*)hid, ids,
                            weights, (const bf16_t*)w_down, (const bf16_t*)shared, shared_gate, (bf16_t*)out, top, D, ff,
                            cols, E, (const bf16_t*)x);

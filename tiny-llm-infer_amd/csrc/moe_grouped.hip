@@ -6,7 +6,7 @@
 //             expert).  How many tiles there are is known on the device only: the products are launched
 //             for the most there can be (pairs / RT + experts) and a workgroup without a tile leaves.
 //   gate/up:  hid[slot, f] = silu(x[row] . Wg_e[f]) * (x[row] . Wu_e[f])          (bfloat16; or the limited form of
-//             common.h's gated_unit)
+//             common.h's gated_unit; or an up matrix alone with an activation: common.h's ExpertUnit)
 //   down:     part[slot, c] = hid[slot] . Wd_e[c]                                 (float32)
 //   combine:  y[row] = sum_j weight[row, j] part[pos[row, j]]  (+ shared gate * shared), in the order of
 //             the choice: a row's result does not depend on which other rows share its tiles, because the
@@ -214,16 +214,17 @@ __device__ __forceinline__ void tile_product(const bf16_t* __restrict__ a1, cons
     }
 }
 
-// gate and up products with the activation: hid[slot, f] (a tile has 16 RB slots)
-template <int RB, int NB>
+// gate and up products (GATED), or the up product alone, with the activation: hid[slot, f] (a tile has 16 RB slots)
+template <int RB, int NB, bool GATED>
 __global__ void __launch_bounds__(256) moe_gate_up_kernel(const bf16_t* __restrict__ x, const int* __restrict__ order,
                                                            const int* __restrict__ tile_expert,
                                                            const int* __restrict__ num_tiles,
                                                            const bf16_t* __restrict__ gate_t,
                                                            const bf16_t* __restrict__ up_t, bf16_t* __restrict__ hid,
-                                                           int top, int D, int ff, float limit, float slope) {
+                                                           int top, int D, int ff, ExpertUnit unit) {
     __shared__ __attribute__((aligned(16))) bf16_t xt[16 * RB * XT_STRIDE];
     __shared__ long long src_off[16 * RB];
+    __shared__ float pair_weight[16 * RB];
     const int tile = blockIdx.y;
     if (tile >= *num_tiles) return;                   // (the whole workgroup)
     const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
@@ -235,6 +236,7 @@ __global__ void __launch_bounds__(256) moe_gate_up_kernel(const bf16_t* __restri
     for (int i = threadIdx.x; i < 16 * RB; i += 256) {
         const int p = order[tile * 16 * RB + i];
         src_off[i] = p >= 0 ? (long long)(p / top) * D : -1;
+        if (!GATED) pair_weight[i] = p >= 0 ? unit.of_pair(p) : 0.f;
     }
     // (a block past the last reads the one before it again and stores nothing)
     const size_t a_step = nb + 1 < nblocks ? (size_t)kblocks * 2048 : 0;
@@ -244,7 +246,10 @@ __global__ void __launch_bounds__(256) moe_gate_up_kernel(const bf16_t* __restri
     for (int i = 0; i < NB; ++i)
 #pragma unroll
         for (int b = 0; b < RB; ++b) ag[i][b] = au[i][b] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    tile_product<RB, NB, true>(gate_t + block0, up_t + block0, a_step, x, src_off, D, active, xt, ag, au);
+    if constexpr (GATED)
+        tile_product<RB, NB, true>(gate_t + block0, up_t + block0, a_step, x, src_off, D, active, xt, ag, au);
+    else
+        tile_product<RB, NB, false>(up_t + block0, nullptr, a_step, x, src_off, D, active, xt, au, ag);
     if (!active) return;
     // the lane holds hidden units (nb + i) * 16 + 4 c .. + 4 of the slots 16 b + r
 #pragma unroll
@@ -256,7 +261,9 @@ __global__ void __launch_bounds__(256) moe_gate_up_kernel(const bf16_t* __restri
             if (src_off[b * 16 + r] < 0) continue;
             float h[4];
 #pragma unroll
-            for (int v = 0; v < 4; ++v) h[v] = gated_unit(ag[i][b][v], au[i][b][v], limit, slope);
+            for (int v = 0; v < 4; ++v)
+                h[v] = GATED ? gated_unit(ag[i][b][v], au[i][b][v], unit.limit, unit.slope)
+                             : act_of(pair_weight[b * 16 + r] * au[i][b][v], unit.kind);
             store4(hid + (size_t)((tile * RB + b) * 16 + r) * ff + n0, h, ff - n0, ff % 4 == 0);
         }
     }
@@ -316,7 +323,7 @@ __global__ void moe_combine_kernel(const float* __restrict__ part, const int* __
         for (int j = 0; j < top; ++j) {
             const int slot = pos[(size_t)t * top + j];           // negative: the expert hands its input on
             const float v = slot >= 0 ? part[(size_t)slot * D + cidx] : bf16_to_f32(x[(size_t)t * D + cidx]);
-            y = fmaf(weights[(size_t)t * top + j], v, y);
+            y = fmaf(weights ? weights[(size_t)t * top + j] : 1.0f, v, y);
         }
         if (shared) y = fmaf(shared_gate ? shared_gate[t] : 1.0f, bf16_to_f32(shared[(size_t)t * D + cidx]), y);
         out[(size_t)t * D + cidx] = f32_to_bf16(y);
@@ -335,13 +342,17 @@ extern "C" int tli_moe_grouped_tile(int pairs, int experts) {
 
 // scratch, all given by the caller: order [tiles_max * RT], pos [pairs], tile_expert [tiles_max],
 // num_tiles [1] (int32); hid [tiles_max * RT, ff] (bfloat16); part [tiles_max * RT, D] (float32);
-// with tiles_max = pairs / RT + experts.  gate_t, up_t: [E] tiled [ff, D]; down_t: [E] tiled [D, ff].
+// with tiles_max = pairs / RT + experts.  gate_t, up_t: [E] tiled [ff, D] (act >= 0: an activation, and no gate_t);
+// down_t: [E] tiled [D, ff]; weight_on_input: see ExpertUnit.
 extern "C" int tli_moe_grouped_bf16(const void* x, const int* ids, const float* weights, const void* gate_t,
                                     const void* up_t, const void* down_t, int* order, int* pos, int* tile_expert,
                                     int* num_tiles, void* hid, float* part, const void* shared,
                                     const float* shared_gate, void* out, int T, int top, int E, int D, int ff, int RT,
-                                    float limit, float slope, void* stream) {
+                                    float limit, float slope, int act, int weight_on_input, void* stream) {
     if (T <= 0) return 0;
+    if (act >= TLI_ACT_KINDS || (act < 0 && (weight_on_input || !gate_t))) return tli_fail("moe_grouped: bad activation");
+    const ExpertUnit unit{act, limit, slope, weight_on_input ? weights : nullptr};
+    if (weight_on_input) weights = nullptr;
     if (top <= 0 || E <= 0 || E > SORT_MAX_EXPERTS || D <= 0 || ff <= 0 || D % 8 || ff % 8)
         return tli_fail("moe_grouped: bad sizes (experts %d (at most %d), width %d and hidden units %d in eights)", E,
                         SORT_MAX_EXPERTS, D, ff);
@@ -354,9 +365,14 @@ extern "C" int tli_moe_grouped_bf16(const void* x, const int* ids, const float* 
     hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, s, ids, (int)pairs, E, RT, (int)tiles_max, order, pos,
                        tile_expert, num_tiles);
 #define TLI_GROUPED(RB, NBG)                                                                                          \
-    hipLaunchKernelGGL((moe_gate_up_kernel<RB, NBG>), dim3((ff + 64 * NBG - 1) / (64 * NBG), (unsigned)tiles_max),      \
-                       dim3(256), 0, s, (const bf16_t*)x, order, tile_expert, num_tiles, (const bf16_t*)gate_t,        \
-                       (const bf16_t*)up_t, (bf16_t*)hid, top, D, ff, limit, slope);                                   \
+    if (act < 0)                                                                                                       \
+        hipLaunchKernelGGL((moe_gate_up_kernel<RB, NBG, true>), dim3((ff + 64 * NBG - 1) / (64 * NBG), (unsigned)tiles_max), \
+                           dim3(256), 0, s, (const bf16_t*)x, order, tile_expert, num_tiles, (const bf16_t*)gate_t,    \
+                           (const bf16_t*)up_t, (bf16_t*)hid, top, D, ff, unit);                                       \
+    else                                                                                                               \
+        hipLaunchKernelGGL((moe_gate_up_kernel<RB, 2, false>), dim3((ff + 127) / 128, (unsigned)tiles_max), dim3(256), 0, s, \
+                           (const bf16_t*)x, order, tile_expert, num_tiles, (const bf16_t*)nullptr, (const bf16_t*)up_t, \
+                           (bf16_t*)hid, top, D, ff, unit);                                                            \
     hipLaunchKernelGGL((moe_down_grouped_kernel<RB, 2>), dim3((D + 127) / 128, (unsigned)tiles_max), dim3(256), 0, s,  \
                        (const bf16_t*)hid, order, tile_expert, num_tiles, (const bf16_t*)down_t, part, D, ff)
     if (RT == 16) { TLI_GROUPED(1, 2); }

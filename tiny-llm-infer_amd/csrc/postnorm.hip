@@ -3,6 +3,12 @@
 // norm_add:       one workgroup a row: the sublayer's output y (the run's type) is read once into registers,
 //                 its mean square summed in float32, the normed row added to the float32 residual, and the
 //                 new residual written in the run's type for the next sublayer to read.
+// norm_add_norm:  the same with the norm of whoever reads the sum next in the same pass: h = w2 * x / sqrt(mean(x^2) + eps2)
+//                 is written instead of x's own rows.  Without y: that norm alone.  With `rows` only those rows of the
+//                 residual are looked at, and it is not written.  With mixes (steps of one row a sequence): h' being the row
+//                 that the sequence's slot keeps (zeros at position 0), h + (h' - h) mu_m for every m is written instead, and
+//                 h replaces the kept row.
+// token_mixes:    those mixes from rows h of portions: h' is the row before in the same sequence.
 // residual_rows:  the residual's rows in the run's type (what the first block reads).
 #include "common.h"
 
@@ -103,6 +109,157 @@ __global__ __launch_bounds__(PN_THREADS) void norm_add_vec_kernel(float* __restr
     }
 }
 
+struct MixArgs {
+    const float* mu;             // [mixes][n], or null: no mixes
+    int mixes;
+    void* kept;                  // [slots][n] in the rows' type
+    const int* slots;            // [seqs]
+    const int* seq_start;        // [seqs]
+    size_t stride;               // elements between two mixes of the output
+};
+
+// h + (h' - h) mu_m for all m; V elements from column c on, of row `row`
+template <typename T, int V>
+__device__ __forceinline__ void put_mixes(const float (&h)[V], const float (&prev)[V], const MixArgs& mix, T* __restrict__ out,
+                                          size_t at, int c, int n) {
+    for (int m = 0; m < mix.mixes; ++m) {
+        const float* mu = mix.mu + (size_t)m * n + c;
+        T* dst = out + (size_t)m * mix.stride + at;
+        float o[V];
+#pragma unroll
+        for (int e = 0; e < V; ++e) o[e] = h[e] + (prev[e] - h[e]) * mu[e];
+        if constexpr (V == 8 && sizeof(T) == 2)
+            *reinterpret_cast<uint4*>(dst) = make_uint4(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]), pack_bf16x2(o[4], o[5]), pack_bf16x2(o[6], o[7]));
+        else
+#pragma unroll
+            for (int e = 0; e < V; ++e) from_f32(dst + e, o[e]);
+    }
+}
+
+// V elements of a row as float32: 1, or 8 of an aligned row
+template <typename T, int V>
+__device__ __forceinline__ void row_load(const T* p, float (&v)[V]) {
+    if constexpr (V == 8 && sizeof(T) == 2) {
+        const uint4 u = *reinterpret_cast<const uint4*>(p);
+        const uint32_t w[4] = {u.x, u.y, u.z, u.w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[2 * e] = __uint_as_float(w[e] << 16), v[2 * e + 1] = __uint_as_float(w[e] & 0xFFFF0000u);
+    } else if constexpr (V == 8) {
+        *reinterpret_cast<float4*>(v) = *reinterpret_cast<const float4*>(p);
+        *reinterpret_cast<float4*>(v + 4) = *reinterpret_cast<const float4*>(p + 4);
+    } else {
+        v[0] = to_f32(*p);
+    }
+}
+template <typename T, int V>
+__device__ __forceinline__ void row_store(T* p, const float (&v)[V]) {
+    if constexpr (V == 8 && sizeof(T) == 2) {
+        *reinterpret_cast<uint4*>(p) = make_uint4(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7]));
+    } else if constexpr (V == 8) {
+        *reinterpret_cast<float4*>(p) = *reinterpret_cast<const float4*>(v);
+        *reinterpret_cast<float4*>(p + 4) = *reinterpret_cast<const float4*>(v + 4);
+    } else {
+        from_f32(p, v[0]);
+    }
+}
+
+// ROUNDS x PN_THREADS x V elements of a row are kept in registers between the sums; a row is no longer than that.
+template <typename T, int V, int ROUNDS>
+__global__ __launch_bounds__(PN_THREADS) void norm_add_norm_kernel(float* __restrict__ resid, const T* __restrict__ y,
+                                                                    const float* __restrict__ w1, float eps1,
+                                                                    const float* __restrict__ w2, float eps2, T* __restrict__ out,
+                                                                    const int* __restrict__ rows, int n, MixArgs mix) {
+    __shared__ float red[16];
+    const size_t row = rows ? rows[blockIdx.x] : blockIdx.x;
+    float* xr = resid + row * n;
+    float v[ROUNDS][V], x[ROUNDS][V];
+    float ssq = 0.f;
+#pragma unroll
+    for (int i = 0; i < ROUNDS; ++i) {
+        const int c = (i * PN_THREADS + threadIdx.x) * V;
+#pragma unroll
+        for (int e = 0; e < V; ++e) v[i][e] = x[i][e] = 0.f;
+        if (c < n) {
+            row_load<float, V>(xr + c, x[i]);
+            if (y) row_load<T, V>(y + row * n + c, v[i]);
+        }
+#pragma unroll
+        for (int e = 0; e < V; ++e) ssq = fmaf(v[i][e], v[i][e], ssq);
+    }
+    if (y) {
+        const float factor = 1.0f / sqrtf(block_sum(ssq, red) / (float)n + eps1);
+#pragma unroll
+        for (int i = 0; i < ROUNDS; ++i) {
+            const int c = (i * PN_THREADS + threadIdx.x) * V;
+            if (c >= n) continue;
+            float g[V];
+            row_load<float, V>(w1 + c, g);
+#pragma unroll
+            for (int e = 0; e < V; ++e) x[i][e] += v[i][e] * factor * g[e];
+            if (!rows) row_store<float, V>(xr + c, x[i]);
+        }
+    }
+    ssq = 0.f;
+#pragma unroll
+    for (int i = 0; i < ROUNDS; ++i)
+#pragma unroll
+        for (int e = 0; e < V; ++e) ssq = fmaf(x[i][e], x[i][e], ssq);
+    const float factor = 1.0f / sqrtf(block_sum(ssq, red) / (float)n + eps2);
+    T* kept = nullptr;
+    bool fresh = true;
+    if (mix.mu) {
+        kept = (T*)mix.kept + (size_t)mix.slots[row] * n;
+        fresh = mix.seq_start[row] <= 0;
+    }
+#pragma unroll
+    for (int i = 0; i < ROUNDS; ++i) {
+        const int c = (i * PN_THREADS + threadIdx.x) * V;
+        if (c >= n) continue;
+        float g[V], h[V];
+        row_load<float, V>(w2 + c, g);
+#pragma unroll
+        for (int e = 0; e < V; ++e) h[e] = x[i][e] * factor * g[e];
+        if (!mix.mu) {
+            row_store<T, V>(out + (size_t)blockIdx.x * n + c, h);
+            continue;
+        }
+        float prev[V];
+#pragma unroll
+        for (int e = 0; e < V; ++e) prev[e] = 0.f;
+        if (!fresh) row_load<T, V>(kept + c, prev);
+        if constexpr (sizeof(T) == 2) {             // h as it is kept: the mixes are made of rounded rows
+#pragma unroll
+            for (int e = 0; e < V; ++e) h[e] = bf16_to_f32(f32_to_bf16(h[e]));
+        }
+        row_store<T, V>(kept + c, h);
+        put_mixes<T, V>(h, prev, mix, out, row * n + c, c, n);
+    }
+}
+
+template <typename T, int V>
+__global__ __launch_bounds__(PN_THREADS) void token_mixes_kernel(const T* __restrict__ h, T* __restrict__ out, const int* __restrict__ seq_of_row,
+                                                                 const int* __restrict__ row_start, int n, MixArgs mix) {
+    const int row = blockIdx.x;
+    const int seq = seq_of_row[row], first = row_start[seq], last = row_start[seq + 1] - 1;
+    // the workgroup of a sequence's first row, having read the kept row, replaces it: each element is read and
+    // written by the same thread
+    T* kept = row == first ? (T*)mix.kept + (size_t)mix.slots[seq] * n : nullptr;
+    const bool fresh = row == first && mix.seq_start[seq] <= 0;
+    for (int c = threadIdx.x * V; c < n; c += PN_THREADS * V) {
+        float cur[V], prev[V];
+        row_load<T, V>(h + (size_t)row * n + c, cur);
+#pragma unroll
+        for (int e = 0; e < V; ++e) prev[e] = 0.f;
+        if (!fresh) row_load<T, V>(kept ? kept + c : h + (size_t)(row - 1) * n + c, prev);
+        if (kept) {
+            float end[V];
+            row_load<T, V>(h + (size_t)last * n + c, end);
+            row_store<T, V>(kept + c, end);
+        }
+        put_mixes<T, V>(cur, prev, mix, out, (size_t)row * n + c, c, n);
+    }
+}
+
 __global__ void residual_rows_kernel(const float* __restrict__ resid, bf16_t* __restrict__ out, long long count) {
     const long long i = ((long long)blockIdx.x * blockDim.x + threadIdx.x) * 4;
     if (i + 3 < count) {
@@ -141,4 +298,83 @@ extern "C" int tli_residual_rows(const float* resid, void* out, long long count,
     const long long threads = (count + 3) / 4;
     residual_rows_kernel<<<(unsigned)((threads + 255) / 256), 256, 0, (hipStream_t)stream>>>(resid, (bf16_t*)out, count);
     return tli_check_launch("residual_rows");
+}
+
+template <typename T>
+static int run_norm_add_norm(float* resid, const T* y, const float* w1, float eps1, const float* w2, float eps2, T* out, const int* rows,
+                             int count, int n, const MixArgs& mix, hipStream_t s) {
+    const bool vec = n % 8 == 0 && !(((uintptr_t)resid | (uintptr_t)y | (uintptr_t)w1 | (uintptr_t)w2 | (uintptr_t)out | (uintptr_t)mix.mu |
+                                      (uintptr_t)mix.kept) & 15);
+#define NAN_RUN(V, R) norm_add_norm_kernel<T, V, R><<<count, PN_THREADS, 0, s>>>(resid, y, w1, eps1, w2, eps2, out, rows, n, mix)
+    if (vec && n <= 8 * PN_THREADS) NAN_RUN(8, 1);
+    else if (vec && n <= 16 * PN_THREADS) NAN_RUN(8, 2);
+    else if (vec && n <= 32 * PN_THREADS) NAN_RUN(8, 4);
+    else if (n <= 4 * PN_THREADS) NAN_RUN(1, 4);
+    else if (n <= 32 * PN_THREADS) NAN_RUN(1, 32);
+    else return tli_fail("norm_add_norm: rows of %d elements (at most %d)", n, 32 * PN_THREADS);
+#undef NAN_RUN
+    return tli_check_launch("norm_add_norm");
+}
+
+// resid [.., n] float32 += w1 * y / rms(y) (y null: nothing), out [count, n] = w2 * resid / rms(resid) in the type of y.
+// rows (or null): the rows of resid and y that `count` counts, resid then unchanged.  mu (or null) [mixes][n], kept
+// [slots][n], slots, seq_start [rows]: out is [mixes][count][n] (rows must be null).
+extern "C" int tli_norm_add_norm(float* resid, const void* y, const float* w1, float eps1, const float* w2, float eps2, void* out,
+                                 const int* rows, int count, int n, const float* mu, int mixes, void* kept, const int* slots,
+                                 const int* seq_start, int dtype, void* stream) {
+    if (count <= 0) return 0;
+    if (n <= 0 || (y && !w1) || !w2 || !out) return tli_fail("norm_add_norm: bad arguments");
+    if (mu && (rows || mixes <= 0 || !kept || !slots || !seq_start)) return tli_fail("norm_add_norm: bad mixes");
+    const MixArgs mix{mu, mixes, kept, slots, seq_start, (size_t)count * n};
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == TLI_F32) return run_norm_add_norm<float>(resid, (const float*)y, w1, eps1, w2, eps2, (float*)out, rows, count, n, mix, s);
+    if (dtype == TLI_BF16) return run_norm_add_norm<bf16_t>(resid, (const bf16_t*)y, w1, eps1, w2, eps2, (bf16_t*)out, rows, count, n, mix, s);
+    return tli_fail("norm_add_norm: unknown dtype %d", dtype);
+}
+
+// h [rows, n]; out [mixes][rows][n]; mu [mixes][n]; kept [slots][n] in the type of h
+extern "C" int tli_token_mixes(const void* h, const float* mu, int mixes, void* kept, void* out, const int* seq_of_row,
+                               const int* row_start, const int* seq_start, const int* slots, int rows, int n, int dtype, void* stream) {
+    if (rows <= 0) return 0;
+    if (n <= 0 || mixes <= 0) return tli_fail("token_mixes: bad sizes");
+    const MixArgs mix{mu, mixes, kept, slots, seq_start, (size_t)rows * n};
+    const bool vec = n % 8 == 0 && !(((uintptr_t)h | (uintptr_t)mu | (uintptr_t)kept | (uintptr_t)out) & 15);
+    hipStream_t s = (hipStream_t)stream;
+#define TM_RUN(T, V) token_mixes_kernel<T, V><<<rows, PN_THREADS, 0, s>>>((const T*)h, (T*)out, seq_of_row, row_start, n, mix)
+    if (dtype == TLI_F32) { if (vec) TM_RUN(float, 8); else TM_RUN(float, 1); }
+    else if (dtype == TLI_BF16) { if (vec) TM_RUN(bf16_t, 8); else TM_RUN(bf16_t, 1); }
+    else return tli_fail("token_mixes: unknown dtype %d", dtype);
+#undef TM_RUN
+    return tli_check_launch("token_mixes");
+}
+
+// out [rows, n] = w * x / sqrt(mean(x^2) + eps) for n elements of rows that lie ld elements apart.  A wave a row.
+template <typename T>
+__global__ __launch_bounds__(PN_THREADS) void norm_rows_kernel(const T* __restrict__ x, int ld, const float* __restrict__ w, T* __restrict__ out,
+                                                               int rows, int n, float eps) {
+    const int lane = threadIdx.x % TLI_WAVE;
+    const int row = blockIdx.x * (PN_THREADS / TLI_WAVE) + threadIdx.x / TLI_WAVE;
+    if (row >= rows) return;
+    const T* src = x + (size_t)row * ld;
+    float ssq = 0.f;
+    for (int c = lane; c < n; c += TLI_WAVE) {
+        const float v = to_f32(src[c]);
+        ssq = fmaf(v, v, ssq);
+    }
+    const float factor = 1.0f / sqrtf(wave_sum(ssq) / (float)n + eps);
+    for (int c = lane; c < n; c += TLI_WAVE) from_f32(out + (size_t)row * n + c, to_f32(src[c]) * factor * w[c]);
+}
+
+extern "C" int tli_norm_rows(const void* x, int ld, const float* w, void* out, int rows, int n, float eps, int dtype, void* stream) {
+    if (rows <= 0) return 0;
+    if (n <= 0 || ld < n) return tli_fail("norm_rows: bad sizes");
+    hipStream_t s = (hipStream_t)stream;
+    const int per = PN_THREADS / TLI_WAVE;
+    if (dtype == TLI_F32)
+        norm_rows_kernel<float><<<(rows + per - 1) / per, PN_THREADS, 0, s>>>((const float*)x, ld, w, (float*)out, rows, n, eps);
+    else if (dtype == TLI_BF16)
+        norm_rows_kernel<bf16_t><<<(rows + per - 1) / per, PN_THREADS, 0, s>>>((const bf16_t*)x, ld, w, (bf16_t*)out, rows, n, eps);
+    else
+        return tli_fail("norm_rows: unknown dtype %d", dtype);
+    return tli_check_launch("norm_rows");
 }

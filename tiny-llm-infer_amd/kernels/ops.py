@@ -113,22 +113,22 @@ def load_library():
         "tli_delta_state_floats": [I, I],
         "tli_gated_rmsnorm": [P, P, I, P, P, I, I, I, F, I, P],
         "tli_moe_route": [P, ctypes.c_longlong, ctypes.c_longlong, P, P, P, I, I, I, I, I, F, I, I, I, I, P, P],
-        "tli_moe_experts": [P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, F, P],
+        "tli_moe_experts": [P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, F, I, I, P],
         "tli_norm_add": [P, P, P, P, I, I, F, I, P],
         "tli_residual_rows": [P, P, ctypes.c_longlong, P],
         "tli_attention_sized_plain": [P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, F, I, I, I, I, P, P],
         "tli_attention_sized_mfma_takes": [I, I, I, I],
         "tli_head_products_mfma_takes": [I, I] + [ctypes.c_longlong] * 4,
         "tli_head_products_mfma_bf16": [P, ctypes.c_longlong, ctypes.c_longlong, P, P, ctypes.c_longlong, ctypes.c_longlong,
-                                        I, I, I, I, P],
+                                        I, I, I, I, P, I, P],
         "tli_attention_sized_mfma_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, I, F, I, I, I, I, P, P],
         "tli_diff_prepare": [P, I, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P, F, I, P],
         "tli_diff_combine": [P, P, I, I, P, I, I, I, F, F, F, I, P],
-        "tli_latent_prepare": [P, I, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P, F, P, P, I, P],
+        "tli_latent_prepare": [P, I, P, I, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P, F, P, P, I, P],
         "tli_head_products_plain": [P, ctypes.c_longlong, ctypes.c_longlong, P, P, ctypes.c_longlong, ctypes.c_longlong,
-                                    I, I, I, I, I, P],
+                                    I, I, I, I, P, I, I, P],
         "tli_moe_grouped_tile": [I, I],
-        "tli_moe_grouped_bf16": [P, P, P, P, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, F, P],
+        "tli_moe_grouped_bf16": [P, P, P, P, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, F, I, I, P],
         "tli_keyed_prepare": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P, I, I, I, P],
         "tli_add_bias": [P, P, I, I, I, P],
         "tli_lightning_recurrence": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
@@ -146,6 +146,12 @@ def load_library():
         "tli_pooled_prefill_takes": [I, I, I, I, I, I],
         "tli_pooled_prefill_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
         "tli_attention_pooled_mfma_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, I, P, P],
+        "tli_norm_add_norm": [P, P, P, F, P, F, P, P, I, I, P, I, P, P, P, I, P],
+        "tli_token_mixes": [P, P, I, P, P, P, P, P, P, I, I, I, P],
+        "tli_norm_rows": [P, I, P, P, I, I, F, I, P],
+        "tli_token_gate": [P, P, P, P, I, I, I, I, I, I, I, P],
+        "tli_wkv_decays": [P, ctypes.c_longlong, ctypes.c_longlong, P, P, P, I, I, I, I, P],
+        "tli_wkv_rows": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, P],
         "tli_sample": [P, I, I, P, P, P, P, P, P],
         "tli_sample_scratch_bytes": [I],
         "tli_random_normal": [P, ctypes.c_longlong, ctypes.c_uint32, ctypes.c_uint32, ctypes.c_uint32, P, F, F, I, P],
@@ -943,7 +949,7 @@ class HipOps:
         return out
 
     # ---- feed-forward without a gate, soft cap -----------------------------------------
-    ACTIVATIONS = {"relu2": 0, "relu": 1, "silu": 2, "gelu_tanh": 3}
+    ACTIVATIONS = {"relu2": 0, "relu": 1, "silu": 2, "gelu_tanh": 3, "gelu": 4}
 
     def check_activation(self, name: str) -> None:
         if name not in self.ACTIVATIONS:
@@ -1253,16 +1259,17 @@ class HipOps:
         if hidden * 4 > 64 * 1024 or top * inter * 4 > 64 * 1024:
             raise KernelError("a row, or the hidden units of a row's experts, do not fit a workgroup's memory")
 
-    def pack_experts(self, w_gate_up, w_down):
+    def pack_experts(self, w_gate_up, w_down, gated=True):
         """The experts' matrices in the tiled layout that the matrix-core kernels read (``tile_matrix`` of every
-        expert's gate, up and down matrix), or None where those kernels do not apply (float32, sizes that are no
-        multiples of 8, the plain kernels asked for): then ``apply_experts`` works from the row-major matrices."""
-        E, two_ff, n = w_gate_up.shape
-        ff = two_ff // 2
+        expert's gate, up and down matrix; ``gated`` false: ``w_gate_up`` is [E, ff, n], up matrices alone), or None
+        where those kernels do not apply (float32, sizes that are no multiples of 8, the plain kernels asked for): then
+        ``apply_experts`` works from the row-major matrices."""
+        E, rows, n = w_gate_up.shape
+        ff = rows // 2 if gated else rows
         if w_gate_up.dtype != torch.bfloat16 or n % 8 or ff % 8 or E > 2048 or self.plain_products:
             return None
-        return {"gate": torch.stack([self.tile_matrix(w_gate_up[e, :ff]) for e in range(E)]),
-                "up": torch.stack([self.tile_matrix(w_gate_up[e, ff:]) for e in range(E)]),
+        return {"gate": torch.stack([self.tile_matrix(w_gate_up[e, :ff]) for e in range(E)]) if gated else None,
+                "up": torch.stack([self.tile_matrix(w_gate_up[e, ff:] if gated else w_gate_up[e]) for e in range(E)]),
                 "down": torch.stack([self.tile_matrix(w_down[e]) for e in range(E)]),
                 "experts": E, "hidden": n, "inter": ff}
 
@@ -1296,14 +1303,24 @@ class HipOps:
                    self.ROUTER_GROUP_SCORES.index(group_score), 1 if normalize else 0, _ptr(correction), self._stream())
         return ids, weights, gate
 
-    def apply_experts(self, x, ids, weights, w_gate_up, w_down, packed, shared, shared_gate, limit=0.0, slope=1.0):
+    def apply_experts(self, x, ids, weights, w_gate_up, w_down, packed, shared, shared_gate, limit=0.0, slope=1.0,
+                      activation=None, weight_on_input=False):
         """sum_j weights[t, j] * expert ids[t, j] (x[t])  (+ shared_gate[t] * shared[t], or + shared[t] without a
         gate);  ``w_gate_up`` [E, 2 ff, n] (an expert's gate rows, then its up rows), ``w_down`` [E, n, ff]; with
         ``packed`` (what ``pack_experts`` gave) the row-major matrices may be None.  An id from E on is an expert
         that hands its input on: its term is weights[t, j] * x[t].  ``limit`` > 0: the experts' hidden units are the
-        limited form (see ``swiglu``) instead of silu(gate) * up."""
+        limited form (see ``swiglu``) instead of silu(gate) * up.  ``activation`` (one of ``ACTIVATIONS``): experts
+        without a gate matrix, down(act(up x)), ``w_gate_up`` being [E, ff, n]; with ``weight_on_input`` a pair's weight
+        multiplies the expert's input and not its output."""
         T, n = x.shape
         top = ids.shape[1]
+        act = -1
+        if activation is not None:
+            self.check_activation(activation)
+            act = self.ACTIVATIONS[activation]
+        elif weight_on_input:
+            raise KernelError("weights on the experts' inputs are for experts without a gate")
+        on_input = 1 if weight_on_input else 0
         self._want(x, "expert input")
         self._want(ids, "chosen experts", torch.int32, (T, top))
         self._want(weights, "experts' weights", torch.float32, (T, top))
@@ -1321,6 +1338,8 @@ class HipOps:
             nb, kb = (ff + 15) // 16, (n + 127) // 128
             for role, shape in (("gate", (E, nb, kb, 4, 4, 16, 8)), ("up", (E, nb, kb, 4, 4, 16, 8)),
                                 ("down", (E, (n + 15) // 16, (ff + 127) // 128, 4, 4, 16, 8))):
+                if role == "gate" and act >= 0:
+                    continue
                 self._want(packed[role], f"experts' {role} matrices (tiled)", torch.bfloat16, shape)
             a_call = max(1, (65535 - E) * 16 // top)                 # (a launch's grid holds 65,535 tiles)
             for t0 in range(0, T, a_call):
@@ -1334,17 +1353,18 @@ class HipOps:
                 hid = torch.empty((slots, ff), dtype=torch.bfloat16, device=self.device)
                 part = torch.empty((slots, n), dtype=torch.float32, device=self.device)
                 self._call(self.lib.tli_moe_grouped_bf16, x[t0:t1].data_ptr(), ids[t0:t1].data_ptr(), weights[t0:t1].data_ptr(),
-                           packed["gate"].data_ptr(), packed["up"].data_ptr(), packed["down"].data_ptr(), order.data_ptr(),
+                           None if act >= 0 else packed["gate"].data_ptr(), packed["up"].data_ptr(), packed["down"].data_ptr(), order.data_ptr(),
                            pos.data_ptr(), tile_expert.data_ptr(), num_tiles.data_ptr(), hid.data_ptr(), part.data_ptr(),
                            None if shared is None else shared[t0:t1].data_ptr(),
                            None if (shared is None or shared_gate is None) else shared_gate[t0:t1].data_ptr(),
-                           out[t0:t1].data_ptr(), t1 - t0, top, E, n, ff, RT, float(limit), float(slope), self._stream())
+                           out[t0:t1].data_ptr(), t1 - t0, top, E, n, ff, RT, float(limit), float(slope), act, on_input,
+                           self._stream())
             return out
         if w_gate_up is None or w_down is None:
             raise KernelError("the experts' row-major matrices were not kept and the tiled ones do not apply here")
-        E, two_ff, _ = w_gate_up.shape
-        ff = two_ff // 2
-        self._want(w_gate_up, "experts' gate and up matrices", x.dtype, (E, 2 * ff, n))
+        E, rows, _ = w_gate_up.shape
+        ff = rows if act >= 0 else rows // 2
+        self._want(w_gate_up, "experts' gate and up matrices", x.dtype, (E, ff if act >= 0 else 2 * ff, n))
         self._want(w_down, "experts' down matrices", x.dtype, (E, n, ff))
         hid = torch.empty((T * top, ff), dtype=x.dtype, device=self.device)
         for t0 in range(0, T, 32768):
@@ -1353,8 +1373,8 @@ class HipOps:
                        w_gate_up.data_ptr(), w_down.data_ptr(), hid[t0 * top:].data_ptr(),
                        None if shared is None else shared[t0:t1].data_ptr(),
                        None if (shared is None or shared_gate is None) else shared_gate[t0:t1].data_ptr(),
-                       out[t0:t1].data_ptr(), t1 - t0, top, n, ff, E, _dtype_code(x.dtype), float(limit), float(slope),
-                       self._stream())
+                       out[t0:t1].data_ptr(), t1 - t0, top, n, ff, E, _dtype_code(x.dtype), float(limit), float(slope), act,
+                       on_input, self._stream())
         return out
 
     # ---- blocks that norm what a sublayer gives ------------------------------------------------------------
@@ -1380,6 +1400,80 @@ class HipOps:
         out = resid if out_dtype == torch.float32 else torch.empty((total, n), dtype=out_dtype, device=self.device)
         self._call(self.lib.tli_norm_add, resid.data_ptr(), y.data_ptr(), weight.data_ptr(),
                    None if out is resid else out.data_ptr(), total, n, float(eps), _dtype_code(out_dtype), self._stream())
+        return out
+
+    # ---- blocks that norm what a sublayer reads and what it gives ---------------------------------------------
+    def norm_add_norm(self, resid, y, w_out, eps_out, w_in, eps_in, out_dtype, rows=None, num_rows=None):
+        """resid (float32 [T, n]) += w_out * y / sqrt(mean(y^2) + eps_out) for ``y`` [T, n] in the run's type or an unfinished
+        product (None: nothing is added); returns w_in * resid / sqrt(mean(resid^2) + eps_in) in the run's type.  With
+        ``rows`` (int32 on the device, the first ``num_rows`` of them) only those rows, and ``resid`` is left as it is."""
+        return self._norm_add_norm(resid, y, w_out, eps_out, w_in, eps_in, out_dtype, rows, num_rows, None, None)
+
+    def norm_add_norm_mixes(self, resid, y, w_out, eps_out, w_in, eps_in, out_dtype, mixes, step):
+        """``norm_add_norm`` and the ``token_mixes`` of its rows in one pass, [mixes, T, n], for a step of one row a sequence;
+        None for other steps, with nothing done.  ``mixes`` = (mu [m, n], kept rows)."""
+        if not self._single_rows(step):
+            return None
+        return self._norm_add_norm(resid, y, w_out, eps_out, w_in, eps_in, out_dtype, None, None, mixes, step)
+
+    def _norm_add_norm(self, resid, y, w_out, eps_out, w_in, eps_in, out_dtype, rows, num_rows, mixes, step):
+        total, n = resid.shape
+        self._want(resid, "residual", torch.float32)
+        self._want(w_in, "norm weight", torch.float32, (n,))
+        if y is not None:
+            y = self.resolve(y)
+            self._want(y, "sublayer output", out_dtype, (total, n))
+            self._want(w_out, "norm weight", torch.float32, (n,))
+        count = total
+        if rows is not None:
+            self._want(rows, "rows", torch.int32)
+            count = int(num_rows)
+            if count > rows.numel():
+                raise KernelError(f"{count} rows wanted, {rows.numel()} are named")
+        mu, kept, m, slots, starts = None, None, 0, None, None
+        if mixes is not None:
+            mu, kept = mixes
+            m = mu.shape[0]
+            self._check_mixes(mu, kept, step, total, n, out_dtype)
+            slots, starts = step.slots.data_ptr(), step.seq_start.data_ptr()
+        out = torch.empty((count, n) if mixes is None else (m, count, n), dtype=out_dtype, device=self.device)
+        self._call(self.lib.tli_norm_add_norm, resid.data_ptr(), _ptr(y), None if y is None else w_out.data_ptr(), float(eps_out),
+                   w_in.data_ptr(), float(eps_in), out.data_ptr(), _ptr(rows), count, n, _ptr(mu), m, _ptr(kept), slots, starts,
+                   _dtype_code(out_dtype), self._stream())
+        return out
+
+    def _check_mixes(self, mu, kept, step, rows, n, dtype):
+        self._want(mu, "weights of the mixes", torch.float32, (mu.shape[0], n))
+        self._want(kept, "kept rows", dtype, (kept.shape[0], n))
+        if step.num_rows != rows:
+            raise KernelError(f"the step has {step.num_rows} rows, the mixes got {rows}")
+        if max(step.h_slots, default=0) >= kept.shape[0]:
+            raise KernelError("a sequence's slot lies outside the kept rows")
+
+    def token_mixes(self, h, mu, kept, step):
+        """out[m, r] = h[r] + (row before r of its sequence - h[r]) * mu[m], [mixes, rows, n]; the row before a step's
+        first row is the sequence's kept row (nothing at position 0), which the sequence's last row replaces."""
+        rows, n = h.shape
+        self._want(h, "rows to mix")
+        self._check_mixes(mu, kept, step, rows, n, h.dtype)
+        out = torch.empty((mu.shape[0], rows, n), dtype=h.dtype, device=self.device)
+        self._call(self.lib.tli_token_mixes, h.data_ptr(), mu.data_ptr(), mu.shape[0], kept.data_ptr(), out.data_ptr(),
+                   step.seq_of_row.data_ptr(), step.row_start.data_ptr(), step.seq_start.data_ptr(), step.slots.data_ptr(), rows, n,
+                   _dtype_code(h.dtype), self._stream())
+        return out
+
+    def token_gate(self, z, table, at, token_ids, activation):
+        """act(z[t]) * table[token_ids[t], at : at + n], [T, n] in the type of ``z`` [T, n]."""
+        self.check_activation(activation)
+        T, n = z.shape
+        self._want(z, "gate's logits")
+        self._want(table, "tokens' vectors", z.dtype)
+        self._want(token_ids, "token ids", torch.int32)
+        if token_ids.numel() < T or at < 0 or at + n > table.shape[1]:
+            raise KernelError("a token's vector lies outside the table")
+        out = torch.empty((T, n), dtype=z.dtype, device=self.device)
+        self._call(self.lib.tli_token_gate, z.data_ptr(), table.data_ptr(), token_ids.data_ptr(), out.data_ptr(), T, n, table.shape[1],
+                   at, table.shape[0], self.ACTIVATIONS[activation], _dtype_code(z.dtype), self._stream())
         return out
 
     # ---- attention whose keys and values have sizes of their own -------------------------------------------
@@ -1469,12 +1563,20 @@ class HipOps:
                    heads, vdim, float(lam), float(after), float(norm_eps), _dtype_code(proj.dtype), self._stream())
         return out
 
-    def head_products(self, x, x_stride, w, out=None, out_stride=None, x_at=0, out_at=0):
+    def head_products(self, x, x_stride, w, out=None, out_stride=None, x_at=0, out_at=0, gate=None):
         """y[t, h, :] = w[h] x[t, h, :] for a matrix a head, ``w`` [heads, N, K].  ``x`` is [T, columns]: the input of
         head h are the K columns from ``x_at + h * x_stride`` on; ``out`` likewise with ``out_stride`` and ``out_at``
-        (made as [T, heads * N] if not given).  Float32 sums, results in the type of x."""
+        (made as [T, heads * N] if not given).  Float32 sums, results in the type of x.  ``gate`` = (tensor [T, columns],
+        column): head h's results are multiplied by the sigmoid of that tensor's element h columns on."""
         T, ldx = x.shape
         heads, N, K = w.shape
+        gate_ptr, gate_ld = None, 0
+        if gate is not None:
+            z, z_at = gate
+            self._want(z, "heads' gates", x.dtype)
+            if z.dim() != 2 or z.shape[0] != T or z_at < 0 or z_at + heads > z.shape[1]:
+                raise KernelError("the heads' gates lie outside their rows")
+            gate_ptr, gate_ld = z.data_ptr() + z_at * z.element_size(), z.shape[1]
         self._want(x, "heads' inputs")
         self._want(w, "matrices of the heads", x.dtype)
         if x_at < 0 or x_stride < K or x_at + (heads - 1) * x_stride + K > ldx:
@@ -1488,45 +1590,71 @@ class HipOps:
         if (x.dtype == torch.bfloat16 and not self.plain_products and x_at % 4 == 0 and out_at % 4 == 0
                 and self.lib.tli_head_products_mfma_takes(N, K, ldx, x_stride, out.shape[1], out_stride)):
             self._call(self.lib.tli_head_products_mfma_bf16, x.data_ptr() + x_at * es, ldx, x_stride, w.data_ptr(),
-                       out.data_ptr() + out_at * es, out.shape[1], out_stride, T, heads, N, K, self._stream())
+                       out.data_ptr() + out_at * es, out.shape[1], out_stride, T, heads, N, K, gate_ptr, gate_ld, self._stream())
             return out
         self._call(self.lib.tli_head_products_plain, x.data_ptr() + x_at * es, ldx, x_stride, w.data_ptr(),
-                   out.data_ptr() + out_at * es, out.shape[1], out_stride, T, heads, N, K, _dtype_code(x.dtype), self._stream())
+                   out.data_ptr() + out_at * es, out.shape[1], out_stride, T, heads, N, K, gate_ptr, gate_ld, _dtype_code(x.dtype),
+                   self._stream())
         return out
 
-    def latent_attention(self, proj, step, cache, heads, dim, rot, rank, vdim, norm_weight, norm_eps, rotary, scale,
-                         w_qk, w_v, sinks=None):
-        """Attention whose keys and values are made from one latent vector a position, from the raw projections
-        ``proj`` [T, q (heads * (dim + rot)) | latent (rank) | key part (rot)] to the heads' outputs [T, heads * vdim].
+    def norm_rows(self, proj, at, n, weight, eps):
+        """weight * x / sqrt(mean(x^2) + eps) of the ``n`` columns from ``at`` on of every row of ``proj``, [T, n]."""
+        T = proj.shape[0]
+        self._want(proj, "projections")
+        self._want(weight, "norm weight", torch.float32, (n,))
+        if at < 0 or at + n > proj.shape[1]:
+            raise KernelError("the elements to norm lie outside their row")
+        out = torch.empty((T, n), dtype=proj.dtype, device=self.device)
+        self._call(self.lib.tli_norm_rows, proj.data_ptr() + at * proj.element_size(), proj.shape[1], weight.data_ptr(), out.data_ptr(),
+                   T, n, float(eps), _dtype_code(proj.dtype), self._stream())
+        return out
+
+    def latent_attention(self, query, q_at, own, step, cache, heads, dim, rot, rank, vdim, rotary, scale, w_qk, w_v, window=None,
+                         sinks=None, gate=None):
+        """Attention whose keys and values are made from one latent vector a position, from the raw queries
+        ``query[:, q_at:]`` [T, heads * (dim + rot)] to the heads' outputs [T, heads * vdim].  ``own`` = (projections, column,
+        norm weight, eps): latent (rank) | key part (rot) of the step's rows, which are normed, turned and written to the
+        cache here; None: another call of this step has written them.
         The cache (record "latent" [page, rank + rot]) keeps the normed latent vector and the turned key part; a
         head's score is q_plain . (W_uk c) + q_turned . k_turned, computed as (W_uk^T q_plain) . c with ``w_qk``
         [heads, rank, dim] = W_uk^T a head, so that all heads read the one cached vector; the weighted sum of the
-        latent vectors then goes through ``w_v`` [heads, vdim, rank] = W_uv a head.  ``sinks``: as in ``sized_attention``."""
+        latent vectors then goes through ``w_v`` [heads, vdim, rank] = W_uv a head.  ``window``, ``sinks``: as in
+        ``sized_attention``; ``gate``: one number a head, as in ``head_products``."""
         T = step.num_rows
-        width = heads * (dim + rot) + rank + rot
-        self._want(proj, "projections", None, (T, width))
-        self._want(norm_weight, "latent norm weight", torch.float32, (rank,))
-        if cache is None or not cache.writes:
-            raise KernelError("this attention writes its latent vectors into a cache layer of its own")
+        self._want(query, "queries")
+        if query.dim() != 2 or query.shape[0] != T or q_at < 0 or q_at + heads * (dim + rot) > query.shape[1]:
+            raise KernelError(f"the queries have shape {tuple(query.shape)}, expected [{T}, >= {q_at + heads * (dim + rot)}]")
+        if cache is None or cache.writes != (own is not None):
+            raise KernelError("this attention either writes latent vectors of its own or reads those of another layer")
+        es = query.element_size()
+        down_ptr, down_ld, norm_ptr, norm_eps = None, 0, None, 0.0
+        if own is not None:
+            proj, at, norm_weight, norm_eps = own
+            self._want(proj, "projections", query.dtype)
+            if proj.dim() != 2 or proj.shape[0] != T or at < 0 or at + rank + rot > proj.shape[1]:
+                raise KernelError("the latent vector lies outside the projections")
+            self._want(norm_weight, "latent norm weight", torch.float32, (rank,))
+            down_ptr, down_ld, norm_ptr = proj.data_ptr() + at * es, proj.shape[1], norm_weight.data_ptr()
         kc, g = cache.record("latent"), cache.group
         pages = kc.shape[0]
         key = rank + rot
-        self._want(kc, "latent cache", proj.dtype, (pages, g.page_size, key))
+        self._want(kc, "latent cache", query.dtype, (pages, g.page_size, key))
         self._check_tables(g, step)
         cos, sin, rd = self._rotary(rotary, step)
         if rd > rot:
             raise KernelError(f"{rd} turned elements do not fit a key part of {rot}")
-        q = torch.empty((T, heads, key), dtype=proj.dtype, device=self.device)
-        self._call(self.lib.tli_latent_prepare, proj.data_ptr(), width, q.data_ptr(), kc.data_ptr(), step.positions.data_ptr(),
+        q = torch.empty((T, heads, key), dtype=query.dtype, device=self.device)
+        self._call(self.lib.tli_latent_prepare, query.data_ptr() + q_at * es, query.shape[1], down_ptr, down_ld, q.data_ptr(),
+                   kc.data_ptr(), step.positions.data_ptr(),
                    step.seq_of_row.data_ptr(), g.tables.data_ptr(), g.table_width, g.page_size, pages, T, heads, dim, rot,
-                   rank, rd, norm_weight.data_ptr(), float(norm_eps), cos.data_ptr(), sin.data_ptr(),
-                   _dtype_code(proj.dtype), self._stream())
-        self._want(w_qk, "matrices into the latent space", proj.dtype, (heads, rank, dim))
-        self._want(w_v, "matrices out of the latent space", proj.dtype, (heads, vdim, rank))
-        self.head_products(proj, dim + rot, w_qk, out=q.view(T, heads * key), out_stride=key)
+                   rank, rd, norm_ptr, float(norm_eps), cos.data_ptr(), sin.data_ptr(),
+                   _dtype_code(query.dtype), self._stream())
+        self._want(w_qk, "matrices into the latent space", query.dtype, (heads, rank, dim))
+        self._want(w_v, "matrices out of the latent space", query.dtype, (heads, vdim, rank))
+        self.head_products(query, dim + rot, w_qk, out=q.view(T, heads * key), out_stride=key, x_at=q_at)
         o = self.sized_attention(q, step, g, kc.view(pages, 1, g.page_size, key), None, heads, 1, 1, key, rank, scale,
-                                 None, 0, proj.dtype, sinks=sinks)
-        return self.head_products(o.view(T, heads * rank), rank, w_v)
+                                 window, 0, query.dtype, sinks=sinks)
+        return self.head_products(o.view(T, heads * rank), rank, w_v, gate=gate)
 
     # ---- attention with biases and a sink whose values may be its keys ------------------------------------
     def sink_attention(self, proj, step, cache, heads, kv_heads, head_dim, bias, rotary, scale, sinks, window,
@@ -1840,6 +1968,52 @@ class HipOps:
                    step.seq_start.data_ptr(), step.slots.data_ptr(), T, step.num_seqs, int(step.max_rows_per_seq), single,
                    heads, dk, dv, _dtype_code(proj.dtype), int(self.lightning_lanes), self._stream())
         self.head_norm_gate(o, floors, weight, proj, gate_at, heads, dv, eps, "sigmoid", scale, out, out_at)
+
+    # ---- the RWKV's time mixing --------------------------------------------------------------------------------
+    def check_wkv_sizes(self, heads: int, dk: int, dv: int, rank: int) -> None:
+        if heads <= 0 or not 1 <= dk <= 256 or dv < 1 or not 1 <= rank <= 8192:
+            raise KernelError(f"time mixing with {heads} heads of keys of {dk} (1 to 256) and values of {dv}, decays through {rank}, "
+                              "is not supported")
+
+    def wkv_state_shape(self, heads: int, dk: int, dv: int):
+        """The shape of one request's recurrent state (float32): a head's matrix is kept transposed."""
+        return (heads, dv, dk)
+
+    def linear_groups(self, xs, groups):
+        """``xs`` [G + 1, T, n] and a ``GroupedMatrix`` of G matrices and one of few rows: (the G products side by side,
+        [T, sum of their rows] in the run's type, the last one's float32 sums, whether those are transposed)."""
+        count = len(groups.sizes)
+        if xs.dim() != 3 or xs.shape[0] != count + 1:
+            raise KernelError(f"{tuple(xs.shape)} are not the inputs of {count} matrices and one of few rows")
+        proj = torch.cat([self.linear(xs[i], m) for i, m in enumerate(groups.each)], dim=1)
+        return (proj,) + self.small_product(xs[count], groups.few)
+
+    def wkv(self, proj, z, transposed, w2, w0, u, state, step, heads, dk, dv, weight, eps, out_dtype):
+        """From the projections ``proj`` [T, r (H dk) | k (H dk) | v (H dv) | g (H dv)] and the decays' inner rows ``z``
+        (float32 [T, rank]; [rank, T] if ``transposed``) to the layer's rows [T, H dv]: decays d = exp(-exp(w2 tanh(z) + w0)),
+        o = (S + diag(u) k v^T)^T r, S <- diag(d) S + k v^T, then o / sqrt(mean(o^2) + eps) * weight * silu(g), the mean
+        head by head.  ``state``: float32 [slots, H, dv, dk], read (unless a sequence starts at position 0) and replaced."""
+        T = step.num_rows
+        self._recurrent_inputs(proj, 0, state, (heads, dv, dk), step, heads, dk, dv)
+        if proj.shape[1] < 2 * heads * (dk + dv):
+            raise KernelError("the gate lies outside the projections")
+        rank = z.shape[0] if transposed else z.shape[1]
+        self._want(z, "decays' inner rows", torch.float32, (rank, T) if transposed else (T, rank))
+        self._want(w2, "decays' matrix", out_dtype, (heads * dk, rank))
+        self._want(w0, "decays' bias", torch.float32, (heads * dk,))
+        self._want(u, "current token's bonus", torch.float32, (heads, dk))
+        self._want(weight, "norm weight", torch.float32, (heads * dv,))
+        out = torch.empty((T, heads * dv), dtype=out_dtype, device=self.device)
+        z_row, z_col = (1, T) if transposed else (rank, 1)
+        decay = torch.empty((T, heads * dk), dtype=torch.float32, device=self.device)
+        self._call(self.lib.tli_wkv_decays, z.data_ptr(), z_row, z_col, w2.data_ptr(), w0.data_ptr(), decay.data_ptr(), T, rank,
+                   heads * dk, _dtype_code(out_dtype), self._stream())
+        o = torch.empty((T, heads, dv), dtype=torch.float32, device=self.device)
+        self._call(self.lib.tli_wkv_rows, proj.data_ptr(), proj.shape[1], decay.data_ptr(), u.data_ptr(), state.data_ptr(), o.data_ptr(),
+                   step.row_start.data_ptr(), step.seq_start.data_ptr(), step.slots.data_ptr(), step.num_seqs, heads, dk, dv,
+                   _dtype_code(proj.dtype), self._stream())
+        self.head_norm_gate(o, None, weight, proj, 2 * heads * dk + heads * dv, heads, dv, eps, "silu", 1.0, out, 0)
+        return out
 
     OUTPUT_GATES = {"silu": 0, "sigmoid": 1}
 

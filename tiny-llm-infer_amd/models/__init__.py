@@ -5,3 +5,4 @@ from . import kapanex  # noqa: F401
 from . import gimipel  # noqa: F401
 from . import defosun  # noqa: F401
 from . import kosusun  # noqa: F401
+from . import kunitar  # noqa: F401

@@ -1,7 +1,8 @@
 """Interfaces of the parts a model is put together from, and their registries.
 
 Kinds of parts: position encoding, norm, mixer, feed-forward, block
-(arrangement), embedding, head, shift (a mix of each row with the row before it).  A part is built from a ``PartSpec`` alone: its
+(arrangement), embedding, head, shift (a mix of each row with the row before it), side (what a block adds
+behind its sublayers).  A part is built from a ``PartSpec`` alone: its
 sizes and constants are ``spec.params``, the checkpoint names of its weights
 are ``spec.names``, nested parts are ``spec.parts``.  Life cycle:
 
@@ -230,7 +231,7 @@ class Block(Part):
 
 
 _REGISTRIES: Dict[str, Dict[str, Callable[[PartSpec], Part]]] = {
-    "position": {}, "norm": {}, "mixer": {}, "ffn": {}, "block": {}, "embedding": {}, "head": {}, "shift": {},
+    "position": {}, "norm": {}, "mixer": {}, "ffn": {}, "block": {}, "embedding": {}, "head": {}, "shift": {}, "side": {},
 }
 
 

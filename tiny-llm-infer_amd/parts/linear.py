@@ -91,3 +91,23 @@ def fuse_rows(mats: Sequence[torch.Tensor], env: BuildEnv) -> Matrix:
     """Stack matrices that read the same input ([out_i, in] each) into one
     [sum out_i, in], so that one product gives all their outputs."""
     return Matrix(torch.cat([m.to(env.dtype) for m in mats], dim=0), env)
+
+
+class GroupedMatrix:
+    """Matrices [out_i, in] that read inputs of their own, one each, and a last one of few rows (``few``) whose
+    products stay in float32.  Where the sizes allow, the kernel library has them stacked so that one launch
+    multiplies them all (``stacked``: the matrices' rows one behind the other, ``few`` last); otherwise each is
+    a ``Matrix`` of its own."""
+
+    def __init__(self, mats: Sequence[torch.Tensor], env: BuildEnv, few: torch.Tensor):
+        self.sizes = [int(m.shape[0]) for m in mats]
+        self.cols = int(mats[0].shape[1])
+        self.dtype = env.dtype
+        self.few = few.to(env.dtype).contiguous()           # few rows: kept row-major
+        takes = getattr(env.ops, "stacks_groups", None)
+        self.stacked: Optional[Matrix] = None
+        self.each: Sequence[Matrix] = ()
+        if takes is not None and takes(self.sizes, self.cols, env.dtype):
+            self.stacked = fuse_rows(list(mats) + [few], env)
+        else:
+            self.each = [as_matrix(m, env) for m in mats]

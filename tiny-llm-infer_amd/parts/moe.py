@@ -15,6 +15,9 @@ beside an optional shared one that every row uses.
     ``activation`` "limited": an expert's hidden units are g * sigmoid(slope * g) * (u + 1) with
         g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit)  (``limit``, ``gate_slope``; the shared
         expert with ``shared_limit``)
+    ``gated`` false: experts without a gate matrix, expert(h) = W_down act(W_up h), ``activation`` one of the kernel
+        library's; the shared expert likewise
+    ``weight_on`` "input" (experts without a gate): out = sum_j expert_j(weight_j h) + ..
 
 The router's product gives float32 (the row of the shared expert's gate rides along as one more
 row of that matrix); scores, choice and weights are float32.  A row's chosen experts are added
@@ -55,7 +58,11 @@ class RoutedExperts(FeedForward):
                 or not 1 <= self.top <= self.keep * (self.outputs // self.groups):
             raise ValueError(f"{self.outputs} router outputs in {self.groups} groups, {self.keep} kept, cannot give {self.top}")
         self.activation = str(p.get("activation", "silu"))
-        if self.activation not in ("silu", "limited"):
+        self.gated = bool(p.get("gated", True))
+        self.weight_on = str(p.get("weight_on", "output"))
+        if self.weight_on not in ("output", "input") or (self.weight_on == "input" and (self.gated or self.identity)):
+            raise ValueError("an expert's weight goes on its output, or, where experts have no gate and matrices all, on its input")
+        if self.gated and self.activation not in ("silu", "limited"):
             raise ValueError(f"activation '{self.activation}' is not known; known: silu, limited")
         self.limit = float(p.get("limit", 0.0)) if self.activation == "limited" else 0.0
         self.shared_limit = float(p.get("shared_limit", self.limit)) if self.activation == "limited" else 0.0
@@ -74,12 +81,12 @@ class RoutedExperts(FeedForward):
         if self.correction_name is not None:
             out.append(TensorDecl(self.correction_name, (self.outputs,)))
         for j in range(self.experts):
-            out += [TensorDecl(self._expert(j, "gate"), (self.inter, self.hidden)),
-                    TensorDecl(self._expert(j, "up"), (self.inter, self.hidden)),
-                    TensorDecl(self._expert(j, "down"), (self.hidden, self.inter))]
+            out += ([TensorDecl(self._expert(j, "gate"), (self.inter, self.hidden))] if self.gated else []) + \
+                [TensorDecl(self._expert(j, "up"), (self.inter, self.hidden)),
+                 TensorDecl(self._expert(j, "down"), (self.hidden, self.inter))]
         if self.shared_inter is not None:
-            out += [TensorDecl(n["shared_gate"], (self.shared_inter, self.hidden)),
-                    TensorDecl(n["shared_up"], (self.shared_inter, self.hidden)),
+            out += ([TensorDecl(n["shared_gate"], (self.shared_inter, self.hidden))] if self.gated else []) + \
+                   [TensorDecl(n["shared_up"], (self.shared_inter, self.hidden)),
                     TensorDecl(n["shared_down"], (self.hidden, self.shared_inter))]
             if self.shared_gated:
                 out.append(TensorDecl(n["shared_scale"], (1, self.hidden)))
@@ -97,18 +104,24 @@ class RoutedExperts(FeedForward):
         if self.correction_name is not None:
             self.correction = weights[self.correction_name].to(torch.float32).contiguous()
         self.w_router = torch.cat([r.to(env.dtype) for r in rows], dim=0).contiguous()       # few rows: kept row-major
-        # the experts' matrices side by side: [E, 2 ff, hidden] (an expert's gate rows, then its up rows), [E, hidden, ff]
-        self.w_gate_up = torch.stack([torch.cat([weights[self._expert(j, "gate")], weights[self._expert(j, "up")]], dim=0)
+        if not self.gated:
+            env.ops.check_activation(self.activation)
+        # the experts' matrices side by side: [E, 2 ff, hidden] (an expert's gate rows, then its up rows) or [E, ff, hidden]
+        # (without a gate), [E, hidden, ff]
+        roles = ("gate", "up") if self.gated else ("up",)
+        self.w_gate_up = torch.stack([torch.cat([weights[self._expert(j, r)] for r in roles], dim=0)
                                       for j in range(self.experts)]).to(env.dtype).contiguous()
         self.w_down = torch.stack([weights[self._expert(j, "down")] for j in range(self.experts)]).to(env.dtype).contiguous()
         # (where the kernels for the matrix cores apply they read a layout of their own, and the row-major
         # matrices are not kept beside it)
-        self.packed = env.ops.pack_experts(self.w_gate_up, self.w_down)
+        self.packed = env.ops.pack_experts(self.w_gate_up, self.w_down, **({} if self.gated else {"gated": False}))
         if self.packed is not None:
             self.w_gate_up = self.w_down = None
         self.shared_gate_up = self.shared_down = None
         if self.shared_inter is not None:
-            if self.activation == "silu":
+            if not self.gated:
+                self.shared_gate_up = as_matrix(weights[n["shared_up"]], env)
+            elif self.activation == "silu":
                 self.shared_gate_up = GatedMatrix(weights[n["shared_gate"]], weights[n["shared_up"]], env)
             else:       # (the products' own epilogue is silu(gate) * up: gate and up rows stacked, the activation in a pass of its own)
                 self.shared_gate_up = fuse_rows([weights[n["shared_gate"]], weights[n["shared_up"]]], env)
@@ -127,12 +140,16 @@ class RoutedExperts(FeedForward):
                                                       self.has_gate, transposed, **how)
         shared = None
         if self.shared_inter is not None:
-            if self.activation == "silu":
+            if not self.gated:
+                hidden = ops.activation(ops.linear(x, self.shared_gate_up), self.activation)
+            elif self.activation == "silu":
                 hidden = ops.linear_swiglu(x, self.shared_gate_up)
             else:
                 hidden = ops.swiglu(ops.linear(x, self.shared_gate_up), limit=self.shared_limit, slope=self.slope)
             shared = ops.linear(hidden, self.shared_down)
         how = {} if self.activation == "silu" else {"limit": self.limit, "slope": self.slope}
+        if not self.gated:
+            how = {"activation": self.activation, "weight_on_input": self.weight_on == "input"}
         return ops.apply_experts(x, ids, weights, self.w_gate_up, self.w_down, self.packed, shared, shared_gate, **how)
 
 

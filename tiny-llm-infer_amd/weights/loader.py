@@ -24,6 +24,10 @@ import torch
 from .safetensors_io import Checkpoint, write_safetensors
 
 
+class AnySize(int):
+    """A size of a declared shape that the checkpoint says: its value is what random weights take."""
+
+
 @dataclass(frozen=True)
 class TensorDecl:
     name: str
@@ -76,7 +80,7 @@ def check_against(decls: Sequence[TensorDecl], checkpoint: Checkpoint) -> None:
             missing.append(d.name)
             continue
         got = tuple(checkpoint.shape(d.name))
-        if got != tuple(d.shape):
+        if len(got) != len(d.shape) or any(g != w if not isinstance(w, AnySize) else g < 1 for g, w in zip(got, d.shape)):
             wrong.append((d.name, got, tuple(d.shape)))
         dt = checkpoint.dtype(d.name)
         if d.init == "int":
