@@ -66,14 +66,14 @@ DESIGN_SIZES = {
 
 
 def compare_designs(args):
-    """Prefill and decode of the Sinepel design (or, with --design-names, of others: Kapanex, Gimipel, Defosun, Kosusun) beside the Qwen3
+    """Prefill and decode of the Sinepel design (or, with --design-names, of others: Kapanex, Gimipel, Defosun, Kosusun, Kunitar) beside the Qwen3
     dense decoder at equal layer sizes
     (random bfloat16 weights, 4 layers unless --layers says otherwise), through the step function:
     one prompt of --prefill-tokens in one step, and decode steps of --batch and 64 requests at
     --prompt-len tokens of context.  One JSON line."""
     import torch
 
-    from tiny_llm_infer_amd.config import DefosunConfig, GimipelConfig, KapanexConfig, KosusunConfig, Qwen3Config, SinepelConfig
+    from tiny_llm_infer_amd.config import DefosunConfig, GimipelConfig, KapanexConfig, KosusunConfig, KunitarConfig, Qwen3Config, SinepelConfig
     from tiny_llm_infer_amd.engine.loading import random_model
     from tiny_llm_infer_amd.engine.runner import ModelRunner, StepEntry
     import random
@@ -156,7 +156,22 @@ def compare_designs(args):
             "architecture": "Kosusun", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "max_positions": context,
             "embedding": {"scale": 1.0}, "residual_mult": 1.0, "logit_scale": 1.0,
             "layers": [{"type": kmixers[i % 2][0], "mixer": kmixers[i % 2][1], "mlp": {"kind": "dense", "ff": ff}} for i in range(layers)]})
-        known = {"kosusun": ("Kosusun", kosusun), "sinepel": ("Sinepel", sinepel), "kapanex": ("Kapanex", kapanex), "gimipel": ("Gimipel", gimipel),
+        # Kunitar: time mixing (heads as Qwen3's, a state of dim x dim a head) and latent attention (as Gimipel's, over a window
+        # of 1,024, its queries through a latent of half the width) in turn, the second latent layer reading the first one's
+        # vectors; the first layer with the dense feed-forward, the others with 16 experts (without a gate) of a quarter of
+        # its size of which 2 are chosen, beside a shared expert of half of it; a vector of an eighth of the width a token
+        # and layer
+        umoe = {"kind": "moe", "expert": {"ff": ff // 4}, "shared": {"ff": ff // 2}, "router": {"experts": 16, "top": 2}}
+        ulatent = {"heads": heads, "dim": dim, "rot_dim": dim // 2, "vdim": dim, "kv_rank": 4 * dim, "q_rank": width // 2,
+                   "scale": (dim + dim // 2) ** -0.5, "mask": {"size": 1024}, "rot": {"dims": dim // 2, "base": 1e6}}
+        kunitar = KunitarConfig.from_dict({
+            "architecture": "Kunitar", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "max_positions": context,
+            "embedding": {"scale": 1.0}, "token_side": {"dim": width // 8},
+            "layers": [{"type": "wkv", "mixer": {"heads": heads, "dim": dim}, "mlp": umoe if i else {"kind": "dense", "ff": ff}}
+                       if i % 2 == 0 else
+                       {"type": "latent_attention", "mixer": ulatent if i == 1 else dict(ulatent, kv_from=1), "mlp": umoe}
+                       for i in range(layers)]})
+        known = {"kunitar": ("Kunitar", kunitar), "kosusun": ("Kosusun", kosusun), "sinepel": ("Sinepel", sinepel), "kapanex": ("Kapanex", kapanex), "gimipel": ("Gimipel", gimipel),
                  "defosun": ("Defosun", defosun), "qwen3": ("Qwen3ForCausalLM", qwen)}
         names = [n for n in args.design_names.split(",") if n]
         if any(n not in known for n in names):
@@ -238,7 +253,7 @@ def main():
                     help="instead of the default workload: the Sinepel design beside the Qwen3 dense decoder at equal layer "
                          f"sizes, prefill and decode; a list of {','.join(DESIGN_SIZES)} or 'all'")
     ap.add_argument("--design-names", default="sinepel,qwen3",
-                    help="with --designs: which designs are run at every size (sinepel, kapanex, gimipel, defosun, kosusun, qwen3)")
+                    help="with --designs: which designs are run at every size (sinepel, kapanex, gimipel, defosun, kosusun, kunitar, qwen3)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py runs on one GPU only; --gpus {args.gpus} is not supported (single-GPU engine)")

@@ -308,8 +308,9 @@ class CpuOps:
     def wkv_state_shape(self, heads, dk, dv):
         return (heads, dv, dk)
 
-    def linear_groups(self, xs, groups):
-        return (torch.cat([self.linear(x, m) for x, m in zip(xs, groups.each)], dim=1),) + self.small_product(xs[len(groups.each)], groups.few)
+    def linear_groups(self, xs, groups, step=None):
+        z, transposed = self.small_product(xs[len(groups.each)], groups.few)
+        return torch.cat([self.linear(x, m) for x, m in zip(xs, groups.each)], dim=1), z, transposed
 
     def wkv(self, proj, z, transposed, w2, w0, u, state, step, heads, dk, dv, weight, eps, out_dtype):
         T = step.num_rows

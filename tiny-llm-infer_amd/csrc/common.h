@@ -135,6 +135,14 @@ static inline const char* gate_out_fault(const GateOut& g, int cols) {
     return nullptr;
 }
 
+// Several matrices stacked in one whose products read inputs of their own: columns n of the output belong to input
+// n / every, inputs lie `step` elements apart.  every 0: one input.  (A workgroup's columns belong to one input.)
+struct InputGroups {
+    int every;
+    long long step;
+    __device__ __forceinline__ long long at(int n) const { return every > 0 ? (long long)(n / every) * step : 0; }
+};
+
 // Makes LDS writes of this wavefront's lanes visible to its other lanes.
 __device__ __forceinline__ void wave_lds_sync() {
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");

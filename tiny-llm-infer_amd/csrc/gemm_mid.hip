@@ -46,7 +46,7 @@ union Pack16m {
 template <int RT, int WAVES, int DEPTH, int MT, typename TO, bool GATED>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* __restrict__ y,
-                float* __restrict__ part, int M_all, int N, int K, int splits, int steps_per_split, GateOut gate) {
+                float* __restrict__ part, int M_all, int N, int K, int splits, int steps_per_split, GateOut gate, InputGroups inputs) {
     constexpr int ROWS = MT * 16;
     constexpr int STAGES = DEPTH + 1;                        // W: DEPTH slices on their way, one in use
     constexpr int XSLOTS = DEPTH + 2;                        // x: one slice further ahead
@@ -70,7 +70,7 @@ gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* 
         if (group * WAVES * RT >= n_tiles) return;            // (the column groups are rounded up to a multiple of 8)
     }
     const int M = min(ROWS, M_all - row0);
-    x += (size_t)row0 * K;
+    x += (size_t)row0 * K + inputs.at(group * WAVES * RT * 16);
     const int tile0 = (group * WAVES + wave) * RT;            // this wave's first 16-column tile
     const int step_begin = blockIdx.y * steps_per_split;
     const int step_end = min(k_steps, step_begin + steps_per_split);
@@ -268,7 +268,7 @@ gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* 
 
 template <int RT, int WAVES, int DEPTH, int MT>
 static int launch_mid_rows(const bf16_t* x, const bf16_t* w, void* y, float* part, int M, int N, int K,
-                           int y_dtype, GateOut gated, int splits, hipStream_t s) {
+                           int y_dtype, GateOut gated, const InputGroups& inputs, int splits, hipStream_t s) {
     const int n_tiles = (N + 15) / 16, k_steps = (K + 127) / 128;
     const int steps_per_split = (k_steps + splits - 1) / splits;
     const int groups = (n_tiles + RT * WAVES - 1) / (RT * WAVES), row_blocks = (M + MT * 16 - 1) / (MT * 16);
@@ -285,7 +285,7 @@ static int launch_mid_rows(const bf16_t* x, const bf16_t* w, void* y, float* par
                 return tli_fail("gemm_mid: cannot have %zu bytes of LDS", lds);                            \
             allowed = true;                                                                                \
         }                                                                                                  \
-        kernel<<<grid, WAVES * 64, lds, s>>>(x, w, (TO*)y, part, M, N, K, splits, steps_per_split, gated); \
+        kernel<<<grid, WAVES * 64, lds, s>>>(x, w, (TO*)y, part, M, N, K, splits, steps_per_split, gated, inputs); \
     }
     if (gated) MID_LAUNCH(bf16_t, true)
     else if (y_dtype == TLI_BF16) MID_LAUNCH(bf16_t, false)
@@ -303,10 +303,10 @@ static int launch_mid_rows(const bf16_t* x, const bf16_t* w, void* y, float* par
 // Four 16-row tiles of x up to 64 rows, eight beyond.
 template <int RT, int WAVES, int DEPTH>
 static int launch_mid(const bf16_t* x, const bf16_t* w, void* y, float* part, int M, int N, int K,
-                      int y_dtype, GateOut gated, int splits, hipStream_t s) {
-    if (M <= 64) return launch_mid_rows<RT, WAVES, DEPTH, 4>(x, w, y, part, M, N, K, y_dtype, gated, splits, s);
+                      int y_dtype, GateOut gated, const InputGroups& inputs, int splits, hipStream_t s) {
+    if (M <= 64) return launch_mid_rows<RT, WAVES, DEPTH, 4>(x, w, y, part, M, N, K, y_dtype, gated, inputs, splits, s);
     if constexpr (DEPTH <= 3)       // (DEPTH + 2) slices of 32 KiB fit the 160 KiB of LDS
-        return launch_mid_rows<RT, WAVES, DEPTH, 8>(x, w, y, part, M, N, K, y_dtype, gated, splits, s);
+        return launch_mid_rows<RT, WAVES, DEPTH, 8>(x, w, y, part, M, N, K, y_dtype, gated, inputs, splits, s);
     else
         return tli_fail("gemm_mid: more than 64 rows leave LDS for at most 3 slices on their way");
 }
@@ -397,16 +397,8 @@ extern "C" int tli_gemm_mid_splits_rows(int M, int N, int K, int gated) {
     return splits;
 }
 
-// y[M,N] = x[M,K] . W^T for 1 <= M <= 256 (a gated product: 128), W in the decode layout (`gated` as tiled = 2 of
-// tli_gemm_skinny_bf16: y is [M, N/2] bfloat16).  `part`: splits*M*N floats when
-// splits > 1 (splits as returned by tli_gemm_mid_splits, or forced by the caller); with
-// y null the partial sums [splits][M][N] are left for the consumer to add (tli_gemm_mid_reduce,
-// or tli_add_rmsnorm);
-// cfg 0 picks the launch shape, else DEPTH*100 + RT*10 + WAVES.  act, act_scale, y_ld: the output of a gated product
-// (common.h's GateOut; y_ld 0: N/2).
-extern "C" int tli_gemm_mid_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K,
-                                 int y_dtype, int is_gated, int splits, int cfg, int act, float act_scale, int y_ld,
-                                 void* stream) {
+static int gemm_mid(const void* x, const void* w, void* y, float* part, int M, int N, int K, int y_dtype, int is_gated, int splits,
+                    int cfg, int act, float act_scale, int y_ld, const InputGroups& inputs, void* stream) {
     const GateOut gated = gate_out(is_gated, act, act_scale, y_ld, N / 2);
     if (const char* fault = gate_out_fault(gated, N / 2)) return tli_fail("gemm_mid: %s", fault);
     if (M <= 0 || N <= 0) return 0;
@@ -437,13 +429,34 @@ extern "C" int tli_gemm_mid_bf16(const void* x, const void* w, void* y, float* p
         cfg = 200 + 10 * rt + waves;
     }
     if (gated && (cfg / 10) % 10 < 2) return tli_fail("gemm_mid: a gated product needs pairs of row tiles");
-#define MID_CASE(D, R, W) case D * 100 + R * 10 + W: return launch_mid<R, W, D>(xp, wp, y, part, M, N, K, y_dtype, gated, splits, s);
+#define MID_CASE(D, R, W) case D * 100 + R * 10 + W: return launch_mid<R, W, D>(xp, wp, y, part, M, N, K, y_dtype, gated, inputs, splits, s);
     switch (cfg) {
         MID_CASE(2, 1, 4) MID_CASE(3, 1, 4) MID_CASE(2, 1, 8) MID_CASE(4, 1, 8)
         MID_CASE(2, 2, 4) MID_CASE(4, 2, 4) MID_CASE(2, 2, 8)
         MID_CASE(2, 2, 3) MID_CASE(2, 2, 5) MID_CASE(2, 2, 6) MID_CASE(2, 2, 7)
         default: return tli_fail("gemm_mid: unknown configuration %d", cfg);
     }
+}
+
+// y[M,N] = x[M,K] . W^T for 1 <= M <= 256 (a gated product: 128), W in the decode layout (`gated` as tiled = 2 of
+// tli_gemm_skinny_bf16: y is [M, N/2] bfloat16).  `part`: splits*M*N floats when
+// splits > 1 (splits as returned by tli_gemm_mid_splits, or forced by the caller); with
+// y null the partial sums [splits][M][N] are left for the consumer to add (tli_gemm_mid_reduce,
+// or tli_add_rmsnorm);
+// cfg 0 picks the launch shape, else DEPTH*100 + RT*10 + WAVES.  act, act_scale, y_ld: the output of a gated product
+// (common.h's GateOut; y_ld 0: N/2).
+extern "C" int tli_gemm_mid_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K,
+                                 int y_dtype, int is_gated, int splits, int cfg, int act, float act_scale, int y_ld,
+                                 void* stream) {
+    return gemm_mid(x, w, y, part, M, N, K, y_dtype, is_gated, splits, cfg, act, act_scale, y_ld, InputGroups{0, 0}, stream);
+}
+
+// The same, without a gate and for up to 128 rows, of stacked matrices whose inputs differ (common.h's InputGroups; every in
+// 128s: up to eight column tiles a workgroup).
+extern "C" int tli_gemm_mid_groups_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K, int y_dtype, int splits,
+                                        int every, long long step, void* stream) {
+    if (M > 128 || every <= 0 || every % 128 || step < (long long)M * K || step % 8) return tli_fail("gemm_mid: bad input groups");
+    return gemm_mid(x, w, y, part, M, N, K, y_dtype, 0, splits, 0, 0, 1.0f, 0, InputGroups{every, step}, stream);
 }
 
 // y[M,N] = sum over the partial products in `part` [splits][M][N], in split order.

@@ -76,7 +76,7 @@ __device__ __forceinline__ void rows_wait_fragments(Pack16r (&a)[RT][4], int j) 
 template <int RT, int WAVES, int MT, int MH, bool GATED, int KG = 1>
 __global__ void __launch_bounds__(WAVES * KG * 64, WAVES * KG == 4 ? 2 : 1)
 gemm_rows_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf16_t* __restrict__ y,
-                 float* __restrict__ part, int M, int N, int K, int splits, int slices_per_split, GateOut out) {
+                 float* __restrict__ part, int M, int N, int K, int splits, int slices_per_split, GateOut out, InputGroups inputs) {
     constexpr int ROWS = MT * 16;
     constexpr int SLICE = ROWS * 128;                        // elements of a slice of x
     constexpr int XI = ROWS / (4 * WAVES);                   // copies a wave issues for a slice (64 x 16 bytes each)
@@ -121,7 +121,7 @@ gemm_rows_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf1
         row_block = chunk * CHUNK + at % chunk_rows;
         col_group = whole * TLI_DIES + at / chunk_rows;
     }
-    x += (size_t)row_block * ROWS * K;
+    x += (size_t)row_block * ROWS * K + inputs.at(col_group * WAVES * RT * 16);
     const int n_out = GATED ? N / 2 : N;
     y += (size_t)row_block * ROWS * (GATED ? out.ld : N);
     // with splits > 1 the workgroup walks one of `splits` ranges of k and leaves float32 partial sums
@@ -374,7 +374,7 @@ gemm_rows_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, bf1
 
 template <int RT, int WAVES, int MT, int MH, int KG = 1>
 static int launch_rows(const bf16_t* x, const bf16_t* w, bf16_t* y, float* part, int M, int N, int K, GateOut gated,
-                       int splits, hipStream_t s) {
+                       const InputGroups& inputs, int splits, hipStream_t s) {
     const int n_tiles = (N + 15) / 16, k_steps = (K + 127) / 128;
     const long col_groups = (n_tiles + RT * WAVES - 1) / (RT * WAVES), row_blocks = (M + MT * 16 - 1) / (MT * 16);
     const long chunk = 2048 / (MT * 16);                     // as the kernel deals the row blocks out
@@ -397,7 +397,7 @@ static int launch_rows(const bf16_t* x, const bf16_t* w, bf16_t* y, float* part,
                 return tli_fail("gemm_rows: cannot have %zu bytes of LDS", lds);                           \
             allowed = true;                                                                                \
         }                                                                                                  \
-        kernel<<<grid, WAVES * KG * 64, lds, s>>>(x, w, y, part, M, N, K, splits, slices_per_split, gated); \
+        kernel<<<grid, WAVES * KG * 64, lds, s>>>(x, w, y, part, M, N, K, splits, slices_per_split, gated, inputs); \
     }
     if (gated) ROWS_LAUNCH(true)
     else ROWS_LAUNCH(false)
@@ -465,20 +465,8 @@ static int rows_pick(int M, int N, int K, int splits, int gated) {
     return best;
 }
 
-// y[M,N] = x[M,K] . W^T for any number of rows, bfloat16, W in the decode layout (`gated` as
-// tiled = 2 of tli_gemm_skinny_bf16: N counts gate and up, y is [M, N/2]).  `part`: splits*M*N
-// floats when splits > 1 (splits as returned by tli_gemm_rows_splits, or forced by the
-// caller); with y null the partial sums [splits][M][N] are left for the consumer to add
-// (tli_gemm_mid_reduce, or tli_add_rmsnorm).
-// cfg 0 picks the launch shape; 1: 256 x 256 outputs a workgroup of eight waves, 2: 128 x 256
-// and four waves, two workgroups a compute unit, 3: 128 x 512 and eight waves, 4: 128 x 192 and
-// four waves, 5: 128 x 384 and eight waves (in a gated product the waves of 4 and 5, which hold three
-// column tiles each, exchange the sums of one tile in pairs), 6: 128 x 256
-// by two sets of four waves that take the slices of k in turn; cfg >= 10: the tens for a gated product, the
-// ones for the others (measurements).  act, act_scale, y_ld: the output of a gated product (common.h's GateOut; y_ld
-// 0: N/2).
-extern "C" int tli_gemm_rows_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K,
-                                  int is_gated, int splits, int cfg, int act, float act_scale, int y_ld, void* stream) {
+static int gemm_rows(const void* x, const void* w, void* y, float* part, int M, int N, int K, int is_gated, int splits, int cfg, int act,
+                     float act_scale, int y_ld, const InputGroups& inputs, void* stream) {
     const GateOut gated = gate_out(is_gated, act, act_scale, y_ld, N / 2);
     if (const char* fault = gate_out_fault(gated, N / 2)) return tli_fail("gemm_rows: %s", fault);
     if (M <= 0 || N <= 0) return 0;
@@ -494,20 +482,49 @@ extern "C" int tli_gemm_rows_bf16(const void* x, const void* w, void* y, float* 
         return tli_fail("gemm_rows: an operand of 4 GiB or more (offsets are 32 bits)");
     if (cfg >= 10) cfg = gated ? cfg / 10 : cfg % 10;       // measurements: one shape for the gated product, one for the others
     if (cfg == 0) cfg = rows_pick(M, N, K, splits, gated);
-    if (cfg == 1) return launch_rows<2, 8, 16, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, splits, s);
-    if (cfg == 2) return launch_rows<4, 4, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, splits, s);
-    if (cfg == 3) return launch_rows<4, 8, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, splits, s);
+    if (cfg == 1) return launch_rows<2, 8, 16, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, inputs, splits, s);
+    if (cfg == 2) return launch_rows<4, 4, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, inputs, splits, s);
+    if (cfg == 3) return launch_rows<4, 8, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, inputs, splits, s);
     if (cfg == 6) {
         const int k_steps = (K + 127) / 128, per = (k_steps + splits - 1) / splits;
         if (per % 2 || k_steps % per) cfg = 2;       // (an odd number of slices somewhere: one set of waves)
-        else return launch_rows<4, 4, 8, 1, 2>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, splits, s);
+        else return launch_rows<4, 4, 8, 1, 2>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, inputs, splits, s);
     }
-    if (cfg == 2) return launch_rows<4, 4, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, splits, s);
+    if (cfg == 2) return launch_rows<4, 4, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, inputs, splits, s);
     if (cfg == 4) {
-        return launch_rows<3, 4, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, splits, s);
+        return launch_rows<3, 4, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, inputs, splits, s);
     }
     if (cfg == 5) {
-        return launch_rows<3, 8, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, splits, s);
+        return launch_rows<3, 8, 8, 1>((const bf16_t*)x, (const bf16_t*)w, (bf16_t*)y, part, M, N, K, gated, inputs, splits, s);
     }
     return tli_fail("gemm_rows: unknown configuration %d", cfg);
+}
+
+// y[M,N] = x[M,K] . W^T for any number of rows, bfloat16, W in the decode layout (`gated` as
+// tiled = 2 of tli_gemm_skinny_bf16: N counts gate and up, y is [M, N/2]).  `part`: splits*M*N
+// floats when splits > 1 (splits as returned by tli_gemm_rows_splits, or forced by the
+// caller); with y null the partial sums [splits][M][N] are left for the consumer to add
+// (tli_gemm_mid_reduce, or tli_add_rmsnorm).
+// cfg 0 picks the launch shape; 1: 256 x 256 outputs a workgroup of eight waves, 2: 128 x 256
+// and four waves, two workgroups a compute unit, 3: 128 x 512 and eight waves, 4: 128 x 192 and
+// four waves, 5: 128 x 384 and eight waves (in a gated product the waves of 4 and 5, which hold three
+// column tiles each, exchange the sums of one tile in pairs), 6: 128 x 256
+// by two sets of four waves that take the slices of k in turn; cfg >= 10: the tens for a gated product, the
+// ones for the others (measurements).  act, act_scale, y_ld: the output of a gated product (common.h's GateOut; y_ld
+// 0: N/2).
+extern "C" int tli_gemm_rows_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K,
+                                  int is_gated, int splits, int cfg, int act, float act_scale, int y_ld, void* stream) {
+    return gemm_rows(x, w, y, part, M, N, K, is_gated, splits, cfg, act, act_scale, y_ld, InputGroups{0, 0}, stream);
+}
+
+// The same, without a gate, of stacked matrices whose inputs differ (common.h's InputGroups; every in 256s): 128 x 512 outputs
+// a workgroup where `every` is in 512s and that fills the chip, else 128 x 256, by two sets of waves where the slices of k are
+// even in number and one workgroup a compute unit is all there is.
+extern "C" int tli_gemm_rows_groups_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K, int splits, int every,
+                                         long long step, void* stream) {
+    if (every <= 0 || every % 256 || step < (long long)M * K || step % 8) return tli_fail("gemm_rows: bad input groups");
+    const long wgs = (long)((N + 255) / 256) * ((M + 127) / 128) * splits, units = tli_compute_units();
+    const int k_steps = (K + 127) / 128, per = (k_steps + splits - 1) / splits;
+    const int cfg = every % 512 == 0 && wgs >= 3 * units ? 3 : (wgs <= units || wgs > 2 * units) && per % 2 == 0 && k_steps % per == 0 ? 6 : 2;
+    return gemm_rows(x, w, y, part, M, N, K, 0, splits, cfg, 0, 1.0f, 0, InputGroups{every, step}, stream);
 }

@@ -73,6 +73,7 @@ struct SkinnyFuse {
     bf16_t* xw;               // [M][N] bfloat16(norm_w * resid)
     float* ssq_out;           // [ceil(N/16)][M]
     GateOut gate;             // of a gated matrix
+    InputGroups inputs;
 };
 
 template <int RT, int MT, int WAVES, typename TO, bool TILED = false, bool GATED = false, int DEPTH = 2,
@@ -84,6 +85,7 @@ gemm_skinny_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, T
     const int lane = threadIdx.x % 64, wave = threadIdx.x / 64;
     const int r = lane % 16, c = lane / 16;
     const int n_base = blockIdx.x * (16 * RT);
+    if constexpr (FUSE == FUSE_NONE && TILED && !GATED) x += fuse.inputs.at(n_base);
 
     f32x4 acc[RT][MT];
 #pragma unroll
@@ -326,18 +328,19 @@ gemm_skinny_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, T
 
 template <int RT, int MT, int WAVES>
 static int launch_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N, int K, int y_dtype,
-                         int tiled, const GateOut& gate, hipStream_t s) {
+                         int tiled, const GateOut& gate, const InputGroups& inputs, hipStream_t s) {
     SkinnyFuse plain{};
     plain.gate = gate;
+    plain.inputs = inputs;
     const int blocks = (N + 16 * RT - 1) / (16 * RT);
     constexpr int D = (MT == 1 && RT <= 2) ? PIPE_DEPTH : 2;    // deep prefetch where the registers allow
     if (tiled == 2) {       // gated: pairs of row tiles, silu(gate)*up written as bfloat16
         gemm_skinny_kernel<RT, MT, WAVES, bf16_t, true, true, D><<<blocks, WAVES * 64, 0, s>>>(x, w, (bf16_t*)y, M, N, K, plain);
     } else if (tiled) {
         if (y_dtype == TLI_BF16)
-            gemm_skinny_kernel<RT, MT, WAVES, bf16_t, true, false, D><<<blocks, WAVES * 64, 0, s>>>(x, w, (bf16_t*)y, M, N, K, SkinnyFuse{});
+            gemm_skinny_kernel<RT, MT, WAVES, bf16_t, true, false, D><<<blocks, WAVES * 64, 0, s>>>(x, w, (bf16_t*)y, M, N, K, plain);
         else
-            gemm_skinny_kernel<RT, MT, WAVES, float, true, false, D><<<blocks, WAVES * 64, 0, s>>>(x, w, (float*)y, M, N, K, SkinnyFuse{});
+            gemm_skinny_kernel<RT, MT, WAVES, float, true, false, D><<<blocks, WAVES * 64, 0, s>>>(x, w, (float*)y, M, N, K, plain);
     } else {
         if (y_dtype == TLI_BF16)
             gemm_skinny_kernel<RT, MT, WAVES, bf16_t, false><<<blocks, WAVES * 64, 0, s>>>(x, w, (bf16_t*)y, M, N, K, SkinnyFuse{});
@@ -349,32 +352,23 @@ static int launch_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N
 
 template <int MT>
 static int pick_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N, int K, int y_dtype,
-                       int tiled, const GateOut& gate, hipStream_t s, int cfg) {
+                       int tiled, const GateOut& gate, const InputGroups& inputs, hipStream_t s, int cfg) {
     // cfg 0: by shape.  Narrow outputs get one 16-column tile per workgroup so that
     // even N = 4096 gives 256 workgroups; wide outputs share x over two tiles.
     const long tiles = (N + 15) / 16;
     if (cfg == 0) cfg = tiles <= tli_compute_units() ? 18 : (tiles < 4 * tli_compute_units() ? 28 : 24);
     if (tiled == 2 && cfg < 20) cfg = 24;          // gated needs pairs of row tiles
     switch (cfg) {
-        case 14: return launch_skinny<1, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, s);
-        case 18: return launch_skinny<1, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, s);
-        case 24: return launch_skinny<2, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, s);
-        case 28: return launch_skinny<2, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, s);
+        case 14: return launch_skinny<1, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, s);
+        case 18: return launch_skinny<1, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, s);
+        case 24: return launch_skinny<2, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, s);
+        case 28: return launch_skinny<2, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, s);
         default: return tli_fail("gemm_skinny: unknown configuration %d", cfg);
     }
 }
 
-// y[M,N] = x[M,K] . W^T.  `tiled` = 0: w is W[N,K] row-major.  `tiled` = 1: w is the
-// same matrix in blocks of 16 rows x 128 columns, zero-padded to whole blocks, stored
-// [row block][column block][j = 0..3][lane = 16*c + r][8] with element
-// W[16*row block + r][128*column block + 32*c + 8*j + e]: every load instruction of
-// a wave then reads 1 KiB in a row.  `tiled` = 2: tiled, and the 16-row blocks alternate
-// between a gate matrix and an up matrix (block 2t: gate rows 16t.., block 2t+1: up rows
-// 16t..); N counts both, y is [M, N/2] bfloat16 = silu(x.gate^T) * (x.up^T).  cfg 0 picks the launch shape; other values
-// (row tiles * 10 + waves) force one, for measurements.  act, act_scale, y_ld: the output of a gated product (common.h's
-// GateOut: another activation than the silu, a factor, rows y_ld elements apart; y_ld 0: N/2).
-extern "C" int tli_gemm_skinny_bf16(const void* x, const void* w, void* y, int M, int N, int K,
-                                    int y_dtype, int tiled, int cfg, int act, float act_scale, int y_ld, void* stream) {
+static int skinny(const void* x, const void* w, void* y, int M, int N, int K, int y_dtype, int tiled, int cfg, int act,
+                  float act_scale, int y_ld, const InputGroups& inputs, void* stream) {
     const GateOut gate = gate_out(tiled == 2, act, act_scale, y_ld, N / 2);
     if (const char* fault = gate_out_fault(gate, N / 2)) return tli_fail("gemm_skinny: %s", fault);
     if (M <= 0 || N <= 0) return 0;
@@ -389,11 +383,32 @@ extern "C" int tli_gemm_skinny_bf16(const void* x, const void* w, void* y, int M
     const bf16_t* xp = (const bf16_t*)x;
     const bf16_t* wp = (const bf16_t*)w;
     switch ((M + 15) / 16) {
-        case 1: return pick_skinny<1>(xp, wp, y, M, N, K, y_dtype, tiled, gate, s, cfg);
-        case 2: return pick_skinny<2>(xp, wp, y, M, N, K, y_dtype, tiled, gate, s, cfg);
-        case 3: return pick_skinny<3>(xp, wp, y, M, N, K, y_dtype, tiled, gate, s, cfg);
-        default: return pick_skinny<4>(xp, wp, y, M, N, K, y_dtype, tiled, gate, s, cfg);
+        case 1: return pick_skinny<1>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, s, cfg);
+        case 2: return pick_skinny<2>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, s, cfg);
+        case 3: return pick_skinny<3>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, s, cfg);
+        default: return pick_skinny<4>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, s, cfg);
     }
+}
+
+// y[M,N] = x[M,K] . W^T.  `tiled` = 0: w is W[N,K] row-major.  `tiled` = 1: w is the
+// same matrix in blocks of 16 rows x 128 columns, zero-padded to whole blocks, stored
+// [row block][column block][j = 0..3][lane = 16*c + r][8] with element
+// W[16*row block + r][128*column block + 32*c + 8*j + e]: every load instruction of
+// a wave then reads 1 KiB in a row.  `tiled` = 2: tiled, and the 16-row blocks alternate
+// between a gate matrix and an up matrix (block 2t: gate rows 16t.., block 2t+1: up rows
+// 16t..); N counts both, y is [M, N/2] bfloat16 = silu(x.gate^T) * (x.up^T).  cfg 0 picks the launch shape; other values
+// (row tiles * 10 + waves) force one, for measurements.  act, act_scale, y_ld: the output of a gated product (common.h's
+// GateOut: another activation than the silu, a factor, rows y_ld elements apart; y_ld 0: N/2).
+extern "C" int tli_gemm_skinny_bf16(const void* x, const void* w, void* y, int M, int N, int K,
+                                    int y_dtype, int tiled, int cfg, int act, float act_scale, int y_ld, void* stream) {
+    return skinny(x, w, y, M, N, K, y_dtype, tiled, cfg, act, act_scale, y_ld, InputGroups{0, 0}, stream);
+}
+
+// The same, tiled and without a gate, of stacked matrices whose inputs differ (common.h's InputGroups; every in 32s).
+extern "C" int tli_gemm_skinny_groups_bf16(const void* x, const void* w, void* y, int M, int N, int K, int y_dtype, int every,
+                                           long long step, void* stream) {
+    if (every <= 0 || every % 32 || step < (long long)M * K || step % 8) return tli_fail("gemm_skinny: bad input groups");
+    return skinny(x, w, y, M, N, K, y_dtype, 1, 0, 0, 1.0f, 0, InputGroups{every, step}, stream);
 }
 
 template <int RT, int WAVES>

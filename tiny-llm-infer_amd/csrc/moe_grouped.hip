@@ -330,6 +330,36 @@ __global__ void moe_combine_kernel(const float* __restrict__ part, const int* __
     }
 }
 
+// The same four columns a thread (D in fours, all pointers aligned for it): two of a row's slots on their way together.
+__global__ void __launch_bounds__(256) moe_combine4_kernel(const float* __restrict__ part, const int* __restrict__ pos,
+                                                           const float* __restrict__ weights, const bf16_t* __restrict__ shared,
+                                                           const float* __restrict__ shared_gate, bf16_t* __restrict__ out, int top, int D,
+                                                           const bf16_t* __restrict__ x) {
+    const size_t t = blockIdx.y;
+    const int c = (blockIdx.x * 256 + threadIdx.x) * 4;
+    if (c >= D) return;
+    auto load4 = [&](const bf16_t* p) {
+        const uint2 u = *reinterpret_cast<const uint2*>(p);
+        return (f32x4){__uint_as_float(u.x << 16), __uint_as_float(u.x & 0xFFFF0000u), __uint_as_float(u.y << 16), __uint_as_float(u.y & 0xFFFF0000u)};
+    };
+    f32x4 y = {0.f, 0.f, 0.f, 0.f}, own = {0.f, 0.f, 0.f, 0.f};
+    if (shared) own = load4(shared + t * D + c);
+    const float open = shared && shared_gate ? shared_gate[t] : 1.0f;
+#pragma unroll 2
+    for (int j = 0; j < top; ++j) {
+        const int slot = pos[t * top + j];                       // negative: the expert hands its input on
+        const float w = weights ? weights[t * top + j] : 1.0f;
+        const f32x4 v = slot >= 0 ? *reinterpret_cast<const f32x4*>(part + (size_t)slot * D + c) : load4(x + t * D + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y[e] = fmaf(w, v[e], y[e]);
+    }
+    if (shared) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y[e] = fmaf(open, own[e], y[e]);
+    }
+    *reinterpret_cast<uint2*>(out + t * D + c) = make_uint2(pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3]));
+}
+
 // ---------------------------------------------------------------------------------------------
 // C ABI
 // ---------------------------------------------------------------------------------------------
@@ -380,6 +410,11 @@ extern "C" int tli_moe_grouped_bf16(const void* x, const int* ids, const float* 
     else if (RT == 64) { TLI_GROUPED(4, 2); }
     else { TLI_GROUPED(8, 1); }
 #undef TLI_GROUPED
+    if (D % 4 == 0 && T <= 65535 && !(((uintptr_t)part & 15) | (((uintptr_t)shared | (uintptr_t)out | (uintptr_t)x) & 7))) {
+        hipLaunchKernelGGL(moe_combine4_kernel, dim3((D + 1023) / 1024, T), dim3(256), 0, s, part, pos, weights, (const bf16_t*)shared,
+                           shared_gate, (bf16_t*)out, top, D, (const bf16_t*)x);
+        return tli_check_launch("moe_grouped");
+    }
     hipLaunchKernelGGL(moe_combine_kernel, dim3(T), dim3(256), 0, s, part, pos, weights, (const bf16_t*)shared, shared_gate,
                        (bf16_t*)out, top, D, (const bf16_t*)x);
     return tli_check_launch("moe_grouped");

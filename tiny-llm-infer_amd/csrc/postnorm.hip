@@ -348,33 +348,41 @@ extern "C" int tli_token_mixes(const void* h, const float* mu, int mixes, void* 
     return tli_check_launch("token_mixes");
 }
 
-// out [rows, n] = w * x / sqrt(mean(x^2) + eps) for n elements of rows that lie ld elements apart.  A wave a row.
-template <typename T>
+// out [rows, n] = w * x / sqrt(mean(x^2) + eps) for n elements of rows that lie ld elements apart.  A workgroup a row, V elements
+// a thread and round.
+template <typename T, int V>
 __global__ __launch_bounds__(PN_THREADS) void norm_rows_kernel(const T* __restrict__ x, int ld, const float* __restrict__ w, T* __restrict__ out,
-                                                               int rows, int n, float eps) {
-    const int lane = threadIdx.x % TLI_WAVE;
-    const int row = blockIdx.x * (PN_THREADS / TLI_WAVE) + threadIdx.x / TLI_WAVE;
-    if (row >= rows) return;
-    const T* src = x + (size_t)row * ld;
+                                                               int n, float eps) {
+    __shared__ float red[16];
+    const size_t row = blockIdx.x;
+    const T* src = x + row * ld;
     float ssq = 0.f;
-    for (int c = lane; c < n; c += TLI_WAVE) {
-        const float v = to_f32(src[c]);
-        ssq = fmaf(v, v, ssq);
+    for (int c = threadIdx.x * V; c < n; c += PN_THREADS * V) {
+        float v[V];
+        row_load<T, V>(src + c, v);
+#pragma unroll
+        for (int e = 0; e < V; ++e) ssq = fmaf(v[e], v[e], ssq);
     }
-    const float factor = 1.0f / sqrtf(wave_sum(ssq) / (float)n + eps);
-    for (int c = lane; c < n; c += TLI_WAVE) from_f32(out + (size_t)row * n + c, to_f32(src[c]) * factor * w[c]);
+    const float factor = 1.0f / sqrtf(block_sum(ssq, red) / (float)n + eps);
+    for (int c = threadIdx.x * V; c < n; c += PN_THREADS * V) {
+        float v[V], g[V];
+        row_load<T, V>(src + c, v);
+        row_load<float, V>(w + c, g);
+#pragma unroll
+        for (int e = 0; e < V; ++e) v[e] = v[e] * factor * g[e];
+        row_store<T, V>(out + row * n + c, v);
+    }
 }
 
 extern "C" int tli_norm_rows(const void* x, int ld, const float* w, void* out, int rows, int n, float eps, int dtype, void* stream) {
     if (rows <= 0) return 0;
     if (n <= 0 || ld < n) return tli_fail("norm_rows: bad sizes");
+    const bool vec = n % 8 == 0 && ld % 8 == 0 && !(((uintptr_t)x | (uintptr_t)w | (uintptr_t)out) & 15);
     hipStream_t s = (hipStream_t)stream;
-    const int per = PN_THREADS / TLI_WAVE;
-    if (dtype == TLI_F32)
-        norm_rows_kernel<float><<<(rows + per - 1) / per, PN_THREADS, 0, s>>>((const float*)x, ld, w, (float*)out, rows, n, eps);
-    else if (dtype == TLI_BF16)
-        norm_rows_kernel<bf16_t><<<(rows + per - 1) / per, PN_THREADS, 0, s>>>((const bf16_t*)x, ld, w, (bf16_t*)out, rows, n, eps);
-    else
-        return tli_fail("norm_rows: unknown dtype %d", dtype);
+#define NR_RUN(T, V) norm_rows_kernel<T, V><<<rows, PN_THREADS, 0, s>>>((const T*)x, ld, w, (T*)out, n, eps)
+    if (dtype == TLI_F32) { if (vec) NR_RUN(float, 8); else NR_RUN(float, 1); }
+    else if (dtype == TLI_BF16) { if (vec) NR_RUN(bf16_t, 8); else NR_RUN(bf16_t, 1); }
+    else return tli_fail("norm_rows: unknown dtype %d", dtype);
+#undef NR_RUN
     return tli_check_launch("norm_rows");
 }

@@ -1,8 +1,10 @@
-// Decode steps of the recurrent layers whose heads are normed one by one (retention.hip, mlstm.hip): every sequence brings
+// Decode steps of the recurrent layers whose heads are normed one by one (retention.hip, mlstm.hip, wkv.hip): every sequence brings
 // one row, and everything between the layer's products is one launch, a workgroup a (head, row).
 //   retention:  q, k turned, k scaled; S <- c S + k v^T; o = S^T q; unit RMS; silu gate
 //   mLSTM:      the two gates' logits (two dot products over the layer's input, which no other head shares), m, S <- a S +
 //               b k v^T, n likewise, o = S^T q / (max(|n q|, exp(-m)) + 1e-6); RMS times the weight; logistic gate
+//   wkv:        d = exp(-exp(W2 tanh(z) + w0)) a channel; o = (S + diag(u) k v^T)^T r; S <- diag(d) S + k v^T; RMS times the
+//               weight; silu gate
 // A column of S belongs to 16 lanes of a wave, a lane holding R elements of it (as in lightning.hip: pieces of up to four
 // that lie side by side with the other lanes').  A workgroup takes 16 columns at a time and asks for the first GROUPS x 16
 // columns before anything else, so that the state's bytes, which are nearly all that such a step moves, are on their
@@ -20,7 +22,9 @@ __device__ __forceinline__ float rs_sum16(float v) {     // over the 16 lanes of
     return v;
 }
 
-struct StepRows {                                        // what both kinds read and write
+enum { STEP_RETENTION = 0, STEP_MEMORY = 1, STEP_WKV = 2 };
+
+struct StepRows {                                        // what all kinds read and write
     const void* proj;                                    // [rows, ld]: q (H dk) | k (H dk) | v (H dv) | gate (H dv)
     int ld;
     void* out;                                           // rows out_ld elements apart, H dv of each
@@ -52,6 +56,16 @@ struct StepMemory {
     float cap, q_scale;
 };
 
+struct StepTimeMix {
+    const float* z;                                      // the decays' inner rows, before tanh: element i of row r at r z_row + i z_col
+    long long z_row, z_col;
+    const void* w2;                                      // [H dk, rank]
+    const float* w0;                                     // [H dk]
+    int rank;
+    const float* u;                                      // [H, dk]
+    const float* weight;                                 // [H dv]
+};
+
 // elements i .. i + 7 of a row of T where `eight`, else element i alone
 template <typename T>
 __device__ __forceinline__ float rs_dot8(const T* a, const T* b) {
@@ -73,8 +87,10 @@ __device__ __forceinline__ float rs_dot8(const T* a, const T* b) {
     }
 }
 
-template <bool MEMORY, int R, typename T>
-__global__ __launch_bounds__(RS_THREADS) void recurrent_step_kernel(StepRows a, StepRetention ret, StepMemory mem) {
+// T: of the projections; TO: of the output and the matrices
+template <int KIND, int R, typename T, typename TO>
+__global__ __launch_bounds__(RS_THREADS) void recurrent_step_kernel(StepRows a, StepRetention ret, StepMemory mem, StepTimeMix mix) {
+    constexpr bool MEMORY = KIND == STEP_MEMORY, WKV = KIND == STEP_WKV;
     constexpr int L = 16, DKP = L * R, NC = RS_THREADS / L;
     constexpr int GROUPS = R >= 16 ? 4 : R >= 8 ? 8 : 8;               // of NC columns, in flight together
     constexpr int VW = R % 4 == 0 ? 4 : R % 2 == 0 ? 2 : 1;
@@ -86,6 +102,8 @@ __global__ __launch_bounds__(RS_THREADS) void recurrent_step_kernel(StepRows a, 
     float* k_s = q_s + DKP;
     float* o_s = k_s + DKP;                                            // [OV]
     float* v_s = o_s + OV;                                             // [OV]
+    float* d_s = v_s + OV;                                             // wkv: [DKP] decays,
+    float* z_s = d_s + DKP;                                            // [rank]
     auto at = [&](int r) { return (r / VW) * (L * VW) + sub * VW + r % VW; };
     const int slot = a.slots[row];
     const bool fresh = a.seq_start[row] == 0;
@@ -144,8 +162,37 @@ __global__ __launch_bounds__(RS_THREADS) void recurrent_step_kernel(StepRows a, 
     const T* q_src = src + (size_t)h * dk;
     const T* k_src = src + (size_t)(H + h) * dk;
     const T* v_src = src + (size_t)2 * H * dk + (size_t)h * dv;
-    float keep, floor_ = 0.f;
-    if constexpr (MEMORY) {
+    float keep = 0.f, floor_ = 0.f;
+    if constexpr (WKV) {
+        for (int i = tid; i < mix.rank; i += RS_THREADS) z_s[i] = tanhf(mix.z[row * mix.z_row + i * mix.z_col]);
+        for (int e = tid; e < DKP; e += RS_THREADS) {
+            q_s[e] = e < dk ? to_f32(q_src[e]) : 0.f;
+            k_s[e] = e < dk ? to_f32(k_src[e]) : 0.f;
+        }
+        for (int j = tid; j < OV; j += RS_THREADS) v_s[j] = to_f32(v_src[j]);
+        __syncthreads();
+        // a channel's decay: P neighbouring threads share out its row of W2
+        constexpr int P = RS_THREADS / DKP;
+        const int c = tid / P, part = tid % P;
+        const TO* w = (const TO*)mix.w2 + (size_t)(h * dk + min(c, dk - 1)) * mix.rank;
+        float acc = 0.f;
+        if (sizeof(TO) == 2 && mix.rank % 8 == 0) {
+            for (int i = part * 8; i < mix.rank; i += 8 * P) {
+                const uint4 raw = *reinterpret_cast<const uint4*>(w + i);
+                const uint32_t b[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    acc = fmaf(z_s[i + 2 * e], __uint_as_float(b[e] << 16), acc);
+                    acc = fmaf(z_s[i + 2 * e + 1], __uint_as_float(b[e] & 0xFFFF0000u), acc);
+                }
+            }
+        } else {
+            for (int i = part; i < mix.rank; i += P) acc = fmaf(z_s[i], to_f32(w[i]), acc);
+        }
+#pragma unroll
+        for (int off = 1; off < P; off *= 2) acc += __shfl_xor(acc, off, TLI_WAVE);
+        if (part == 0) d_s[c] = c < dk ? expf(-expf(acc + mix.w0[h * dk + c])) : 0.f;
+    } else if constexpr (MEMORY) {
         // the gates' logits: every thread a part of the two dot products
         const T* x = (const T*)mem.x + (size_t)row * mem.n;
         const T* wi = (const T*)mem.w + (size_t)h * mem.n;
@@ -216,16 +263,30 @@ __global__ __launch_bounds__(RS_THREADS) void recurrent_step_kernel(StepRows a, 
     float q[R], k[R];
 #pragma unroll
     for (int r = 0; r < R; ++r) q[r] = q_s[at(r)], k[r] = k_s[at(r)];
+    float d[WKV ? R : 1], bonus = 0.f;                   // wkv: the channels' decays; r diag(u) k
+    if constexpr (WKV) {
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            d[r] = d_s[at(r)];
+            if (at(r) < dk) bonus = fmaf(q[r] * mix.u[h * dk + at(r)], k[r], bonus);
+        }
+        bonus = rs_sum16(bonus);
+    }
     auto walk = [&](int j, auto& c) {                    // (all 16 lanes of a column come here together, or none)
         const float v = v_s[j];
         float acc = 0.f;
 #pragma unroll
         for (int r = 0; r < R; ++r) {
-            c[r] = fmaf(keep, c[r], k[r] * v);
-            acc = fmaf(c[r], q[r], acc);
+            if constexpr (WKV) {
+                acc = fmaf(c[r], q[r], acc);
+                c[r] = fmaf(d[r], c[r], k[r] * v);
+            } else {
+                c[r] = fmaf(keep, c[r], k[r] * v);
+                acc = fmaf(c[r], q[r], acc);
+            }
         }
         acc = rs_sum16(acc);
-        if (sub == 0) o_s[j] = acc;
+        if (sub == 0) o_s[j] = WKV ? fmaf(bonus, v, acc) : acc;
         store_column(j, c);
     };
     if constexpr (MEMORY) {
@@ -246,22 +307,22 @@ __global__ __launch_bounds__(RS_THREADS) void recurrent_step_kernel(StepRows a, 
     }
     const float factor = a.scale * by / sqrtf(block_sum(ss, red) / (float)dv + a.eps);
     const T* g_src = src + (size_t)H * (2 * dk + dv) + (size_t)h * dv;
-    T* dst = (T*)a.out + (size_t)row * a.out_ld + (size_t)h * dv;
+    TO* dst = (TO*)a.out + (size_t)row * a.out_ld + (size_t)h * dv;
     for (int j = tid; j < dv; j += RS_THREADS) {
         const float z = to_f32(g_src[j]);
-        const float open = (MEMORY ? mem.weight[h * dv + j] : z) / (1.f + expf(-z));
+        const float open = (MEMORY ? mem.weight[h * dv + j] : WKV ? z * mix.weight[h * dv + j] : z) / (1.f + expf(-z));
         from_f32(dst + j, o_s[j] * factor * open);
     }
 }
 
-template <bool MEMORY, typename T>
-static int run_step(const StepRows& a, const StepRetention& ret, const StepMemory& mem, hipStream_t s) {
+template <int KIND, typename T, typename TO = T>
+static int run_step(const StepRows& a, const StepRetention& ret, const StepMemory& mem, const StepTimeMix& mix, hipStream_t s) {
     int R = 1;
     while (16 * R < a.dk) R *= 2;
-    const size_t lds = (size_t)(2 * 16 * R + 2 * (a.dv + 1)) * sizeof(float);
+    const size_t lds = (size_t)(2 * 16 * R + 2 * (a.dv + 1) + (KIND == STEP_WKV ? 16 * R + mix.rank : 0)) * sizeof(float);
     if (lds > 65536) return tli_fail("recurrent_step: values of %d do not fit LDS", a.dv);
     const dim3 grid(a.H, a.rows);
-#define RS_CASE(R) case R: recurrent_step_kernel<MEMORY, R, T><<<grid, RS_THREADS, lds, s>>>(a, ret, mem); break;
+#define RS_CASE(R) case R: recurrent_step_kernel<KIND, R, T, TO><<<grid, RS_THREADS, lds, s>>>(a, ret, mem, mix); break;
     switch (R) {
         RS_CASE(1) RS_CASE(2) RS_CASE(4) RS_CASE(8) RS_CASE(16)
         default: return tli_fail("recurrent_step: keys of %d", a.dk);
@@ -288,8 +349,8 @@ extern "C" int tli_retention_step(const void* proj, int ld, const float* decay, 
     if (const char* fault = step_fault(a, 2 * H * (dk + dv))) return tli_fail("retention_step: %s", fault);
     if (cos_table && (dims <= 0 || dims % 2 || dims > dk)) return tli_fail("retention_step: %d turned elements of heads of %d", dims, dk);
     const StepRetention ret{positions, decay, cos_table, sin_table, dims, pairing, table_positions, k_scale};
-    if (dtype == TLI_F32) return run_step<false, float>(a, ret, StepMemory{}, (hipStream_t)stream);
-    if (dtype == TLI_BF16) return run_step<false, bf16_t>(a, ret, StepMemory{}, (hipStream_t)stream);
+    if (dtype == TLI_F32) return run_step<STEP_RETENTION, float>(a, ret, StepMemory{}, StepTimeMix{}, (hipStream_t)stream);
+    if (dtype == TLI_BF16) return run_step<STEP_RETENTION, bf16_t>(a, ret, StepMemory{}, StepTimeMix{}, (hipStream_t)stream);
     return tli_fail("retention_step: unknown dtype %d", dtype);
 }
 
@@ -305,7 +366,24 @@ extern "C" int tli_mlstm_step(const void* proj, int ld, const void* x, const voi
     if (n <= 0 || !(cap > 0.f) || (ssq && parts <= 0)) return tli_fail("mlstm_step: bad gates");
     if (((uintptr_t)x | (uintptr_t)w) & 15) return tli_fail("mlstm_step: operands must be 16-byte aligned");
     const StepMemory mem{x, w, n, RowFactor{ssq, ssq ? parts : 0, rows, 1.0f / (float)n, x_eps}, bias, weight, m_state, cap, q_scale};
-    if (dtype == TLI_F32) return run_step<true, float>(a, StepRetention{}, mem, (hipStream_t)stream);
-    if (dtype == TLI_BF16) return run_step<true, bf16_t>(a, StepRetention{}, mem, (hipStream_t)stream);
+    if (dtype == TLI_F32) return run_step<STEP_MEMORY, float>(a, StepRetention{}, mem, StepTimeMix{}, (hipStream_t)stream);
+    if (dtype == TLI_BF16) return run_step<STEP_MEMORY, bf16_t>(a, StepRetention{}, mem, StepTimeMix{}, (hipStream_t)stream);
     return tli_fail("mlstm_step: unknown dtype %d", dtype);
+}
+
+// proj: rows of ld elements of proj_dtype, r (H dk) | k (H dk) | v (H dv) | gate (H dv) first; z, w2, w0, rank: as for tli_wkv_decays
+// (wkv.hip); u [H, dk]; weight [H dv]; state [slots][H][dv][dk]; out and w2 in `dtype` (proj_dtype: the same, or float32)
+extern "C" int tli_wkv_step(const void* proj, int ld, int proj_dtype, const float* z, long long z_row, long long z_col, const void* w2,
+                            const float* w0, int rank, const float* u, const float* weight, float* state, void* out, int out_ld,
+                            const int* seq_start, const int* slots, float eps, int rows, int H, int dk, int dv, int dtype, void* stream) {
+    if (rows <= 0) return 0;
+    const StepRows a{proj, ld, out, out_ld, state, seq_start, slots, rows, H, dk, dv, eps, 1.0f};
+    if (const char* fault = step_fault(a, 2 * H * (dk + dv))) return tli_fail("wkv_step: %s", fault);
+    if (rank <= 0 || rank > 8192 || ((uintptr_t)w2 & 15)) return tli_fail("wkv_step: bad decays");
+    const StepTimeMix mix{z, z_row, z_col, w2, w0, rank, u, weight};
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == TLI_F32 && proj_dtype == TLI_F32) return run_step<STEP_WKV, float>(a, StepRetention{}, StepMemory{}, mix, s);
+    if (dtype == TLI_BF16 && proj_dtype == TLI_F32) return run_step<STEP_WKV, float, bf16_t>(a, StepRetention{}, StepMemory{}, mix, s);
+    if (dtype == TLI_BF16 && proj_dtype == TLI_BF16) return run_step<STEP_WKV, bf16_t>(a, StepRetention{}, StepMemory{}, mix, s);
+    return tli_fail("wkv_step: unknown dtypes %d, %d", proj_dtype, dtype);
 }

@@ -151,6 +151,12 @@ def load_library():
         "tli_norm_rows": [P, I, P, P, I, I, F, I, P],
         "tli_token_gate": [P, P, P, P, I, I, I, I, I, I, I, P],
         "tli_wkv_decays": [P, ctypes.c_longlong, ctypes.c_longlong, P, P, P, I, I, I, I, P],
+        "tli_gemm_skinny_groups_bf16": [P, P, P, I, I, I, I, I, ctypes.c_longlong, P],
+        "tli_gemm_mid_groups_bf16": [P, P, P, P, I, I, I, I, I, I, ctypes.c_longlong, P],
+        "tli_gemm_rows_groups_bf16": [P, P, P, P, I, I, I, I, I, ctypes.c_longlong, P],
+        "tli_wkv_chunked_takes": [I, I, I],
+        "tli_wkv_chunked_bf16": [P, I, P, ctypes.c_longlong, ctypes.c_longlong, P, P, I, P, P, P, I, P, P, P, P, P, F, I, I, I, I, I, P],
+        "tli_wkv_step": [P, I, I, P, ctypes.c_longlong, ctypes.c_longlong, P, P, I, P, P, P, P, I, P, P, F, I, I, I, I, I, P],
         "tli_wkv_rows": [P, I, P, P, P, P, P, P, P, I, I, I, I, I, P],
         "tli_sample": [P, I, I, P, P, P, P, P, P],
         "tli_sample_scratch_bytes": [I],
@@ -162,6 +168,8 @@ def load_library():
         fn.restype = c_int
     lib.tli_lightning_scratch_floats.argtypes = [I, I, I, I, I, I]
     lib.tli_lightning_scratch_floats.restype = ctypes.c_longlong
+    lib.tli_wkv_chunked_scratch_floats.argtypes = [I, I, I, I, I]
+    lib.tli_wkv_chunked_scratch_floats.restype = ctypes.c_longlong
     lib.tli_chunked_scratch_floats.argtypes = [I, I, I, I, I]
     lib.tli_chunked_scratch_floats.restype = ctypes.c_longlong
     lib.tli_sample_uniform.argtypes = [ctypes.c_uint32, ctypes.c_uint32, ctypes.c_uint32]
@@ -253,7 +261,8 @@ class HipOps:
         self.rows_splits = 0
         self.pooled_prefill = True       # measurements, tests: False sends portions of prompts over windows and pooled blocks through the kernels for sizes of their own
         self.pooled_splits = None        # measurements, tests: into how many splits a decoding row's keys over windows and pooled blocks go (None: the rule)
-        self.recurrence_in_chunks = True    # measurements, tests: False sends the portions of prompts of retention and mLSTM through the recurrence row by row
+        self.recurrence_in_chunks = True    # measurements, tests: False sends the portions of prompts of retention, mLSTM and wkv through the recurrence row by row
+        self.grouped_products = True        # measurements, tests: False multiplies stacked matrices with inputs of their own one by one
 
     @property
     def keep_row_major(self) -> bool:
@@ -1979,32 +1988,93 @@ class HipOps:
         """The shape of one request's recurrent state (float32): a head's matrix is kept transposed."""
         return (heads, dv, dk)
 
-    def linear_groups(self, xs, groups):
-        """``xs`` [G + 1, T, n] and a ``GroupedMatrix`` of G matrices and one of few rows: (the G products side by side,
-        [T, sum of their rows] in the run's type, the last one's float32 sums, whether those are transposed)."""
-        count = len(groups.sizes)
-        if xs.dim() != 3 or xs.shape[0] != count + 1:
-            raise KernelError(f"{tuple(xs.shape)} are not the inputs of {count} matrices and one of few rows")
-        proj = torch.cat([self.linear(xs[i], m) for i, m in enumerate(groups.each)], dim=1)
-        return (proj,) + self.small_product(xs[count], groups.few)
+    def stacks_groups(self, sizes, cols: int, dtype) -> bool:
+        """Whether matrices of these rows, each with an input of its own, are held stacked in one (``linear_groups``)."""
+        return (dtype == torch.bfloat16 and cols % 8 == 0 and len(set(sizes)) == 1 and sizes[0] % 128 == 0
+                and self.many_rows == "own" and not self.plain_products)
 
-    def wkv(self, proj, z, transposed, w2, w0, u, state, step, heads, dk, dv, weight, eps, out_dtype):
-        """From the projections ``proj`` [T, r (H dk) | k (H dk) | v (H dv) | g (H dv)] and the decays' inner rows ``z``
-        (float32 [T, rank]; [rank, T] if ``transposed``) to the layer's rows [T, H dv]: decays d = exp(-exp(w2 tanh(z) + w0)),
-        o = (S + diag(u) k v^T)^T r, S <- diag(d) S + k v^T, then o / sqrt(mean(o^2) + eps) * weight * silu(g), the mean
-        head by head.  ``state``: float32 [slots, H, dv, dk], read (unless a sequence starts at position 0) and replaced."""
+    def linear_groups(self, xs, groups, step=None):
+        """``xs`` [G + 1, T, n] and a ``GroupedMatrix`` of G matrices and one of few rows: (the G products side by side,
+        [T, >= sum of their rows] in the run's type, the last one's float32 sums, the distances of their rows and columns).
+        Where the matrices are stacked one launch multiplies the G; in a ``step`` of one row a sequence it takes the last
+        one with it and the products are float32."""
+        count = len(groups.sizes)
+        if xs.dim() != 3 or xs.shape[0] != count + 1 or xs.shape[2] != groups.cols:
+            raise KernelError(f"{tuple(xs.shape)} are not the inputs of {count} matrices of {groups.cols} columns and one of few rows")
+        self._want(xs, "inputs of several matrices", groups.dtype)
+        M, K = int(xs.shape[1]), groups.cols
+        proj = None
+        if groups.stacked is not None and self.grouped_products and not self.plain_products and M > 0:
+            every, few, apart = groups.sizes[0], groups.few.shape[0], M * K
+            tiled = groups.stacked.tiled
+            together = step is not None and self._single_rows(step) and M <= self.MID_ROWS_TO and few <= every
+            N = count * every + (few if together else 0)
+            dtype = torch.float32 if together else torch.bfloat16
+            if M <= self.MID_ROWS_TO or every % 256 == 0:
+                proj = torch.empty((M, N), dtype=dtype, device=self.device)
+                if M < self.MID_ROWS_FROM:
+                    self._call(self.lib.tli_gemm_skinny_groups_bf16, xs.data_ptr(), tiled.data_ptr(), proj.data_ptr(), M, N, K,
+                               _dtype_code(dtype), every, apart, self._stream())
+                else:
+                    mid = M <= self.MID_ROWS_TO
+                    splits = int(self.lib.tli_gemm_mid_splits_rows(M, N, K, 0) if mid else self.lib.tli_gemm_rows_splits(M, N, K))
+                    part = torch.empty((splits, M, N), dtype=torch.float32, device=self.device) if splits > 1 else None
+                    if mid:
+                        self._call(self.lib.tli_gemm_mid_groups_bf16, xs.data_ptr(), tiled.data_ptr(), proj.data_ptr(), _ptr(part), M, N, K,
+                                   _dtype_code(dtype), splits, every, apart, self._stream())
+                    else:
+                        self._call(self.lib.tli_gemm_rows_groups_bf16, xs.data_ptr(), tiled.data_ptr(), proj.data_ptr(), _ptr(part), M, N, K,
+                                   splits, every, apart, self._stream())
+                if together:
+                    return proj, proj[:, count * every:], (N, 1)
+        if proj is None:
+            if groups.stacked is not None:
+                w, at = groups.stacked.w, 0
+                mats = []
+                for n in groups.sizes:
+                    mats.append(w[at:at + n])
+                    at += n
+            else:
+                mats = groups.each
+            proj = torch.cat([self.linear(xs[i], m) for i, m in enumerate(mats)], dim=1)
+        z, transposed = self.small_product(xs[count], groups.few)
+        return proj, z, ((1, M) if transposed else (groups.few.shape[0], 1))
+
+    def wkv(self, proj, z, z_strides, w2, w0, u, state, step, heads, dk, dv, weight, eps, out_dtype):
+        """From the projections ``proj`` [T, r (H dk) | k (H dk) | v (H dv) | g (H dv) | ..] and the decays' inner rows ``z``
+        (float32, ``z_strides`` the distances of its rows and columns) to the layer's rows [T, H dv]: decays
+        d = exp(-exp(w2 tanh(z) + w0)), o = (S + diag(u) k v^T)^T r, S <- diag(d) S + k v^T, then o / sqrt(mean(o^2) + eps) *
+        weight * silu(g), the mean head by head.  ``state``: float32 [slots, H, dv, dk], read (unless a sequence starts at
+        position 0) and replaced."""
         T = step.num_rows
         self._recurrent_inputs(proj, 0, state, (heads, dv, dk), step, heads, dk, dv)
         if proj.shape[1] < 2 * heads * (dk + dv):
             raise KernelError("the gate lies outside the projections")
-        rank = z.shape[0] if transposed else z.shape[1]
-        self._want(z, "decays' inner rows", torch.float32, (rank, T) if transposed else (T, rank))
+        rank = w2.shape[1]
+        z_row, z_col = z_strides
+        if z.dtype != torch.float32 or z.device.type != "cuda" or tuple(z.shape) not in ((T, rank), (rank, T)) \
+                or tuple(z.stride()) not in ((z_row, z_col), (z_col, z_row)):
+            raise KernelError(f"the decays' inner rows have shape {tuple(z.shape)} and strides {tuple(z.stride())}, not {rank} a row")
         self._want(w2, "decays' matrix", out_dtype, (heads * dk, rank))
         self._want(w0, "decays' bias", torch.float32, (heads * dk,))
         self._want(u, "current token's bonus", torch.float32, (heads, dk))
         self._want(weight, "norm weight", torch.float32, (heads * dv,))
         out = torch.empty((T, heads * dv), dtype=out_dtype, device=self.device)
-        z_row, z_col = (1, T) if transposed else (rank, 1)
+        if self._single_rows(step):
+            self._call(self.lib.tli_wkv_step, proj.data_ptr(), proj.shape[1], _dtype_code(proj.dtype), z.data_ptr(), z_row, z_col,
+                       w2.data_ptr(), w0.data_ptr(), rank, u.data_ptr(), weight.data_ptr(), state.data_ptr(), out.data_ptr(), heads * dv,
+                       step.seq_start.data_ptr(), step.slots.data_ptr(), float(eps), T, heads, dk, dv, _dtype_code(out_dtype),
+                       self._stream())
+            return out
+        if (self.recurrence_in_chunks and proj.dtype == torch.bfloat16 and not self.force_plain and proj.shape[1] % 8 == 0
+                and self.lib.tli_wkv_chunked_takes(dk, dv, rank)):
+            scratch = torch.empty((int(self.lib.tli_wkv_chunked_scratch_floats(T, step.num_seqs, heads, dk, dv)),), dtype=torch.float32,
+                                  device=self.device)
+            self._call(self.lib.tli_wkv_chunked_bf16, proj.data_ptr(), proj.shape[1], z.data_ptr(), z_row, z_col, w2.data_ptr(), w0.data_ptr(),
+                       rank, u.data_ptr(), state.data_ptr(), out.data_ptr(), heads * dv, weight.data_ptr(), scratch.data_ptr(),
+                       step.row_start.data_ptr(), step.seq_start.data_ptr(), step.slots.data_ptr(), float(eps), T, step.num_seqs, heads,
+                       dk, dv, self._stream())
+            return out
         decay = torch.empty((T, heads * dk), dtype=torch.float32, device=self.device)
         self._call(self.lib.tli_wkv_decays, z.data_ptr(), z_row, z_col, w2.data_ptr(), w0.data_ptr(), decay.data_ptr(), T, rank,
                    heads * dk, _dtype_code(out_dtype), self._stream())

@@ -83,8 +83,8 @@ class TimeMix(Mixer):
         """x: normed rows [T, hidden], or their mixes [5, T, hidden] where the norm before has made them."""
         ops = self.env.ops
         mixes = x if x.dim() == 3 else ops.token_mixes(x, self.mu, step.state["last"], step)
-        proj, z, transposed = ops.linear_groups(mixes, self.w_in)
-        y = ops.wkv(proj, z, transposed, self.w2, self.w0, self.u, step.state["S"], step, self.heads, self.dk, self.dv, self.norm,
+        proj, z, z_strides = ops.linear_groups(mixes, self.w_in, step)
+        y = ops.wkv(proj, z, z_strides, self.w2, self.w0, self.u, step.state["S"], step, self.heads, self.dk, self.dv, self.norm,
                     self.eps, self.env.dtype)
         return ops.linear(y, self.w_o, deferred=True)
 
