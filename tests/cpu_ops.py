@@ -36,6 +36,10 @@ class CpuOps:
     def activation(self, x, name):
         return self._act(x.to(torch.float32), name).to(x.dtype)
 
+    def linear_act(self, x, matrix, activation, token=None):
+        z = self.linear(x, matrix)
+        return self.activation(z, activation) if token is None else self.token_gate(z, token[0], token[1], token[2], activation)
+
     @staticmethod
     def _act(z, name):
         if name == "relu2":

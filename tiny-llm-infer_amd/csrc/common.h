@@ -135,6 +135,32 @@ static inline const char* gate_out_fault(const GateOut& g, int cols) {
     return nullptr;
 }
 
+// What a product without a gate does to its sums before it writes them: kind < 0 nothing; else act_of(sum, kind), times element n
+// of the row's token's own vector (row id of a bfloat16 table, rows `width` apart) where there is one.
+struct OutUnit {
+    int kind;
+    const bf16_t* table;         // at the vector's first element, or null
+    const int* ids;              // [rows]
+    int width, vocab;
+    __device__ __forceinline__ void apply(float (&v)[4], int row, int n0, int left) const {
+        if (kind < 0) return;
+        const bf16_t* own = nullptr;
+        if (table) {
+            const int id = ids[row];
+            own = table + (size_t)(id < 0 || id >= vocab ? 0 : id) * width + n0;
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            if (i < left) v[i] = act_of(v[i], kind) * (own ? bf16_to_f32(own[i]) : 1.0f);
+    }
+};
+static inline OutUnit no_unit() { return OutUnit{-1, nullptr, nullptr, 0, 0}; }
+static inline const char* out_unit_fault(const OutUnit& u, int cols) {
+    if (u.kind < 0 || u.kind >= TLI_ACT_KINDS) return "unknown activation of a product's outputs";
+    if (u.table && (!u.ids || u.width < cols || u.vocab <= 0)) return "bad tokens' vectors";
+    return nullptr;
+}
+
 // Several matrices stacked in one whose products read inputs of their own: columns n of the output belong to input
 // n / every, inputs lie `step` elements apart.  every 0: one input.  (A workgroup's columns belong to one input.)
 struct InputGroups {

@@ -46,7 +46,7 @@ union Pack16m {
 template <int RT, int WAVES, int DEPTH, int MT, typename TO, bool GATED>
 __global__ void __launch_bounds__(WAVES * 64)
 gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* __restrict__ y,
-                float* __restrict__ part, int M_all, int N, int K, int splits, int steps_per_split, GateOut gate, InputGroups inputs) {
+                float* __restrict__ part, int M_all, int N, int K, int splits, int steps_per_split, GateOut gate, InputGroups inputs, OutUnit unit) {
     constexpr int ROWS = MT * 16;
     constexpr int STAGES = DEPTH + 1;                        // W: DEPTH slices on their way, one in use
     constexpr int XSLOTS = DEPTH + 2;                        // x: one slice further ahead
@@ -260,7 +260,8 @@ gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* 
         for (int m = 0; m < MT; ++m) {
             const int row = m * 16 + r;
             if (row >= M) continue;
-            const float o[4] = {acc[t][m][0], acc[t][m][1], acc[t][m][2], acc[t][m][3]};
+            float o[4] = {acc[t][m][0], acc[t][m][1], acc[t][m][2], acc[t][m][3]};
+            unit.apply(o, row0 + row, n0, N - n0);
             store4(y + (size_t)row * N + n0, o, N - n0, (N & 3) == 0);
         }
     }
@@ -268,7 +269,7 @@ gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, TO* 
 
 template <int RT, int WAVES, int DEPTH, int MT>
 static int launch_mid_rows(const bf16_t* x, const bf16_t* w, void* y, float* part, int M, int N, int K,
-                           int y_dtype, GateOut gated, const InputGroups& inputs, int splits, hipStream_t s) {
+                           int y_dtype, GateOut gated, const InputGroups& inputs, const OutUnit& unit, int splits, hipStream_t s) {
     const int n_tiles = (N + 15) / 16, k_steps = (K + 127) / 128;
     const int steps_per_split = (k_steps + splits - 1) / splits;
     const int groups = (n_tiles + RT * WAVES - 1) / (RT * WAVES), row_blocks = (M + MT * 16 - 1) / (MT * 16);
@@ -285,7 +286,7 @@ static int launch_mid_rows(const bf16_t* x, const bf16_t* w, void* y, float* par
                 return tli_fail("gemm_mid: cannot have %zu bytes of LDS", lds);                            \
             allowed = true;                                                                                \
         }                                                                                                  \
-        kernel<<<grid, WAVES * 64, lds, s>>>(x, w, (TO*)y, part, M, N, K, splits, steps_per_split, gated, inputs); \
+        kernel<<<grid, WAVES * 64, lds, s>>>(x, w, (TO*)y, part, M, N, K, splits, steps_per_split, gated, inputs, unit); \
     }
     if (gated) MID_LAUNCH(bf16_t, true)
     else if (y_dtype == TLI_BF16) MID_LAUNCH(bf16_t, false)
@@ -303,10 +304,10 @@ static int launch_mid_rows(const bf16_t* x, const bf16_t* w, void* y, float* par
 // Four 16-row tiles of x up to 64 rows, eight beyond.
 template <int RT, int WAVES, int DEPTH>
 static int launch_mid(const bf16_t* x, const bf16_t* w, void* y, float* part, int M, int N, int K,
-                      int y_dtype, GateOut gated, const InputGroups& inputs, int splits, hipStream_t s) {
-    if (M <= 64) return launch_mid_rows<RT, WAVES, DEPTH, 4>(x, w, y, part, M, N, K, y_dtype, gated, inputs, splits, s);
+                      int y_dtype, GateOut gated, const InputGroups& inputs, const OutUnit& unit, int splits, hipStream_t s) {
+    if (M <= 64) return launch_mid_rows<RT, WAVES, DEPTH, 4>(x, w, y, part, M, N, K, y_dtype, gated, inputs, unit, splits, s);
     if constexpr (DEPTH <= 3)       // (DEPTH + 2) slices of 32 KiB fit the 160 KiB of LDS
-        return launch_mid_rows<RT, WAVES, DEPTH, 8>(x, w, y, part, M, N, K, y_dtype, gated, inputs, splits, s);
+        return launch_mid_rows<RT, WAVES, DEPTH, 8>(x, w, y, part, M, N, K, y_dtype, gated, inputs, unit, splits, s);
     else
         return tli_fail("gemm_mid: more than 64 rows leave LDS for at most 3 slices on their way");
 }
@@ -398,7 +399,7 @@ extern "C" int tli_gemm_mid_splits_rows(int M, int N, int K, int gated) {
 }
 
 static int gemm_mid(const void* x, const void* w, void* y, float* part, int M, int N, int K, int y_dtype, int is_gated, int splits,
-                    int cfg, int act, float act_scale, int y_ld, const InputGroups& inputs, void* stream) {
+                    int cfg, int act, float act_scale, int y_ld, const InputGroups& inputs, const OutUnit& unit, void* stream) {
     const GateOut gated = gate_out(is_gated, act, act_scale, y_ld, N / 2);
     if (const char* fault = gate_out_fault(gated, N / 2)) return tli_fail("gemm_mid: %s", fault);
     if (M <= 0 || N <= 0) return 0;
@@ -429,7 +430,7 @@ static int gemm_mid(const void* x, const void* w, void* y, float* part, int M, i
         cfg = 200 + 10 * rt + waves;
     }
     if (gated && (cfg / 10) % 10 < 2) return tli_fail("gemm_mid: a gated product needs pairs of row tiles");
-#define MID_CASE(D, R, W) case D * 100 + R * 10 + W: return launch_mid<R, W, D>(xp, wp, y, part, M, N, K, y_dtype, gated, inputs, splits, s);
+#define MID_CASE(D, R, W) case D * 100 + R * 10 + W: return launch_mid<R, W, D>(xp, wp, y, part, M, N, K, y_dtype, gated, inputs, unit, splits, s);
     switch (cfg) {
         MID_CASE(2, 1, 4) MID_CASE(3, 1, 4) MID_CASE(2, 1, 8) MID_CASE(4, 1, 8)
         MID_CASE(2, 2, 4) MID_CASE(4, 2, 4) MID_CASE(2, 2, 8)
@@ -448,7 +449,7 @@ static int gemm_mid(const void* x, const void* w, void* y, float* part, int M, i
 extern "C" int tli_gemm_mid_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K,
                                  int y_dtype, int is_gated, int splits, int cfg, int act, float act_scale, int y_ld,
                                  void* stream) {
-    return gemm_mid(x, w, y, part, M, N, K, y_dtype, is_gated, splits, cfg, act, act_scale, y_ld, InputGroups{0, 0}, stream);
+    return gemm_mid(x, w, y, part, M, N, K, y_dtype, is_gated, splits, cfg, act, act_scale, y_ld, InputGroups{0, 0}, no_unit(), stream);
 }
 
 // The same, without a gate and for up to 128 rows, of stacked matrices whose inputs differ (common.h's InputGroups; every in
@@ -456,7 +457,27 @@ extern "C" int tli_gemm_mid_bf16(const void* x, const void* w, void* y, float* p
 extern "C" int tli_gemm_mid_groups_bf16(const void* x, const void* w, void* y, float* part, int M, int N, int K, int y_dtype, int splits,
                                         int every, long long step, void* stream) {
     if (M > 128 || every <= 0 || every % 128 || step < (long long)M * K || step % 8) return tli_fail("gemm_mid: bad input groups");
-    return gemm_mid(x, w, y, part, M, N, K, y_dtype, 0, splits, 0, 0, 1.0f, 0, InputGroups{every, step}, stream);
+    return gemm_mid(x, w, y, part, M, N, K, y_dtype, 0, splits, 0, 0, 1.0f, 0, InputGroups{every, step}, no_unit(), stream);
+}
+
+// The same, without a gate, k whole, for up to 128 rows and bfloat16, its outputs through common.h's OutUnit.
+extern "C" int tli_gemm_mid_unit_bf16(const void* x, const void* w, void* y, int M, int N, int K, int kind, const void* table, const int* ids,
+                                      int width, int vocab, void* stream) {
+    const OutUnit unit{kind, (const bf16_t*)table, ids, width, vocab};
+    if (const char* fault = out_unit_fault(unit, N)) return tli_fail("gemm_mid: %s", fault);
+    if (M > 128) return tli_fail("gemm_mid: %d rows", M);
+    return gemm_mid(x, w, y, nullptr, M, N, K, TLI_BF16, 0, 1, 0, 0, 1.0f, 0, InputGroups{0, 0}, unit, stream);
+}
+
+// tli_gemm_mid_reduce to bfloat16, its sums through common.h's OutUnit
+extern "C" int tli_gemm_reduce_unit_bf16(const float* part, void* y, int M, int N, int splits, int kind, const void* table, const int* ids,
+                                         int width, int vocab, void* stream) {
+    if (M <= 0 || N <= 0) return 0;
+    const OutUnit unit{kind, (const bf16_t*)table, ids, width, vocab};
+    if (const char* fault = out_unit_fault(unit, N)) return tli_fail("gemm_reduce: %s", fault);
+    if (!part || !y || splits < 1) return tli_fail("gemm_reduce: bad arguments");
+    launch_gemm_reduce(part, (bf16_t*)y, M, N, splits, GateOut{}, (hipStream_t)stream, unit);
+    return tli_check_launch("gemm_reduce");
 }
 
 // y[M,N] = sum over the partial products in `part` [splits][M][N], in split order.

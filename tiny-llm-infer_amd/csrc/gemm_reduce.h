@@ -7,7 +7,7 @@
 // gate column (j/16)*32 + j%16 and up column 16 further.
 template <typename TO>
 __global__ void gemm_mid_reduce_kernel(const float* __restrict__ part, TO* __restrict__ y, int M, int N,
-                                       int splits, GateOut gated) {
+                                       int splits, GateOut gated, OutUnit unit) {
     const int n_out = gated ? N / 2 : N;
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= (size_t)M * n_out) return;
@@ -24,7 +24,9 @@ __global__ void gemm_mid_reduce_kernel(const float* __restrict__ part, TO* __res
     } else {
         float v = 0.f;
         for (int s = 0; s < splits; ++s) v += part[s * plane + (size_t)row * N + j];
-        from_f32(y + idx, v);
+        float o[4] = {v, 0.f, 0.f, 0.f};
+        unit.apply(o, row, j, 1);
+        from_f32(y + idx, o[0]);
     }
 }
 
@@ -32,7 +34,7 @@ __global__ void gemm_mid_reduce_kernel(const float* __restrict__ part, TO* __res
 // 16-byte load a plane and one store.
 template <typename TO>
 __global__ void gemm_mid_reduce4_kernel(const float* __restrict__ part, TO* __restrict__ y, int M, int N,
-                                        int splits, GateOut gated) {
+                                        int splits, GateOut gated, OutUnit unit) {
     const int n_out = gated ? N / 2 : N, quads = n_out / 4;
     const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= (size_t)M * quads) return;
@@ -56,19 +58,21 @@ __global__ void gemm_mid_reduce4_kernel(const float* __restrict__ part, TO* __re
             const float4 a = *reinterpret_cast<const float4*>(part + s * plane + (size_t)row * N + j);
             o[0] += a.x; o[1] += a.y; o[2] += a.z; o[3] += a.w;
         }
+        unit.apply(o, row, j, 4);
     }
     store4(y + (size_t)row * (gated ? gated.ld : n_out) + j, o, 4, true);
 }
 
 // Launches the pass: four columns a thread where the sizes and addresses allow it.
 template <typename TO>
-static inline void launch_gemm_reduce(const float* part, TO* y, int M, int N, int splits, GateOut gated, hipStream_t s) {
+static inline void launch_gemm_reduce(const float* part, TO* y, int M, int N, int splits, GateOut gated, hipStream_t s,
+                                      OutUnit unit = no_unit()) {
     const int n_out = gated ? N / 2 : N;
     if (N % 4 == 0 && n_out % 4 == 0 && (!gated || gated.ld % 4 == 0) && !(((uintptr_t)part | (uintptr_t)y) & 15)) {
         const size_t total = (size_t)M * (n_out / 4);
-        gemm_mid_reduce4_kernel<TO><<<(unsigned)((total + 255) / 256), 256, 0, s>>>(part, y, M, N, splits, gated);
+        gemm_mid_reduce4_kernel<TO><<<(unsigned)((total + 255) / 256), 256, 0, s>>>(part, y, M, N, splits, gated, unit);
     } else {
         const size_t total = (size_t)M * n_out;
-        gemm_mid_reduce_kernel<TO><<<(unsigned)((total + 255) / 256), 256, 0, s>>>(part, y, M, N, splits, gated);
+        gemm_mid_reduce_kernel<TO><<<(unsigned)((total + 255) / 256), 256, 0, s>>>(part, y, M, N, splits, gated, unit);
     }
 }

@@ -74,6 +74,7 @@ struct SkinnyFuse {
     float* ssq_out;           // [ceil(N/16)][M]
     GateOut gate;             // of a gated matrix
     InputGroups inputs;
+    OutUnit unit;             // of a product without a gate and norm
 };
 
 template <int RT, int MT, int WAVES, typename TO, bool TILED = false, bool GATED = false, int DEPTH = 2,
@@ -318,7 +319,10 @@ gemm_skinny_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, T
 #pragma unroll
             for (int i = 0; i < 4; ++i) s[i] *= rstd[m];
         }
-        if (row < M) store4(y + (size_t)row * N + n0, s, N - n0, (N & 3) == 0);
+        if (row < M) {
+            if constexpr (FUSE == FUSE_NONE && TILED) fuse.unit.apply(s, row, n0, N - n0);
+            store4(y + (size_t)row * N + n0, s, N - n0, (N & 3) == 0);
+        }
     }
 }
 
@@ -328,8 +332,9 @@ gemm_skinny_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, T
 
 template <int RT, int MT, int WAVES>
 static int launch_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N, int K, int y_dtype,
-                         int tiled, const GateOut& gate, const InputGroups& inputs, hipStream_t s) {
+                         int tiled, const GateOut& gate, const InputGroups& inputs, const OutUnit& unit, hipStream_t s) {
     SkinnyFuse plain{};
+    plain.unit = unit;
     plain.gate = gate;
     plain.inputs = inputs;
     const int blocks = (N + 16 * RT - 1) / (16 * RT);
@@ -352,23 +357,23 @@ static int launch_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N
 
 template <int MT>
 static int pick_skinny(const bf16_t* x, const bf16_t* w, void* y, int M, int N, int K, int y_dtype,
-                       int tiled, const GateOut& gate, const InputGroups& inputs, hipStream_t s, int cfg) {
+                       int tiled, const GateOut& gate, const InputGroups& inputs, const OutUnit& unit, hipStream_t s, int cfg) {
     // cfg 0: by shape.  Narrow outputs get one 16-column tile per workgroup so that
     // even N = 4096 gives 256 workgroups; wide outputs share x over two tiles.
     const long tiles = (N + 15) / 16;
     if (cfg == 0) cfg = tiles <= tli_compute_units() ? 18 : (tiles < 4 * tli_compute_units() ? 28 : 24);
     if (tiled == 2 && cfg < 20) cfg = 24;          // gated needs pairs of row tiles
     switch (cfg) {
-        case 14: return launch_skinny<1, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, s);
-        case 18: return launch_skinny<1, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, s);
-        case 24: return launch_skinny<2, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, s);
-        case 28: return launch_skinny<2, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, s);
+        case 14: return launch_skinny<1, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, unit, s);
+        case 18: return launch_skinny<1, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, unit, s);
+        case 24: return launch_skinny<2, MT, 4>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, unit, s);
+        case 28: return launch_skinny<2, MT, 8>(x, w, y, M, N, K, y_dtype, tiled, gate, inputs, unit, s);
         default: return tli_fail("gemm_skinny: unknown configuration %d", cfg);
     }
 }
 
 static int skinny(const void* x, const void* w, void* y, int M, int N, int K, int y_dtype, int tiled, int cfg, int act,
-                  float act_scale, int y_ld, const InputGroups& inputs, void* stream) {
+                  float act_scale, int y_ld, const InputGroups& inputs, const OutUnit& unit, void* stream) {
     const GateOut gate = gate_out(tiled == 2, act, act_scale, y_ld, N / 2);
     if (const char* fault = gate_out_fault(gate, N / 2)) return tli_fail("gemm_skinny: %s", fault);
     if (M <= 0 || N <= 0) return 0;
@@ -383,10 +388,10 @@ static int skinny(const void* x, const void* w, void* y, int M, int N, int K, in
     const bf16_t* xp = (const bf16_t*)x;
     const bf16_t* wp = (const bf16_t*)w;
     switch ((M + 15) / 16) {
-        case 1: return pick_skinny<1>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, s, cfg);
-        case 2: return pick_skinny<2>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, s, cfg);
-        case 3: return pick_skinny<3>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, s, cfg);
-        default: return pick_skinny<4>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, s, cfg);
+        case 1: return pick_skinny<1>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, unit, s, cfg);
+        case 2: return pick_skinny<2>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, unit, s, cfg);
+        case 3: return pick_skinny<3>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, unit, s, cfg);
+        default: return pick_skinny<4>(xp, wp, y, M, N, K, y_dtype, tiled, gate, inputs, unit, s, cfg);
     }
 }
 
@@ -401,14 +406,22 @@ static int skinny(const void* x, const void* w, void* y, int M, int N, int K, in
 // GateOut: another activation than the silu, a factor, rows y_ld elements apart; y_ld 0: N/2).
 extern "C" int tli_gemm_skinny_bf16(const void* x, const void* w, void* y, int M, int N, int K,
                                     int y_dtype, int tiled, int cfg, int act, float act_scale, int y_ld, void* stream) {
-    return skinny(x, w, y, M, N, K, y_dtype, tiled, cfg, act, act_scale, y_ld, InputGroups{0, 0}, stream);
+    return skinny(x, w, y, M, N, K, y_dtype, tiled, cfg, act, act_scale, y_ld, InputGroups{0, 0}, no_unit(), stream);
 }
 
 // The same, tiled and without a gate, of stacked matrices whose inputs differ (common.h's InputGroups; every in 32s).
 extern "C" int tli_gemm_skinny_groups_bf16(const void* x, const void* w, void* y, int M, int N, int K, int y_dtype, int every,
                                            long long step, void* stream) {
     if (every <= 0 || every % 32 || step < (long long)M * K || step % 8) return tli_fail("gemm_skinny: bad input groups");
-    return skinny(x, w, y, M, N, K, y_dtype, 1, 0, 0, 1.0f, 0, InputGroups{every, step}, stream);
+    return skinny(x, w, y, M, N, K, y_dtype, 1, 0, 0, 1.0f, 0, InputGroups{every, step}, no_unit(), stream);
+}
+
+// The same, tiled, without a gate and bfloat16, its outputs through common.h's OutUnit.
+extern "C" int tli_gemm_skinny_unit_bf16(const void* x, const void* w, void* y, int M, int N, int K, int kind, const void* table,
+                                         const int* ids, int width, int vocab, void* stream) {
+    const OutUnit unit{kind, (const bf16_t*)table, ids, width, vocab};
+    if (const char* fault = out_unit_fault(unit, N)) return tli_fail("gemm_skinny: %s", fault);
+    return skinny(x, w, y, M, N, K, TLI_BF16, 1, 0, 0, 1.0f, 0, InputGroups{0, 0}, unit, stream);
 }
 
 template <int RT, int WAVES>

@@ -4,7 +4,9 @@
 //                 its mean square summed in float32, the normed row added to the float32 residual, and the
 //                 new residual written in the run's type for the next sublayer to read.
 // norm_add_norm:  the same with the norm of whoever reads the sum next in the same pass: h = w2 * x / sqrt(mean(x^2) + eps2)
-//                 is written instead of x's own rows.  Without y: that norm alone.  With `rows` only those rows of the
+//                 is written instead of x's own rows.  Without y: that norm alone;
+//                 without w2: x's own rows.  y may come as float32 partial sums of a product, which are added in order and
+//                 rounded as the product would have.  With `rows` only those rows of the
 //                 residual are looked at, and it is not written.  With mixes (steps of one row a sequence): h' being the row
 //                 that the sequence's slot keeps (zeros at position 0), h + (h' - h) mu_m for every m is written instead, and
 //                 h replaces the kept row.
@@ -166,37 +168,67 @@ __device__ __forceinline__ void row_store(T* p, const float (&v)[V]) {
 // ROUNDS x PN_THREADS x V elements of a row are kept in registers between the sums; a row is no longer than that.
 template <typename T, int V, int ROUNDS>
 __global__ __launch_bounds__(PN_THREADS) void norm_add_norm_kernel(float* __restrict__ resid, const T* __restrict__ y,
+                                                                    const float* __restrict__ sums, int parts, size_t plane,
                                                                     const float* __restrict__ w1, float eps1,
                                                                     const float* __restrict__ w2, float eps2, T* __restrict__ out,
                                                                     const int* __restrict__ rows, int n, MixArgs mix) {
     __shared__ float red[16];
     const size_t row = rows ? rows[blockIdx.x] : blockIdx.x;
     float* xr = resid + row * n;
-    float v[ROUNDS][V], x[ROUNDS][V];
+    float v[ROUNDS][V], x[ROUNDS][V], g1[ROUNDS][V], g2[ROUNDS][V];
     float ssq = 0.f;
+    const bool add = y || parts > 0;
+    // everything but the mixes' weights is asked for before the first sum is taken
 #pragma unroll
     for (int i = 0; i < ROUNDS; ++i) {
         const int c = (i * PN_THREADS + threadIdx.x) * V;
 #pragma unroll
-        for (int e = 0; e < V; ++e) v[i][e] = x[i][e] = 0.f;
+        for (int e = 0; e < V; ++e) v[i][e] = x[i][e] = g1[i][e] = g2[i][e] = 0.f;
         if (c < n) {
-            row_load<float, V>(xr + c, x[i]);
             if (y) row_load<T, V>(y + row * n + c, v[i]);
+            for (int p = 0; p < parts; ++p) {
+                float a[V];
+                row_load<float, V>(sums + p * plane + row * n + c, a);
+#pragma unroll
+                for (int e = 0; e < V; ++e) v[i][e] += a[e];
+            }
+            if constexpr (sizeof(T) == 2) {
+                if (parts > 0) {
+#pragma unroll
+                    for (int e = 0; e < V; ++e) v[i][e] = bf16_to_f32(f32_to_bf16(v[i][e]));
+                }
+            }
+            row_load<float, V>(xr + c, x[i]);
+            if (add) row_load<float, V>(w1 + c, g1[i]);
+            if (w2) row_load<float, V>(w2 + c, g2[i]);
         }
 #pragma unroll
         for (int e = 0; e < V; ++e) ssq = fmaf(v[i][e], v[i][e], ssq);
     }
-    if (y) {
+    if (add) {
         const float factor = 1.0f / sqrtf(block_sum(ssq, red) / (float)n + eps1);
 #pragma unroll
         for (int i = 0; i < ROUNDS; ++i) {
             const int c = (i * PN_THREADS + threadIdx.x) * V;
             if (c >= n) continue;
-            float g[V];
-            row_load<float, V>(w1 + c, g);
 #pragma unroll
-            for (int e = 0; e < V; ++e) x[i][e] += v[i][e] * factor * g[e];
+            for (int e = 0; e < V; ++e) x[i][e] += v[i][e] * factor * g1[i][e];
             if (!rows) row_store<float, V>(xr + c, x[i]);
+            if (!w2 && out) row_store<T, V>(out + (size_t)blockIdx.x * n + c, x[i]);
+        }
+    }
+    if (!w2) return;
+    T* kept = nullptr;
+    bool fresh = true;
+    if (mix.mu) {
+        kept = (T*)mix.kept + (size_t)mix.slots[row] * n;
+        fresh = mix.seq_start[row] <= 0;
+#pragma unroll
+        for (int i = 0; i < ROUNDS; ++i) {           // (v now holds the kept row)
+            const int c = (i * PN_THREADS + threadIdx.x) * V;
+#pragma unroll
+            for (int e = 0; e < V; ++e) v[i][e] = 0.f;
+            if (c < n && !fresh) row_load<T, V>(kept + c, v[i]);
         }
     }
     ssq = 0.f;
@@ -205,34 +237,23 @@ __global__ __launch_bounds__(PN_THREADS) void norm_add_norm_kernel(float* __rest
 #pragma unroll
         for (int e = 0; e < V; ++e) ssq = fmaf(x[i][e], x[i][e], ssq);
     const float factor = 1.0f / sqrtf(block_sum(ssq, red) / (float)n + eps2);
-    T* kept = nullptr;
-    bool fresh = true;
-    if (mix.mu) {
-        kept = (T*)mix.kept + (size_t)mix.slots[row] * n;
-        fresh = mix.seq_start[row] <= 0;
-    }
 #pragma unroll
     for (int i = 0; i < ROUNDS; ++i) {
         const int c = (i * PN_THREADS + threadIdx.x) * V;
         if (c >= n) continue;
-        float g[V], h[V];
-        row_load<float, V>(w2 + c, g);
+        float h[V];
 #pragma unroll
-        for (int e = 0; e < V; ++e) h[e] = x[i][e] * factor * g[e];
+        for (int e = 0; e < V; ++e) h[e] = x[i][e] * factor * g2[i][e];
         if (!mix.mu) {
             row_store<T, V>(out + (size_t)blockIdx.x * n + c, h);
             continue;
         }
-        float prev[V];
-#pragma unroll
-        for (int e = 0; e < V; ++e) prev[e] = 0.f;
-        if (!fresh) row_load<T, V>(kept + c, prev);
         if constexpr (sizeof(T) == 2) {             // h as it is kept: the mixes are made of rounded rows
 #pragma unroll
             for (int e = 0; e < V; ++e) h[e] = bf16_to_f32(f32_to_bf16(h[e]));
         }
         row_store<T, V>(kept + c, h);
-        put_mixes<T, V>(h, prev, mix, out, row * n + c, c, n);
+        put_mixes<T, V>(h, v[i], mix, out, row * n + c, c, n);
     }
 }
 
@@ -301,11 +322,11 @@ extern "C" int tli_residual_rows(const float* resid, void* out, long long count,
 }
 
 template <typename T>
-static int run_norm_add_norm(float* resid, const T* y, const float* w1, float eps1, const float* w2, float eps2, T* out, const int* rows,
+static int run_norm_add_norm(float* resid, const T* y, const float* sums, int parts, size_t plane, const float* w1, float eps1, const float* w2, float eps2, T* out, const int* rows,
                              int count, int n, const MixArgs& mix, hipStream_t s) {
-    const bool vec = n % 8 == 0 && !(((uintptr_t)resid | (uintptr_t)y | (uintptr_t)w1 | (uintptr_t)w2 | (uintptr_t)out | (uintptr_t)mix.mu |
+    const bool vec = n % 8 == 0 && !(((uintptr_t)resid | (uintptr_t)y | (uintptr_t)sums | (uintptr_t)w1 | (uintptr_t)w2 | (uintptr_t)out | (uintptr_t)mix.mu |
                                       (uintptr_t)mix.kept) & 15);
-#define NAN_RUN(V, R) norm_add_norm_kernel<T, V, R><<<count, PN_THREADS, 0, s>>>(resid, y, w1, eps1, w2, eps2, out, rows, n, mix)
+#define NAN_RUN(V, R) norm_add_norm_kernel<T, V, R><<<count, PN_THREADS, 0, s>>>(resid, y, sums, parts, plane, w1, eps1, w2, eps2, out, rows, n, mix)
     if (vec && n <= 8 * PN_THREADS) NAN_RUN(8, 1);
     else if (vec && n <= 16 * PN_THREADS) NAN_RUN(8, 2);
     else if (vec && n <= 32 * PN_THREADS) NAN_RUN(8, 4);
@@ -316,19 +337,26 @@ static int run_norm_add_norm(float* resid, const T* y, const float* w1, float ep
     return tli_check_launch("norm_add_norm");
 }
 
-// resid [.., n] float32 += w1 * y / rms(y) (y null: nothing), out [count, n] = w2 * resid / rms(resid) in the type of y.
-// rows (or null): the rows of resid and y that `count` counts, resid then unchanged.  mu (or null) [mixes][n], kept
-// [slots][n], slots, seq_start [rows]: out is [mixes][count][n] (rows must be null).
-extern "C" int tli_norm_add_norm(float* resid, const void* y, const float* w1, float eps1, const float* w2, float eps2, void* out,
-                                 const int* rows, int count, int n, const float* mu, int mixes, void* kept, const int* slots,
+// resid [total, n] float32 += w1 * y / rms(y) (y null: nothing), out [count, n] = w2 * resid / rms(resid) in the type of y (w2 null:
+// resid's rows; out may then be null).  parts > 0: y is float32 partial sums [parts][total][n].  rows (or null): the rows of resid
+// and y that `count` counts, resid then unchanged; without them count is total.  mu (or null) [mixes][n], kept [slots][n],
+// slots, seq_start [rows]: out is [mixes][count][n] (rows must be null).
+extern "C" int tli_norm_add_norm(float* resid, const void* y, int parts, int total, const float* w1, float eps1, const float* w2, float eps2,
+                                 void* out, const int* rows, int count, int n, const float* mu, int mixes, void* kept, const int* slots,
                                  const int* seq_start, int dtype, void* stream) {
     if (count <= 0) return 0;
-    if (n <= 0 || (y && !w1) || !w2 || !out) return tli_fail("norm_add_norm: bad arguments");
+    if (n <= 0 || (y && !w1) || (w2 && !out) || (!w2 && (!y || rows || mu)) || parts < 0 || (parts && !y) || count > total)
+        return tli_fail("norm_add_norm: bad arguments");
     if (mu && (rows || mixes <= 0 || !kept || !slots || !seq_start)) return tli_fail("norm_add_norm: bad mixes");
     const MixArgs mix{mu, mixes, kept, slots, seq_start, (size_t)count * n};
+    const float* sums = parts ? (const float*)y : nullptr;
+    const size_t plane = (size_t)total * n;
+    if (parts) y = nullptr;
     hipStream_t s = (hipStream_t)stream;
-    if (dtype == TLI_F32) return run_norm_add_norm<float>(resid, (const float*)y, w1, eps1, w2, eps2, (float*)out, rows, count, n, mix, s);
-    if (dtype == TLI_BF16) return run_norm_add_norm<bf16_t>(resid, (const bf16_t*)y, w1, eps1, w2, eps2, (bf16_t*)out, rows, count, n, mix, s);
+    if (dtype == TLI_F32)
+        return run_norm_add_norm<float>(resid, (const float*)y, sums, parts, plane, w1, eps1, w2, eps2, (float*)out, rows, count, n, mix, s);
+    if (dtype == TLI_BF16)
+        return run_norm_add_norm<bf16_t>(resid, (const bf16_t*)y, sums, parts, plane, w1, eps1, w2, eps2, (bf16_t*)out, rows, count, n, mix, s);
     return tli_fail("norm_add_norm: unknown dtype %d", dtype);
 }
 

@@ -146,7 +146,10 @@ def load_library():
         "tli_pooled_prefill_takes": [I, I, I, I, I, I],
         "tli_pooled_prefill_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, P],
         "tli_attention_pooled_mfma_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, F, I, P, P, P, I, I, I, I, P, I, F, I, P, P],
-        "tli_norm_add_norm": [P, P, P, F, P, F, P, P, I, I, P, I, P, P, P, I, P],
+        "tli_norm_add_norm": [P, P, I, I, P, F, P, F, P, P, I, I, P, I, P, P, P, I, P],
+        "tli_gemm_skinny_unit_bf16": [P, P, P, I, I, I, I, P, P, I, I, P],
+        "tli_gemm_mid_unit_bf16": [P, P, P, I, I, I, I, P, P, I, I, P],
+        "tli_gemm_reduce_unit_bf16": [P, P, I, I, I, I, P, P, I, I, P],
         "tli_token_mixes": [P, P, I, P, P, P, P, P, P, I, I, I, P],
         "tli_norm_rows": [P, I, P, P, I, I, F, I, P],
         "tli_token_gate": [P, P, P, P, I, I, I, I, I, I, I, P],
@@ -262,6 +265,7 @@ class HipOps:
         self.pooled_prefill = True       # measurements, tests: False sends portions of prompts over windows and pooled blocks through the kernels for sizes of their own
         self.pooled_splits = None        # measurements, tests: into how many splits a decoding row's keys over windows and pooled blocks go (None: the rule)
         self.recurrence_in_chunks = True    # measurements, tests: False sends the portions of prompts of retention, mLSTM and wkv through the recurrence row by row
+        self.separate_activations = False   # measurements, tests: True leaves the activations of products without a gate to a pass of their own
         self.grouped_products = True        # measurements, tests: False multiplies stacked matrices with inputs of their own one by one
 
     @property
@@ -972,6 +976,49 @@ class HipOps:
                    _dtype_code(x.dtype), self._stream())
         return out
 
+    def linear_act(self, x, matrix, activation: str, token=None):
+        """``activation`` of x W^T, one of ``ACTIVATIONS``; with ``token`` = (table, column, ids) times row ids[t] of the table from that
+        column on (``token_gate``).  Products of up to 128 rows, and those whose k is cut into ranges, do it where they write
+        their sums; others are followed by a pass."""
+        self.check_activation(activation)
+        tiled = getattr(matrix, "tiled", None)
+        M, K = x.shape
+        N = _shape_of(matrix)[0]
+        kind = self.ACTIVATIONS[activation]
+        if (tiled is not None and x.dtype == torch.bfloat16 and not self.plain_products and self.many_rows == "own" and K % 8 == 0 and M > 0
+                and K == _shape_of(matrix)[1] and not self.separate_activations):
+            self._want(x, "linear input")
+            table, ids, width, vocab = None, None, 0, 0
+            if token is not None:
+                table, at, ids = token
+                self._want(table, "tokens' vectors", torch.bfloat16)
+                self._want(ids, "token ids", torch.int32)
+                if ids.numel() < M or at < 0 or at + N > table.shape[1]:
+                    raise KernelError("a token's vector lies outside the table")
+                vocab, width = table.shape
+                table, ids = table.data_ptr() + 2 * at, ids.data_ptr()
+            unit = (kind, table, ids, width, vocab, self._stream())
+            y = torch.empty((M, N), dtype=torch.bfloat16, device=self.device)
+            if M < self.MID_ROWS_FROM:
+                self._call(self.lib.tli_gemm_skinny_unit_bf16, x.data_ptr(), tiled.data_ptr(), y.data_ptr(), M, N, K, *unit)
+                return y
+            mid = M <= self.MID_ROWS_TO
+            splits = int(self.lib.tli_gemm_mid_splits_rows(M, N, K, 0)) if mid else int(self.lib.tli_gemm_rows_splits(M, N, K))
+            if mid and splits == 1:
+                self._call(self.lib.tli_gemm_mid_unit_bf16, x.data_ptr(), tiled.data_ptr(), y.data_ptr(), M, N, K, *unit)
+                return y
+            if splits > 1:
+                product = self._linear_mid(x, tiled, y, M, N, K, 0, True) if mid else self._linear_rows(x, tiled, y, M, N, K, 0, True)
+                if isinstance(product, DeferredSum):
+                    self._call(self.lib.tli_gemm_reduce_unit_bf16, product.parts.data_ptr(), y.data_ptr(), M, N, product.parts.shape[0], *unit)
+                    return y
+                z = product
+            else:
+                z = self._linear_rows(x, tiled, y, M, N, K, 0)
+        else:
+            z = self.linear(x, matrix)
+        return self.activation(z, activation) if token is None else self.token_gate(z, token[0], token[1], token[2], activation)
+
     def softcap(self, logits: torch.Tensor, cap: float) -> torch.Tensor:
         """logits <- cap * tanh(logits / cap), in place (float32)."""
         self._want(logits, "logits", torch.float32)
@@ -1401,6 +1448,8 @@ class HipOps:
     def norm_add(self, resid, y, weight, eps, out_dtype):
         """resid (float32 [T, n]) += weight * y / sqrt(mean(y^2) + eps) with ``y`` [T, n] in the run's type (or an
         unfinished product); returns the new residual's rows in the run's type (the residual itself in a float32 run)."""
+        if isinstance(y, DeferredSum) and y.dtype == out_dtype == torch.bfloat16 and resid.shape[1] <= 8192:
+            return self._norm_add_norm(resid, y, weight, eps, None, 0.0, out_dtype, None, None, None, None)
         y = self.resolve(y)
         total, n = resid.shape
         self._want(resid, "residual", torch.float32)
@@ -1428,10 +1477,16 @@ class HipOps:
     def _norm_add_norm(self, resid, y, w_out, eps_out, w_in, eps_in, out_dtype, rows, num_rows, mixes, step):
         total, n = resid.shape
         self._want(resid, "residual", torch.float32)
-        self._want(w_in, "norm weight", torch.float32, (n,))
+        if w_in is not None:
+            self._want(w_in, "norm weight", torch.float32, (n,))
+        parts = 0
         if y is not None:
-            y = self.resolve(y)
-            self._want(y, "sublayer output", out_dtype, (total, n))
+            if isinstance(y, DeferredSum) and y.dtype == out_dtype == torch.bfloat16:
+                y, parts = y.parts, y.parts.shape[0]
+                self._want(y, "partial sums of a sublayer's output", torch.float32, (parts, total, n))
+            else:
+                y = self.resolve(y)
+                self._want(y, "sublayer output", out_dtype, (total, n))
             self._want(w_out, "norm weight", torch.float32, (n,))
         count = total
         if rows is not None:
@@ -1446,8 +1501,8 @@ class HipOps:
             self._check_mixes(mu, kept, step, total, n, out_dtype)
             slots, starts = step.slots.data_ptr(), step.seq_start.data_ptr()
         out = torch.empty((count, n) if mixes is None else (m, count, n), dtype=out_dtype, device=self.device)
-        self._call(self.lib.tli_norm_add_norm, resid.data_ptr(), _ptr(y), None if y is None else w_out.data_ptr(), float(eps_out),
-                   w_in.data_ptr(), float(eps_in), out.data_ptr(), _ptr(rows), count, n, _ptr(mu), m, _ptr(kept), slots, starts,
+        self._call(self.lib.tli_norm_add_norm, resid.data_ptr(), _ptr(y), parts, total, None if y is None else w_out.data_ptr(),
+                   float(eps_out), _ptr(w_in), float(eps_in), out.data_ptr(), _ptr(rows), count, n, _ptr(mu), m, _ptr(kept), slots, starts,
                    _dtype_code(out_dtype), self._stream())
         return out
 

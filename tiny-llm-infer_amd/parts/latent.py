@@ -147,7 +147,7 @@ class LatentAttention(Mixer):
         o = ops.latent_attention(query, q_at, own, step, step.cache, self.heads, self.dim, self.rot, self.rank, self.vdim,
                                  self.rotary, self.scale, self.w_qk, self.w_v, window=self.window, sinks=self.sinks,
                                  gate=(proj, self.at["gate"]) if self.gated else None)
-        return ops.linear(o, self.w_o)
+        return ops.linear(o, self.w_o, deferred=True)
 
 
 register_part("mixer", "latent_attention", LatentAttention)

@@ -74,7 +74,7 @@ class DenseFF(FeedForward):
 
     def forward(self, x: torch.Tensor, step: StepView) -> torch.Tensor:
         ops = self.env.ops
-        return ops.linear(ops.activation(ops.linear(x, self.w_up), self.activation), self.w_down, deferred=True)
+        return ops.linear(ops.linear_act(x, self.w_up, self.activation), self.w_down, deferred=True)
 
 
 register_part("ffn", "swiglu", SwiGLU)

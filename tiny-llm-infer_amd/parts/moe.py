@@ -141,7 +141,7 @@ class RoutedExperts(FeedForward):
         shared = None
         if self.shared_inter is not None:
             if not self.gated:
-                hidden = ops.activation(ops.linear(x, self.shared_gate_up), self.activation)
+                hidden = ops.linear_act(x, self.shared_gate_up, self.activation)
             elif self.activation == "silu":
                 hidden = ops.linear_swiglu(x, self.shared_gate_up)
             else:

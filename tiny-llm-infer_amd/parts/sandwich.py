@@ -65,7 +65,7 @@ class TokenSide(Part):
     def forward(self, x: torch.Tensor, step: StepView):
         """x: the residual's rows in the run's type; returns y, not normed."""
         ops = self.env.ops
-        z = ops.token_gate(ops.linear(x, self.w_gate), self.table, self.at, step.token_ids, self.activation)
+        z = ops.linear_act(x, self.w_gate, self.activation, token=(self.table, self.at, step.token_ids))
         return ops.linear(z, self.w_proj, deferred=True)
 
 
