@@ -634,7 +634,7 @@ class HipOps:
             return y, y.data_ptr(), cols
         y, at = into
         self._want(y, "shared rows of outputs", dtype)
-        if y.dim() != 2 or y.shape[0] != rows or at < 0 or at % 8 or at + cols > y.shape[1] or y.shape[1] % 8:
+        if y.dim() != 2 or y.shape[0] != rows or at < 0 or at % 8 or at + cols > y.shape[1] or (y.shape[1] % 8 and cols != y.shape[1]):
             raise KernelError(f"{cols} columns from {at} on (a multiple of 8) do not fit shared rows of shape {tuple(y.shape)}")
         return y, y.data_ptr() + at * y.element_size(), y.shape[1]
 
@@ -2107,8 +2107,11 @@ class HipOps:
             raise KernelError("the gate lies outside the projections")
         rank = w2.shape[1]
         z_row, z_col = z_strides
-        if z.dtype != torch.float32 or z.device.type != "cuda" or tuple(z.shape) not in ((T, rank), (rank, T)) \
-                or tuple(z.stride()) not in ((z_row, z_col), (z_col, z_row)):
+
+        def lies(shape, strides):            # (the distance of a dimension of one element says nothing)
+            return tuple(z.shape) == shape and all(n == 1 or a == b for n, a, b in zip(shape, z.stride(), strides))
+        if z.dtype != torch.float32 or z.device.type != "cuda" \
+                or not (lies((T, rank), (z_row, z_col)) or lies((rank, T), (z_col, z_row))):
             raise KernelError(f"the decays' inner rows have shape {tuple(z.shape)} and strides {tuple(z.stride())}, not {rank} a row")
         self._want(w2, "decays' matrix", out_dtype, (heads * dk, rank))
         self._want(w0, "decays' bias", torch.float32, (heads * dk,))
