@@ -239,6 +239,10 @@ class CpuOps:
         w = w / (w.sum(-1, keepdim=True) + 1e-20) * scale if normalize else w * scale
         return ids.to(torch.int32), w, (torch.sigmoid(z[:, experts]) if has_shared else None)
 
+    def router(self, x, w_rows, experts, top, groups, keep, scale, has_shared, **how):
+        z, transposed = self.small_product(x, w_rows)
+        return self.route_experts(z, experts, top, groups, keep, scale, has_shared, transposed, **how)
+
     def apply_experts(self, x, ids, weights, w_gate_up, w_down, packed, shared, shared_gate, limit=0.0, slope=1.0,
                       activation=None, weight_on_input=False):
         T, n = x.shape

@@ -303,6 +303,31 @@ def test_activations_and_tokens_vectors_where_sums_are_written(ops, rows, n, out
                 ops.separate_activations = False
 
 
+# ---------------------------------------------------------------------------- the router ---
+@pytest.mark.parametrize("experts, top, groups, keep", [(16, 1, 1, 1), (6, 2, 1, 1), (64, 6, 8, 3), (130, 5, 10, 2), (256, 32, 1, 1), (3, 3, 1, 1), (48, 2, 48, 2)])
+@pytest.mark.parametrize("score, group_score, normalize", [("sigmoid", "top2", False), ("sigmoid", "top2", True), ("softmax", "max", False)])
+@pytest.mark.parametrize("corrected, shared", [(False, True), (True, False)])
+def test_a_router_in_one_launch_chooses_as_the_one_in_two(ops, experts, top, groups, keep, score, group_score, normalize, corrected, shared):
+    """Small whole numbers, so that logits are exact in any order and many scores are equal: ties go to the lower index."""
+    g = torch.Generator().manual_seed(experts + top)
+    n = 72
+    for rows in (1, 5, 128):
+        x = torch.randint(-1, 2, (rows, n), generator=g).to(torch.bfloat16).cuda()
+        w = (torch.randint(-1, 2, (experts + shared, n), generator=g) * 0.25).to(torch.bfloat16).cuda()
+        correction = torch.randint(-2, 3, (experts,), generator=g).float().cuda() * 0.125 if corrected else None
+        how = dict(score=score, group_score=group_score, normalize=normalize, correction=correction)
+        ids, weights, gate = ops.router(x, w, experts, top, groups, keep, 1.5, shared, **how)
+        z = (x.double() @ w.double().t()).float().contiguous()
+        ids2, weights2, gate2 = ops.route_experts(z, experts, top, groups, keep, 1.5, shared, False, **how)
+        assert torch.equal(ids, ids2)
+        _close(weights, weights2.cpu(), 5e-6, "weights")
+        if shared:
+            _close(gate, gate2.cpu(), 1e-6, "gate of the shared expert")
+        s = torch.sigmoid(z[:, :experts].double()) if score == "sigmoid" else torch.softmax(z[:, :experts].double(), dim=-1)
+        chosen = s.gather(1, ids.long()).cpu()
+        _close(weights, (chosen / (chosen.sum(-1, keepdim=True) + 1e-20) if normalize else chosen) * 1.5, 1e-5, "weights of the chosen")
+
+
 # --------------------------------------------------------------- experts without a gate ---
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("rows", [1, 9, 130, 600])

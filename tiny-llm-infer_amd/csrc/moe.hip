@@ -9,6 +9,8 @@
 //          or s_j * scale without that division.  One more logit behind the E, if present, is the gate of
 //          a shared expert: sigmoid of it.  Ids from `experts` on (see the kernels below) are experts that
 //          hand their input on: they have no matrices.
+//          Two kernels: from logits, a thread a row; and, for few rows of bfloat16, a workgroup a row that makes the
+//          logits itself (float32 sums) and chooses with one wave.
 // hidden:  for the pair (row, chosen expert e): a_f = silu(x . Wg_e[f]) * (x . Wu_e[f]), or the limited form of
 //          common.h's gated_unit (limit > 0); or, of experts without a gate, a_f = act(x . Wu_e[f]), the weight
 //          multiplied in before the activation where it belongs on the expert's input (common.h's ExpertUnit)
@@ -88,6 +90,100 @@ __global__ void moe_route_kernel(const float* __restrict__ z, long long z_row, l
         ids[(size_t)t * top + n] = chosen[n];
         weights[(size_t)t * top + n] = s[chosen[n]] * norm;
     }
+}
+
+// The largest of the lanes' values, ties to the lower index; every lane gets both.  (index < 0: the lane has none)
+__device__ __forceinline__ void wave_best(float& v, int& index) {
+#pragma unroll
+    for (int off = TLI_WAVE / 2; off > 0; off >>= 1) {
+        const float ov = __shfl_xor(v, off, TLI_WAVE);
+        const int oi = __shfl_xor(index, off, TLI_WAVE);
+        if (oi >= 0 && (index < 0 || ov > v || (ov == v && oi < index))) v = ov, index = oi;
+    }
+}
+
+#define ROUTER_THREADS 1024
+__global__ __launch_bounds__(ROUTER_THREADS) void moe_router_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, int D,
+                                                                    int* __restrict__ ids, float* __restrict__ weights,
+                                                                    float* __restrict__ shared_gate, int E, int top, int groups,
+                                                                    int keep, float scale, int has_shared, int softmax_scores,
+                                                                    int group_by_max, int normalize, const float* __restrict__ correction) {
+    extern __shared__ float rt_lds[];              // the row's logits [E + 1], then its scores; then the choice scores [E]
+    float* s = rt_lds;
+    float* c = rt_lds + E + 1;
+    const size_t t = blockIdx.x;
+    const int lane = threadIdx.x % TLI_WAVE, wave = threadIdx.x / TLI_WAVE;
+    const bf16_t* xr = x + t * D;
+    for (int e = wave; e < E + (has_shared ? 1 : 0); e += ROUTER_THREADS / TLI_WAVE) {
+        const bf16_t* we = w + (size_t)e * D;
+        float a = 0.f;
+#pragma unroll 4
+        for (int i = lane * 8; i < D; i += TLI_WAVE * 8) {
+            const uint4 p = *reinterpret_cast<const uint4*>(xr + i), q = *reinterpret_cast<const uint4*>(we + i);
+            const uint32_t u[4] = {p.x, p.y, p.z, p.w}, v[4] = {q.x, q.y, q.z, q.w};
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                a = fmaf(__uint_as_float(u[k] << 16), __uint_as_float(v[k] << 16), a);
+                a = fmaf(__uint_as_float(u[k] & 0xFFFF0000u), __uint_as_float(v[k] & 0xFFFF0000u), a);
+            }
+        }
+        a = wave_sum(a);
+        if (lane == 0) s[e] = a;
+    }
+    __syncthreads();
+    if (wave > 0) return;
+    if (has_shared && lane == 0) shared_gate[t] = 1.0f / (1.0f + expf(-s[E]));
+    if (softmax_scores) {
+        float top_z = -INFINITY, sum = 0.f;
+        for (int e = lane; e < E; e += TLI_WAVE) top_z = fmaxf(top_z, s[e]);
+        top_z = wave_max(top_z);
+        for (int e = lane; e < E; e += TLI_WAVE) {
+            s[e] = expf(s[e] - top_z);
+            sum += s[e];
+        }
+        sum = wave_sum(sum);
+        for (int e = lane; e < E; e += TLI_WAVE) s[e] /= sum;
+    } else {
+        for (int e = lane; e < E; e += TLI_WAVE) s[e] = 1.0f / (1.0f + expf(-s[e]));
+    }
+    for (int e = lane; e < E; e += TLI_WAVE) c[e] = correction ? s[e] + correction[e] : s[e];
+    wave_lds_sync();
+    const int per = E / groups;
+    unsigned long long open = ~0ull;               // the `keep` best groups, a bit each (groups <= 64: one a lane)
+    if (keep < groups) {
+        open = 0ull;
+        float a = -INFINITY, b = -INFINITY;        // the two largest of this lane's group
+        if (lane < groups)
+            for (int e = lane * per; e < (lane + 1) * per; ++e) {
+                const float v = c[e];
+                if (v > a) { b = a; a = v; }
+                else if (v > b) b = v;
+            }
+        const float score = (b > -INFINITY && !group_by_max) ? a + b : a;
+        for (int n = 0; n < keep; ++n) {
+            float v = score;
+            int g = lane < groups && !((open >> lane) & 1ull) ? lane : -1;
+            wave_best(v, g);
+            if (g >= 0) open |= 1ull << g;
+        }
+    }
+    uint32_t taken = 0u;                           // of this lane's experts lane, lane + 64, .. (E <= 2048)
+    float total = 0.f, mine = 0.f;                 // the weight of this lane's place in the choice (top <= 32)
+    for (int n = 0; n < top; ++n) {
+        float v = -INFINITY;
+        int best = -1;
+        for (int e = lane, k = 0; e < E; e += TLI_WAVE, ++k)
+            if (!((taken >> k) & 1u) && ((open >> (e / per)) & 1ull) && (best < 0 || c[e] > v)) v = c[e], best = e;
+        wave_best(v, best);
+        if (best < 0) best = 0;                    // (not with sizes that the host lets through)
+        if (best % TLI_WAVE == lane) taken |= 1u << (best / TLI_WAVE);
+        total += s[best];
+        if (lane == n) {
+            mine = s[best];
+            ids[t * top + n] = best;
+        }
+    }
+    if (lane < top) weights[t * top + lane] = mine * (normalize ? scale / (total + 1e-20f) : scale);
 }
 
 // one workgroup a pair; a wave takes every (waves)th hidden unit, its lanes share out k
@@ -175,6 +271,22 @@ extern "C" int tli_moe_route(const float* z, long long z_row, long long z_col, i
                        (size_t)threads * (2 * E + 1) * sizeof(float), (hipStream_t)stream, z, z_row, z_col, ids, weights, shared_gate,
                        T, E, top, groups, keep, scale, has_shared, softmax_scores, group_by_max, normalize, correction);
     return tli_check_launch("moe_route");
+}
+
+// x [T, D], w [E (+ 1), D] bfloat16: the product and the choice of tli_moe_route in one launch, a workgroup a row
+extern "C" int tli_moe_router_bf16(const void* x, const void* w, int D, int* ids, float* weights, float* shared_gate, int T, int E, int top,
+                                   int groups, int keep, float scale, int has_shared, int softmax_scores, int group_by_max,
+                                   int normalize, const float* correction, void* stream) {
+    if (T <= 0) return 0;
+    if (E <= 0 || E > 2048 || top <= 0 || top > E || top > MOE_MAX_TOP || groups <= 0 || groups > 64 || E % groups || keep <= 0 ||
+        keep > groups || (long long)keep * (E / groups) < top || D <= 0 || D % 8)
+        return tli_fail("moe_router: bad sizes (experts %d, top %d (at most %d), groups %d (at most 64), keep %d, width %d)", E, top,
+                        MOE_MAX_TOP, groups, keep, D);
+    if (((uintptr_t)x | (uintptr_t)w) & 15) return tli_fail("moe_router: operands must be 16-byte aligned");
+    moe_router_kernel<<<T, ROUTER_THREADS, (size_t)(2 * E + 1) * sizeof(float), (hipStream_t)stream>>>(
+        (const bf16_t*)x, (const bf16_t*)w, D, ids, weights, shared_gate, E, top, groups, keep, scale, has_shared, softmax_scores,
+        group_by_max, normalize, correction);
+    return tli_check_launch("moe_router");
 }
 
 // x [T, D]; ids, weights [T, top]; w_gu [E, 2 ff, D] (an expert's gate rows, then its up rows), or [E, ff, D] (up rows)

@@ -113,6 +113,7 @@ def load_library():
         "tli_delta_state_floats": [I, I],
         "tli_gated_rmsnorm": [P, P, I, P, P, I, I, I, F, I, P],
         "tli_moe_route": [P, ctypes.c_longlong, ctypes.c_longlong, P, P, P, I, I, I, I, I, F, I, I, I, I, P, P],
+        "tli_moe_router_bf16": [P, P, I, P, P, P, I, I, I, I, I, F, I, I, I, I, P, P],
         "tli_moe_experts": [P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, F, I, I, P],
         "tli_norm_add": [P, P, P, P, I, I, F, I, P],
         "tli_residual_rows": [P, P, ctypes.c_longlong, P],
@@ -1355,6 +1356,28 @@ class HipOps:
         weights = torch.empty((T, top), dtype=torch.float32, device=self.device)
         gate = torch.empty((T,), dtype=torch.float32, device=self.device) if has_shared else None
         self._call(self.lib.tli_moe_route, z.data_ptr(), z_row, z_col, ids.data_ptr(), weights.data_ptr(), _ptr(gate), T,
+                   experts, top, groups, keep, float(scale), 1 if has_shared else 0, self.ROUTER_SCORES.index(score),
+                   self.ROUTER_GROUP_SCORES.index(group_score), 1 if normalize else 0, _ptr(correction), self._stream())
+        return ids, weights, gate
+
+    ROUTER_ROWS = 128            # up to so many rows the router's product and its choice are one launch
+
+    def router(self, x, w_rows, experts, top, groups, keep, scale, has_shared, score="sigmoid", group_score="top2", normalize=True,
+               correction=None):
+        """``route_experts`` of the logits x w_rows^T (float32 sums); ``w_rows`` [E (+ 1), n]."""
+        T, n = x.shape
+        if x.dtype != torch.bfloat16 or n % 8 or not 0 < T <= self.ROUTER_ROWS or self.plain_products:
+            z, transposed = self.small_product(x, w_rows)
+            return self.route_experts(z, experts, top, groups, keep, scale, has_shared, transposed, score, group_score, normalize, correction)
+        self.check_router(score, group_score)
+        self._want(x, "router input")
+        self._want(w_rows, "router rows", torch.bfloat16, (experts + (1 if has_shared else 0), n))
+        if correction is not None:
+            self._want(correction, "router correction", torch.float32, (experts,))
+        ids = torch.empty((T, top), dtype=torch.int32, device=self.device)
+        weights = torch.empty((T, top), dtype=torch.float32, device=self.device)
+        gate = torch.empty((T,), dtype=torch.float32, device=self.device) if has_shared else None
+        self._call(self.lib.tli_moe_router_bf16, x.data_ptr(), w_rows.data_ptr(), n, ids.data_ptr(), weights.data_ptr(), _ptr(gate), T,
                    experts, top, groups, keep, float(scale), 1 if has_shared else 0, self.ROUTER_SCORES.index(score),
                    self.ROUTER_GROUP_SCORES.index(group_score), 1 if normalize else 0, _ptr(correction), self._stream())
         return ids, weights, gate

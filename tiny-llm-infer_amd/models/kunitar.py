@@ -60,7 +60,7 @@ def kunitar_spec(cfg: KunitarConfig) -> ModelSpec:
     def feed_forward(i: int) -> PartSpec:
         f, p = cfg.layers[i].mlp, f"l{i}.mlp."
         if isinstance(f, KunitarDense):
-            return PartSpec("dense_act", {"hidden_size": cfg.width, "intermediate_size": f.ff, "activation": "gelu"},
+            return PartSpec("dense_act", {"hidden_size": cfg.width, "intermediate_size": f.ff, "activation": "gelu", "on_sums": True},
                             {"up": p + "up", "down": p + "down"})
         names = {"router": p + "router", "experts": p + "e{}."}
         if f.shared_ff is not None:

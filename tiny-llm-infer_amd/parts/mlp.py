@@ -48,7 +48,8 @@ class SwiGLU(FeedForward):
 
 class DenseFF(FeedForward):
     """Dense feed-forward without a gate: down( act(up(x)) ).  ``activation`` names the
-    function, one of the kernel library's ``ACTIVATIONS`` ("relu2" is relu(z)^2)."""
+    function, one of the kernel library's ``ACTIVATIONS`` ("relu2" is relu(z)^2).  ``on_sums``: it is taken
+    of the product's float32 sums, where the product's kernel can, and not of their rounding."""
     replayable = True
 
     def __init__(self, spec):
@@ -56,6 +57,7 @@ class DenseFF(FeedForward):
         self.hidden = int(spec.params["hidden_size"])
         self.inter = int(spec.params["intermediate_size"])
         self.activation = str(spec.params["activation"])
+        self.on_sums = bool(spec.params.get("on_sums", False))
 
     def tensors(self) -> List[TensorDecl]:
         n = self.spec.names
@@ -74,7 +76,11 @@ class DenseFF(FeedForward):
 
     def forward(self, x: torch.Tensor, step: StepView) -> torch.Tensor:
         ops = self.env.ops
-        return ops.linear(ops.linear_act(x, self.w_up, self.activation), self.w_down, deferred=True)
+        if self.on_sums:
+            hidden = ops.linear_act(x, self.w_up, self.activation)
+        else:
+            hidden = ops.activation(ops.linear(x, self.w_up), self.activation)
+        return ops.linear(hidden, self.w_down, deferred=True)
 
 
 register_part("ffn", "swiglu", SwiGLU)

@@ -132,12 +132,11 @@ class RoutedExperts(FeedForward):
 
     def forward(self, x: torch.Tensor, step: StepView):
         ops = self.env.ops
-        z, transposed = ops.small_product(x, self.w_router)
         how = {}
         if (self.score, self.group_score, self.normalize, self.correction) != ("sigmoid", "top2", True, None):
             how = dict(score=self.score, group_score=self.group_score, normalize=self.normalize, correction=self.correction)
-        ids, weights, shared_gate = ops.route_experts(z, self.outputs, self.top, self.groups, self.keep, self.scale,
-                                                      self.has_gate, transposed, **how)
+        ids, weights, shared_gate = ops.router(x, self.w_router, self.outputs, self.top, self.groups, self.keep, self.scale,
+                                               self.has_gate, **how)
         shared = None
         if self.shared_inter is not None:
             if not self.gated:
