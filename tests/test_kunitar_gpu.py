@@ -361,7 +361,7 @@ def test_experts_without_a_gate(ops, dtype, rows, experts, top, n, ff, shared):
 # ------------------------------------------------- a window over cached latent vectors ---
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("heads, dim, rot, rank, vdim, page", [(4, 16, 16, 32, 24, 16), (8, 64, 16, 128, 80, 16), (3, 12, 6, 18, 10, 8), (20, 32, 32, 64, 32, 32)])
-def test_one_key_at_every_edge_of_the_window(ops, dtype, heads, dim, rot, rank, vdim, page):
+def test_one_key_at_every_edge_of_the_window(ops, dtype, heads, dim, rot, rank, vdim, page, monkeypatch):
     """A layer that reads vectors which another has cached: one key stands out and is placed just inside and just outside the
     window, at pages' borders and at the first position; rows decoded alone and in portions; one gate a head."""
     from tiny_llm_infer_amd.parts.base import GroupView, LayerCache
@@ -394,12 +394,45 @@ def test_one_key_at_every_edge_of_the_window(ops, dtype, heads, dim, rot, rank, 
             for first in (i, max(0, i - 13)):                                          # alone, and as the last row of a portion
                 step = _view([first], [i + 1 - first], [0])
                 rows = slice(first, i + 1)
-                got = ops.latent_attention(query[rows].cuda(), 0, None, step, LayerCache(group, 0, False), heads, dim, rot, rank, vdim,
-                                           (cos, sin, rot), scale, w_qk.cuda(), w_v.cuda(), window=size, gate=(gates[rows].cuda(), 2))
                 kd = keys.double()[:, None, :].expand(n, heads, key)
-                want = plain_kunitar.windowed(q_lat, kd, kd[..., :rank], scale, size)[i]
+                want = plain_kunitar.windowed(q_lat[:i + 1], kd[:i + 1], kd[:i + 1, :, :rank], scale, size)[i]
                 want = torch.einsum("hn,hen->he", want, w_v.double()) * torch.sigmoid(gates[i, 2:2 + heads].double())[:, None]
-                _close(got[-1], want.reshape(-1), 1e-5 if dtype == "float32" else 2.5e-2, f"row {i}, key {j}, window {size}, from {first}")
+                for splits in ((None, 1, 3, 64) if first == i else (None,)):           # workgroups that share out a decoded row's keys
+                    monkeypatch.setattr(ops, "sized_splits", splits)
+                    got = ops.latent_attention(query[rows].cuda(), 0, None, step, LayerCache(group, 0, False), heads, dim, rot, rank, vdim,
+                                               (cos, sin, rot), scale, w_qk.cuda(), w_v.cuda(), window=size, gate=(gates[rows].cuda(), 2))
+                    _close(got[-1], want.reshape(-1), 1e-5 if dtype == "float32" else 2.5e-2,
+                           f"row {i}, key {j}, window {size}, from {first}, {splits} splits")
+
+
+@pytest.mark.parametrize("sinks", [False, True])
+@pytest.mark.parametrize("window, keep", [(None, 0), (50, 0), (70, 20)])
+def test_decoded_rows_whose_keys_are_shared_out(ops, sinks, window, keep, monkeypatch):
+    """Rows of unequal length at once, all heads over one cached vector a position: any number of workgroups a row gives what one
+    gives, kept first keys and sinks included."""
+    from tiny_llm_infer_amd.parts.base import GroupView
+    g = torch.Generator().manual_seed(4)
+    lengths, page, heads, key, value = [1, 16, 17, 200, 333], 16, 20, 96, 64
+    need = [-(-n // page) for n in lengths]
+    ids, width, at = torch.randperm(sum(need), generator=g).to(torch.int32), max(need), 0
+    tables = torch.full((len(lengths), width), -1, dtype=torch.int32)
+    for i, n in enumerate(need):
+        tables[i, :n] = ids[at:at + n]
+        at += n
+    kc = torch.randn(sum(need), 1, page, key, generator=g).to(torch.bfloat16).cuda()
+    q = torch.randn(len(lengths), heads, key, generator=g).to(torch.bfloat16).cuda()
+    group = GroupView(tensors={}, tables=tables.cuda(), table_width=width, page_size=page, window=window)
+    step = _view([n - 1 for n in lengths], [1] * len(lengths), range(len(lengths)))
+    extra = torch.randn(heads, generator=g).cuda() if sinks else None
+    outs = []
+    for splits in (1, 2, 5, 22, 64, None):
+        monkeypatch.setattr(ops, "sized_splits", splits)
+        outs.append(ops.sized_attention(q, step, group, kc, None, heads, 1, 1, key, value, 0.2, window, keep, torch.bfloat16, sinks=extra))
+    monkeypatch.setattr(ops, "force_plain", True)
+    plain = ops.sized_attention(q, step, group, kc, None, heads, 1, 1, key, value, 0.2, window, keep, torch.bfloat16, sinks=extra)
+    for y in outs:
+        _close(y, plain.cpu(), 2e-2, "against the plain kernel")
+        _close(y, outs[0].cpu(), 1e-2, "against one workgroup")
 
 
 # ------------------------------------------------------- one mixer alone, every cut ---

@@ -405,7 +405,9 @@ __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
     const bf16_t* __restrict__ v_cache, const int* __restrict__ row_start, const int* __restrict__ seq_start,
     int num_seqs, const int* __restrict__ tables, int table_width, int page_size, int num_pages, int heads,
     int kv_heads, int maps, int nk_arg, int nv_arg, float scale, int window, int keep_first, int grouped,
-    const float* __restrict__ sinks, PooledKeys pooled, int out_ld, float out_scale) {
+    const float* __restrict__ sinks, PooledKeys pooled, int out_ld, float out_scale, float* __restrict__ parts) {
+    // a row's tiles of keys may be shared out over gridDim.z workgroups, in runs; their sums go to `parts`
+    constexpr bool SPLITS = VKEY && !POOLED && sizeof(TO) == 2;
     const int nk = EXACT ? NKM : nk_arg, nv = EXACT ? NVM : nv_arg;
     const int DK = nk * 16, DV = nv * 16, LD = DK + ASM_PAD;
     const int pieces = 2 * nk;                                          // 16-byte pieces of one key
@@ -488,6 +490,12 @@ __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
     const int blocks_my = POOLED ? pooled_blocks_seen(qpos, window, pooled.pool) : 0;
     const int* block_table = POOLED ? pooled.tables + (size_t)seq * pooled.width : nullptr;
     const int n_tiles = n_tokens + (blocks_hi + 15) / 16;
+    int t_begin = 0, t_end = n_tiles;
+    if (SPLITS && parts) {
+        const int per = (n_tiles + (int)gridDim.z - 1) / (int)gridDim.z;
+        t_begin = min((int)blockIdx.z * per, n_tiles);
+        t_end = min(t_begin + per, n_tiles);
+    }
     auto is_block = [&](int i) { return POOLED && i >= n_tokens; };
     auto tile_key = [&](int i) {
         return is_block(i) ? 16 * (i - n_tokens) : i < n_main ? k_top - 16 * i : 16 * (i - n_main);
@@ -548,12 +556,14 @@ __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
         }
     };
 
-    fetch(0);
-    store(lds);
+    if (t_begin < t_end) {                                              // (the same for the whole workgroup)
+        fetch(t_begin);
+        store(lds + (size_t)(t_begin & 1) * buf_elems);
+    }
     __syncthreads();
-    for (int it = 0; it < n_tiles; ++it) {
+    for (int it = t_begin; it < t_end; ++it) {
         const int k0 = tile_key(it);
-        const bool more = it + 1 < n_tiles;
+        const bool more = it + 1 < t_end;
         if (more) fetch(it + 1);
         const bool block = is_block(it);
         const bf16_t* kt = lds + (size_t)(it & 1) * buf_elems;
@@ -617,6 +627,17 @@ __global__ __launch_bounds__(64 * WAVES) void attention_sized_shared_kernel(
         __syncthreads();                                // the next tile is written; this one is read by all
     }
     if (!stores || col >= live) return;
+    if (SPLITS && parts) {                              // the sums as they are, with m and l behind them
+        float* part = parts + (((size_t)row * units + unit) * gridDim.z + blockIdx.z) * (DV + 4);
+        if (grp == 0) {
+            part[DV] = m;
+            part[DV + 1] = l;
+        }
+#pragma unroll
+        for (int j = 0; j < NVM; ++j)
+            if (j < nv) asm_store4(part + j * 16 + grp * 4, acc[j], 1.0f);
+        return;
+    }
     float inv = l > 0.f ? 1.0f / l : 0.f;
     if (sinks) inv = asm_sink_factor(sinks[unit], m, l);
     inv *= out_scale;
@@ -667,7 +688,7 @@ static int run_sized_mfma(
         const int waves = (!grouped && !v_cache && !out_f32 && nk == 36 && nv == 32 && (long long)tiles * per_kv >= 8 * 512) ? 8 : 4;
         const long long wgs = ((long long)tiles * (grouped ? col_groups : per_kv) + waves - 1) / waves + num_seqs;
         if (wgs > 0x7fffffffLL || kv_heads * maps > 65535) return tli_fail("attention: too many tiles for one launch");
-        const dim3 sgrid((unsigned)wgs, (unsigned)(kv_heads * maps));
+        const dim3 sgrid((unsigned)wgs, (unsigned)(kv_heads * maps), (unsigned)splits);
         const size_t sbytes = ast_lds_bytes(key_dim, value_dim);
 #define AST_ONE(NKM, NVM, VKEY, TO, EXACT, WAVES) AST_RUN(NKM, NVM, VKEY, TO, EXACT, WAVES, false)
 #define AST_RUN(NKM, NVM, VKEY, TO, EXACT, WAVES, POOLED)                                                                  \
@@ -682,7 +703,7 @@ static int run_sized_mfma(
         }                                                                                                                  \
         kernel<<<sgrid, 64 * WAVES, sbytes, s>>>((const bf16_t*)q, (TO*)out, (const bf16_t*)k_cache, (const bf16_t*)v_cache,      \
                                           row_start, seq_start, num_seqs, tables, table_width, page_size, num_pages,      \
-                                          heads, kv_heads, maps, nk, nv, scale, window, keep_first, grouped, sinks, pooled, out_ld, out_scale); \
+                                          heads, kv_heads, maps, nk, nv, scale, window, keep_first, grouped, sinks, pooled, out_ld, out_scale, splits > 1 ? parts : nullptr); \
     }
 #define AST_SIZES(VKEY, TO)                                                   \
     if (nk <= 8 && nv <= 8) AST_ONE(8, 8, VKEY, TO, false, 4)                 \
@@ -758,14 +779,24 @@ static int run_sized_mfma(
 // tiles: an upper bound of the sum over the sequences of ceil(rows / 16) (of the rows, with `grouped`);
 // grouped: a tile is one row and its columns are the query heads of one key head, 16 at a time;
 // sinks: float32 [heads * maps] or null
+// splits: with `grouped`, values that are the keys' first elements and bfloat16 outputs, a row's keys may be shared out over 2
+// to 64 workgroups, whose sums go to `parts` (float32, 16-byte aligned: [rows, heads * maps, splits, value_dim + 4]) and are put
+// together by a second launch; `tiles` is then the number of rows.  Else 1.
 extern "C" int tli_attention_sized_mfma_bf16(
     const void* q, void* out, const void* k_cache, const void* v_cache, const int* row_start, const int* seq_start,
     int num_seqs, int tiles, const int* tables, int table_width, int page_size, int num_pages, int heads, int kv_heads,
     int maps, int key_dim, int value_dim, float scale, int window, int keep_first, int grouped, int out_f32,
-    const float* sinks, void* stream) {
-    return run_sized_mfma(q, out, k_cache, v_cache, row_start, seq_start, num_seqs, tiles, tables, table_width, page_size,
+    const float* sinks, int splits, float* parts, void* stream) {
+    if (splits < 1 || splits > 64 || (splits > 1 && (!grouped || v_cache || out_f32 || !parts || ((uintptr_t)parts & 15))))
+        return tli_fail("attention: %d splits", splits);
+    const int rc = run_sized_mfma(q, out, k_cache, v_cache, row_start, seq_start, num_seqs, tiles, tables, table_width, page_size,
                           num_pages, heads, kv_heads, maps, key_dim, value_dim, scale, window, keep_first, grouped, out_f32, sinks,
-                          PooledKeys{}, heads * maps * value_dim, 1.0f, 1, nullptr, stream);
+                          PooledKeys{}, heads * maps * value_dim, 1.0f, splits, parts, stream);
+    if (rc || splits == 1 || num_seqs <= 0 || tiles <= 0) return rc;
+    const int pairs = tiles * heads * maps;
+    attention_parts_merge_kernel<<<(pairs + 3) / 4, 256, 0, (hipStream_t)stream>>>(parts, splits, pairs, heads * maps, value_dim, sinks,
+                                                                                   (bf16_t*)out, heads * maps * value_dim, 1.0f);
+    return tli_check_launch("attention_parts_merge");
 }
 
 // The same over a window and the pooled blocks before it (pooled.h; their caches hold kv_heads heads): one map, values of

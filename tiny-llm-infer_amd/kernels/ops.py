@@ -122,7 +122,7 @@ def load_library():
         "tli_head_products_mfma_takes": [I, I] + [ctypes.c_longlong] * 4,
         "tli_head_products_mfma_bf16": [P, ctypes.c_longlong, ctypes.c_longlong, P, P, ctypes.c_longlong, ctypes.c_longlong,
                                         I, I, I, I, P, I, P],
-        "tli_attention_sized_mfma_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, I, F, I, I, I, I, P, P],
+        "tli_attention_sized_mfma_bf16": [P, P, P, P, P, P, I, I, P, I, I, I, I, I, I, I, I, F, I, I, I, I, P, I, P, P],
         "tli_diff_prepare": [P, I, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P, F, I, P],
         "tli_diff_combine": [P, P, I, I, P, I, I, I, F, F, F, I, P],
         "tli_latent_prepare": [P, I, P, I, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P, F, P, P, I, P],
@@ -264,6 +264,7 @@ class HipOps:
         self.lightning_lanes = int(os.environ.get("TLI_LIGHTNING_LANES", "0"))   # measurements, tests: 16 or 64 lanes a column of the lightning recurrence's state (0: the launch rule)
         self.rows_splits = 0
         self.pooled_prefill = True       # measurements, tests: False sends portions of prompts over windows and pooled blocks through the kernels for sizes of their own
+        self.sized_splits = None         # measurements, tests: the same of a decoding row's cached vectors that all heads read (None: the rule)
         self.pooled_splits = None        # measurements, tests: into how many splits a decoding row's keys over windows and pooled blocks go (None: the rule)
         self.recurrence_in_chunks = True    # measurements, tests: False sends the portions of prompts of retention, mLSTM and wkv through the recurrence row by row
         self.separate_activations = False   # measurements, tests: True leaves the activations of products without a gate to a pass of their own
@@ -1607,10 +1608,16 @@ class HipOps:
             grouped = 1 if step.max_rows_per_seq == 1 else 0
             starts = step.h_row_start
             tiles = T if grouped else sum((starts[i + 1] - starts[i] + 15) // 16 for i in range(step.num_seqs))
+            splits, parts = 1, None
+            if grouped and vc is None and out_dtype == torch.bfloat16 and step.num_seqs == T:
+                splits = self._sized_splits(T, step.reach, heads * maps, kv_heads * maps, window, keep)
+                if splits > 1:
+                    parts = torch.empty((T * heads * maps * splits * (value_dim + 4),), dtype=torch.float32, device=self.device)
             self._call(self.lib.tli_attention_sized_mfma_bf16, q.data_ptr(), out.data_ptr(), kc.data_ptr(), _ptr(vc),
                        step.row_start.data_ptr(), step.seq_start.data_ptr(), step.num_seqs, tiles, g.tables.data_ptr(),
                        g.table_width, g.page_size, pages, heads, kv_heads, maps, key_dim, value_dim, float(scale),
-                       int(window or 0), keep, grouped, 1 if out_dtype == torch.float32 else 0, _ptr(sinks), self._stream())
+                       int(window or 0), keep, grouped, 1 if out_dtype == torch.float32 else 0, _ptr(sinks), splits, _ptr(parts),
+                       self._stream())
             return out
         self._call(self.lib.tli_attention_sized_plain, q.data_ptr(), out.data_ptr(), kc.data_ptr(), _ptr(vc),
                    step.positions.data_ptr(), step.seq_of_row.data_ptr(), g.tables.data_ptr(), g.table_width, g.page_size,
@@ -1649,6 +1656,17 @@ class HipOps:
         self._call(self.lib.tli_diff_combine, maps.data_ptr(), proj.data_ptr(), width, width - heads, out.data_ptr(), T,
                    heads, vdim, float(lam), float(after), float(norm_eps), _dtype_code(proj.dtype), self._stream())
         return out
+
+    SIZED_WORKGROUPS = 256           # decoding rows whose keys are shared out: the workgroups aimed at,
+    SIZED_SPLIT_KEYS = 32            # and the fewest keys of a split (two tiles of 16)
+
+    def _sized_splits(self, T, reach, units, key_heads, window, keep) -> int:
+        """Over how many workgroups the keys of one (row, key head) that decodes are shared out, where all heads read one cached
+        vector; ``reach``: a power of two that the longest sequence fits.  A workgroup takes a row's tiles of 16 keys one
+        after the other."""
+        keys = min(reach, (window + 15 if window else reach) + keep)
+        groups = T * key_heads * ((units // key_heads + 63) // 64)
+        return max(1, self.sized_splits or min(self.SIZED_WORKGROUPS // groups, keys // self.SIZED_SPLIT_KEYS, 64))
 
     def head_products(self, x, x_stride, w, out=None, out_stride=None, x_at=0, out_at=0, gate=None):
         """y[t, h, :] = w[h] x[t, h, :] for a matrix a head, ``w`` [heads, N, K].  ``x`` is [T, columns]: the input of
