@@ -364,15 +364,19 @@ __global__ __launch_bounds__(256) void attention_parts_merge_kernel(
     float inv = l > 0.f ? 1.0f / l : 0.f;
     if (sinks) inv = asm_sink_factor(sinks[head], mt, l);
     inv *= out_scale;
-    for (int d0 = 0; d0 < DV; d0 += 256) {              // (every lane stays in for the exchanges)
+    for (int d0 = blockIdx.y * 256; d0 < DV; d0 += 256 * gridDim.y) {              // (every lane stays in for the exchanges)
         const int d = d0 + lane * 4;
+        const float* src = mine + min(d, DV - 4);
         f32x4 a = (f32x4){0.f, 0.f, 0.f, 0.f};
-        for (int s = 0; s < splits; ++s) {
-            const float fs = __shfl(f, s);
-            if (d < DV) {
-                const f32x4 t = *reinterpret_cast<const f32x4*>(mine + (size_t)s * (DV + 4) + d);
+        for (int s = 0; s < splits; s += 8) {            // eight splits' sums on their way together
+            f32x4 t[8];
 #pragma unroll
-                for (int i = 0; i < 4; ++i) a[i] += t[i] * fs;
+            for (int k = 0; k < 8; ++k) t[k] = *reinterpret_cast<const f32x4*>(src + (size_t)min(s + k, splits - 1) * (DV + 4));
+#pragma unroll
+            for (int k = 0; k < 8; ++k) {
+                const float fs = s + k < splits ? __shfl(f, s + k) : 0.f;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) a[i] += t[k][i] * fs;
             }
         }
         if (d < DV) asm_store4(out + (size_t)row * out_ld + (size_t)head * DV + d, a, inv);
@@ -794,7 +798,7 @@ extern "C" int tli_attention_sized_mfma_bf16(
                           PooledKeys{}, heads * maps * value_dim, 1.0f, splits, parts, stream);
     if (rc || splits == 1 || num_seqs <= 0 || tiles <= 0) return rc;
     const int pairs = tiles * heads * maps;
-    attention_parts_merge_kernel<<<(pairs + 3) / 4, 256, 0, (hipStream_t)stream>>>(parts, splits, pairs, heads * maps, value_dim, sinks,
+    attention_parts_merge_kernel<<<dim3((pairs + 3) / 4, (value_dim + 255) / 256), 256, 0, (hipStream_t)stream>>>(parts, splits, pairs, heads * maps, value_dim, sinks,
                                                                                    (bf16_t*)out, heads * maps * value_dim, 1.0f);
     return tli_check_launch("attention_parts_merge");
 }
@@ -819,7 +823,7 @@ extern "C" int tli_attention_pooled_mfma_bf16(
                           PooledKeys{pooled_k, pooled_v, pooled_tables, pooled_width, pooled_pages, pool}, out_ld, out_scale, splits, parts, stream);
     if (rc || splits == 1 || num_seqs <= 0 || tiles <= 0) return rc;
     const int pairs = tiles * heads;
-    attention_parts_merge_kernel<<<(pairs + 3) / 4, 256, 0, (hipStream_t)stream>>>(parts, splits, pairs, heads, value_dim, sinks,
+    attention_parts_merge_kernel<<<dim3((pairs + 3) / 4, (value_dim + 255) / 256), 256, 0, (hipStream_t)stream>>>(parts, splits, pairs, heads, value_dim, sinks,
                                                                                    (bf16_t*)out, out_ld, out_scale);
     return tli_check_launch("attention_parts_merge");
 }
