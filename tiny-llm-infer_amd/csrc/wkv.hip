@@ -1,5 +1,5 @@
 // The RWKV's recurrence row by row: for the rows of one sequence, head by head (key size dk, value size dv),
-//   o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t,   S_t = diag(d_t) S_(t-1) + k_t v_t^T
+//   o_t = S_(t-1)^T r_t + (r_t . u k_t) v_t,   row c of S_t = d_t(c) (row c of S_(t-1)) + k_t(c) v_t
 // float32, S zero before position 0.  d_t = exp(-exp(W2 tanh(z_t) + w0)), a number a channel.
 //
 // wkv_decays:  d of a step's rows, [T, H dk].
